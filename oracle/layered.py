@@ -1,0 +1,119 @@
+"""Plain, slow restatement of the layered decoder models (test infrastructure), one function per
+mechanism, token by token where the mechanism is a recurrence.  numpy only; `dtype` is the type of
+every intermediate (float64 unless a caller wants otherwise).  Weights come as a dictionary
+name -> array, linear weights [out, in]."""
+import numpy as np
+
+UNIT_EPS = 1e-6
+
+
+def rms_norm(x, w, eps):
+    return x / np.sqrt(np.mean(x * x, axis=-1, keepdims=True) + eps) * w
+
+
+def silu(x):
+    return x / (1.0 + np.exp(-x))
+
+
+def sigmoid(x):
+    return 1.0 / (1.0 + np.exp(-x))
+
+
+def softplus(x):
+    return np.logaddexp(0.0, x)
+
+
+def unit(x):
+    return x / np.sqrt(np.sum(x * x, axis=-1, keepdims=True) + UNIT_EPS)
+
+
+def short_conv(x, taps):
+    """x [T, C], taps [C, K]: y[t, c] = silu(sum_j taps[c, j] x[t - (K - 1) + j, c]), zeros before 0."""
+    T, K = x.shape[0], taps.shape[1]
+    y = np.zeros_like(x)
+    for t in range(T):
+        for j in range(K):
+            s = t - (K - 1) + j
+            if s >= 0:
+                y[t] = y[t] + taps[:, j] * x[s]
+    return silu(y)
+
+
+def delta_rule(q, k, v, beta, decay, state=None):
+    """One head.  q, k [T, d], v [T, e], beta, decay [T]; state [d, e].  Returns (o [T, e], state)."""
+    S = np.zeros((q.shape[1], v.shape[1]), dtype=q.dtype) if state is None else state.copy()
+    out = np.zeros_like(v)
+    for t in range(q.shape[0]):
+        S = decay[t] * S
+        u = beta[t] * (v[t] - S.T @ k[t])
+        S = S + np.outer(k[t], u)
+        out[t] = S.T @ q[t]
+    return out, S
+
+
+def gated_delta_mixer(x, W, p, m, eps):
+    """x [T, width]; p = tensor prefix ('l0.mix'), m = the mixer's sizes."""
+    H, KH, d, e = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    T = x.shape[0]
+    q = short_conv(x @ W[p + ".q"].T, W[p + ".q.conv"]).reshape(T, KH, d)
+    k = short_conv(x @ W[p + ".k"].T, W[p + ".k.conv"]).reshape(T, KH, d)
+    v = short_conv(x @ W[p + ".v"].T, W[p + ".v.conv"]).reshape(T, H, e)
+    q, k = unit(q) * d ** -0.5, unit(k)
+    beta = sigmoid(x @ W[p + ".b"].T)
+    decay = np.exp(-np.exp(W[p + ".A_log"]) * softplus(x @ W[p + ".a"].T + W[p + ".dt_bias"]))
+    gate = silu(x @ W[p + ".g"].T).reshape(T, H, e)
+    o = np.zeros((T, H, e), dtype=x.dtype)
+    for h in range(H):
+        hk = h // (H // KH)
+        o[:, h], _ = delta_rule(q[:, hk], k[:, hk], v[:, h], beta[:, h], decay[:, h])
+    o = rms_norm(o, W[p + ".norm"], eps) * gate
+    return o.reshape(T, H * e) @ W[p + ".o"].T
+
+
+def masked_attention(q, k, v, scale, window):
+    """One head: q, k [T, d], v [T, e]; i sees j with 0 <= i - j < window (window None: all j <= i)."""
+    T = q.shape[0]
+    out = np.zeros((T, v.shape[1]), dtype=q.dtype)
+    for i in range(T):
+        lo = 0 if window is None else max(0, i - window + 1)
+        s = k[lo:i + 1] @ q[i] * scale
+        a = np.exp(s - s.max())
+        out[i] = (a / a.sum()) @ v[lo:i + 1]
+    return out
+
+
+def latent_attention_mixer(x, W, p, m, eps):
+    H, d, e, T = m["heads"], m["dim"], m["vdim"], x.shape[0]
+    cq = rms_norm(x @ W[p + ".dq"].T, W[p + ".dq.norm"], eps)
+    q = (cq @ W[p + ".uq"].T).reshape(T, H, d)
+    c = rms_norm(x @ W[p + ".dkv"].T, W[p + ".dkv.norm"], eps)
+    k = (c @ W[p + ".uk"].T).reshape(T, H, d)
+    v = (c @ W[p + ".uv"].T).reshape(T, H, e)
+    window = (m.get("mask") or {}).get("size")
+    o = np.stack([masked_attention(q[:, h], k[:, h], v[:, h], m["scale"], window) for h in range(H)], axis=1)
+    return o.reshape(T, H * e) @ W[p + ".o"].T
+
+
+def dense_ff(x, W, p):
+    return (silu(x @ W[p + ".gate"].T) * (x @ W[p + ".up"].T)) @ W[p + ".down"].T
+
+
+MIXERS = {"delta": gated_delta_mixer, "delta_2": gated_delta_mixer, "latent_attention": latent_attention_mixer}
+
+
+def forward(cfg, weights, tokens, dtype=np.float64, layers_out=None):
+    """Logits [T, vocab] of a "Bofirax" configuration; layers_out (a list) receives the residual stream
+    after every layer."""
+    W = {n: np.asarray(a, dtype=dtype) for n, a in weights.items()}
+    eps = dtype(cfg["norm"]["eps"])
+    x = W["embed"][np.asarray(tokens, dtype=np.int64)]
+    for i, layer in enumerate(cfg["layers"]):
+        p = f"l{i}"
+        y = MIXERS[layer["type"]](x, W, p + ".mix", layer["mixer"], eps)
+        x = x + rms_norm(y, W[p + ".norm1"], eps) * W[p + ".ls1"]
+        if layer["mlp"] is not None:
+            y = dense_ff(x, W, p + ".mlp")
+            x = x + rms_norm(y, W[p + ".norm2"], eps) * W[p + ".ls2"]
+        if layers_out is not None:
+            layers_out.append(x)
+    return rms_norm(x, W["final.norm"], eps) @ W["embed"].T
