@@ -39,6 +39,12 @@ class CConfig(C.Structure):
     ]
 
 
+class CLoadOptions(C.Structure):
+    """coeus_load_options: storage type and limits of a layered model."""
+
+    _fields_ = [("weight_dtype", C.c_uint32), ("max_seq_len", C.c_uint64), ("max_batch", C.c_uint64)]
+
+
 # name -> (restype, argtypes); this table is also what the symbol-export test walks
 _u64, _u32, _f32 = C.c_uint64, C.c_uint32, C.c_float
 _vp, _cfgp = C.c_void_p, C.POINTER(CConfig)
@@ -68,6 +74,10 @@ SIGNATURES = {
     "coeus_positional_encoding": (C.c_int, [_u64, _u64, _vp]),
     "coeus_model_create": (C.c_int, [_cfgp, _vp, _u64, C.POINTER(_vp)]),
     "coeus_model_create_seeded": (C.c_int, [_cfgp, _u64, C.POINTER(_vp)]),
+    "coeus_model_load": (C.c_int, [C.c_char_p, C.POINTER(CLoadOptions), C.POINTER(_vp)]),
+    "coeus_model_create_layered": (C.c_int, [C.c_char_p, _u64, C.POINTER(CLoadOptions), _u64, C.POINTER(_vp)]),
+    "coeus_layered_config_check": (C.c_int, [C.c_char_p, _u64, C.POINTER(_u64)]),
+    "coeus_layered_check": (C.c_int, [C.c_char_p, C.POINTER(_u64)]),
     "coeus_model_forward": (C.c_int, [_vp, _vp, _u64, _vp]),
     "coeus_model_forward_all": (C.c_int, [_vp, _vp, _u64, _vp]),
     "coeus_model_num_parameters": (_u64, [_vp]),
@@ -78,6 +88,7 @@ SIGNATURES = {
     "coeus_model_destroy": (None, [_vp]),
     "coeus_session_create": (C.c_int, [_vp, _u64, _u64, C.POINTER(_vp)]),
     "coeus_session_prefill": (C.c_int, [_vp, _vp, _u64, _vp]),
+    "coeus_session_feed": (C.c_int, [_vp, _vp, _u64, _vp, _u64, _vp, _vp]),
     "coeus_session_decode": (C.c_int, [_vp, _vp, _vp]),
     "coeus_session_decode_greedy": (C.c_int, [_vp, _vp, _u64, _vp]),
     "coeus_session_generate": (C.c_int, [_vp, _vp, _u64, _vp, _vp]),

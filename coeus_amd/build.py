@@ -76,9 +76,17 @@ def build(force=False, verbose=True):
     return LIB
 
 
-# The sources without device code (errors, configuration, parameter layout, .rustllm files, the
-# tokenizer): what the sanitizer build of the host logic is made of.
-HOST_ONLY = ["host.hip", "rustllm_file.hip", "bpe.hip"]
+def ensure_built():
+    """The library's path; compiles only if it is missing or older than a source."""
+    srcs = glob.glob(os.path.join(CSRC, "*.h*")) + [os.path.join(HERE, "..", "include", "coeus.h")]
+    if os.path.exists(LIB) and os.path.getmtime(LIB) >= max(os.path.getmtime(s) for s in srcs):
+        return LIB
+    return build(verbose=False)
+
+
+# The sources without device code (errors, configuration, parameter layout, .rustllm files, layered
+# configurations and their weight files, the tokenizer): what the sanitizer build of the host logic is made of.
+HOST_ONLY = ["host.hip", "rustllm_file.hip", "bpe.hip", "layered_config.hip", "safetensors.hip"]
 HOST_ASAN_LIB = os.path.join(OBJ, "libcoeus_host_asan.so")
 
 

@@ -130,6 +130,29 @@ int coeus_model_create_seeded(const coeus_config *cfg, uint64_t seed, coeus_mode
     return create_common(cfg, nullptr, 0, seed, out);
 }
 
+int coeus_model_load(const char *dir, const coeus_load_options *opt, coeus_model **out) {
+    COEUS_GUARD_BEGIN
+    if (!dir || !opt || !out) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    *out = nullptr;
+    Model *m = nullptr;
+    COEUS_TRY(layered_load(dir, *opt, &m));
+    *out = reinterpret_cast<coeus_model *>(m);
+    return COEUS_OK;
+    COEUS_GUARD_END
+}
+
+int coeus_model_create_layered(const char *json, uint64_t len, const coeus_load_options *opt, uint64_t seed,
+                               coeus_model **out) {
+    COEUS_GUARD_BEGIN
+    if (!json || !opt || !out) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    *out = nullptr;
+    Model *m = nullptr;
+    COEUS_TRY(layered_create_seeded(json, len, *opt, seed, &m));
+    *out = reinterpret_cast<coeus_model *>(m);
+    return COEUS_OK;
+    COEUS_GUARD_END
+}
+
 static Model *M(coeus_model *m) { return reinterpret_cast<Model *>(m); }
 static const Model *M(const coeus_model *m) { return reinterpret_cast<const Model *>(m); }
 static Session *S(coeus_session *s) { return reinterpret_cast<Session *>(s); }
@@ -150,7 +173,9 @@ int coeus_model_forward_all(coeus_model *m, const uint64_t *ids, uint64_t seq_le
 
 uint64_t coeus_model_num_parameters(const coeus_model *m) { return m ? M(m)->n_params : 0; }
 const coeus_config *coeus_model_config(const coeus_model *m) { return m ? &M(m)->cfg : nullptr; }
-const char *coeus_model_name(const coeus_model *m) { (void)m; return "TransformerModel"; }  // MT:782-784
+const char *coeus_model_name(const coeus_model *m) {  // MT:782-784
+    return m && M(m)->stack ? M(m)->stack->cfg.architecture.c_str() : "TransformerModel";
+}
 uint64_t coeus_model_weight_bytes(const coeus_model *m) { return m ? M(m)->weight_bytes : 0; }
 uint64_t coeus_model_resident_bytes(const coeus_model *m) {
     if (!m) return 0;
@@ -176,6 +201,14 @@ int coeus_session_prefill(coeus_session *s, const uint64_t *ids, uint64_t n, flo
     COEUS_GUARD_BEGIN
     if (!s) return fail(COEUS_INVALID_INPUT, "null session");
     return session_prefill(*S(s), ids, n, logits_out);
+    COEUS_GUARD_END
+}
+
+int coeus_session_feed(coeus_session *s, const uint64_t *ids, uint64_t n, const uint64_t *want, uint64_t n_want,
+                       float *logits_out, float *residuals_out) {
+    COEUS_GUARD_BEGIN
+    if (!s) return fail(COEUS_INVALID_INPUT, "null session");
+    return session_feed(*S(s), ids, n, want, n_want, logits_out, residuals_out);
     COEUS_GUARD_END
 }
 
@@ -253,9 +286,9 @@ uint64_t coeus_session_position(const coeus_session *s) {
 
 int coeus_session_reset(coeus_session *s) {
     if (!s) return fail(COEUS_INVALID_INPUT, "null session");
-    std::lock_guard<std::mutex> lock(S(s)->m->mu);
-    S(s)->pos = 0;
-    return COEUS_OK;
+    COEUS_GUARD_BEGIN
+    return session_reset(*S(s));
+    COEUS_GUARD_END
 }
 
 void coeus_session_destroy(coeus_session *s) { delete S(s); }

@@ -251,6 +251,13 @@ int launch_norm(uint32_t kind, uint32_t scope, const float *x, uint64_t rows, ui
                 const float *scale, const float *bias, float eps, float *y, __half *y_xq,
                 uint32_t bp, hipStream_t st, const LpOut *y_lp = nullptr, double *partials = nullptr);
 size_t norm_sequence_scratch_bytes();
+// h += RMSNorm(y; scale, eps) * ls (nullable: 1) row by row; h_lp (nullable) receives 16-bit rows of the new h
+int launch_norm_residual(const float *y, uint64_t rows, uint64_t hidden, const float *scale, const float *ls,
+                         float eps, float *h, hipStream_t st, const LpOut *h_lp = nullptr);
+// dst[i, :] = src[rows_dev[i], :] for i < count (row numbers are checked by the caller)
+int launch_gather_rows(const float *src, const uint64_t *rows_dev, uint64_t count, uint64_t hidden, float *dst,
+                       hipStream_t st);
+// pe nullable: no positional term
 int launch_embed(const void *table, bool table_bf16, const float *pe, const uint64_t *ids,
                  uint64_t rows, uint64_t rows_per_seq, uint64_t pos0, const uint32_t *pos_dev,
                  uint64_t hidden, float *x, float2 *stats, hipStream_t st, const float *g_scale = nullptr,

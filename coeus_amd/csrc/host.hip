@@ -1,7 +1,7 @@
 // Host-only part of libcoeus_mi355x.so: errors, Transformer250MConfig (default, validate),
 // the parameter layout, the sinusoidal table, and the extern "C" entry points that never touch
 // the device (configuration, .rustllm files, the reference's initialisation loop).  Together with
-// rustllm_file.hip and bpe.hip this file builds without any device code, which is what the
+// rustllm_file.hip, layered_config.hip, safetensors.hip and bpe.hip this file builds without any device code, which is what the
 // address / undefined-behaviour sanitizer build of the host logic links.
 #include "model.hpp"
 
@@ -200,6 +200,36 @@ int coeus_config_validate(const coeus_config *c) {
 
 uint64_t coeus_config_num_parameters(const coeus_config *c) { return c ? make_layout(*c).total_params : 0; }
 uint64_t coeus_config_used_parameters(const coeus_config *c) { return c ? make_layout(*c).used_params : 0; }
+
+// ---- layered models: configuration and weight files
+static uint64_t count_params(const LayeredConfig &c) {
+    uint64_t n = 0;
+    for (const TensorSpec &t : layered_tensors(c)) n += t.elems();
+    return n;
+}
+int coeus_layered_config_check(const char *json, uint64_t len, uint64_t *n_params_out) {
+    COEUS_GUARD_BEGIN
+    if (!json) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    LayeredConfig c;
+    COEUS_TRY(layered_config_parse(json, len, c));
+    if (n_params_out) *n_params_out = count_params(c);
+    return COEUS_OK;
+    COEUS_GUARD_END
+}
+int coeus_layered_check(const char *dir, uint64_t *n_params_out) {
+    COEUS_GUARD_BEGIN
+    if (!dir) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    std::string text;
+    LayeredConfig c;
+    COEUS_TRY(read_text_file(std::string(dir) + "/config.json", text));
+    COEUS_TRY(layered_config_parse(text.data(), text.size(), c));
+    SafeTensors file;
+    COEUS_TRY(file.open(std::string(dir) + "/model.safetensors"));
+    COEUS_TRY(check_tensors(file, layered_tensors(c)));
+    if (n_params_out) *n_params_out = count_params(c);
+    return COEUS_OK;
+    COEUS_GUARD_END
+}
 
 uint64_t coeus_rustllm_checksum(const float *params, uint64_t n) {
     return params || n == 0 ? rustllm_checksum(params, n) : 0;

@@ -78,14 +78,15 @@ void Workspace::release() {
     h.release(); x.release(); qkv.release(); att.release(); ff.release(); ids.release();
     a_lp.release(); b_lp.release(); w_lp.release(); logits.release(); xq.release(); norm_part.release();
     gemm_part.release();
+    mix.release(); lat.release(); q_lp.release(); kv_lp.release();
     rows = 0;
 }
 
 // ---------------------------------------------------------------- model construction
 Model::~Model() {
     for (auto &l : layers) { weight_free(l.qkv); weight_free(l.o); weight_free(l.up); weight_free(l.down); }
+    if (embed && embed != out.data) (void)hipFree(embed);  // (tied embeddings: one tensor)
     weight_free(out);
-    if (embed) (void)hipFree(embed);
     if (pe) (void)hipFree(pe);
     if (small) (void)hipFree(small);
     ws.release();
@@ -94,7 +95,7 @@ Model::~Model() {
     if (stream) (void)hipStreamDestroy(stream);
 }
 
-static int check_device() {
+int check_device() {
     int n = 0;
     hipError_t e = hipGetDeviceCount(&n);
     if (e != hipSuccess || n == 0)
@@ -268,8 +269,9 @@ int model_create(const coeus_config &cfg, const float *params, uint64_t n_params
 // ---------------------------------------------------------------- forward over rows (prefill path)
 // Runs embedding + all blocks for `batch` sequences of n new rows each (positions pos0..),
 // appending K/V to `cache`; leaves the residual stream in ws.h.  Uses the matrix-core matmul.
+// `residuals` (nullable, host): [layer][rows][H], the stream behind every block.
 int run_blocks_prefill(Model &m, Workspace &ws, const Cache &cache, uint64_t batch, uint64_t n,
-                       uint64_t pos0, hipStream_t st) {
+                       uint64_t pos0, hipStream_t st, float *residuals = nullptr) {
     const coeus_config &c = m.cfg;
     const uint64_t H = c.hidden_dim, rows = batch * n, hd = m.L.head_dim;
     float *h = (float *)ws.h.p, *x = (float *)ws.x.p, *qkv = (float *)ws.qkv.p,
@@ -325,6 +327,8 @@ int run_blocks_prefill(Model &m, Workspace &ws, const Cache &cache, uint64_t bat
         Epilogue e4;
         e4.bias = lw.b_down; e4.residual = h; e4.out_f32 = h;
         COEUS_TRY(launch_gemm(lw.down, lp ? (const void *)ws.b_lp.p : (const void *)ff, rows, e4, ws.gs, st, lp));
+        if (residuals)
+            COEUS_HIP(hipMemcpyAsync(residuals + l * rows * H, h, rows * H * 4, hipMemcpyDeviceToHost, st));
     }
     return COEUS_OK;
 }
@@ -357,24 +361,10 @@ static int check_ids(const Model &m, const uint64_t *ids, uint64_t count) {
     return COEUS_OK;
 }
 
-int model_forward(Model &m, const uint64_t *ids, uint64_t seq_len, float *logits_out, bool all_rows) {
+// The rows of m.ws.h -> logits on the host (enqueued).
+static int finish_forward(Model &m, uint64_t seq_len, float *logits_out, bool all_rows, hipStream_t st) {
     const coeus_config &c = m.cfg;
-    if (!ids || !logits_out) return fail(COEUS_INVALID_INPUT, "null pointer argument");
-    if (seq_len == 0 || seq_len > c.max_seq_len)  // MT:797-802 (empty input panics there, MT:915)
-        return fail(COEUS_INVALID_INPUT, "Sequence length %llu out of range [1, %llu]",
-                    (unsigned long long)seq_len, (unsigned long long)c.max_seq_len);
-    COEUS_TRY(check_ids(m, ids, seq_len));
-    std::lock_guard<std::mutex> lock(m.mu);
-    hipStream_t st = m.stream;
     const uint64_t H = c.hidden_dim, V = c.vocab_size;
-    COEUS_TRY(m.ws.ensure(m, seq_len, all_rows ? seq_len : 1));
-    // single-layer scratch cache: the stateless forward needs K/V only inside a layer
-    const uint64_t cache_bytes = c.num_heads * seq_len * m.L.head_dim * kv_elem_size(c.kv_dtype);
-    COEUS_TRY(m.tmp_k.ensure(cache_bytes));
-    COEUS_TRY(m.tmp_v.ensure(cache_bytes));
-    Cache cache{m.tmp_k.p, m.tmp_v.p, seq_len, 0, false};
-    COEUS_HIP(hipMemcpyAsync(m.ws.ids.p, ids, seq_len * 8, hipMemcpyHostToDevice, st));
-    COEUS_TRY(run_blocks_prefill(m, m.ws, cache, 1, seq_len, 0, st));
     float *h = (float *)m.ws.h.p, *x = (float *)m.ws.x.p, *logits = (float *)m.ws.logits.p;
     // final normalisation over the whole slice, then the last row (MT:903-916) or every row
     COEUS_TRY(launch_norm(c.norm, c.norm_scope, h, seq_len, H, m.fin_s, m.fin_b, c.layer_norm_eps, x,
@@ -388,6 +378,44 @@ int model_forward(Model &m, const uint64_t *ids, uint64_t seq_len, float *logits
     }
     COEUS_HIP(hipMemcpyAsync(logits_out, logits, (all_rows ? seq_len : 1) * V * 4,
                              hipMemcpyDeviceToHost, st));
+    return COEUS_OK;
+}
+
+int model_forward(Model &m, const uint64_t *ids, uint64_t seq_len, float *logits_out, bool all_rows) {
+    const coeus_config &c = m.cfg;
+    if (!ids || !logits_out) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    if (seq_len == 0 || seq_len > c.max_seq_len)  // MT:797-802 (empty input panics there, MT:915)
+        return fail(COEUS_INVALID_INPUT, "Sequence length %llu out of range [1, %llu]",
+                    (unsigned long long)seq_len, (unsigned long long)c.max_seq_len);
+    COEUS_TRY(check_ids(m, ids, seq_len));
+    std::lock_guard<std::mutex> lock(m.mu);
+    hipStream_t st = m.stream;
+    const uint64_t V = c.vocab_size;
+    if (m.stack) {
+        // a sequence of its own: fresh state, dropped at the end
+        LayeredState state;
+        struct Drop { LayeredState &s; ~Drop() { s.release(); } } drop{state};
+        COEUS_TRY(state.create(*m.stack, c.weight_dtype == COEUS_W_BF16, 1, seq_len));
+        COEUS_TRY(state.clear(st));
+        COEUS_TRY(layered_workspace(m, m.ws, 1, seq_len, 0));
+        COEUS_TRY(m.ws.logits.ensure((all_rows ? seq_len : 1) * V * 4));
+        COEUS_HIP(hipMemcpyAsync(m.ws.ids.p, ids, seq_len * 8, hipMemcpyHostToDevice, st));
+        COEUS_TRY(layered_prefill(m, m.ws, state, 1, seq_len, 0, nullptr, st));
+        const int rc = finish_forward(m, seq_len, logits_out, all_rows, st);
+        const hipError_t e = hipStreamSynchronize(st);  // (also on failure: the state goes away below)
+        COEUS_TRY(rc);
+        COEUS_HIP(e);
+        return COEUS_OK;
+    }
+    COEUS_TRY(m.ws.ensure(m, seq_len, all_rows ? seq_len : 1));
+    // single-layer scratch cache: the stateless forward needs K/V only inside a layer
+    const uint64_t cache_bytes = c.num_heads * seq_len * m.L.head_dim * kv_elem_size(c.kv_dtype);
+    COEUS_TRY(m.tmp_k.ensure(cache_bytes));
+    COEUS_TRY(m.tmp_v.ensure(cache_bytes));
+    Cache cache{m.tmp_k.p, m.tmp_v.p, seq_len, 0, false};
+    COEUS_HIP(hipMemcpyAsync(m.ws.ids.p, ids, seq_len * 8, hipMemcpyHostToDevice, st));
+    COEUS_TRY(run_blocks_prefill(m, m.ws, cache, 1, seq_len, 0, st));
+    COEUS_TRY(finish_forward(m, seq_len, logits_out, all_rows, st));
     COEUS_HIP(hipStreamSynchronize(st));
     return COEUS_OK;
 }
@@ -396,7 +424,8 @@ int model_forward(Model &m, const uint64_t *ids, uint64_t seq_len, float *logits
 Session::~Session() {
     if (graph_exec) (void)hipGraphExecDestroy(graph_exec);
     if (graph) (void)hipGraphDestroy(graph);
-    kc.release(); vc.release(); ws.release();
+    kc.release(); vc.release(); state.release(); ws.release();
+    dmix.release(); dscratch.release(); drows.release(); dwant.release();
     dh.release(); dx.release(); dqkv.release(); datt.release(); dff.release(); dlogits.release();
     dids.release(); dpos.release(); dhist.release(); dpart.release(); dcount.release(); dstats.release();
     xq_h.release(); xq_inner.release(); xq_ff.release(); xq_g.release();
@@ -421,6 +450,11 @@ int session_create(Model &m, uint64_t batch, uint64_t max_ctx, Session **out) {
     s->use_graph = graph_replay_forbidden() == nullptr;
     const uint64_t H = c.hidden_dim, I = c.intermediate_dim, V = c.vocab_size,
                    inner = m.L.inner_dim, hd = m.L.head_dim;
+    if (m.stack) {
+        COEUS_TRY(layered_session_init(*s));
+        *out = s.release();
+        return COEUS_OK;
+    }
     s->layer_bytes = batch * c.num_heads * max_ctx * hd * kv_elem_size(c.kv_dtype);
     COEUS_TRY(s->kc.ensure(s->layer_bytes * c.num_layers));
     COEUS_TRY(s->vc.ensure(s->layer_bytes * c.num_layers));
@@ -457,24 +491,38 @@ int session_create(Model &m, uint64_t batch, uint64_t max_ctx, Session **out) {
     return COEUS_OK;
 }
 
+// The n tokens of every sequence at positions s.pos ..: blocks over all of them, cache and state
+// moved on, the residual stream left in s.ws.h.  Called under the model's lock.
+static int feed_rows(Session &s, const uint64_t *ids, uint64_t n, float *residuals_out, hipStream_t st) {
+    Model &m = *s.m;
+    if (n == 0 || n > s.max_ctx || s.pos + n > s.max_ctx)
+        return fail(COEUS_INVALID_INPUT, "Sequence length %llu out of range [1, %llu]",
+                    (unsigned long long)(s.pos + n), (unsigned long long)s.max_ctx);
+    COEUS_TRY(check_ids(m, ids, s.batch * n));
+    const uint64_t rows = s.batch * n;
+    if (m.stack) COEUS_TRY(layered_workspace(m, s.ws, s.batch, n, s.pos));
+    else COEUS_TRY(s.ws.ensure(m, rows, 0));
+    COEUS_HIP(hipMemcpyAsync(s.ws.ids.p, ids, rows * 8, hipMemcpyHostToDevice, st));
+    if (m.stack) {
+        COEUS_TRY(layered_prefill(m, s.ws, s.state, s.batch, n, s.pos, residuals_out, st));
+    } else {
+        Cache cache{s.kc.p, s.vc.p, s.max_ctx, s.layer_bytes, true};
+        COEUS_TRY(run_blocks_prefill(m, s.ws, cache, s.batch, n, s.pos, st, residuals_out));
+    }
+    s.pos += n;
+    return COEUS_OK;
+}
+
 int session_prefill(Session &s, const uint64_t *ids, uint64_t n, float *logits_out) {
     Model &m = *s.m;
     const coeus_config &c = m.cfg;
     if (!ids) return fail(COEUS_INVALID_INPUT, "null pointer argument");
     // the position is read and advanced under the lock: two threads stepping one session must not
-    // both pass the bound below and then write a cache row past the end
+    // both pass the bound check and then write a cache row past the end
     std::lock_guard<std::mutex> lock(m.mu);
-    if (n == 0 || n > s.max_ctx || s.pos + n > s.max_ctx)
-        return fail(COEUS_INVALID_INPUT, "Sequence length %llu out of range [1, %llu]",
-                    (unsigned long long)(s.pos + n), (unsigned long long)s.max_ctx);
-    COEUS_TRY(check_ids(m, ids, s.batch * n));
     hipStream_t st = m.stream;
-    const uint64_t H = c.hidden_dim, V = c.vocab_size, rows = s.batch * n;
-    COEUS_TRY(s.ws.ensure(m, rows, 0));
-    Cache cache{s.kc.p, s.vc.p, s.max_ctx, s.layer_bytes, true};
-    COEUS_HIP(hipMemcpyAsync(s.ws.ids.p, ids, rows * 8, hipMemcpyHostToDevice, st));
-    COEUS_TRY(run_blocks_prefill(m, s.ws, cache, s.batch, n, s.pos, st));
-    s.pos += n;
+    const uint64_t H = c.hidden_dim, V = c.vocab_size;
+    COEUS_TRY(feed_rows(s, ids, n, nullptr, st));
     if (logits_out) {
         // last row of every sequence -> contiguous [batch, H], final norm, decode matmul
         float *h = (float *)s.ws.h.p, *last = (float *)s.dh.p, *x = (float *)s.dx.p;
@@ -489,13 +537,51 @@ int session_prefill(Session &s, const uint64_t *ids, uint64_t n, float *logits_o
     return COEUS_OK;
 }
 
+int session_feed(Session &s, const uint64_t *ids, uint64_t n, const uint64_t *want, uint64_t n_want,
+                 float *logits_out, float *residuals_out) {
+    Model &m = *s.m;
+    const coeus_config &c = m.cfg;
+    if (!ids || (n_want && (!want || !logits_out))) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    for (uint64_t i = 0; i < n_want; i++)
+        if (want[i] >= n)
+            return fail(COEUS_INVALID_INPUT, "Row %llu out of range [0, %llu)", (unsigned long long)want[i], (unsigned long long)n);
+    std::lock_guard<std::mutex> lock(m.mu);
+    hipStream_t st = m.stream;
+    COEUS_TRY(feed_rows(s, ids, n, residuals_out, st));
+    const uint64_t H = c.hidden_dim, V = c.vocab_size, total = s.batch * n_want;
+    std::vector<uint64_t> rows(total);  // (lives until the stream is synchronised)
+    if (total) {
+        for (uint64_t b = 0; b < s.batch; b++)
+            for (uint64_t i = 0; i < n_want; i++) rows[b * n_want + i] = b * n + want[i];
+        COEUS_TRY(s.drows.ensure(total * 8));
+        COEUS_TRY(s.dwant.ensure(total * H * 4));
+        COEUS_TRY(s.ws.logits.ensure(total * V * 4));
+        COEUS_HIP(hipMemcpyAsync(s.drows.p, rows.data(), total * 8, hipMemcpyHostToDevice, st));
+        float *x = (float *)s.dwant.p;
+        COEUS_TRY(launch_gather_rows((const float *)s.ws.h.p, (const uint64_t *)s.drows.p, total, H, x, st));
+        COEUS_TRY(launch_norm(c.norm, COEUS_SCOPE_TOKEN, x, total, H, m.fin_s, m.fin_b, c.layer_norm_eps, x, nullptr, 0, st));
+        COEUS_TRY(logits_gemv(m, s.ws, x, total, (float *)s.ws.logits.p, st));
+        COEUS_HIP(hipMemcpyAsync(logits_out, s.ws.logits.p, total * V * 4, hipMemcpyDeviceToHost, st));
+    }
+    COEUS_HIP(hipStreamSynchronize(st));
+    return COEUS_OK;
+}
+
+int session_reset(Session &s) {
+    Model &m = *s.m;
+    std::lock_guard<std::mutex> lock(m.mu);
+    s.pos = 0;
+    if (m.stack) {
+        COEUS_TRY(s.state.clear(m.stream));
+        COEUS_HIP(hipStreamSynchronize(m.stream));
+    }
+    return COEUS_OK;
+}
+
 // One decode step for every sequence of the session, reading the token ids from s.dids and the
 // position from the device (s.dpos[0]); only enqueues kernels, so it can be graph-captured.
-static uint64_t gemv_algorithmic_bytes(const Weight &w, uint64_t batch, bool gated, bool normed);
-
 // `only` (roofline measurements): enqueue just the decode matmuls (with their fused staging and
 // epilogues) or just the attention launches, and count them and their algorithmic bytes.
-enum { STEP_ALL = 0, STEP_MATMULS = 1, STEP_ATTENTION = 2 };
 static int enqueue_decode_step(Session &s, hipStream_t st, int only = STEP_ALL,
                                uint64_t *launches = nullptr, uint64_t *bytes = nullptr) {
     const bool matmuls_only = only != STEP_ALL;  // everything that is not a matmul or the attention is skipped
@@ -518,6 +604,12 @@ static int enqueue_decode_step(Session &s, hipStream_t st, int only = STEP_ALL,
     const bool gpath = stats && c.norm == COEUS_NORM_RMSNORM && gemv_can_fuse_norm(m.layers[0].qkv, B) &&
                        gemv_can_fuse_norm(m.layers[0].up, B) && gemv_can_fuse_norm(m.out, B);
     float *xq_g = gpath ? (float *)s.xq_g.p : nullptr;
+    if (m.stack) {
+        if (!matmuls_only)
+            COEUS_TRY(launch_embed(m.embed, m.embed_bf16, nullptr, (const uint64_t *)s.dids.p, B, 1, 0, pos_dev, H, h,
+                                   nullptr, st));
+        return layered_decode(s, st, only, launches, bytes);
+    }
     if (!matmuls_only)
         COEUS_TRY(launch_embed(m.embed, m.embed_bf16, m.pe, (const uint64_t *)s.dids.p, B, 1, 0,
                                pos_dev, H, h, stats, st, gpath ? m.layers[0].ln1_s : nullptr, xq_g));
@@ -698,7 +790,7 @@ int session_decode_greedy(Session &s, const uint64_t *first_ids, uint64_t n_step
 // Algorithmic bytes one launch of the decode matmul moves: the weight in its stored form
 // (quants + scales, padding excluded) plus the activation rows in (f32 when the norm is folded
 // into the launch, else the matrix-core input type) and out.
-static uint64_t gemv_algorithmic_bytes(const Weight &w, uint64_t batch, bool gated, bool normed) {
+uint64_t gemv_algorithmic_bytes(const Weight &w, uint64_t batch, bool gated, bool normed) {
     uint64_t wb;
     switch (w.dtype) {
         case COEUS_W_F32: wb = w.k * w.n * 4; break;

@@ -4,6 +4,8 @@
 #include <memory>
 
 #include "common.hpp"
+#include "layered.hpp"
+#include "mixers.hpp"
 
 namespace coeus {
 
@@ -26,12 +28,45 @@ struct LayerWeights {
     const float *b_qkv = nullptr, *b_o = nullptr, *b_up = nullptr, *b_down = nullptr;
 };
 
+// One layer of a layered model on the device.
+struct LayeredLayer {
+    LayerSpec spec;
+    Weight in, o, up, down;  // fused input projection, output projection; up: interleaved (gate, up) rows
+    Weight uq, ukv;          // latent attention: query expansion; key and value expansions, one behind the other
+    DeltaParams delta{};
+    const float *dq_norm = nullptr, *dkv_norm = nullptr;
+    const float *norm1 = nullptr, *ls1 = nullptr, *norm2 = nullptr, *ls2 = nullptr;
+    DeltaDims delta_dims() const;
+    LatentDims latent_dims() const;
+};
+struct LayeredStack {
+    LayeredConfig cfg;
+    std::vector<LayeredLayer> layers;
+    float *small = nullptr;  // every f32 vector of every layer
+    ~LayeredStack();
+};
+// What the sequences of a session carry from token to token, layer by layer: matrix states and
+// convolution rings of recurrent layers, rings of cached latents of attention layers.
+struct LayeredState {
+    struct Layer {
+        DeltaState delta{};
+        LatentCache latent{};
+    };
+    std::vector<Layer> layers;
+    DeviceBuf mem;
+    uint64_t batch = 0, recurrent_bytes = 0;  // the recurrent part comes first in `mem` and starts at zero
+    int create(const LayeredStack &stack, bool bf16, uint64_t batch, uint64_t max_ctx);
+    int clear(hipStream_t st);  // start of a sequence
+    void release() { mem.release(); layers.clear(); }
+};
+
 struct Model;
 
 // Activation buffers of the matrix-core (prefill) path, grown on demand.
 struct Workspace {
     uint64_t rows = 0;
     DeviceBuf h, x, qkv, att, ff, ids, a_lp, b_lp, w_lp, logits, xq, norm_part, gemm_part;
+    DeviceBuf mix, lat, q_lp, kv_lp;  // layered models: mixer operands, latents, 16-bit queries / keys and values
     GemmScratch gs;
     int ensure(const Model &m, uint64_t rows_needed, uint64_t logit_rows);
     void release();
@@ -61,6 +96,7 @@ struct Model {
     // HBM that resident f16 copies of quantised weights may still take (prefill matmul operands)
     static constexpr uint64_t kExpandBudget = 64ull << 30;
     uint64_t expand_budget = kExpandBudget;
+    std::unique_ptr<LayeredStack> stack;  // set: the blocks are the stack's layers, not `layers`
     ~Model();
 };
 
@@ -72,8 +108,11 @@ struct Session {
     bool fuse = true;  // fold norms into the decode matmuls where possible
     uint32_t host_pos[2] = {0, 0};
     DeviceBuf kc, vc;
+    LayeredState state;  // layered models (instead of kc / vc)
     Workspace ws;  // prefill
     DeviceBuf dh, dx, dqkv, datt, dff, dlogits, dids, dpos, dhist, dpart, dcount, dstats, xq_h, xq_inner, xq_ff, xq_g;
+    DeviceBuf drows, dwant;    // rows whose logits session_feed was asked for
+    DeviceBuf dmix, dscratch;  // layered models: latent queries of a decode step, attention partials
     hipGraph_t graph = nullptr;
     hipGraphExec_t graph_exec = nullptr;
     ~Session();
@@ -84,6 +123,9 @@ int model_create(const coeus_config &cfg, const float *params, uint64_t n_params
 int model_forward(Model &m, const uint64_t *ids, uint64_t seq_len, float *logits_out, bool all_rows);
 int session_create(Model &m, uint64_t batch, uint64_t max_ctx, Session **out);
 int session_prefill(Session &s, const uint64_t *ids, uint64_t n, float *logits_out);
+int session_feed(Session &s, const uint64_t *ids, uint64_t n, const uint64_t *want, uint64_t n_want,
+                 float *logits_out, float *residuals_out);
+int session_reset(Session &s);
 int session_decode(Session &s, const uint64_t *ids, float *logits_out);
 int session_decode_greedy(Session &s, const uint64_t *first_ids, uint64_t n_steps, uint64_t *out_ids,
                           const coeus_sampling *sampling = nullptr);
@@ -92,5 +134,20 @@ int session_time_decode_matmuls(Session &s, uint64_t reps, float *ms_out, uint64
                                 uint64_t *bytes_out);
 int session_time_decode_attention(Session &s, uint64_t reps, float *ms_out, uint64_t *launches_out,
                                   uint64_t *bytes_out);
+
+// ---------------------------------------------------------------- layered models (layered.hip)
+int layered_load(const char *dir, const coeus_load_options &opt, Model **out);
+int layered_create_seeded(const char *json, uint64_t len, const coeus_load_options &opt, uint64_t seed, Model **out);
+int layered_workspace(const Model &m, Workspace &ws, uint64_t batch, uint64_t n, uint64_t pos0);
+// All layers over n new rows per sequence; the residual stream is in ws.h.  residuals (nullable, host):
+// [layer][batch * n][width] after every layer.
+int layered_prefill(Model &m, Workspace &ws, LayeredState &state, uint64_t batch, uint64_t n, uint64_t pos0,
+                    float *residuals, hipStream_t st);
+int layered_session_init(Session &s);
+// Parts of a decode step: everything, only the matmuls, or only the mixers.
+enum { STEP_ALL = 0, STEP_MATMULS = 1, STEP_ATTENTION = 2 };
+int layered_decode(Session &s, hipStream_t st, int only, uint64_t *launches, uint64_t *bytes);
+uint64_t gemv_algorithmic_bytes(const Weight &w, uint64_t batch, bool gated, bool normed);
+int check_device();
 
 }  // namespace coeus

@@ -6,6 +6,7 @@
 //                         MT:469,488,906): ONE mean/variance over the whole [rows*hidden] slice,
 //                         scale/bias indexed i % hidden.
 //   embed_kernel          x[s,:] = E[id_s,:] + PE[pos0+s,:]  (MT:812-835)
+//   norm_residual_kernel  h += RMSNorm(y) * layer_scale: norms that stand behind a sublayer
 #include "device_utils.hpp"
 
 namespace coeus {
@@ -329,6 +330,81 @@ int launch_norm(uint32_t kind, uint32_t scope, const float *x, uint64_t rows, ui
     return COEUS_OK;
 }
 
+// Norm behind a sublayer: h[row, :] += y[row, :] / rms(y[row, :]) * scale (* ls), and the 16-bit copy of
+// the new h for the next matmul.  One workgroup per row; rows of up to 8192 elements are read once.
+__global__ __launch_bounds__(256) void norm_residual_kernel(const float *__restrict__ y, uint32_t hidden,
+                                                            const float *__restrict__ scale,
+                                                            const float *__restrict__ ls, float eps, float *h,
+                                                            uint16_t *h_lp, uint64_t lp_ld, bool lp_bf16) {
+    __shared__ float sh[16];
+    const uint64_t row = blockIdx.x;
+    const float *yr = y + row * hidden;
+    float *hr = h + row * hidden;
+    constexpr int VMAX = 8;
+    if ((hidden & 3) == 0 && hidden <= 4u * 256u * VMAX && (lp_ld & 3) == 0) {
+        const uint32_t n4 = hidden / 4;
+        float4 v[VMAX];
+        float s2 = 0.f;
+#pragma unroll
+        for (int u = 0; u < VMAX; u++) {
+            const uint32_t i = threadIdx.x + 256 * u;
+            v[u] = i < n4 ? *(const float4 *)(yr + 4 * i) : make_float4(0.f, 0.f, 0.f, 0.f);
+            s2 = fmaf(v[u].x, v[u].x, s2); s2 = fmaf(v[u].y, v[u].y, s2);
+            s2 = fmaf(v[u].z, v[u].z, s2); s2 = fmaf(v[u].w, v[u].w, s2);
+        }
+        const float rs = 1.0f / sqrtf(block_sum(s2, sh) / (float)hidden + eps);
+#pragma unroll
+        for (int u = 0; u < VMAX; u++) {
+            const uint32_t i = threadIdx.x + 256 * u;
+            if (i >= n4) continue;
+            const float4 sc = *(const float4 *)(scale + 4 * i);
+            const float4 l4 = ls ? *(const float4 *)(ls + 4 * i) : make_float4(1.f, 1.f, 1.f, 1.f);
+            float4 o = *(const float4 *)(hr + 4 * i);
+            o.x = fmaf(v[u].x * rs * sc.x, l4.x, o.x); o.y = fmaf(v[u].y * rs * sc.y, l4.y, o.y);
+            o.z = fmaf(v[u].z * rs * sc.z, l4.z, o.z); o.w = fmaf(v[u].w * rs * sc.w, l4.w, o.w);
+            *(float4 *)(hr + 4 * i) = o;
+            if (h_lp) {
+                uint2 p;
+                p.x = (uint32_t)f32_to_lp_bits(o.x, lp_bf16) | ((uint32_t)f32_to_lp_bits(o.y, lp_bf16) << 16);
+                p.y = (uint32_t)f32_to_lp_bits(o.z, lp_bf16) | ((uint32_t)f32_to_lp_bits(o.w, lp_bf16) << 16);
+                *(uint2 *)(h_lp + row * lp_ld + 4 * i) = p;
+            }
+        }
+        return;
+    }
+    float s2 = 0.f;
+    for (uint32_t i = threadIdx.x; i < hidden; i += blockDim.x) s2 = fmaf(yr[i], yr[i], s2);
+    const float rs = 1.0f / sqrtf(block_sum(s2, sh) / (float)hidden + eps);
+    for (uint32_t i = threadIdx.x; i < hidden; i += blockDim.x) {
+        const float o = fmaf(yr[i] * rs * scale[i], ls ? ls[i] : 1.0f, hr[i]);
+        hr[i] = o;
+        if (h_lp) h_lp[row * lp_ld + i] = f32_to_lp_bits(o, lp_bf16);
+    }
+}
+
+int launch_norm_residual(const float *y, uint64_t rows, uint64_t hidden, const float *scale, const float *ls,
+                         float eps, float *h, hipStream_t st, const LpOut *h_lp) {
+    if (rows == 0 || hidden == 0 || hidden > 0xffffffffull) return fail(COEUS_INVALID_INPUT, "bad normalisation shape");
+    hipLaunchKernelGGL(norm_residual_kernel, dim3((unsigned)rows), dim3(256), 0, st, y, (uint32_t)hidden, scale, ls,
+                       eps, h, h_lp ? (uint16_t *)h_lp->p : nullptr, h_lp ? h_lp->ld : 0, h_lp && h_lp->bf16);
+    COEUS_HIP(hipGetLastError());
+    return COEUS_OK;
+}
+
+// dst[i, :] = src[rows[i], :]
+__global__ __launch_bounds__(256) void gather_rows_kernel(const float *__restrict__ src, const uint64_t *__restrict__ rows,
+                                                          uint64_t hidden, float *__restrict__ dst) {
+    const uint64_t r = rows[blockIdx.x];
+    for (uint64_t i = threadIdx.x; i < hidden; i += blockDim.x) dst[blockIdx.x * hidden + i] = src[r * hidden + i];
+}
+
+int launch_gather_rows(const float *src, const uint64_t *rows_dev, uint64_t count, uint64_t hidden, float *dst, hipStream_t st) {
+    if (count == 0) return COEUS_OK;
+    hipLaunchKernelGGL(gather_rows_kernel, dim3((unsigned)count), dim3(256), 0, st, src, rows_dev, hidden, dst);
+    COEUS_HIP(hipGetLastError());
+    return COEUS_OK;
+}
+
 // ids are range-checked on the host before upload (MT:816-822).  pos_dev (nullable) holds the
 // position of row 0 on the device so a captured graph can be replayed as the context grows;
 // with several sequences (rows == batch, one new token each) every row sits at that position.
@@ -356,7 +432,7 @@ __global__ __launch_bounds__(1024) void embed_kernel(const void *__restrict__ ta
             if (i < hidden) {
                 const float ev = BF16 ? bf16_bits_to_f32(((const uint16_t *)table)[id * hidden + i])
                                       : ((const float *)table)[id * hidden + i];
-                v[u] = ev + pe[pos * hidden + i];
+                v[u] = pe ? ev + pe[pos * hidden + i] : ev;
             }
         }
 #pragma unroll

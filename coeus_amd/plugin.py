@@ -7,6 +7,8 @@ over the C ABI of libcoeus_mi355x.so.  Names, argument meaning and error behavio
 reference; `Result<T>` becomes "return T or raise".  All arithmetic runs on the GPU.
 """
 import ctypes as C
+import json
+import os
 from dataclasses import dataclass, fields
 
 import numpy as np
@@ -292,6 +294,101 @@ class TransformerModel:
             pass
 
 
+# ---------------------------------------------------------------- layered models
+@dataclass
+class LayeredConfig:
+    """A layered decoder (its config.json as a dictionary) with the storage type and the limits the
+    model is built with.  No counterpart in the reference."""
+
+    config: dict
+    weight_dtype: str = "bf16"        # "bf16" | "f32"
+    max_seq_len: int = 1 << 20
+    max_batch: int = 1
+
+    _WD = {"f32": 0, "bf16": 1}
+
+    @property
+    def vocab_size(self):
+        return int(self.config["vocab"])
+
+    @property
+    def hidden_dim(self):
+        return int(self.config["width"])
+
+    def text(self):
+        return json.dumps(self.config).encode()
+
+    def options(self):
+        if self.weight_dtype not in self._WD:
+            raise ConfigError(f"Invalid configuration: weight_dtype = {self.weight_dtype!r}: unknown value")
+        if int(self.max_seq_len) < 1 or int(self.max_batch) < 1:
+            raise ConfigError("Invalid configuration: max_seq_len and max_batch must be at least 1")
+        return _lib.CLoadOptions(self._WD[self.weight_dtype], int(self.max_seq_len), int(self.max_batch))
+
+    def validate(self):
+        self.num_parameters()
+
+    def num_parameters(self):
+        n, text = C.c_uint64(), self.text()
+        _check(_lib.load().coeus_layered_config_check(text, len(text), C.byref(n)))
+        return int(n.value)
+
+
+class LayeredModelPlugin:
+    """The plugin surface of the transformer family for layered decoders (coeus_model_load)."""
+
+    def id(self):
+        return "layered_model"
+
+    def version(self):
+        return (0, 1, 0)
+
+    def capabilities(self):
+        return ("model_building", "gated_delta_rule", "latent_attention", "sliding_window")
+
+    def create_builder(self):
+        return LayeredModelBuilder()
+
+
+class LayeredModelBuilder:
+    def build(self, config, seed=0):
+        """A model of the configuration's shape with synthetic weights."""
+        config.validate()
+        handle, text, opt = C.c_void_p(), config.text(), config.options()
+        _check(_lib.load().coeus_model_create_layered(text, len(text), C.byref(opt), int(seed), C.byref(handle)))
+        return LayeredModel(config, handle)
+
+    def load(self, path, **overrides):
+        """A folder with config.json and model.safetensors; `overrides` are LayeredConfig fields."""
+        try:
+            with open(os.path.join(path, "config.json"), encoding="utf-8") as f:
+                config = LayeredConfig(json.load(f), **overrides)
+        except (OSError, ValueError) as e:
+            raise ConfigError(f"Invalid configuration: {path}: {e}") from e
+        handle, opt = C.c_void_p(), config.options()
+        _check(_lib.load().coeus_model_load(os.fsencode(path), C.byref(opt), C.byref(handle)))
+        return LayeredModel(config, handle)
+
+
+class LayeredModel(TransformerModel):
+    """forward / sessions / generation as for any model of the library."""
+
+    def write_to(self, path):
+        raise ProcessingError("Processing error: layered models are read from safetensors folders; "
+                              "the .rustllm format has no place for their layers")
+
+
+# ---------------------------------------------------------------- registry
+PLUGINS = {p.id(): p for p in (TransformerModelPlugin(), LayeredModelPlugin())}
+
+
+def load_model(path, **overrides):
+    """Loads what `path` holds: a .rustllm file (transformer) or a folder whose config.json names an
+    architecture (layered).  `overrides` go to the family's configuration."""
+    family = "layered_model" if os.path.isdir(path) else "transformer_model"
+    return PLUGINS[family].create_builder().load(path, **overrides)
+
+
 class Session:
     """KV-cache generation state (an extension: the reference recomputes the whole sequence)."""
 
@@ -316,6 +413,20 @@ class Session:
         _check(_lib.load().coeus_session_prefill(self._h, ids.ctypes.data, ids.shape[1],
                                                  out.ctypes.data if want_logits else None))
         return out
+
+    def feed(self, ids, want=(), want_residuals=False):
+        """prefill with the logits of chosen rows: `want` are places among the fed tokens, the result is
+        [batch, len(want), vocab]; with want_residuals also [layers, batch * n, hidden], the residual
+        stream behind every layer."""
+        ids = self._ids2d(ids)
+        cfg = _lib.load().coeus_model_config(self._model._h).contents
+        w = np.ascontiguousarray(want, dtype=np.uint64).ravel()
+        out = np.empty((self.batch, w.size, int(cfg.vocab_size)), dtype=np.float32)
+        res = (np.empty((int(cfg.num_layers), ids.size, int(cfg.hidden_dim)), dtype=np.float32)
+               if want_residuals else None)
+        _check(_lib.load().coeus_session_feed(self._h, ids.ctypes.data, ids.shape[1], w.ctypes.data, w.size,
+                                              out.ctypes.data, res.ctypes.data if want_residuals else None))
+        return (out, res) if want_residuals else out
 
     def decode(self, ids):
         ids = TransformerModel._ids(ids).ravel()

@@ -196,6 +196,27 @@ int coeus_model_create(const coeus_config *cfg, const float *params, uint64_t n_
  * mean 1 for norm scales and 0 elsewhere.  No reference counterpart (the reference has one
  * fixed init, MT:604-611); exists so multi-GB configurations need no host-side buffer. */
 int coeus_model_create_seeded(const coeus_config *cfg, uint64_t seed, coeus_model **out);
+/* ---- layered models (no counterpart in the reference) --------------------------------------
+ * Decoders whose layers name their own token mixer: a gated delta rule with short convolutions, or
+ * attention through low-rank latents in a sliding window.  A folder holds config.json (its
+ * "architecture" selects the design from the library's registry: "Bofirax") and model.safetensors
+ * (BF16 or F32).  The handle is a coeus_model like any other: coeus_model_forward*, sessions,
+ * generation and sampling work on it; coeus_model_config reports width, depth, vocabulary, storage
+ * types and limits.  Weight storage COEUS_W_BF16 (16-bit matrix products, bf16 latents in the cache;
+ * norms, recurrences, scores and the residual stream in f32) or COEUS_W_F32 (everything in f32). */
+typedef struct coeus_load_options {
+    uint32_t weight_dtype; /* COEUS_W_BF16 or COEUS_W_F32 */
+    uint64_t max_seq_len;  /* 0 => 1048576: upper bound of a session's positions */
+    uint64_t max_batch;    /* 0 => 1 */
+} coeus_load_options;
+int coeus_model_load(const char *dir, const coeus_load_options *opt, coeus_model **out);
+/* The same from a config.json text with synthetic weights generated on the device. */
+int coeus_model_create_layered(const char *config_json, uint64_t len, const coeus_load_options *opt,
+                               uint64_t seed, coeus_model **out);
+/* Reads and checks a config.json text without a device; *n_params_out (nullable) = its parameters. */
+int coeus_layered_config_check(const char *config_json, uint64_t len, uint64_t *n_params_out);
+/* The same for a folder: config.json and the names, types and shapes in model.safetensors. */
+int coeus_layered_check(const char *dir, uint64_t *n_params_out);
 /* ForwardModel::forward (MT:791-919): token ids in, the LAST token's logits out
  * (logits_out[vocab_size]).  Errors as the reference: seq_len > max_seq_len ->
  * "Sequence length {} out of range [1, {}]" (MT:797-802); id >= vocab ->
@@ -225,6 +246,11 @@ int coeus_session_create(coeus_model *m, uint64_t batch, uint64_t max_ctx, coeus
  * keys/values to the cache, writes the logits of the last fed token: logits_out[batch][vocab]
  * (nullable). */
 int coeus_session_prefill(coeus_session *s, const uint64_t *ids, uint64_t n, float *logits_out);
+/* coeus_session_prefill with the logits of chosen rows: want[n_want] are places in 0 .. n - 1 of the
+ * fed tokens (the same for every sequence), logits_out[batch][n_want][vocab].  residuals_out
+ * (nullable): the residual stream behind every layer, [num_layers][batch * n][hidden_dim]. */
+int coeus_session_feed(coeus_session *s, const uint64_t *ids, uint64_t n, const uint64_t *want,
+                       uint64_t n_want, float *logits_out, float *residuals_out);
 /* One token per sequence: ids[batch] -> logits_out[batch][vocab]. */
 int coeus_session_decode(coeus_session *s, const uint64_t *ids, float *logits_out);
 /* n_steps greedy steps entirely on the device: step 0 consumes first_ids[batch], every later
