@@ -337,29 +337,6 @@ __global__ void attn_merge_kernel(const float *__restrict__ part, uint32_t heads
 // Within a wave a key tile is a strict chain (scores -> softmax on the VALU -> P.V), so the
 // matrix cores are only kept busy by other waves of the SIMD: the register budget is capped at
 // what lets three workgroups share a CU (measured: 17 % faster than two).
-// Which (query tile, head) a workgroup of a prefill grid (x = query tiles, y = heads) works on.
-// Causal work grows with the query tile: the last (longest) tiles are dispatched first, so that
-// the short ones fill in behind them instead of the long ones forming the tail.  The hardware
-// deals consecutive workgroups round-robin to the 8 XCDs: with a multiple of 8 heads the numbering
-// is permuted so that all query tiles of a head run on one XCD and its keys and values are fetched
-// into one L2 instead of eight (measured on 32 heads x 4024 rows: 292 -> 184 us).
-__device__ __forceinline__ void prefill_tile_of_block(uint32_t &qt, uint32_t &h) {
-    qt = gridDim.x - 1 - blockIdx.x;
-    h = blockIdx.y;
-    if ((gridDim.y & 7) == 0) {
-        const uint32_t lin = blockIdx.x + gridDim.x * blockIdx.y, idx = lin >> 3, hpx = gridDim.y >> 3;
-        h = (lin & 7) + 8 * (idx % hpx);
-        qt = gridDim.x - 1 - idx / hpx;
-    }
-}
-
-// Maximum of a value over lanes i and i ^ 32 (v_permlane32_swap hands every lane both values: a
-// register move, no trip through LDS); the sum is xor32_sum.
-__device__ __forceinline__ float both_halves_max(float v) {
-    const auto r = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
-    return fmaxf(__uint_as_float(r[0]), __uint_as_float(r[1]));
-}
-
 template <int HD, bool BF16>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(3, 4))) void attn_prefill_kernel(const float *__restrict__ qkv,
                                                            const uint16_t *__restrict__ kc,

@@ -188,6 +188,13 @@ struct NormFuse {
     // records (Epilogue::g_out, launch_embed).  The consuming matmul then stages half the bytes
     // (16 KB instead of 32 KB per workgroup at k = 4096) and multiplies by 1 / rms.
     const float *g = nullptr;
+    // Dense weights only: row stride of h (0: k), for rows that are part of a wider buffer.
+    uint64_t ld = 0;
+    // Dense weights only, instead of a norm in front: the norm stands behind the previous sublayer, whose
+    // bare output is y [batch, k].  The matmul multiplies h + y / rms(y) * scale (* ls) and stores these
+    // rows to h_out (not h: every workgroup reads h).
+    const float *y = nullptr, *ls = nullptr;
+    float *h_out = nullptr;
 };
 // True when launch_gemv can take `nf` for this weight and batch (quantised weights whose whole
 // activation block fits in LDS).
@@ -195,6 +202,8 @@ bool gemv_can_fuse_norm(const Weight &w, uint64_t batch);
 // The same for f32 / bf16 weights (the normalised block [batch, k] f32 has to fit in LDS; the
 // statistics are computed inside the launch, NormFuse::stats is not used).
 bool gemv_can_fuse_norm_dense(const Weight &w, uint64_t batch);
+// ... and for the norm behind a sublayer (NormFuse::y): two rows per sequence have to fit.
+bool gemv_can_fuse_post_norm(const Weight &w, uint64_t batch);
 // The same normalisation as a launch of its own (batches too large for the folded form):
 // nf.h rows -> xq, row statistics merged from nf.stats.  Padding rows of xq are not written.
 int launch_norm_from_stats(const NormFuse &nf, uint64_t batch, uint64_t k, uint64_t k_pad, __half *xq,

@@ -3,7 +3,9 @@
 //
 //   delta_prepare_kernel  prompt: convolution + SiLU of q, k, v, unit norms, step sizes and decays
 //   delta_ring_kernel     prompt: the last projections of every sequence into the convolution ring
-//   delta_scan_kernel     prompt: the recurrence token by token, state in registers
+//   delta_scan_kernel     short prompts: the recurrence token by token, state in registers
+//   delta_chunk_kernel    prompt: everything of a chunk of 64 tokens that does not need the state
+//   delta_carry_kernel    prompt: the state through the chunks, on the matrix cores
 //   delta_gate_kernel     prompt: per-head RMS norm of the read-out times silu(gate)
 //   delta_step_kernel     decode: all of it for one token per sequence
 //
@@ -164,17 +166,308 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaDims dm, DeltaOper
             if (sub * R + r < dm.d) sp[(uint64_t)(sub * R + r) * dm.e] = s[r];
 }
 
+// ---------------------------------------------------------------- the recurrence, chunk by chunk
+// With G_i the sum of the log decays of a chunk's tokens up to i and S0 the state in front of it:
+//   (I + A) U = beta (V - e^G K S0),   A_ij = beta_i e^(G_i - G_j) (k_i . k_j) for j < i
+//   O   = e^G Q S0 + P U,              P_ij = e^(G_i - G_j) (q_i . k_j) for j <= i
+//   S_C = e^(G_C) S0 + K^T (e^(G_C - G) U)
+// U = V' - W S0 where (I + A) [W | V'] = beta [e^G K | V] is solved by forward substitution: every exponent
+// is of a sum of log decays that lie between two tokens, so nothing overflows however fast the state decays.
+// delta_chunk_kernel does everything that does not need S0, for all chunks at once; delta_carry_kernel
+// then walks the chunks with one workgroup per head and 16 columns of S.  All products are f32
+// (v_mfma_f32_16x16x4_f32, or fused multiply-adds in the substitution).
+//
+// A reduction index of a matrix instruction is only a label: instruction i of a 16-wide step sums over
+// {4 g + i : g = lane / 16}, so a lane's operand pieces are 16 consecutive bytes, and an accumulator
+// tile (rows 4 g + i) is the next product's right operand as it stands.
+constexpr uint32_t kChunk = 64;
+constexpr uint64_t kSegment = 4096;  // tokens whose chunk operands are in memory at once
+
+struct ChunkBuf {
+    float *w, *vp, *p, *eg, *ed, *kt;
+    uint32_t chunks;  // per sequence
+};
+static uint32_t chunk_dim(uint32_t d) { return (uint32_t)round_up(d, 64); }
+static uint64_t chunk_floats(const DeltaDims &dm, uint64_t batch, uint64_t chunks) {
+    const uint64_t dq = chunk_dim(dm.d);
+    return batch * chunks * (dm.heads * (kChunk * (dq + dm.e + kChunk) + 2 * kChunk) + (uint64_t)dm.kv_heads * dq * kChunk);
+}
+
+__device__ __forceinline__ float4_t mfma4(const float4 &a, const float4_t &b, float4_t acc) {
+    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b[0], acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b[1], acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b[2], acc, 0, 0, 0);
+    return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b[3], acc, 0, 0, 0);
+}
+
+// One workgroup of 256 per (chunk, head, sequence).  dp: row length of the prepared q and k.
+template <int NT>  // 16-wide steps of the padded query/key size
+__global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaDims dm, DeltaOperands op, uint32_t dp, uint64_t n,
+                                                          uint64_t t0, uint64_t seg, ChunkBuf cb) {
+    constexpr uint32_t DQ = 16 * NT, KLD = DQ + 4, ALD = kChunk + 4;
+    extern __shared__ float lds[];
+    float *kl = lds, *al = kl + kChunk * KLD;  // K [64][KLD], A [64][ALD]
+    __shared__ float gs[kChunk], es[kChunk], bs[kChunk];
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
+    const uint32_t chunk = blockIdx.x, h = blockIdx.y, H = dm.heads, KH = dm.kv_heads, hk = h / (H / KH);
+    const uint64_t b = blockIdx.z, first = t0 + (uint64_t)chunk * kChunk, left = seg - (uint64_t)chunk * kChunk;
+    const uint32_t live = left < kChunk ? (uint32_t)left : kChunk;  // tokens behind the end: beta = 0, k = q = v = 0
+    const uint64_t row0 = b * n + first, ci = ((b * H + h) * cb.chunks + chunk);
+    if (wave == 0) {
+        float lg = lane < live ? op.lg[(row0 + lane) * H + h] : 0.f;
+#pragma unroll
+        for (int off = 1; off < 64; off <<= 1) {
+            const float o = __shfl_up(lg, off, 64);
+            if ((int)lane >= off) lg += o;
+        }
+        const float be = lane < live ? op.beta[(row0 + lane) * H + h] : 0.f;
+        gs[lane] = lg;
+        es[lane] = expf(lg);
+        bs[lane] = be;
+        cb.eg[ci * kChunk + lane] = es[lane];
+        cb.ed[ci * kChunk + lane] = expf(__shfl(lg, 63, 64) - lg);
+    }
+    for (uint32_t i = tid; i < kChunk * (DQ / 4); i += 256) {
+        const uint32_t r = i / (DQ / 4), q4 = 4 * (i % (DQ / 4));
+        float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (r < live && q4 < dp) v = *(const float4 *)(op.k + ((row0 + r) * KH + hk) * dp + q4);
+        *(float4 *)(kl + r * KLD + q4) = v;
+    }
+    __syncthreads();
+    // rows 16 wave .. + 15 of K K^T and Q K^T, tiles up to the diagonal
+    {
+        const uint32_t r = 16 * wave + c;
+        float4 ka[NT], qa[NT];
+#pragma unroll
+        for (int m = 0; m < NT; m++) {
+            const uint32_t q4 = 16 * m + 4 * g;
+            ka[m] = *(const float4 *)(kl + r * KLD + q4);
+            qa[m] = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (r < live && q4 < dp) qa[m] = *(const float4 *)(op.q + ((row0 + r) * KH + hk) * dp + q4);
+        }
+        for (uint32_t t = 0; t < 4; t++) {
+            float4_t akk = {0.f, 0.f, 0.f, 0.f}, aqk = {0.f, 0.f, 0.f, 0.f};
+            if (t <= wave) {
+#pragma unroll
+                for (int m = 0; m < NT; m++) {
+                    const float4_t kb = *(const float4_t *)(kl + (16 * t + c) * KLD + 16 * m + 4 * g);
+                    akk = mfma4(ka[m], kb, akk);
+                    aqk = mfma4(qa[m], kb, aqk);
+                }
+            }
+            const uint32_t j = 16 * t + c;
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const uint32_t ri = 16 * wave + 4 * g + i;
+                const float e = j <= ri ? expf(gs[ri] - gs[j]) : 0.f;
+                al[ri * ALD + j] = j < ri ? bs[ri] * e * akk[i] : 0.f;
+                cb.p[(ci * kChunk + ri) * kChunk + j] = e * aqk[i];
+            }
+        }
+    }
+    __syncthreads();
+    // forward substitution, a column of [W | V'] per thread
+    for (uint32_t col = tid; col < DQ + dm.e; col += 256) {
+        const bool is_w = col < DQ;
+        const float *vp = op.v + (row0 * H + h) * dm.e + (col - DQ);
+        float x[kChunk];
+#pragma unroll
+        for (uint32_t i = 0; i < kChunk; i++) {
+            float r;
+            if (is_w) r = es[i] * kl[i * KLD + col];
+            else r = i < live ? vp[(uint64_t)i * H * dm.e] : 0.f;
+            x[i] = bs[i] * r;
+        }
+#pragma unroll
+        for (uint32_t i = 1; i < kChunk; i++) {
+            float a0 = 0.f, a1 = 0.f;
+#pragma unroll
+            for (uint32_t j = 0; j < i; j += 4) {
+                const float4 a = *(const float4 *)(al + i * ALD + j);  // (zeros from the diagonal on)
+                a0 = fmaf(a.x, x[j], a0);
+                if (j + 1 < i) a1 = fmaf(a.y, x[j + 1], a1);
+                if (j + 2 < i) a0 = fmaf(a.z, x[j + 2], a0);
+                if (j + 3 < i) a1 = fmaf(a.w, x[j + 3], a1);
+            }
+            x[i] -= a0 + a1;
+        }
+        float *dst = is_w ? cb.w + ci * kChunk * DQ + col : cb.vp + ci * kChunk * dm.e + (col - DQ);
+        const uint32_t ld = is_w ? DQ : dm.e;
+#pragma unroll
+        for (uint32_t i = 0; i < kChunk; i++) dst[(uint64_t)i * ld] = x[i];
+    }
+    if (h % (H / KH) == 0) {  // K^T once per query/key head
+        float *kt = cb.kt + ((b * KH + hk) * cb.chunks + chunk) * DQ * kChunk;
+        for (uint32_t i = tid; i < DQ * kChunk; i += 256) kt[i] = kl[(i % kChunk) * KLD + i / kChunk];
+    }
+}
+
+// One workgroup of four waves per (16 columns of S, head, sequence).  Wave w keeps rows 16 QW w .. of the
+// state in accumulators, computes tokens 16 w .. of U and O, and hands both to the others through LDS.
+template <int QW>
+__global__ __launch_bounds__(256) void delta_carry_kernel(DeltaDims dm, const float *__restrict__ q, uint32_t dp, uint64_t n,
+                                                          uint64_t t0, uint64_t seg, ChunkBuf cb, float *state,
+                                                          float *__restrict__ o, uint32_t blocks, uint32_t units) {
+    constexpr uint32_t NT = 4 * QW, DQ = 16 * NT;
+    __shared__ float4_t sl[2][NT][64], ul[2][4][64];
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
+    const uint32_t H = dm.heads, KH = dm.kv_heads;
+    // all column blocks of a head on one XCD (consecutive workgroups go round the 8 XCDs): its chunk
+    // operands are fetched into one L2
+    uint32_t blk = blockIdx.x % blocks, unit = blockIdx.x / blocks;
+    if ((units & 7) == 0) {
+        const uint32_t idx = blockIdx.x >> 3;
+        blk = idx % blocks;
+        unit = (blockIdx.x & 7) + 8 * (idx / blocks);
+    }
+    const uint32_t h = unit % H, hk = h / (H / KH);
+    const uint64_t b = unit / H;
+    const uint32_t col = blk * 16 + c, colc = min(col, dm.e - 1);
+    float *sp = state + ((b * H + h) * (uint64_t)dm.d) * dm.e + colc;
+    float4_t s[QW];
+#pragma unroll
+    for (int t = 0; t < QW; t++)
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const uint32_t r = 16 * (QW * wave + t) + 4 * g + i;
+            s[t][i] = r < dm.d ? sp[(uint64_t)r * dm.e] : 0.f;
+        }
+    const uint32_t tok = 16 * wave + c;  // this lane's row of the left operands
+    float4 wa[NT], qa[NT], pa[4], ka[QW][4];
+    float4 eg4, ed4[4];
+    float v4[4], egc;
+    auto fetch = [&](uint32_t ch) {
+        const uint64_t ci = (b * H + h) * cb.chunks + ch;
+        const float *wp = cb.w + (ci * kChunk + tok) * DQ + 4 * g;
+        const uint64_t qrow = min((uint64_t)ch * kChunk + tok, seg - 1);  // (rows behind the end are not stored)
+        const float *qp = q + ((b * n + t0 + qrow) * KH + hk) * dp;
+#pragma unroll
+        for (uint32_t m = 0; m < NT; m++) {
+            wa[m] = *(const float4 *)(wp + 16 * m);
+            qa[m] = *(const float4 *)(qp + min(16 * m + 4 * g, dp - 4));  // (the state is zero behind d)
+        }
+        const float *pp = cb.p + (ci * kChunk + tok) * kChunk + 4 * g;
+        const float *kp = cb.kt + (((b * KH + hk) * cb.chunks + ch) * DQ + 16 * QW * wave + c) * kChunk + 4 * g;
+#pragma unroll
+        for (int t = 0; t < 4; t++) {
+            pa[t] = *(const float4 *)(pp + 16 * t);
+#pragma unroll
+            for (int u = 0; u < QW; u++) ka[u][t] = *(const float4 *)(kp + 16 * u * kChunk + 16 * t);
+            ed4[t] = *(const float4 *)(cb.ed + ci * kChunk + 16 * t + 4 * g);
+        }
+        eg4 = *(const float4 *)(cb.eg + ci * kChunk + 16 * wave + 4 * g);
+        egc = cb.eg[ci * kChunk + kChunk - 1];
+#pragma unroll
+        for (int i = 0; i < 4; i++) v4[i] = cb.vp[(ci * kChunk + 16 * wave + 4 * g + i) * dm.e + colc];
+    };
+    const uint32_t chunks = (uint32_t)((seg + kChunk - 1) / kChunk);
+    fetch(0);
+    for (uint32_t ch = 0; ch < chunks; ch++) {
+        const uint32_t buf = ch & 1;
+#pragma unroll
+        for (int t = 0; t < QW; t++) sl[buf][QW * wave + t][lane] = s[t];
+        lds_barrier();
+        float4_t au = {0.f, 0.f, 0.f, 0.f}, ao = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (uint32_t m = 0; m < NT; m++) {
+            const float4_t sb = sl[buf][m][lane];
+            au = mfma4(wa[m], sb, au);
+            ao = mfma4(qa[m], sb, ao);
+        }
+        float4_t u;
+#pragma unroll
+        for (int i = 0; i < 4; i++) u[i] = v4[i] - au[i];
+        ul[buf][wave][lane] = u;
+        ao[0] *= eg4.x; ao[1] *= eg4.y; ao[2] *= eg4.z; ao[3] *= eg4.w;
+        lds_barrier();
+        float4_t ub[4];
+#pragma unroll
+        for (int t = 0; t < 4; t++) ub[t] = ul[buf][t][lane];
+#pragma unroll
+        for (int t = 0; t < 4; t++)
+            if (t <= (int)wave) ao = mfma4(pa[t], ub[t], ao);
+#pragma unroll
+        for (int t = 0; t < 4; t++) { ub[t][0] *= ed4[t].x; ub[t][1] *= ed4[t].y; ub[t][2] *= ed4[t].z; ub[t][3] *= ed4[t].w; }
+#pragma unroll
+        for (int w = 0; w < QW; w++) {
+            s[w] *= egc;
+#pragma unroll
+            for (int t = 0; t < 4; t++) s[w] = mfma4(ka[w][t], ub[t], s[w]);
+        }
+        fetch(ch + 1 < chunks ? ch + 1 : ch);
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const uint64_t r = (uint64_t)ch * kChunk + 16 * wave + 4 * g + i;
+            if (r < seg && col < dm.e) o[((b * n + t0 + r) * H + h) * dm.e + col] = ao[i];
+        }
+    }
+    if (col < dm.e)
+#pragma unroll
+        for (int t = 0; t < QW; t++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const uint32_t r = 16 * (QW * wave + t) + 4 * g + i;
+                if (r < dm.d) sp[(uint64_t)r * dm.e] = s[t][i];
+            }
+}
+
+// A few dozen tokens are quicker one by one than through two launches of chunks.
+constexpr uint64_t kChunkedFrom = 48;
+
 uint64_t delta_prompt_scratch_bytes(const DeltaDims &dm, uint64_t batch, uint64_t n) {
-    (void)dm; (void)batch; (void)n;
-    return 0;
+    if (n < kChunkedFrom) return 0;
+    return chunk_floats(dm, batch, ceil_div(n < kSegment ? n : kSegment, kChunk)) * 4;
+}
+
+template <int QW>
+static int launch_chunks(const DeltaDims &dm, const DeltaOperands &op, const DeltaState &state, uint64_t batch, uint64_t n,
+                         float *o, float *scratch, hipStream_t st) {
+    constexpr uint32_t DQ = 64 * QW;
+    const uint32_t dp = delta_padded_dim(dm.d);
+    const size_t lds = (kChunk * (DQ + 4) + kChunk * (kChunk + 4)) * 4;
+    static const bool once = [] {
+        (void)hipFuncSetAttribute((const void *)delta_chunk_kernel<4 * QW>, hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024);
+        return true;
+    }();
+    (void)once;
+    for (uint64_t t0 = 0; t0 < n; t0 += kSegment) {
+        const uint64_t seg = n - t0 < kSegment ? n - t0 : kSegment;
+        ChunkBuf cb;
+        cb.chunks = (uint32_t)ceil_div(seg, kChunk);
+        float *p = scratch;
+        const uint64_t hc = batch * cb.chunks * dm.heads;
+        auto take = [&](uint64_t k) { float *r = p; p += k; return r; };
+        cb.w = take(hc * kChunk * DQ);
+        cb.p = take(hc * kChunk * kChunk);
+        cb.eg = take(hc * kChunk);
+        cb.ed = take(hc * kChunk);
+        cb.kt = take(batch * cb.chunks * dm.kv_heads * DQ * kChunk);
+        cb.vp = take(hc * kChunk * dm.e);  // last: its rows need no alignment
+        hipLaunchKernelGGL((delta_chunk_kernel<4 * QW>), dim3(cb.chunks, dm.heads, (unsigned)batch), dim3(256), lds, st, dm,
+                           op, dp, n, t0, seg, cb);
+        const uint32_t blocks = (uint32_t)ceil_div(dm.e, 16), units = (uint32_t)(dm.heads * batch);
+        hipLaunchKernelGGL((delta_carry_kernel<QW>), dim3(blocks * units), dim3(256), 0, st, dm, op.q, dp, n, t0, seg, cb,
+                           state.s, o, blocks, units);
+    }
+    COEUS_HIP(hipGetLastError());
+    return COEUS_OK;
 }
 
 int launch_delta_prompt(const DeltaDims &dm, const DeltaOperands &op, const DeltaState &state, uint64_t batch,
                         uint64_t n, float *o, float *scratch, uint64_t scratch_bytes, hipStream_t st) {
-    (void)scratch; (void)scratch_bytes;
     COEUS_TRY(check_dims(dm));
     COEUS_TRY(check_rows(batch, n));
-    if (dm.heads > 65535) return fail(COEUS_INVALID_INPUT, "delta rule: too many heads");
+    if (dm.heads > 65535 || (uint64_t)dm.heads * batch * ceil_div(dm.e, 16) > 0x7fffffffull)
+        return fail(COEUS_INVALID_INPUT, "delta rule: too many heads");
+    const uint64_t want = delta_prompt_scratch_bytes(dm, batch, n);
+    if (want && scratch && scratch_bytes >= want) {
+        switch (chunk_dim(dm.d) / 64) {
+            case 1: return launch_chunks<1>(dm, op, state, batch, n, o, scratch, st);
+            case 2: return launch_chunks<2>(dm, op, state, batch, n, o, scratch, st);
+            case 3: return launch_chunks<3>(dm, op, state, batch, n, o, scratch, st);
+            default: return launch_chunks<4>(dm, op, state, batch, n, o, scratch, st);
+        }
+    }
     const dim3 grid((unsigned)ceil_div(dm.e, 16), dm.heads, (unsigned)batch);
 #define COEUS_DS(RV) \
     case RV: hipLaunchKernelGGL(delta_scan_kernel<RV>, grid, dim3(256), 0, st, dm, op, state.s, n, o); break

@@ -995,12 +995,20 @@ static int launch_gemv_quant(const Weight &w, const __half *xq, uint64_t batch, 
 // and its waves read the normalised rows from there: no separate norm launch.  Wave b computes
 // the statistics of batch row b on its own (two passes over the row), while every wave already
 // has its first weights on the way.
+// NORM = 3: the norm of the sublayer before stands behind it.  x is the residual stream h, y the
+// sublayer's bare output: the workgroup stages h + y / rms(y) * scale (* ls), and the first one stores
+// these rows as the new residual stream.  LDS: y rows (then the sums), [2][k] scales, h rows behind them.
+struct PostNorm {
+    const float *y, *ls;
+    float *h_out;
+};
 template <bool BF16, int BP, int NORM>
 __global__ __launch_bounds__(1024) void gemv_dense_kernel(const void *__restrict__ wdata,
                                                           const float *__restrict__ x, uint64_t k,
                                                           uint32_t batch, EpiArgs e,
                                                           const float *__restrict__ nscale,
-                                                          const float *__restrict__ nbias, float eps) {
+                                                          const float *__restrict__ nbias, float eps,
+                                                          uint64_t ldx, PostNorm post) {
     extern __shared__ float xn[];  // NORM: [BP][k] rows, [2][k] scale and bias, partial sums, statistics
     const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nwaves = blockDim.x >> 6;
     const uint64_t j = (uint64_t)blockIdx.x * nwaves + wave;
@@ -1034,17 +1042,20 @@ __global__ __launch_bounds__(1024) void gemv_dense_kernel(const void *__restrict
         float *gs = xn + (size_t)BP * k, *bs = gs + k;  // scale, bias
         float *red = bs + k;                            // [16 waves][BP] partial sums
         float *stat = red + 16 * BP;                    // [0][b] mean, [1][b] standard deviation
+        float *hs = stat + 32;                          // NORM == 3: [BP][k] residual rows
         float ps[BP];
 #pragma unroll
         for (int b = 0; b < BP; b++) ps[b] = 0.f;
         for (uint64_t i = threadIdx.x; i < k; i += blockDim.x) {
             gs[i] = nscale[i];
             if (NORM == 1) bs[i] = nbias[i];
+            if (NORM == 3) bs[i] = post.ls ? post.ls[i] : 1.0f;
 #pragma unroll
             for (int b = 0; b < BP; b++)
                 if (b < (int)batch) {
-                    const float v = x[(uint64_t)b * k + i];
+                    const float v = NORM == 3 ? post.y[(uint64_t)b * k + i] : x[(uint64_t)b * ldx + i];
                     xn[(uint64_t)b * k + i] = v;
+                    if (NORM == 3) hs[(uint64_t)b * k + i] = x[(uint64_t)b * ldx + i];
                     ps[b] += v;
                 }
         }
@@ -1070,7 +1081,7 @@ __global__ __launch_bounds__(1024) void gemv_dense_kernel(const void *__restrict
         }
 #pragma unroll
         for (int b = 0; b < BP; b++) ps[b] = 0.f;
-        if (NORM == 2) __syncthreads();  // the rows and the zero means are in LDS
+        if (NORM >= 2) __syncthreads();  // the rows and the zero means are in LDS
         for (uint64_t i = threadIdx.x; i < k; i += blockDim.x)
 #pragma unroll
             for (int b = 0; b < BP; b++)
@@ -1087,8 +1098,15 @@ __global__ __launch_bounds__(1024) void gemv_dense_kernel(const void *__restrict
             const float g = gs[i], bi = NORM == 1 ? bs[i] : 0.f;
 #pragma unroll
             for (int b = 0; b < BP; b++)
-                if (b < (int)batch)
-                    xn[(uint64_t)b * k + i] = g * (xn[(uint64_t)b * k + i] - stat[b]) / stat[16 + b] + bi;
+                if (b < (int)batch) {
+                    if (NORM == 3) {
+                        const float v = fmaf(xn[(uint64_t)b * k + i] / stat[16 + b] * g, bs[i], hs[(uint64_t)b * k + i]);
+                        xn[(uint64_t)b * k + i] = v;
+                        if (blockIdx.x == 0) post.h_out[(uint64_t)b * k + i] = v;
+                    } else {
+                        xn[(uint64_t)b * k + i] = g * (xn[(uint64_t)b * k + i] - stat[b]) / stat[16 + b] + bi;
+                    }
+                }
         }
         __syncthreads();
         xs = xn;
@@ -1175,26 +1193,38 @@ bool gemv_can_fuse_norm_dense(const Weight &w, uint64_t batch) {
     return gemv_dense_norm_lds(w.k, pad_batch(batch)) <= kDenseNormLdsLimit;
 }
 
+static size_t gemv_dense_post_lds(uint64_t k, uint32_t bp) { return gemv_dense_norm_lds(k, bp) + (size_t)bp * k * 4; }
+bool gemv_can_fuse_post_norm(const Weight &w, uint64_t batch) {
+    if (w.dtype >= COEUS_W_Q8_0 || batch < 1 || batch > 16) return false;
+    return gemv_dense_post_lds(w.k, pad_batch(batch)) <= kDenseNormLdsLimit;
+}
+
 template <bool BF16>
 static int launch_gemv_dense(const Weight &w, const float *x, uint64_t batch, const EpiArgs &e,
                              hipStream_t st, const NormFuse *nf) {
     const uint32_t bp = pad_batch(batch), b = (uint32_t)batch;
-    if (nf && !gemv_can_fuse_norm_dense(w, batch))
+    const bool post_norm = nf && nf->y;
+    if (nf && !(post_norm ? gemv_can_fuse_post_norm(w, batch) : gemv_can_fuse_norm_dense(w, batch)))
         return fail(COEUS_INVALID_INPUT, "norm fusion needs the normalised activations to fit in LDS");
-    if (nf && (!nf->h || !nf->scale || (nf->kind == COEUS_NORM_LAYERNORM && !nf->bias)))
+    if (post_norm && (!nf->h || !nf->scale || !nf->h_out || nf->h_out == nf->h || nf->kind != COEUS_NORM_RMSNORM))
+        return fail(COEUS_INVALID_INPUT, "a norm behind the previous sublayer needs its output, the residual rows and "
+                                         "a place for the new ones");
+    if (nf && !post_norm && (!nf->h || !nf->scale || (nf->kind == COEUS_NORM_LAYERNORM && !nf->bias)))
         return fail(COEUS_INVALID_INPUT, "null pointer argument");
     // plain: 4 rows per workgroup; folded norm: 16, so that the block is normalised once per 16 rows
     const uint32_t waves = nf ? 16 : 4;
     const dim3 grid((unsigned)ceil_div(w.n, waves)), block(waves * 64);
-    const size_t lds = nf ? gemv_dense_norm_lds(w.k, bp) : 0;
-    const int norm = !nf ? 0 : nf->kind == COEUS_NORM_RMSNORM ? 2 : 1;
+    const size_t lds = !nf ? 0 : post_norm ? gemv_dense_post_lds(w.k, bp) : gemv_dense_norm_lds(w.k, bp);
+    const int norm = !nf ? 0 : post_norm ? 3 : nf->kind == COEUS_NORM_RMSNORM ? 2 : 1;
+    const uint64_t ldx = nf && nf->ld ? nf->ld : w.k;
+    const PostNorm post = post_norm ? PostNorm{nf->y, nf->ls, nf->h_out} : PostNorm{nullptr, nullptr, nullptr};
     const float *xin = nf ? nf->h : x;
     const float *ns = nf ? nf->scale : nullptr, *nb = nf ? nf->bias : nullptr;
     const float eps = nf ? nf->eps : 0.f;
 #define COEUS_GEMVD2(BPV, NV) \
-    hipLaunchKernelGGL((gemv_dense_kernel<BF16, BPV, NV>), grid, block, lds, st, w.data, xin, w.k, b, e, ns, nb, eps)
+    hipLaunchKernelGGL((gemv_dense_kernel<BF16, BPV, NV>), grid, block, lds, st, w.data, xin, w.k, b, e, ns, nb, eps, ldx, post)
 #define COEUS_GEMVD(BPV) \
-    do { if (norm == 0) COEUS_GEMVD2(BPV, 0); else if (norm == 1) COEUS_GEMVD2(BPV, 1); else COEUS_GEMVD2(BPV, 2); } while (0)
+    do { if (norm == 0) COEUS_GEMVD2(BPV, 0); else if (norm == 1) COEUS_GEMVD2(BPV, 1); else if (norm == 2) COEUS_GEMVD2(BPV, 2); else COEUS_GEMVD2(BPV, 3); } while (0)
     switch (bp) {
         case 1: COEUS_GEMVD(1); break;
         case 2: COEUS_GEMVD(2); break;

@@ -2,9 +2,14 @@
 //
 //   latent_norm_kernel        RMS norms of the query latent and of the key/value latent
 //   latent_gather / append    cached latents in front of a prompt's portion / its own into the ring
-//   window_attn_kernel        prompt: one wave per (row, head) on expanded keys and values
-//   latent_decode_kernel      decode: the query is taken into latent space (W_uk^T q), scored against the
-//                             cached latents, and the weighted latent is expanded by W_uv
+//   window_prefill_kernel     prompt, bf16: expanded keys and values on the matrix cores
+//   window_attn_kernel        prompt: one wave per (row, head), any size and type
+// Decode takes the query into latent space (W_uk^T q), scores it against the cached latents, which all
+// heads share, and expands the weighted latent by W_uv:
+//   latent_absorb_kernel      W_uk^T q of every head; the new token's latent, normalised, into the ring
+//   latent_scores_kernel      bf16: 16 heads against a share of the ring on the matrix cores
+//   latent_expand_kernel      merge of the shares, W_uv
+//   latent_decode_kernel      all of it in one workgroup per head, any size and type
 #include "device_utils.hpp"
 #include "mixers.hpp"
 
@@ -29,17 +34,18 @@ static int check_dims(const LatentDims &dm, const LatentCache &cache) {
     return COEUS_OK;
 }
 
-// blockIdx.y 0: the query latent, 1: the key/value latent.
+// blockIdx.y + part0 0: the query latent, 1: the key/value latent.
 template <bool BF16>
 __global__ __launch_bounds__(256) void latent_norm_kernel(const float *__restrict__ proj, LatentDims dm,
                                                           const float *__restrict__ q_scale,
                                                           const float *__restrict__ c_scale, float eps, uint64_t n,
                                                           float *cq, uint16_t *cq_lp, uint64_t cq_ld, bool lp_bf16,
                                                           void *lat, uint64_t lat_ld, uint64_t lat_rows,
-                                                          uint64_t lat_off, uint32_t cap, const uint32_t *pos_dev) {
+                                                          uint64_t lat_off, uint32_t cap, const uint32_t *pos_dev,
+                                                          uint32_t part0) {
     __shared__ float sh[4];
     const uint64_t row = blockIdx.x;
-    const bool is_q = blockIdx.y == 0;
+    const bool is_q = blockIdx.y + part0 == 0;
     const uint32_t len = is_q ? dm.q_rank : dm.rank, tid = threadIdx.x;
     const float *x = proj + row * dm.in_ld + (is_q ? 0 : dm.q_rank);
     float s2 = 0.f;
@@ -68,17 +74,18 @@ int launch_latent_norm(const float *proj, const LatentDims &dm, const float *q_s
     COEUS_TRY(check_dims(dm, cache));
     if (batch == 0 || n == 0 || batch * n > 0x7fffffffull || (pos_dev && n != 1))
         return fail(COEUS_INVALID_INPUT, "latent attention: rows out of range");
-    const dim3 grid((unsigned)(batch * n), 2);
+    const uint32_t part0 = cq || cq_lp ? 0 : 1;  // no place for the query latent: its consumer normalises it
+    const dim3 grid((unsigned)(batch * n), 2 - part0);
     uint16_t *lp = cq_lp ? (uint16_t *)cq_lp->p : nullptr;
     const uint64_t ld = cq_lp ? cq_lp->ld : 0;
     const bool lp_bf = cq_lp && cq_lp->bf16;
     void *dst = pos_dev ? cache.c : lat;
     if (cache.bf16)
         hipLaunchKernelGGL(latent_norm_kernel<true>, grid, dim3(256), 0, st, proj, dm, q_scale, c_scale, eps, n, cq, lp, ld,
-                           lp_bf, dst, lat_ld, lat_rows, lat_off, cache.cap, pos_dev);
+                           lp_bf, dst, lat_ld, lat_rows, lat_off, cache.cap, pos_dev, part0);
     else
         hipLaunchKernelGGL(latent_norm_kernel<false>, grid, dim3(256), 0, st, proj, dm, q_scale, c_scale, eps, n, cq, lp, ld,
-                           lp_bf, dst, lat_ld, lat_rows, lat_off, cache.cap, pos_dev);
+                           lp_bf, dst, lat_ld, lat_rows, lat_off, cache.cap, pos_dev, part0);
     COEUS_HIP(hipGetLastError());
     return COEUS_OK;
 }
@@ -177,6 +184,175 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const void *__restrict
     }
 }
 
+// ---------------------------------------------------------------- prompt attention on the matrix cores
+// The scheme of attn_prefill_kernel (scores and outputs transposed, so that a query stays in its lanes and
+// the weights never leave registers) with key and value sizes of their own, rounded up to DK and DV (a
+// piece behind the end re-reads the last one: its query dims are zero / its outputs are not stored), and a
+// lower edge.  The f32 weights enter the product with V as a sum of two bf16 numbers.
+__device__ __forceinline__ void split_bf16(float a, __bf16 &hi, __bf16 &lo) {
+    hi = (__bf16)a;
+    lo = (__bf16)(a - (float)hi);
+}
+
+template <int DK, int DV>
+__global__ __launch_bounds__(256) void window_prefill_kernel(const uint16_t *__restrict__ q, uint64_t q_ld,
+                                                             const uint16_t *__restrict__ kv, uint64_t kv_ld,
+                                                             LatentDims dm, uint32_t n, uint32_t hist,
+                                                             float *__restrict__ out, uint16_t *__restrict__ out_lp,
+                                                             uint64_t lp_ld, bool lp_bf16) {
+    constexpr int KT = 32, KLD = DK + 8, VLD = 36, NKS = DK / 16, NDT = DV / 32, KP = DK / 64, VP = (DV + 127) / 128;
+    extern __shared__ __attribute__((aligned(16))) uint16_t lds16[];
+    uint16_t *const ks = lds16, *const vt = lds16 + 2 * KT * KLD;  // [2][key][dim], [2][dim][key]
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, qi = lane & 31, hf = lane >> 5;
+    uint32_t qt, h;
+    prefill_tile_of_block(qt, h);
+    const uint64_t b = blockIdx.z;
+    const uint32_t r0 = qt * 128 + wave * 32, r = r0 + qi, rc = min(r, n - 1);
+    const uint32_t qkey = hist + rc, W = dm.window ? dm.window : 0xffffffffu;  // row rc is key qkey, sees (qkey - W, qkey]
+    const float scale2 = 1.4426950408889634f * dm.scale;
+    bf16x8_t qf[NKS];
+    {
+        const uint16_t *qp = q + (b * n + rc) * q_ld + h * dm.d;
+#pragma unroll
+        for (int s = 0; s < NKS; s++) {
+            union { uint4 u; bf16x8_t v; } cv;
+            const uint32_t d0 = 16 * s + 8 * hf;
+            cv.u = *(const uint4 *)(qp + min(d0, dm.d - 8));
+            if (d0 >= dm.d) cv.u = make_uint4(0, 0, 0, 0);
+            qf[s] = cv.v;
+        }
+    }
+    const uint16_t *kb = kv + b * (hist + n) * kv_ld + h * dm.d;
+    const uint16_t *vb = kv + b * (hist + n) * kv_ld + dm.heads * dm.d + h * dm.e;
+    const uint32_t first_q = hist + qt * 128, kmax = hist + min(n, qt * 128 + 128) - 1;
+    const uint32_t t_begin = (first_q >= W ? first_q - W + 1 : 0) / KT, t_end = kmax / KT + 1;
+    const uint32_t wave_lo = hist + min(r0, n - 1), wave_hi = hist + min(r0 + 31, n - 1);
+    const bool wave_live = r0 < n;
+
+    const uint32_t kkey = tid >> 3, kpc = tid & 7, va = tid & 15, vdp = tid >> 4;
+    uint4 rk[KP], rv[VP][2];
+    auto gload = [&](uint32_t t) {
+        const uint64_t krow = (uint64_t)min(t * KT + kkey, kmax) * kv_ld;
+#pragma unroll
+        for (int u = 0; u < KP; u++) rk[u] = *(const uint4 *)(kb + krow + min(8 * (kpc + 8 * u), dm.d - 8));
+#pragma unroll
+        for (int u = 0; u < VP; u++)
+            if (DV >= 128 || vdp < DV / 8) {
+                const uint32_t d0 = min(8 * (vdp + 16 * u), dm.e - 8);
+                rv[u][0] = *(const uint4 *)(vb + (uint64_t)min(t * KT + 2 * va, kmax) * kv_ld + d0);
+                rv[u][1] = *(const uint4 *)(vb + (uint64_t)min(t * KT + 2 * va + 1, kmax) * kv_ld + d0);
+            }
+    };
+    auto lstore = [&](uint32_t buf) {
+#pragma unroll
+        for (int u = 0; u < KP; u++) *(uint4 *)(ks + buf * KT * KLD + kkey * KLD + 8 * (kpc + 8 * u)) = rk[u];
+#pragma unroll
+        for (int u = 0; u < VP; u++)
+            if (DV >= 128 || vdp < DV / 8) {
+                const uint32_t a[4] = {rv[u][0].x, rv[u][0].y, rv[u][0].z, rv[u][0].w};
+                const uint32_t c[4] = {rv[u][1].x, rv[u][1].y, rv[u][1].z, rv[u][1].w};
+                uint32_t *dst = (uint32_t *)(vt + buf * DV * VLD) + (vdp + 16 * u) * (8 * VLD / 2) + va;
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    dst[e * VLD] = __builtin_amdgcn_perm(c[e], a[e], 0x05040100u);
+                    dst[e * VLD + VLD / 2] = __builtin_amdgcn_perm(c[e], a[e], 0x07060302u);
+                }
+            }
+    };
+    float16_t o[NDT];
+#pragma unroll
+    for (int d = 0; d < NDT; d++)
+#pragma unroll
+        for (int i = 0; i < 16; i++) o[d][i] = 0.f;
+    float m = -1e30f, l = 0.f;  // (finite: a tile may hold no key that this query sees)
+
+    gload(t_begin);
+    lstore(t_begin & 1);
+    gload(min(t_begin + 1, t_end - 1));
+    for (uint32_t t = t_begin; t < t_end; t++) {
+        __syncthreads();
+        lstore((t + 1) & 1);
+        gload(min(t + 2, t_end - 1));
+        const uint32_t k0 = t * KT;
+        if (!wave_live || k0 > wave_hi || (wave_lo >= W && k0 + KT - 1 <= wave_lo - W)) continue;  // wave-uniform
+        const uint16_t *kt_ = ks + (t & 1) * KT * KLD, *vt_ = vt + (t & 1) * DV * VLD;
+        float16_t sc;
+#pragma unroll
+        for (int i = 0; i < 16; i++) sc[i] = 0.f;
+#pragma unroll
+        for (int s = 0; s < NKS; s++)
+            sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8_t *)(kt_ + qi * KLD + 16 * s + 8 * hf), qf[s], sc, 0, 0, 0);
+        float tmax = -INFINITY;
+#pragma unroll
+        for (int i = 0; i < 16; i++) sc[i] *= scale2;
+        if (k0 + KT - 1 > wave_lo || (wave_hi >= W && k0 <= wave_hi - W)) {  // an edge crosses the tile
+#pragma unroll
+            for (int i = 0; i < 16; i++) {
+                const uint32_t key = k0 + 4 * hf + 8 * (i >> 2) + (i & 3);
+                sc[i] = key > qkey || qkey - key >= W ? -INFINITY : sc[i];
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < 16; i++) tmax = fmaxf(tmax, sc[i]);
+        const float m_new = fmaxf(m, both_halves_max(tmax));
+        float psum = 0.f, pv[16];
+#pragma unroll
+        for (int i = 0; i < 16; i++) {
+            pv[i] = __builtin_amdgcn_exp2f(sc[i] - m_new);  // 2^(-inf) = 0 for keys that are not seen
+            psum += pv[i];
+        }
+        if (__builtin_amdgcn_ballot_w64(m_new != m) != 0) {
+            const float corr = __builtin_amdgcn_exp2f(m - m_new);
+            l *= corr;
+#pragma unroll
+            for (int d = 0; d < NDT; d++)
+#pragma unroll
+                for (int i = 0; i < 16; i++) o[d][i] *= corr;
+        }
+        l += psum;
+        m = m_new;
+        bf16x8_t ph[2], pl[2];
+#pragma unroll
+        for (int j = 0; j < 2; j++)
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                __bf16 hi, lo;
+                split_bf16(pv[8 * j + e], hi, lo);
+                ph[j][e] = hi;
+                pl[j][e] = lo;
+            }
+#pragma unroll
+        for (int d = 0; d < NDT; d++)
+#pragma unroll
+            for (int j = 0; j < 2; j++) {
+                const uint16_t *vp = vt_ + (d * 32 + qi) * VLD + 16 * j + 4 * hf;
+                const uint2 v0 = *(const uint2 *)vp, v1 = *(const uint2 *)(vp + 8);
+                union { uint4 u; bf16x8_t v; } vf;
+                vf.u = make_uint4(v0.x, v0.y, v1.x, v1.y);
+                o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf.v, pl[j], o[d], 0, 0, 0);
+                o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf.v, ph[j], o[d], 0, 0, 0);
+            }
+    }
+    if (r >= n) return;
+    const float inv = 1.0f / xor32_sum(l);
+    const uint64_t row = b * n + r;
+#pragma unroll
+    for (int d = 0; d < NDT; d++)
+#pragma unroll
+        for (int gq = 0; gq < 4; gq++) {
+            const uint32_t c0 = d * 32 + 8 * gq + 4 * hf;  // e % 8 == 0: four columns are all in or all out
+            if (c0 >= dm.e) continue;
+            const float v[4] = {o[d][4 * gq] * inv, o[d][4 * gq + 1] * inv, o[d][4 * gq + 2] * inv, o[d][4 * gq + 3] * inv};
+            if (out) *(float4 *)(out + row * dm.heads * dm.e + h * dm.e + c0) = make_float4(v[0], v[1], v[2], v[3]);
+            if (out_lp) {
+                uint2 p;
+                p.x = (uint32_t)f32_to_lp_bits(v[0], lp_bf16) | ((uint32_t)f32_to_lp_bits(v[1], lp_bf16) << 16);
+                p.y = (uint32_t)f32_to_lp_bits(v[2], lp_bf16) | ((uint32_t)f32_to_lp_bits(v[3], lp_bf16) << 16);
+                *(uint2 *)(out_lp + row * lp_ld + h * dm.e + c0) = p;
+            }
+        }
+}
+
 int launch_window_attention(const void *q, uint64_t q_ld, const void *kv, uint64_t kv_ld, bool bf16,
                             const LatentDims &dm, uint64_t batch, uint64_t n, uint64_t hist, float *out,
                             const LpOut *out_lp, hipStream_t st) {
@@ -186,6 +362,27 @@ int launch_window_attention(const void *q, uint64_t q_ld, const void *kv, uint64
     uint16_t *lp = out_lp ? (uint16_t *)out_lp->p : nullptr;
     const uint64_t lp_ld = out_lp ? out_lp->ld : 0;
     const bool lp_bf = out_lp && out_lp->bf16;
+    // the matrix-core kernel moves 8 dims at a time
+    if (bf16 && dm.d % 8 == 0 && dm.e % 8 == 0 && q_ld % 8 == 0 && kv_ld % 8 == 0 && lp_ld % 4 == 0) {
+        const dim3 pgrid((unsigned)ceil_div(n, 128), dm.heads, (unsigned)batch);
+#define COEUS_WP(DKV, DVV)                                                                                           \
+    do {                                                                                                             \
+        static const bool once = hipFuncSetAttribute((const void *)window_prefill_kernel<DKV, DVV>,                  \
+                                                     hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024) == hipSuccess; \
+        (void)once;                                                                                                  \
+        hipLaunchKernelGGL((window_prefill_kernel<DKV, DVV>), pgrid, dim3(256), (2 * 32 * (DKV + 8) + 2 * DVV * 36) * 2, st, \
+                           (const uint16_t *)q, q_ld, (const uint16_t *)kv, kv_ld, dm, (uint32_t)n, (uint32_t)hist, out, lp, \
+                           lp_ld, lp_bf);                                                                            \
+    } while (0)
+#define COEUS_WPV(DKV) do { if (dm.e <= 64) COEUS_WP(DKV, 64); else if (dm.e <= 128) COEUS_WP(DKV, 128); else COEUS_WP(DKV, 256); } while (0)
+        if (dm.d <= 64) COEUS_WPV(64);
+        else if (dm.d <= 128) COEUS_WPV(128);
+        else COEUS_WPV(256);
+#undef COEUS_WPV
+#undef COEUS_WP
+        COEUS_HIP(hipGetLastError());
+        return COEUS_OK;
+    }
     const dim3 grid((unsigned)ceil_div(n, 4), dm.heads, (unsigned)batch);
     const size_t lds = 4 * (dm.d + 64) * sizeof(float);
     if (bf16)
@@ -255,17 +452,256 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const float *__restr
     }
 }
 
-uint64_t latent_decode_scratch_bytes(const LatentDims &dm, uint32_t cap, uint64_t batch) {
-    (void)dm; (void)cap; (void)batch;
-    return 0;
+// ---------------------------------------------------------------- decode, 16-bit cache
+constexpr uint32_t kKeyTile = 64, kMaxShares = 32;
+
+static bool latent_decode_fast(const LatentDims &dm, bool bf16) {
+    return bf16 && dm.rank % 32 == 0 && dm.rank <= 1024 && dm.d % 4 == 0;
+}
+static uint32_t latent_shares(uint32_t cap) {
+    const uint64_t tiles = ceil_div(cap, kKeyTile);
+    return (uint32_t)(tiles < kMaxShares ? tiles : kMaxShares);
+}
+
+// W_uk^T q, [batch][heads][rank]: one workgroup per (128 columns of the rank, head) and every sequence, so
+// that the weights are read once.  Thread (g, r): column pair r, rows g, g + 4, ..
+template <int BP>
+__global__ __launch_bounds__(256) void latent_absorb_kernel(const float *__restrict__ q, const uint16_t *__restrict__ ukv,
+                                                            LatentDims dm, uint32_t batch, float *__restrict__ qa) {
+    extern __shared__ float lds[];  // q [BP][d], partial sums [4][BP][128]
+    const uint32_t tid = threadIdx.x, g = tid >> 6, rp = tid & 63, h = blockIdx.y, d = dm.d, R = dm.rank;
+    const uint32_t r = blockIdx.x * 128 + 2 * rp, rc = min(r, R - 2);
+    float *qs = lds, *red = lds + BP * d;
+    const uint16_t *w = ukv + (uint64_t)h * d * R + rc;
+    for (uint32_t i = tid; i < BP * d; i += 256) {
+        const uint32_t b = i / d;
+        qs[i] = b < batch ? q[(uint64_t)b * dm.heads * d + h * d + i % d] : 0.f;
+    }
+    float a0[BP], a1[BP];
+#pragma unroll
+    for (int b = 0; b < BP; b++) a0[b] = a1[b] = 0.f;
+    __syncthreads();
+    constexpr int U = 16;  // rows of a thread in flight
+    for (uint32_t t0 = g; t0 < d; t0 += 4 * U) {
+        uint32_t x[U];
+#pragma unroll
+        for (int u = 0; u < U; u++) x[u] = *(const uint32_t *)(w + (uint64_t)min(t0 + 4 * u, d - 1) * R);
+#pragma unroll
+        for (int u = 0; u < U; u++) {
+            const uint32_t t = t0 + 4 * u;
+            const float lo = __uint_as_float(x[u] << 16), hi = __uint_as_float(x[u] & 0xffff0000u);
+#pragma unroll
+            for (int b = 0; b < BP; b++) {
+                const float qv = t < d ? qs[b * d + t] : 0.f;
+                a0[b] = fmaf(qv, lo, a0[b]);
+                a1[b] = fmaf(qv, hi, a1[b]);
+            }
+        }
+    }
+#pragma unroll
+    for (int b = 0; b < BP; b++) *(float2 *)(red + (g * BP + b) * 128 + 2 * rp) = make_float2(a0[b], a1[b]);
+    __syncthreads();
+    for (uint32_t i = tid; i < batch * 128; i += 256) {
+        const uint32_t b = i / 128, cc = i % 128, rr = blockIdx.x * 128 + cc;
+        if (rr < R)
+            qa[((uint64_t)b * dm.heads + h) * R + rr] = (red[b * 128 + cc] + red[(BP + b) * 128 + cc]) +
+                                                        (red[(2 * BP + b) * 128 + cc] + red[(3 * BP + b) * 128 + cc]);
+    }
+}
+
+// One workgroup of four waves per (share of the ring, 16 heads, sequence).  A wave scores 16 of a tile's 64
+// latents for 16 heads, the softmax of the tile runs over LDS, then a wave accumulates a quarter of the
+// rank.  Absorbed queries and weights are f32: both enter the products as sums of two bf16 numbers.
+// The share's record: maximum (base 2), sum, weighted latent.
+__global__ __launch_bounds__(256) void latent_scores_kernel(const float *__restrict__ qa, LatentDims dm,
+                                                            const uint16_t *__restrict__ cache, uint32_t cap,
+                                                            const uint32_t *pos_dev, uint32_t keys_per_share,
+                                                            float *__restrict__ part) {
+    constexpr uint32_t VLD = kKeyTile + 8, PLD = kKeyTile + 8;
+    extern __shared__ __attribute__((aligned(16))) uint16_t lds16[];
+    uint16_t *ct = lds16;                                    // latents of the tile, [rank][VLD]
+    uint16_t *ph = ct + dm.rank * VLD, *pl = ph + 16 * PLD;  // weights, high and low parts, [16][PLD]
+    float *ss = (float *)(pl + 16 * PLD);                    // scores [16][PLD]
+    float *ms = ss + 16 * PLD, *ls = ms + 16, *cs = ls + 16; // running maximum and sum, correction, per head
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4, R = dm.rank;
+    const uint32_t share = blockIdx.x, h0 = blockIdx.y * 16, hc = min(h0 + c, dm.heads - 1);
+    const uint64_t b = blockIdx.z;
+    const uint32_t nv = min(*pos_dev + 1, cap), k_begin = share * keys_per_share, k_end = min(nv, k_begin + keys_per_share);
+    const float scale2 = 1.4426950408889634f * dm.scale;
+    if (tid < 16) { ms[tid] = -1e30f; ls[tid] = 0.f; }
+    const float *qp = qa + (b * dm.heads + hc) * R + 8 * g;
+    const uint16_t *cb = cache + b * cap * R;
+    const uint32_t per = ((R / 16) + 3) / 4;  // 16-wide column tiles of a wave (at most 16)
+    float4_t acc[16];
+#pragma unroll
+    for (int t = 0; t < 16; t++) acc[t] = float4_t{0.f, 0.f, 0.f, 0.f};
+    for (uint32_t k0 = k_begin; k0 < k_end; k0 += kKeyTile) {
+        // transposed latents: two keys a dword
+        for (uint32_t i = tid; i < 256 * ((R / 8 + 7) / 8); i += 256) {  // 8 pieces x 32 key pairs a round
+            const uint32_t piece = (i & 7) + 8 * (i / 256), a = (i >> 3) & 31;
+            if (piece < R / 8) {
+                const uint4 x = *(const uint4 *)(cb + (uint64_t)min(k0 + 2 * a, k_end - 1) * R + 8 * piece);
+                const uint4 y = *(const uint4 *)(cb + (uint64_t)min(k0 + 2 * a + 1, k_end - 1) * R + 8 * piece);
+                const uint32_t xs[4] = {x.x, x.y, x.z, x.w}, ys[4] = {y.x, y.y, y.z, y.w};
+                uint32_t *dst = (uint32_t *)ct + piece * (8 * VLD / 2) + a;
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    dst[e * VLD] = __builtin_amdgcn_perm(ys[e], xs[e], 0x05040100u);
+                    dst[e * VLD + VLD / 2] = __builtin_amdgcn_perm(ys[e], xs[e], 0x07060302u);
+                }
+            }
+        }
+        // scores of keys k0 + 16 wave + c
+        float4_t sc = {0.f, 0.f, 0.f, 0.f}, sc2 = {0.f, 0.f, 0.f, 0.f};
+        const uint16_t *kp = cb + (uint64_t)min(k0 + 16 * wave + c, k_end - 1) * R + 8 * g;
+#pragma unroll 4
+        for (uint32_t s = 0; s < R / 32; s++) {
+            const float4 q0 = *(const float4 *)(qp + 32 * s), q1 = *(const float4 *)(qp + 32 * s + 4);
+            const float qv[8] = {q0.x, q0.y, q0.z, q0.w, q1.x, q1.y, q1.z, q1.w};
+            bf16x8_t qh, ql;
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                __bf16 hi, lo;
+                split_bf16(qv[e], hi, lo);
+                qh[e] = hi;
+                ql[e] = lo;
+            }
+            const bf16x8_t kf = *(const bf16x8_t *)(kp + 32 * s);
+            sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh, kf, sc, 0, 0, 0);
+            sc2 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ql, kf, sc2, 0, 0, 0);
+        }
+        const uint32_t key = k0 + 16 * wave + c;
+#pragma unroll
+        for (int i = 0; i < 4; i++) ss[(4 * g + i) * PLD + 16 * wave + c] = key < k_end ? (sc[i] + sc2[i]) * scale2 : -INFINITY;
+        __syncthreads();
+        // wave w: the softmax of heads 4 w .. 4 w + 3, a key per lane
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const uint32_t hh = 4 * wave + i;
+            const float s = ss[hh * PLD + lane], m_old = ms[hh];
+            const float m_new = fmaxf(m_old, wave_max(s)), p = __builtin_amdgcn_exp2f(s - m_new);
+            const float sum = wave_sum(p), corr = __builtin_amdgcn_exp2f(m_old - m_new);
+            __bf16 hi, lo;
+            split_bf16(p, hi, lo);
+            ((__bf16 *)ph)[hh * PLD + lane] = hi;
+            ((__bf16 *)pl)[hh * PLD + lane] = lo;
+            if (lane == 0) { ms[hh] = m_new; ls[hh] = ls[hh] * corr + sum; cs[hh] = corr; }
+        }
+        __syncthreads();
+        float cr[4];
+#pragma unroll
+        for (int i = 0; i < 4; i++) cr[i] = cs[4 * g + i];
+        bf16x8_t pah[2], pal[2];
+#pragma unroll
+        for (int j = 0; j < 2; j++) {
+            pah[j] = *(const bf16x8_t *)(ph + c * PLD + 32 * j + 8 * g);
+            pal[j] = *(const bf16x8_t *)(pl + c * PLD + 32 * j + 8 * g);
+        }
+#pragma unroll
+        for (int t = 0; t < 16; t++) {
+            const uint32_t tile = wave * per + t;
+            if (t < (int)per && 16 * tile < R) {  // wave-uniform
+#pragma unroll
+                for (int i = 0; i < 4; i++) acc[t][i] *= cr[i];
+#pragma unroll
+                for (int j = 0; j < 2; j++) {
+                    const bf16x8_t vf = *(const bf16x8_t *)(ct + (16 * tile + c) * VLD + 32 * j + 8 * g);
+                    acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pal[j], vf, acc[t], 0, 0, 0);
+                    acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pah[j], vf, acc[t], 0, 0, 0);
+                }
+            }
+        }
+        __syncthreads();  // everybody is done with this tile
+    }
+    if (k_begin >= k_end) __syncthreads();  // an empty share: the initial maxima and sums are its record
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        const uint32_t hh = h0 + 4 * g + i;
+        if (hh >= dm.heads) continue;
+        float *rec = part + ((b * dm.heads + hh) * gridDim.x + share) * (R + 2);
+        if (wave == 0 && c == 0) { rec[0] = ms[4 * g + i]; rec[1] = ls[4 * g + i]; }
+#pragma unroll
+        for (int t = 0; t < 16; t++) {
+            const uint32_t r = 16 * (wave * per + t) + c;
+            if (t < (int)per && r < R) rec[2 + r] = acc[t][i];
+        }
+    }
+}
+
+// One workgroup per (32 value dims, head, sequence): merges the shares, then W_uv rows against the result.
+__global__ __launch_bounds__(256) void latent_expand_kernel(const float *__restrict__ part, const uint16_t *__restrict__ ukv,
+                                                            LatentDims dm, uint32_t shares, float *__restrict__ out) {
+    extern __shared__ float lds[];  // merged latent [rank]
+    __shared__ float ws[kMaxShares], lt_s;
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.y, R = dm.rank;
+    const uint64_t b = blockIdx.z;
+    const float *rec = part + (b * dm.heads + h) * shares * (R + 2);
+    if (wave == 0) {
+        const float m = lane < shares ? rec[lane * (R + 2)] : -1e30f, mm = wave_max(m);
+        const float w = lane < shares ? __builtin_amdgcn_exp2f(m - mm) : 0.f;
+        const float lt = wave_sum(lane < shares ? rec[lane * (R + 2) + 1] * w : 0.f);
+        if (lane < shares) ws[lane] = w;
+        if (lane == 0) lt_s = lt;
+    }
+    __syncthreads();
+    for (uint32_t r = tid; r < R; r += 256) {
+        float a = 0.f;
+        for (uint32_t s = 0; s < shares; s++) a = fmaf(ws[s], rec[s * (R + 2) + 2 + r], a);
+        lds[r] = a / lt_s;
+    }
+    __syncthreads();
+    const uint32_t c_end = min(dm.e, blockIdx.x * 32 + 32);
+    for (uint32_t cc = blockIdx.x * 32 + wave; cc < c_end; cc += 4) {
+        const uint16_t *w = ukv + ((uint64_t)dm.heads * dm.d + h * dm.e + cc) * R;
+        float a = 0.f;
+        for (uint32_t r = lane * 8; r < R; r += 512) {
+            const uint4 x = *(const uint4 *)(w + r);
+            const uint32_t xs[4] = {x.x, x.y, x.z, x.w};
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                a = fmaf(__uint_as_float(xs[e] << 16), lds[r + 2 * e], a);
+                a = fmaf(__uint_as_float(xs[e] & 0xffff0000u), lds[r + 2 * e + 1], a);
+            }
+        }
+        a = wave_sum(a);
+        if (lane == 0) out[b * dm.heads * dm.e + h * dm.e + cc] = a;
+    }
+}
+
+uint64_t latent_decode_scratch_bytes(const LatentDims &dm, const LatentCache &cache, uint64_t batch) {
+    if (!latent_decode_fast(dm, cache.bf16)) return 0;
+    // absorbed queries, then a record per (sequence, head, share)
+    return batch * dm.heads * (dm.rank + latent_shares(cache.cap) * (dm.rank + 2ull)) * 4;
 }
 
 int launch_latent_decode(const float *q, const void *ukv, const LatentDims &dm, const LatentCache &cache,
                          uint64_t batch, const uint32_t *pos_dev, float *out, float *scratch, uint64_t scratch_bytes,
                          hipStream_t st) {
-    (void)scratch; (void)scratch_bytes;
     COEUS_TRY(check_dims(dm, cache));
     if (batch == 0 || batch > 65535 || !pos_dev) return fail(COEUS_INVALID_INPUT, "latent attention: rows out of range");
+    const uint64_t want = latent_decode_scratch_bytes(dm, cache, batch);
+    if (want && batch <= 16 && scratch && scratch_bytes >= want) {
+        const uint16_t *w = (const uint16_t *)ukv, *cc = (const uint16_t *)cache.c;
+        float *qa = scratch, *part = scratch + batch * dm.heads * dm.rank;
+        const uint32_t shares = latent_shares(cache.cap), bp = pad_batch(batch), R = dm.rank;
+        const uint32_t per_share = (uint32_t)round_up(ceil_div(cache.cap, shares), kKeyTile);
+        const dim3 agrid((unsigned)ceil_div(R, 128), dm.heads);
+        const size_t alds = (bp * (size_t)dm.d + 4 * bp * 128) * 4;
+#define COEUS_LA(BPV) \
+    case BPV: hipLaunchKernelGGL(latent_absorb_kernel<BPV>, agrid, dim3(256), alds, st, q, w, dm, (uint32_t)batch, qa); break
+        switch (bp) { COEUS_LA(1); COEUS_LA(2); COEUS_LA(4); COEUS_LA(8); COEUS_LA(16); }
+#undef COEUS_LA
+        static const bool once = hipFuncSetAttribute((const void *)latent_scores_kernel,
+                                                     hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) == hipSuccess;
+        (void)once;
+        const size_t slds = ((size_t)R * (kKeyTile + 8) + 2 * 16 * (kKeyTile + 8)) * 2 + (16 * (kKeyTile + 8) + 48) * 4;
+        hipLaunchKernelGGL(latent_scores_kernel, dim3(shares, (unsigned)ceil_div(dm.heads, 16), (unsigned)batch), dim3(256),
+                           slds, st, qa, dm, cc, cache.cap, pos_dev, per_share, part);
+        hipLaunchKernelGGL(latent_expand_kernel, dim3((unsigned)ceil_div(dm.e, 32), dm.heads, (unsigned)batch), dim3(256),
+                           (size_t)R * 4, st, part, w, dm, shares, out);
+        COEUS_HIP(hipGetLastError());
+        return COEUS_OK;
+    }
     const dim3 grid(dm.heads, (unsigned)batch);
     const size_t lds = 5 * (size_t)dm.rank * 4;
     if (cache.bf16)

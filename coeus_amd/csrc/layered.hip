@@ -489,10 +489,11 @@ int layered_session_init(Session &s) {
         up(ff, ly.spec.ff);
         if (mx.kind == MixerKind::LatentAttention) {
             up(q, mx.q_rank + mx.heads * mx.dim);
-            up(sc, latent_decode_scratch_bytes(ly.latent_dims(), s.state.layers[l].latent.cap, B));
+            up(sc, latent_decode_scratch_bytes(ly.latent_dims(), s.state.layers[l].latent, B));
         }
     }
     COEUS_TRY(s.dh.ensure(B * W * 4));
+    COEUS_TRY(s.dh2.ensure(B * W * 4));
     COEUS_TRY(s.dx.ensure(B * W * 4));
     COEUS_TRY(s.dqkv.ensure(B * in * 4));
     COEUS_TRY(s.datt.ensure(B * att * 4));
@@ -509,30 +510,62 @@ int layered_session_init(Session &s) {
 }
 
 // One decode step behind the embedding (s.dh holds the residual stream): only enqueues kernels.
+// The norm behind a sublayer is folded into the matmul that reads the stream next, like the norms in front
+// of the transformer's matmuls: `pending` is the sublayer output that the stream has not taken in yet.  The
+// folded form reads the stream and writes the new one, so the two buffers change places.
 int layered_decode(Session &s, hipStream_t st, int only, uint64_t *launches, uint64_t *bytes) {
     Model &m = *s.m;
     const LayeredStack &stack = *m.stack;
     const uint64_t B = s.batch, W = stack.cfg.width;
     const bool matmuls = only != STEP_ATTENTION, mixers = only != STEP_MATMULS, rest = only == STEP_ALL;
     const uint32_t *pos = (const uint32_t *)s.dpos.p;
-    float *h = (float *)s.dh.p, *y = (float *)s.dx.p, *proj = (float *)s.dqkv.p, *att = (float *)s.datt.p, *ff = (float *)s.dff.p;
+    float *h = (float *)s.dh.p, *h_other = (float *)s.dh2.p, *y = (float *)s.dx.p, *proj = (float *)s.dqkv.p,
+          *att = (float *)s.datt.p, *ff = (float *)s.dff.p;
     const float eps = stack.cfg.eps;
+    struct { const float *norm = nullptr, *ls = nullptr; } pending;
     uint64_t n_launch = 0, n_bytes = 0;
-    auto gemv = [&](const Weight &w, const float *x, float *dst, uint32_t act = COEUS_EPI_NONE) -> int {
+    auto count = [&](const Weight &w, bool gated) {
+        n_launch++;
+        n_bytes += gemv_algorithmic_bytes(w, B, gated, true);
+    };
+    auto gemv = [&](const Weight &w, const float *x, float *dst) -> int {
         if (!matmuls) return COEUS_OK;
         Epilogue e;
         e.out_f32 = dst;
-        e.act = act;
-        n_launch++;
-        n_bytes += gemv_algorithmic_bytes(w, B, act == COEUS_EPI_SILU_GATE, false);
+        count(w, false);
         return launch_gemv(w, x, B, e, st);
     };
-    auto add = [&](const float *norm, const float *ls) { return rest ? launch_norm_residual(y, B, W, norm, ls, eps, h, st) : COEUS_OK; };
+    auto settle = [&]() -> int {  // the pending sublayer output into the stream, as a launch of its own
+        if (rest && pending.norm) COEUS_TRY(launch_norm_residual(y, B, W, pending.norm, pending.ls, eps, h, st));
+        pending.norm = nullptr;
+        return COEUS_OK;
+    };
+    // a matmul of the residual stream (the same limit on the output rows as for norms in front of it: every
+    // workgroup of 16 rows repeats the norm)
+    auto stream_gemv = [&](const Weight &w, float *dst, uint32_t act = COEUS_EPI_NONE) -> int {
+        Epilogue e;
+        e.out_f32 = dst;
+        e.act = act;
+        if (s.fuse && pending.norm && w.n <= 16384 && gemv_can_fuse_post_norm(w, B)) {
+            if (!matmuls) return COEUS_OK;
+            NormFuse nf;
+            nf.h = h; nf.scale = pending.norm; nf.ls = pending.ls; nf.y = y; nf.h_out = h_other;
+            nf.eps = eps; nf.kind = COEUS_NORM_RMSNORM;
+            pending.norm = nullptr;
+            std::swap(h, h_other);
+            count(w, act == COEUS_EPI_SILU_GATE);
+            return launch_gemv(w, nullptr, B, e, st, &nf);
+        }
+        COEUS_TRY(settle());
+        if (!matmuls) return COEUS_OK;
+        count(w, act == COEUS_EPI_SILU_GATE);
+        return launch_gemv(w, h, B, e, st);
+    };
     for (size_t l = 0; l < stack.layers.size(); l++) {
         const LayeredLayer &ly = stack.layers[l];
         const LayeredState::Layer &sl = s.state.layers[l];
         const MixerSpec &mx = ly.spec.mixer;
-        COEUS_TRY(gemv(ly.in, h, proj));
+        COEUS_TRY(stream_gemv(ly.in, proj));
         if (mx.kind == MixerKind::GatedDelta) {
             if (mixers) {
                 COEUS_TRY(launch_delta_step(proj, ly.delta_dims(), ly.delta, sl.delta, B, pos, att, st));
@@ -545,9 +578,20 @@ int layered_decode(Session &s, hipStream_t st, int only, uint64_t *launches, uin
         } else {
             const LatentDims dm = ly.latent_dims();
             float *cq = (float *)s.dmix.p, *q = cq + B * mx.q_rank;
+            const bool fold = s.fuse && gemv_can_fuse_norm_dense(ly.uq, B);
             if (rest)
-                COEUS_TRY(launch_latent_norm(proj, dm, ly.dq_norm, ly.dkv_norm, eps, B, 1, cq, nullptr, nullptr, 0, 0, 0, sl.latent, pos, st));
-            COEUS_TRY(gemv(ly.uq, cq, q));
+                COEUS_TRY(launch_latent_norm(proj, dm, ly.dq_norm, ly.dkv_norm, eps, B, 1, fold ? nullptr : cq, nullptr, nullptr,
+                                             0, 0, 0, sl.latent, pos, st));
+            if (fold && matmuls) {  // the query latent's norm rides on its expansion
+                Epilogue e;
+                e.out_f32 = q;
+                NormFuse nf;
+                nf.h = proj; nf.ld = ly.in.n; nf.scale = ly.dq_norm; nf.eps = eps; nf.kind = COEUS_NORM_RMSNORM;
+                count(ly.uq, false);
+                COEUS_TRY(launch_gemv(ly.uq, nullptr, B, e, st, &nf));
+            } else if (!fold) {
+                COEUS_TRY(gemv(ly.uq, cq, q));
+            }
             if (mixers) {
                 COEUS_TRY(launch_latent_decode(q, ly.ukv.data, dm, sl.latent, B, pos, att, (float *)s.dscratch.p, s.dscratch.bytes, st));
                 if (only == STEP_ATTENTION) {
@@ -558,13 +602,16 @@ int layered_decode(Session &s, hipStream_t st, int only, uint64_t *launches, uin
             }
         }
         COEUS_TRY(gemv(ly.o, att, y));
-        COEUS_TRY(add(ly.norm1, ly.ls1));
+        pending.norm = ly.norm1;
+        pending.ls = ly.ls1;
         if (ly.spec.ff) {
-            COEUS_TRY(gemv(ly.up, h, ff, COEUS_EPI_SILU_GATE));
+            COEUS_TRY(stream_gemv(ly.up, ff, COEUS_EPI_SILU_GATE));
             COEUS_TRY(gemv(ly.down, ff, y));
-            COEUS_TRY(add(ly.norm2, ly.ls2));
+            pending.norm = ly.norm2;
+            pending.ls = ly.ls2;
         }
     }
+    COEUS_TRY(settle());
     if (rest)
         COEUS_TRY(launch_norm(COEUS_NORM_RMSNORM, COEUS_SCOPE_TOKEN, h, B, W, m.fin_s, nullptr, eps, y, nullptr, 0, st));
     COEUS_TRY(gemv(m.out, y, (float *)s.dlogits.p));

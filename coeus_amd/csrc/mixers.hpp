@@ -66,7 +66,7 @@ struct LatentCache {
     uint32_t cap;
     bool bf16;  // else f32
 };
-// Normalises both latents of every row.  cq: f32 rows (cq) and / or 16-bit rows (cq_lp).  c goes to
+// Normalises both latents of every row.  cq: f32 rows (cq) and / or 16-bit rows (cq_lp); neither: only c.  c goes to
 // `lat`, rows of lat_ld elements in the cache's type, row (b, i) at b * lat_rows + lat_off + i; with
 // `pos_dev` (one row per sequence) it goes to the cache slot of position *pos_dev instead.
 int launch_latent_norm(const float *proj, const LatentDims &dm, const float *q_scale, const float *c_scale, float eps,
@@ -90,6 +90,6 @@ int launch_window_attention(const void *q, uint64_t q_ld, const void *kv, uint64
 int launch_latent_decode(const float *q, const void *ukv, const LatentDims &dm, const LatentCache &cache,
                          uint64_t batch, const uint32_t *pos_dev, float *out, float *scratch, uint64_t scratch_bytes,
                          hipStream_t st);
-uint64_t latent_decode_scratch_bytes(const LatentDims &dm, uint32_t cap, uint64_t batch);
+uint64_t latent_decode_scratch_bytes(const LatentDims &dm, const LatentCache &cache, uint64_t batch);
 
 }  // namespace coeus

@@ -425,7 +425,7 @@ Session::~Session() {
     if (graph_exec) (void)hipGraphExecDestroy(graph_exec);
     if (graph) (void)hipGraphDestroy(graph);
     kc.release(); vc.release(); state.release(); ws.release();
-    dmix.release(); dscratch.release(); drows.release(); dwant.release();
+    dh2.release(); dmix.release(); dscratch.release(); drows.release(); dwant.release();
     dh.release(); dx.release(); dqkv.release(); datt.release(); dff.release(); dlogits.release();
     dids.release(); dpos.release(); dhist.release(); dpart.release(); dcount.release(); dstats.release();
     xq_h.release(); xq_inner.release(); xq_ff.release(); xq_g.release();

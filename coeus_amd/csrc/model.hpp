@@ -112,6 +112,7 @@ struct Session {
     Workspace ws;  // prefill
     DeviceBuf dh, dx, dqkv, datt, dff, dlogits, dids, dpos, dhist, dpart, dcount, dstats, xq_h, xq_inner, xq_ff, xq_g;
     DeviceBuf drows, dwant;    // rows whose logits session_feed was asked for
+    DeviceBuf dh2;             // layered models: the residual stream changes buffers at every folded norm
     DeviceBuf dmix, dscratch;  // layered models: latent queries of a decode step, attention partials
     hipGraph_t graph = nullptr;
     hipGraphExec_t graph_exec = nullptr;
