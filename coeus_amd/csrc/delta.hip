@@ -25,52 +25,90 @@ __device__ __forceinline__ float sigmoid(float x) { return 1.0f / (1.0f + expf(-
 // log of the decay: -exp(A_log) softplus(a + dt_bias)
 __device__ __forceinline__ float log_decay(float a, float exp_a, float dt_bias) { return -exp_a * softplus(a + dt_bias); }
 
-// Convolution + SiLU of channel c at row i of sequence b (position pos0 + i).
-__device__ __forceinline__ float conv_silu(const float *__restrict__ proj, const float *__restrict__ ring,
-                                           const float *__restrict__ taps_w, uint32_t taps, uint32_t channels,
-                                           uint64_t in_ld, uint64_t b, uint64_t n, uint64_t i, uint64_t pos0, uint32_t c) {
-    float acc = 0.f;
-    for (uint32_t j = 0; j < taps; j++) {
-        const uint32_t back = taps - 1 - j;  // this tap looks `back` positions behind
-        float x = 0.f;
-        if (back <= i) x = proj[(b * n + i - back) * in_ld + c];
-        else if (back <= pos0 + i) x = ring[(b * taps + (pos0 + i - back) % taps) * channels + c];
-        acc = fmaf(taps_w[(uint64_t)j * channels + c], x, acc);
-    }
-    return silu(acc);
+// Input of the convolution `back` positions before row i of sequence b (position pos0 + i): a row of this
+// prompt, a slot of the ring, or zero in front of the sequence.
+__device__ __forceinline__ float conv_input(const float *__restrict__ proj, const float *__restrict__ ring, uint32_t taps,
+                                            uint32_t channels, uint64_t in_ld, uint64_t b, uint64_t n, uint64_t i,
+                                            uint64_t pos0, uint32_t back, uint32_t c) {
+    if (back <= i) return proj[(b * n + i - back) * in_ld + c];
+    if (back <= pos0 + i) return ring[(b * taps + (pos0 + i - back) % taps) * channels + c];
+    return 0.f;
 }
 
-// One wave per (row, unit); a unit is one head of q, k or v, or the gates of all heads.
+// One wave per (strip of rows, unit).  A unit is a head of q or k, 256 channels of v, or the gates of all heads;
+// lane l owns channels l, l + 64, .. of it.  T taps (1 .. 4) slide through registers, so that every input is
+// read once; four rows are requested at a time.
+constexpr uint32_t kStrip = 16;
+template <int T>
 __global__ __launch_bounds__(256) void delta_prepare_kernel(const float *__restrict__ proj, DeltaDims dm, DeltaParams pr,
                                                             const float *__restrict__ ring, uint64_t n, uint64_t pos0,
                                                             uint32_t dp, DeltaOperands op) {
     const uint32_t lane = threadIdx.x & 63, unit = blockIdx.y * 4 + (threadIdx.x >> 6);
-    const uint64_t row = blockIdx.x, b = row / n, i = row % n;
-    const uint32_t KH = dm.kv_heads, H = dm.heads, C = dm.channels();
-    if (unit < 2 * KH) {
-        const bool is_q = unit < KH;
-        const uint32_t c0 = unit * dm.d;  // q heads, then k heads
-        float v[4], s2 = 0.f;             // d <= 256
-#pragma unroll
-        for (int t = 0; t < 4; t++) {
-            const uint32_t c = lane + 64 * t;
-            v[t] = c < dm.d ? conv_silu(proj, ring, pr.conv, dm.taps, C, dm.in_ld, b, n, i, pos0, c0 + c) : 0.f;
-            s2 = fmaf(v[t], v[t], s2);
-        }
-        const float r = (is_q ? 1.0f / sqrtf((float)dm.d) : 1.0f) / sqrtf(wave_sum(s2) + kUnitEps);
-        float *dst = (is_q ? op.q : op.k) + (row * KH + (is_q ? unit : unit - KH)) * dp;
-#pragma unroll
-        for (int t = 0; t < 4; t++)
-            if (lane + 64 * t < dp) dst[lane + 64 * t] = v[t] * r;  // (zeros behind d)
-    } else if (unit < 2 * KH + H) {
-        const uint32_t h = unit - 2 * KH, c0 = 2 * KH * dm.d + h * dm.e;
-        for (uint32_t c = lane; c < dm.e; c += 64)
-            op.v[(row * H + h) * dm.e + c] = conv_silu(proj, ring, pr.conv, dm.taps, C, dm.in_ld, b, n, i, pos0, c0 + c);
-    } else if (unit == 2 * KH + H) {
-        const float *p = proj + row * dm.in_ld;
-        for (uint32_t h = lane; h < H; h += 64) {
+    const uint64_t b = blockIdx.z, i0 = (uint64_t)blockIdx.x * kStrip, i1 = min(i0 + kStrip, n);
+    const uint32_t KH = dm.kv_heads, H = dm.heads, C = dm.channels(), V = H * dm.e, vunits = (V + 255) / 256;
+    if (unit > 2 * KH + vunits) return;
+    if (unit == 2 * KH + vunits) {
+        for (uint64_t t = lane; t < (i1 - i0) * H; t += 64) {
+            const uint64_t row = b * n + i0 + t / H;
+            const uint32_t h = (uint32_t)(t % H);
+            const float *p = proj + row * dm.in_ld;
             op.beta[row * H + h] = sigmoid(p[dm.beta_off() + h]);
             op.lg[row * H + h] = log_decay(p[dm.decay_off() + h], pr.exp_a[h], pr.dt_bias[h]);
+        }
+        return;
+    }
+    const bool is_v = unit >= 2 * KH;
+    const uint32_t vu = unit - 2 * KH, c0 = is_v ? 2 * KH * dm.d + 256 * vu : unit * dm.d;
+    const uint32_t len = is_v ? min(256u, V - 256 * vu) : dm.d;  // d <= 256
+    float *dst = is_v ? op.v + 256 * vu : (unit < KH ? op.q + unit * dp : op.k + (unit - KH) * dp);
+    const uint64_t dst_ld = is_v ? V : (uint64_t)KH * dp;
+    const uint32_t dst_len = is_v ? len : dp;  // (q and k: zeros behind d)
+    const float post = unit < KH ? 1.0f / sqrtf((float)dm.d) : 1.0f;
+    constexpr int TT = T ? T : 1;
+    float w[TT][4], x[TT][4];
+#pragma unroll
+    for (int j = 0; j < T; j++)
+#pragma unroll
+        for (int s = 0; s < 4; s++) {
+            const uint32_t c = lane + 64 * s;
+            w[j][s] = c < len ? pr.conv[(uint64_t)j * C + c0 + c] : 0.f;
+            x[j][s] = j + 1 < T && c < len ? conv_input(proj, ring, dm.taps, C, dm.in_ld, b, n, i0, pos0, T - 1 - j, c0 + c) : 0.f;
+        }
+    for (uint64_t ib = i0; ib < i1; ib += 4) {
+        float in[4][4];
+#pragma unroll
+        for (int u = 0; u < 4; u++)
+#pragma unroll
+            for (int s = 0; s < 4; s++) {
+                const uint32_t c = lane + 64 * s;
+                in[u][s] = c < len && ib + u < i1 ? proj[(b * n + ib + u) * dm.in_ld + c0 + c] : 0.f;
+            }
+#pragma unroll
+        for (int u = 0; u < 4; u++) {
+            if (ib + u >= i1) break;
+            float y[4], s2 = 0.f;
+#pragma unroll
+            for (int s = 0; s < 4; s++) {
+                float acc = 0.f;
+                if (T) {
+                    x[TT - 1][s] = in[u][s];
+#pragma unroll
+                    for (int j = 0; j < T; j++) acc = fmaf(w[j][s], x[j][s], acc);
+#pragma unroll
+                    for (int j = 0; j + 1 < T; j++) x[j][s] = x[j + 1][s];
+                } else if (lane + 64 * s < len) {  // any number of taps
+                    for (uint32_t j = 0; j < dm.taps; j++)
+                        acc = fmaf(pr.conv[(uint64_t)j * C + c0 + lane + 64 * s],
+                                   conv_input(proj, ring, dm.taps, C, dm.in_ld, b, n, ib + u, pos0, dm.taps - 1 - j, c0 + lane + 64 * s), acc);
+                }
+                y[s] = fast_silu(acc);
+                s2 = fmaf(y[s], y[s], s2);
+            }
+            const float r = is_v ? 1.0f : post / sqrtf(wave_sum(s2) + kUnitEps);
+            float *o = dst + (b * n + ib + u) * dst_ld;
+#pragma unroll
+            for (int s = 0; s < 4; s++)
+                if (lane + 64 * s < dst_len) o[lane + 64 * s] = y[s] * r;
         }
     }
 }
@@ -92,9 +130,18 @@ int launch_delta_prepare(const float *proj, const DeltaDims &dm, const DeltaPara
                          uint64_t batch, uint64_t n, uint64_t pos0, const DeltaOperands &op, hipStream_t st) {
     COEUS_TRY(check_dims(dm));
     COEUS_TRY(check_rows(batch, n));
-    const dim3 grid((unsigned)(batch * n), (unsigned)ceil_div(2 * dm.kv_heads + dm.heads + 1, 4));
-    hipLaunchKernelGGL(delta_prepare_kernel, grid, dim3(256), 0, st, proj, dm, pr, state.ring, n, pos0,
-                       delta_padded_dim(dm.d), op);
+    const dim3 grid((unsigned)ceil_div(n, kStrip), (unsigned)ceil_div(2 * dm.kv_heads + ceil_div((uint64_t)dm.heads * dm.e, 256) + 1, 4),
+                    (unsigned)batch);
+#define COEUS_DP(TV) \
+    hipLaunchKernelGGL(delta_prepare_kernel<TV>, grid, dim3(256), 0, st, proj, dm, pr, state.ring, n, pos0, delta_padded_dim(dm.d), op)
+    switch (dm.taps) {
+        case 1: COEUS_DP(1); break;
+        case 2: COEUS_DP(2); break;
+        case 3: COEUS_DP(3); break;
+        case 4: COEUS_DP(4); break;
+        default: COEUS_DP(0); break;
+    }
+#undef COEUS_DP
     COEUS_HIP(hipGetLastError());
     return COEUS_OK;
 }
@@ -204,9 +251,9 @@ __device__ __forceinline__ float4_t mfma4(const float4 &a, const float4_t &b, fl
 template <int NT>  // 16-wide steps of the padded query/key size
 __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaDims dm, DeltaOperands op, uint32_t dp, uint64_t n,
                                                           uint64_t t0, uint64_t seg, ChunkBuf cb) {
-    constexpr uint32_t DQ = 16 * NT, KLD = DQ + 4, ALD = kChunk + 4;
+    constexpr uint32_t DQ = 16 * NT, KLD = DQ + 4, ALD = kChunk + 4, TLD = 20;
     extern __shared__ float lds[];
-    float *kl = lds, *al = kl + kChunk * KLD;  // K [64][KLD], A [64][ALD]
+    float *kl = lds, *al = kl + kChunk * KLD, *tl = al + kChunk * ALD;  // K [64][KLD], A [64][ALD], -T [64][TLD]
     __shared__ float gs[kChunk], es[kChunk], bs[kChunk];
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
     const uint32_t chunk = blockIdx.x, h = blockIdx.y, H = dm.heads, KH = dm.kv_heads, hk = h / (H / KH);
@@ -234,67 +281,93 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaDims dm, DeltaOpe
         *(float4 *)(kl + r * KLD + q4) = v;
     }
     __syncthreads();
-    // rows 16 wave .. + 15 of K K^T and Q K^T, tiles up to the diagonal
-    {
-        const uint32_t r = 16 * wave + c;
-        float4 ka[NT], qa[NT];
+    // 16 x 16 tiles of K K^T and Q K^T up to the diagonal, rows block by block, five tiles a wave: (K, rows
+    // 3) + (Q, 0), (Q, 3) + (K, 0), (K, 2) + (Q, 1), (Q, 2) + (K, 1)
+#pragma unroll
+    for (int part = 0; part < 2; part++) {
+        const uint32_t blk = part == 0 ? 3 - (wave >> 1) : wave >> 1;
+        const bool is_q = ((wave & 1) ^ part) != 0;
+        const uint32_t r = 16 * blk + c;
+        float4 ra[NT];
 #pragma unroll
         for (int m = 0; m < NT; m++) {
             const uint32_t q4 = 16 * m + 4 * g;
-            ka[m] = *(const float4 *)(kl + r * KLD + q4);
-            qa[m] = make_float4(0.f, 0.f, 0.f, 0.f);
-            if (r < live && q4 < dp) qa[m] = *(const float4 *)(op.q + ((row0 + r) * KH + hk) * dp + q4);
+            if (!is_q) {
+                ra[m] = *(const float4 *)(kl + r * KLD + q4);
+            } else {
+                ra[m] = make_float4(0.f, 0.f, 0.f, 0.f);
+                if (r < live && q4 < dp) ra[m] = *(const float4 *)(op.q + ((row0 + r) * KH + hk) * dp + q4);
+            }
         }
         for (uint32_t t = 0; t < 4; t++) {
-            float4_t akk = {0.f, 0.f, 0.f, 0.f}, aqk = {0.f, 0.f, 0.f, 0.f};
-            if (t <= wave) {
+            float4_t acc = {0.f, 0.f, 0.f, 0.f};
+            if (t <= blk) {
 #pragma unroll
-                for (int m = 0; m < NT; m++) {
-                    const float4_t kb = *(const float4_t *)(kl + (16 * t + c) * KLD + 16 * m + 4 * g);
-                    akk = mfma4(ka[m], kb, akk);
-                    aqk = mfma4(qa[m], kb, aqk);
-                }
+                for (int m = 0; m < NT; m++) acc = mfma4(ra[m], *(const float4_t *)(kl + (16 * t + c) * KLD + 16 * m + 4 * g), acc);
             }
             const uint32_t j = 16 * t + c;
 #pragma unroll
             for (int i = 0; i < 4; i++) {
-                const uint32_t ri = 16 * wave + 4 * g + i;
-                const float e = j <= ri ? expf(gs[ri] - gs[j]) : 0.f;
-                al[ri * ALD + j] = j < ri ? bs[ri] * e * akk[i] : 0.f;
-                cb.p[(ci * kChunk + ri) * kChunk + j] = e * aqk[i];
+                const uint32_t ri = 16 * blk + 4 * g + i;
+                const float e = j <= ri ? expf(gs[ri] - gs[j]) * acc[i] : 0.f;
+                if (is_q) cb.p[(ci * kChunk + ri) * kChunk + j] = e;
+                else al[ri * ALD + j] = j < ri ? bs[ri] * e : 0.f;
             }
         }
     }
     __syncthreads();
-    // forward substitution, a column of [W | V'] per thread
-    for (uint32_t col = tid; col < DQ + dm.e; col += 256) {
-        const bool is_w = col < DQ;
-        const float *vp = op.v + (row0 * H + h) * dm.e + (col - DQ);
-        float x[kChunk];
+    // Forward substitution by blocks of 16 tokens: X_I = T_I (R_I - sum_J<I A_IJ X_J) with T_I the inverse of the
+    // diagonal block I + A_II, which wave I finds column by column.  -T is kept: the products accumulate A X - R.
+    {
+        float t[16];
 #pragma unroll
-        for (uint32_t i = 0; i < kChunk; i++) {
-            float r;
-            if (is_w) r = es[i] * kl[i * KLD + col];
-            else r = i < live ? vp[(uint64_t)i * H * dm.e] : 0.f;
-            x[i] = bs[i] * r;
+        for (int i = 0; i < 16; i++) {
+            float x = i == (int)c ? 1.f : 0.f;
+#pragma unroll
+            for (int k = 0; k < i; k++) x = fmaf(-al[(16 * wave + i) * ALD + 16 * wave + k], t[k], x);
+            t[i] = x;
         }
+        if (lane < 16)
 #pragma unroll
-        for (uint32_t i = 1; i < kChunk; i++) {
-            float a0 = 0.f, a1 = 0.f;
+            for (int i = 0; i < 16; i++) tl[(16 * wave + i) * TLD + lane] = -t[i];
+    }
+    __syncthreads();
+    float4 ta[4], aa[6];
 #pragma unroll
-            for (uint32_t j = 0; j < i; j += 4) {
-                const float4 a = *(const float4 *)(al + i * ALD + j);  // (zeros from the diagonal on)
-                a0 = fmaf(a.x, x[j], a0);
-                if (j + 1 < i) a1 = fmaf(a.y, x[j + 1], a1);
-                if (j + 2 < i) a0 = fmaf(a.z, x[j + 2], a0);
-                if (j + 3 < i) a1 = fmaf(a.w, x[j + 3], a1);
+    for (int i = 0; i < 4; i++) ta[i] = *(const float4 *)(tl + (16 * i + c) * TLD + 4 * g);
+#pragma unroll
+    for (int i = 1, k = 0; i < 4; i++)
+#pragma unroll
+        for (int j = 0; j < i; j++, k++) aa[k] = *(const float4 *)(al + (16 * i + c) * ALD + 16 * j + 4 * g);
+    const uint32_t tiles = NT + (dm.e + 15) / 16;
+    for (uint32_t t = wave; t < tiles; t += 4) {
+        const bool is_w = t < NT;
+        const uint32_t col = 16 * (is_w ? t : t - NT) + c;
+        float4_t x[4];
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+#pragma unroll
+            for (int k = 0; k < 4; k++) {
+                const uint32_t r = 16 * i + 4 * g + k;
+                float v = 0.f;
+                if (is_w) v = es[r] * kl[r * KLD + col];
+                else if (r < live && col < dm.e) v = op.v[((row0 + r) * H + h) * dm.e + col];
+                x[i][k] = -bs[r] * v;
             }
-            x[i] -= a0 + a1;
-        }
-        float *dst = is_w ? cb.w + ci * kChunk * DQ + col : cb.vp + ci * kChunk * dm.e + (col - DQ);
-        const uint32_t ld = is_w ? DQ : dm.e;
 #pragma unroll
-        for (uint32_t i = 0; i < kChunk; i++) dst[(uint64_t)i * ld] = x[i];
+        for (int i = 0, k = 0; i < 4; i++) {
+#pragma unroll
+            for (int j = 0; j < i; j++, k++) x[i] = mfma4(aa[k], x[j], x[i]);
+            x[i] = mfma4(ta[i], x[i], float4_t{0.f, 0.f, 0.f, 0.f});
+        }
+        if (is_w || col < dm.e) {
+            float *dst = is_w ? cb.w + ci * kChunk * DQ + col : cb.vp + ci * kChunk * dm.e + col;
+            const uint32_t ld = is_w ? DQ : dm.e;
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+#pragma unroll
+                for (int k = 0; k < 4; k++) dst[(uint64_t)(16 * i + 4 * g + k) * ld] = x[i][k];
+        }
     }
     if (h % (H / KH) == 0) {  // K^T once per query/key head
         float *kt = cb.kt + ((b * KH + hk) * cb.chunks + chunk) * DQ * kChunk;
@@ -336,7 +409,9 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(DeltaDims dm, const fl
     float4 wa[NT], qa[NT], pa[4], ka[QW][4];
     float4 eg4, ed4[4];
     float v4[4], egc;
-    auto fetch = [&](uint32_t ch) {
+    // A chunk's operands are requested as soon as the registers of the chunk before are free: W, Q and V' while
+    // P U and the state are computed, P, K^T and the decays behind them.
+    auto fetch_wq = [&](uint32_t ch) {
         const uint64_t ci = (b * H + h) * cb.chunks + ch;
         const float *wp = cb.w + (ci * kChunk + tok) * DQ + 4 * g;
         const uint64_t qrow = min((uint64_t)ch * kChunk + tok, seg - 1);  // (rows behind the end are not stored)
@@ -346,6 +421,11 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(DeltaDims dm, const fl
             wa[m] = *(const float4 *)(wp + 16 * m);
             qa[m] = *(const float4 *)(qp + min(16 * m + 4 * g, dp - 4));  // (the state is zero behind d)
         }
+#pragma unroll
+        for (int i = 0; i < 4; i++) v4[i] = cb.vp[(ci * kChunk + 16 * wave + 4 * g + i) * dm.e + colc];
+    };
+    auto fetch_pk = [&](uint32_t ch) {
+        const uint64_t ci = (b * H + h) * cb.chunks + ch;
         const float *pp = cb.p + (ci * kChunk + tok) * kChunk + 4 * g;
         const float *kp = cb.kt + (((b * KH + hk) * cb.chunks + ch) * DQ + 16 * QW * wave + c) * kChunk + 4 * g;
 #pragma unroll
@@ -357,13 +437,12 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(DeltaDims dm, const fl
         }
         eg4 = *(const float4 *)(cb.eg + ci * kChunk + 16 * wave + 4 * g);
         egc = cb.eg[ci * kChunk + kChunk - 1];
-#pragma unroll
-        for (int i = 0; i < 4; i++) v4[i] = cb.vp[(ci * kChunk + 16 * wave + 4 * g + i) * dm.e + colc];
     };
     const uint32_t chunks = (uint32_t)((seg + kChunk - 1) / kChunk);
-    fetch(0);
+    fetch_wq(0);
+    fetch_pk(0);
     for (uint32_t ch = 0; ch < chunks; ch++) {
-        const uint32_t buf = ch & 1;
+        const uint32_t buf = ch & 1, next = ch + 1 < chunks ? ch + 1 : ch;
 #pragma unroll
         for (int t = 0; t < QW; t++) sl[buf][QW * wave + t][lane] = s[t];
         lds_barrier();
@@ -378,6 +457,9 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(DeltaDims dm, const fl
 #pragma unroll
         for (int i = 0; i < 4; i++) u[i] = v4[i] - au[i];
         ul[buf][wave][lane] = u;
+        __builtin_amdgcn_sched_barrier(0);
+        fetch_wq(next);
+        __builtin_amdgcn_sched_barrier(0);
         ao[0] *= eg4.x; ao[1] *= eg4.y; ao[2] *= eg4.z; ao[3] *= eg4.w;
         lds_barrier();
         float4_t ub[4];
@@ -389,12 +471,14 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(DeltaDims dm, const fl
 #pragma unroll
         for (int t = 0; t < 4; t++) { ub[t][0] *= ed4[t].x; ub[t][1] *= ed4[t].y; ub[t][2] *= ed4[t].z; ub[t][3] *= ed4[t].w; }
 #pragma unroll
-        for (int w = 0; w < QW; w++) {
-            s[w] *= egc;
+        for (int w = 0; w < QW; w++) s[w] *= egc;
 #pragma unroll
-            for (int t = 0; t < 4; t++) s[w] = mfma4(ka[w][t], ub[t], s[w]);
-        }
-        fetch(ch + 1 < chunks ? ch + 1 : ch);
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int w = 0; w < QW; w++) s[w] = mfma4(ka[w][t], ub[t], s[w]);
+        __builtin_amdgcn_sched_barrier(0);
+        fetch_pk(next);
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
         for (int i = 0; i < 4; i++) {
             const uint64_t r = (uint64_t)ch * kChunk + 16 * wave + 4 * g + i;
@@ -424,7 +508,7 @@ static int launch_chunks(const DeltaDims &dm, const DeltaOperands &op, const Del
                          float *o, float *scratch, hipStream_t st) {
     constexpr uint32_t DQ = 64 * QW;
     const uint32_t dp = delta_padded_dim(dm.d);
-    const size_t lds = (kChunk * (DQ + 4) + kChunk * (kChunk + 4)) * 4;
+    const size_t lds = (kChunk * (DQ + 4) + kChunk * (kChunk + 4) + kChunk * 20) * 4;
     static const bool once = [] {
         (void)hipFuncSetAttribute((const void *)delta_chunk_kernel<4 * QW>, hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024);
         return true;
@@ -480,23 +564,48 @@ int launch_delta_prompt(const DeltaDims &dm, const DeltaOperands &op, const Delt
     return COEUS_OK;
 }
 
-// One wave per (row, head); out may be o itself.
+// One wave per (row, head); out may be o itself.  With LG lanes a head (e = 4 LG), 64 / LG heads per wave in
+// 16-byte pieces instead.
+template <int LG>
 __global__ __launch_bounds__(256) void delta_gate_kernel(const float *o, const float *__restrict__ proj,
                                                          DeltaDims dm, const float *__restrict__ norm, float eps,
-                                                         uint64_t units, float *out,
-                                                         uint16_t *__restrict__ out_lp, uint64_t lp_ld, bool lp_bf16) {
+                                                         uint64_t units, float *out, uint16_t *__restrict__ out_lp,
+                                                         uint64_t lp_ld, bool lp_bf16) {
     const uint32_t lane = threadIdx.x & 63, H = dm.heads;
-    const uint64_t unit = (uint64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (unit >= units) return;
-    const uint64_t row = unit / H;
-    const uint32_t h = (uint32_t)(unit % H);
-    const float *op = o + unit * dm.e, *gp = proj + row * dm.in_ld + dm.gate_off() + h * dm.e;
+    const uint64_t wave = (uint64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (LG) {
+        constexpr uint32_t PER = LG ? 64 / LG : 1, GL = LG ? LG : 1;
+        const uint64_t unit = wave * PER + lane / GL, uc = unit < units ? unit : units - 1, row = uc / H;
+        const uint32_t h = (uint32_t)(uc % H), c = 4 * (lane % GL);
+        const float4 v = *(const float4 *)(o + uc * dm.e + c);
+        const float4 gt = *(const float4 *)(proj + row * dm.in_ld + dm.gate_off() + h * dm.e + c);
+        const float4 nw = *(const float4 *)(norm + c);
+        float s2 = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, v.w * v.w)));
+#pragma unroll
+        for (uint32_t off = 1; off < GL; off <<= 1) s2 += __shfl_xor(s2, (int)off, 64);
+        const float rs = 1.0f / sqrtf(s2 / (float)dm.e + eps);
+        if (unit >= units) return;
+        const float4 r = make_float4(v.x * rs * nw.x * fast_silu(gt.x), v.y * rs * nw.y * fast_silu(gt.y),
+                                     v.z * rs * nw.z * fast_silu(gt.z), v.w * rs * nw.w * fast_silu(gt.w));
+        if (out) *(float4 *)(out + unit * dm.e + c) = r;
+        if (out_lp) {
+            uint2 p;
+            p.x = (uint32_t)f32_to_lp_bits(r.x, lp_bf16) | ((uint32_t)f32_to_lp_bits(r.y, lp_bf16) << 16);
+            p.y = (uint32_t)f32_to_lp_bits(r.z, lp_bf16) | ((uint32_t)f32_to_lp_bits(r.w, lp_bf16) << 16);
+            *(uint2 *)(out_lp + row * lp_ld + h * dm.e + c) = p;
+        }
+        return;
+    }
+    if (wave >= units) return;
+    const uint64_t row = wave / H;
+    const uint32_t h = (uint32_t)(wave % H);
+    const float *op = o + wave * dm.e, *gp = proj + row * dm.in_ld + dm.gate_off() + h * dm.e;
     float s2 = 0.f;
     for (uint32_t c = lane; c < dm.e; c += 64) s2 = fmaf(op[c], op[c], s2);
     const float rs = 1.0f / sqrtf(wave_sum(s2) / (float)dm.e + eps);
     for (uint32_t c = lane; c < dm.e; c += 64) {
-        const float v = op[c] * rs * norm[c] * silu(gp[c]);
-        if (out) out[unit * dm.e + c] = v;
+        const float v = op[c] * rs * norm[c] * fast_silu(gp[c]);
+        if (out) out[wave * dm.e + c] = v;
         if (out_lp) out_lp[row * lp_ld + h * dm.e + c] = f32_to_lp_bits(v, lp_bf16);
     }
 }
@@ -506,8 +615,20 @@ int launch_delta_gate(const float *o, const float *proj, const DeltaDims &dm, co
     COEUS_TRY(check_dims(dm));
     COEUS_TRY(check_rows(1, rows));
     const uint64_t units = rows * dm.heads;
-    hipLaunchKernelGGL(delta_gate_kernel, dim3((unsigned)ceil_div(units, 4)), dim3(256), 0, st, o, proj, dm, pr.norm, pr.eps,
-                       units, out, out_lp ? (uint16_t *)out_lp->p : nullptr, out_lp ? out_lp->ld : 0, out_lp && out_lp->bf16);
+    uint16_t *lp = out_lp ? (uint16_t *)out_lp->p : nullptr;
+    const uint64_t ld = out_lp ? out_lp->ld : 0;
+    const bool lp_bf = out_lp && out_lp->bf16;
+    // 16-byte pieces: heads of 16, 32, .. 256 values behind a gate that starts on a boundary
+    const bool vec = dm.in_ld % 4 == 0 && dm.gate_off() % 4 == 0 && ld % 4 == 0;
+#define COEUS_DG(LGV, PERV) \
+    hipLaunchKernelGGL(delta_gate_kernel<LGV>, dim3((unsigned)ceil_div(units, 4 * PERV)), dim3(256), 0, st, o, proj, dm, pr.norm, \
+                       pr.eps, units, out, lp, ld, lp_bf)
+    if (vec && dm.e == 32) COEUS_DG(8, 8);
+    else if (vec && dm.e == 64) COEUS_DG(16, 4);
+    else if (vec && dm.e == 128) COEUS_DG(32, 2);
+    else if (vec && dm.e == 256) COEUS_DG(64, 1);
+    else COEUS_DG(0, 1);
+#undef COEUS_DG
     COEUS_HIP(hipGetLastError());
     return COEUS_OK;
 }
@@ -516,7 +637,7 @@ int launch_delta_gate(const float *o, const float *proj, const DeltaDims &dm, co
 // One workgroup of 512 per (head, sequence).  Both products with the state are taken of the old state in
 // one pass (o = exp(lg) S^T q + (k . q) u), thread (g, c) of the pass owning columns VW c .. of rows
 // g, g + DG, ..: up to RM of them stay in registers between the products and the update.
-template <int VW, int RM>
+template <int VW, int RM, int T>  // T taps (1 .. 4), 0: any number
 __global__ __launch_bounds__(512) void delta_step_kernel(const float *__restrict__ proj, DeltaDims dm, DeltaParams pr,
                                                          float *state, float *ring, const uint32_t *pos_dev,
                                                          float *__restrict__ out) {
@@ -546,16 +667,34 @@ __global__ __launch_bounds__(512) void delta_step_kernel(const float *__restrict
         for (int t = 0; t < VW; t++) sr[i][t] = 0.f;
         if (live && r < d) load_row(r, sr[i]);
     }
-    // convolution ring: every workgroup that shares a channel writes the same value
+    // Convolution ring: every workgroup that shares a channel writes the same value.  All slots are requested
+    // without knowing the position (one trip to memory); the position then says which tap each slot meets.
+    // Slots in front of the sequence hold the zeros that a cleared state starts with.
     auto channel = [&](uint32_t c) -> float {
         const float x = p[c];
-        float acc = pr.conv[(uint64_t)(dm.taps - 1) * C + c] * x;
-        for (uint32_t back = 1; back < dm.taps; back++) {
-            if (back > pos) break;
-            acc = fmaf(pr.conv[(uint64_t)(dm.taps - 1 - back) * C + c], ring[(b * dm.taps + (pos - back) % dm.taps) * C + c], acc);
+        float acc;
+        if (T) {
+            constexpr uint32_t TT = T ? T : 1;
+            float r[TT], w[TT];
+#pragma unroll
+            for (uint32_t j = 0; j < TT; j++) {
+                r[j] = ring[(b * TT + j) * C + c];
+                w[j] = pr.conv[(uint64_t)j * C + c];
+            }
+            acc = w[TT - 1] * x;
+            const uint32_t slot = pos % TT;
+#pragma unroll
+            for (uint32_t k = 0; k < TT; k++)  // slot k is uniform: one of these runs
+                if (slot == k)
+#pragma unroll
+                    for (uint32_t back = 1; back < TT; back++) acc = fmaf(w[TT - 1 - back], r[(k + TT - back) % TT], acc);
+        } else {
+            acc = pr.conv[(uint64_t)(dm.taps - 1) * C + c] * x;
+            for (uint32_t back = 1; back < dm.taps && back <= pos; back++)
+                acc = fmaf(pr.conv[(uint64_t)(dm.taps - 1 - back) * C + c], ring[(b * dm.taps + (pos - back) % dm.taps) * C + c], acc);
         }
         ring[(b * dm.taps + pos % dm.taps) * C + c] = x;
-        return silu(acc);
+        return fast_silu(acc);
     };
     if (wave < 2) {  // wave 0: q, wave 1: k
         const uint32_t base = (wave * KH + hk) * d;
@@ -608,6 +747,7 @@ __global__ __launch_bounds__(512) void delta_step_kernel(const float *__restrict
     float s2 = 0.f;
     for (uint32_t c = tid; c < e; c += 512) {
         float sk = 0.f, sq = 0.f;
+#pragma unroll 8
         for (uint32_t i = 0; i < DG; i++) { sk += pk[i * e + c]; sq += pq[i * e + c]; }
         const float u = beta * (vs[c] - g * sk);
         us[c] = u;
@@ -647,7 +787,7 @@ __global__ __launch_bounds__(512) void delta_step_kernel(const float *__restrict
     for (int w = 0; w < 8; w++) tot += red[w];
     const float rs = 1.0f / sqrtf(tot / (float)e + pr.eps);
     for (uint32_t c = tid; c < e; c += 512)
-        out[(b * H + h) * e + c] = vs[c] * rs * pr.norm[c] * silu(p[dm.gate_off() + h * e + c]);
+        out[(b * H + h) * e + c] = vs[c] * rs * pr.norm[c] * fast_silu(p[dm.gate_off() + h * e + c]);
 }
 
 int launch_delta_step(const float *proj, const DeltaDims &dm, const DeltaParams &pr, const DeltaState &state,
@@ -660,11 +800,22 @@ int launch_delta_step(const float *proj, const DeltaDims &dm, const DeltaParams 
     const uint32_t DG = 512 / cg, per = (uint32_t)ceil_div(dm.d, DG);
     const size_t lds = (2 * dm.d + 2 * dm.e + 2 * (size_t)DG * dm.e) * 4;
     const dim3 grid(dm.heads, (unsigned)batch);
-#define COEUS_DST(VWV, RMV) \
-    hipLaunchKernelGGL((delta_step_kernel<VWV, RMV>), grid, dim3(512), lds, st, proj, dm, pr, state.s, state.ring, pos_dev, out)
+#define COEUS_DST2(VWV, RMV, TV) \
+    hipLaunchKernelGGL((delta_step_kernel<VWV, RMV, TV>), grid, dim3(512), lds, st, proj, dm, pr, state.s, state.ring, pos_dev, out)
+#define COEUS_DST(VWV, RMV)                            \
+    do {                                               \
+        switch (dm.taps) {                             \
+            case 1: COEUS_DST2(VWV, RMV, 1); break;    \
+            case 2: COEUS_DST2(VWV, RMV, 2); break;    \
+            case 3: COEUS_DST2(VWV, RMV, 3); break;    \
+            case 4: COEUS_DST2(VWV, RMV, 4); break;    \
+            default: COEUS_DST2(VWV, RMV, 0); break;   \
+        }                                              \
+    } while (0)
     if (vec) { if (per <= 8) COEUS_DST(4, 8); else COEUS_DST(4, 16); }
     else { if (per <= 8) COEUS_DST(1, 8); else COEUS_DST(1, 32); }
 #undef COEUS_DST
+#undef COEUS_DST2
     COEUS_HIP(hipGetLastError());
     return COEUS_OK;
 }

@@ -230,34 +230,38 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(const uint16_t *__r
     const bool wave_live = r0 < n;
 
     const uint32_t kkey = tid >> 3, kpc = tid & 7, va = tid & 15, vdp = tid >> 4;
-    uint4 rk[KP], rv[VP][2];
+    uint4 rk0, rk1, rk2, rk3, rv0, rv1, rv2, rv3;  // (named: arrays captured by the lambdas end up in scratch memory)
+    rk0 = rk1 = rk2 = rk3 = rv0 = rv1 = rv2 = rv3 = make_uint4(0, 0, 0, 0);
+    auto kload = [&](uint64_t krow, uint32_t u, uint4 &x) { x = *(const uint4 *)(kb + krow + min(8 * (kpc + 8 * u), dm.d - 8)); };
+    auto vload = [&](uint32_t t, uint32_t u, uint4 &x, uint4 &y) {
+        const uint32_t d0 = min(8 * (vdp + 16 * u), dm.e - 8);
+        x = *(const uint4 *)(vb + (uint64_t)min(t * KT + 2 * va, kmax) * kv_ld + d0);
+        y = *(const uint4 *)(vb + (uint64_t)min(t * KT + 2 * va + 1, kmax) * kv_ld + d0);
+    };
     auto gload = [&](uint32_t t) {
         const uint64_t krow = (uint64_t)min(t * KT + kkey, kmax) * kv_ld;
+        kload(krow, 0, rk0);
+        if (KP > 1) kload(krow, 1, rk1);
+        if (KP > 2) { kload(krow, 2, rk2); kload(krow, 3, rk3); }
+        if (DV >= 128 || vdp < DV / 8) vload(t, 0, rv0, rv1);
+        if (VP > 1) vload(t, 1, rv2, rv3);
+    };
+    auto kstore = [&](uint32_t buf, uint32_t u, const uint4 &x) { *(uint4 *)(ks + buf * KT * KLD + kkey * KLD + 8 * (kpc + 8 * u)) = x; };
+    auto vstore = [&](uint32_t buf, uint32_t u, const uint4 &x, const uint4 &y) {
+        uint32_t *dst = (uint32_t *)(vt + buf * DV * VLD) + (vdp + 16 * u) * (8 * VLD / 2) + va;
+        const uint32_t a[4] = {x.x, x.y, x.z, x.w}, c[4] = {y.x, y.y, y.z, y.w};
 #pragma unroll
-        for (int u = 0; u < KP; u++) rk[u] = *(const uint4 *)(kb + krow + min(8 * (kpc + 8 * u), dm.d - 8));
-#pragma unroll
-        for (int u = 0; u < VP; u++)
-            if (DV >= 128 || vdp < DV / 8) {
-                const uint32_t d0 = min(8 * (vdp + 16 * u), dm.e - 8);
-                rv[u][0] = *(const uint4 *)(vb + (uint64_t)min(t * KT + 2 * va, kmax) * kv_ld + d0);
-                rv[u][1] = *(const uint4 *)(vb + (uint64_t)min(t * KT + 2 * va + 1, kmax) * kv_ld + d0);
-            }
+        for (int e = 0; e < 4; e++) {
+            dst[e * VLD] = __builtin_amdgcn_perm(c[e], a[e], 0x05040100u);
+            dst[e * VLD + VLD / 2] = __builtin_amdgcn_perm(c[e], a[e], 0x07060302u);
+        }
     };
     auto lstore = [&](uint32_t buf) {
-#pragma unroll
-        for (int u = 0; u < KP; u++) *(uint4 *)(ks + buf * KT * KLD + kkey * KLD + 8 * (kpc + 8 * u)) = rk[u];
-#pragma unroll
-        for (int u = 0; u < VP; u++)
-            if (DV >= 128 || vdp < DV / 8) {
-                const uint32_t a[4] = {rv[u][0].x, rv[u][0].y, rv[u][0].z, rv[u][0].w};
-                const uint32_t c[4] = {rv[u][1].x, rv[u][1].y, rv[u][1].z, rv[u][1].w};
-                uint32_t *dst = (uint32_t *)(vt + buf * DV * VLD) + (vdp + 16 * u) * (8 * VLD / 2) + va;
-#pragma unroll
-                for (int e = 0; e < 4; e++) {
-                    dst[e * VLD] = __builtin_amdgcn_perm(c[e], a[e], 0x05040100u);
-                    dst[e * VLD + VLD / 2] = __builtin_amdgcn_perm(c[e], a[e], 0x07060302u);
-                }
-            }
+        kstore(buf, 0, rk0);
+        if (KP > 1) kstore(buf, 1, rk1);
+        if (KP > 2) { kstore(buf, 2, rk2); kstore(buf, 3, rk3); }
+        if (DV >= 128 || vdp < DV / 8) vstore(buf, 0, rv0, rv1);
+        if (VP > 1) vstore(buf, 1, rv2, rv3);
     };
     float16_t o[NDT];
 #pragma unroll
@@ -463,11 +467,11 @@ static uint32_t latent_shares(uint32_t cap) {
     return (uint32_t)(tiles < kMaxShares ? tiles : kMaxShares);
 }
 
-// W_uk^T q, [batch][heads][rank]: one workgroup per (128 columns of the rank, head) and every sequence, so
+// W_uk^T q as two bf16 numbers per element, [batch][heads][high, low][rank]: one workgroup per (128 columns of the rank, head) and every sequence, so
 // that the weights are read once.  Thread (g, r): column pair r, rows g, g + 4, ..
 template <int BP>
 __global__ __launch_bounds__(256) void latent_absorb_kernel(const float *__restrict__ q, const uint16_t *__restrict__ ukv,
-                                                            LatentDims dm, uint32_t batch, float *__restrict__ qa) {
+                                                            LatentDims dm, uint32_t batch, uint16_t *__restrict__ qa) {
     extern __shared__ float lds[];  // q [BP][d], partial sums [4][BP][128]
     const uint32_t tid = threadIdx.x, g = tid >> 6, rp = tid & 63, h = blockIdx.y, d = dm.d, R = dm.rank;
     const uint32_t r = blockIdx.x * 128 + 2 * rp, rc = min(r, R - 2);
@@ -481,7 +485,7 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(const float *__restr
 #pragma unroll
     for (int b = 0; b < BP; b++) a0[b] = a1[b] = 0.f;
     __syncthreads();
-    constexpr int U = 16;  // rows of a thread in flight
+    constexpr int U = BP > 4 ? 8 : 16;  // rows of a thread in flight
     for (uint32_t t0 = g; t0 < d; t0 += 4 * U) {
         uint32_t x[U];
 #pragma unroll
@@ -503,17 +507,20 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(const float *__restr
     __syncthreads();
     for (uint32_t i = tid; i < batch * 128; i += 256) {
         const uint32_t b = i / 128, cc = i % 128, rr = blockIdx.x * 128 + cc;
-        if (rr < R)
-            qa[((uint64_t)b * dm.heads + h) * R + rr] = (red[b * 128 + cc] + red[(BP + b) * 128 + cc]) +
-                                                        (red[(2 * BP + b) * 128 + cc] + red[(3 * BP + b) * 128 + cc]);
+        if (rr >= R) continue;
+        __bf16 hi, lo;
+        split_bf16((red[b * 128 + cc] + red[(BP + b) * 128 + cc]) + (red[(2 * BP + b) * 128 + cc] + red[(3 * BP + b) * 128 + cc]), hi, lo);
+        __bf16 *dst = (__bf16 *)qa + ((uint64_t)b * dm.heads + h) * 2 * R + rr;
+        dst[0] = hi;
+        dst[R] = lo;
     }
 }
 
 // One workgroup of four waves per (share of the ring, 16 heads, sequence).  A wave scores 16 of a tile's 64
 // latents for 16 heads, the softmax of the tile runs over LDS, then a wave accumulates a quarter of the
-// rank.  Absorbed queries and weights are f32: both enter the products as sums of two bf16 numbers.
+// rank.  Absorbed queries and weights enter the products as sums of two bf16 numbers each.
 // The share's record: maximum (base 2), sum, weighted latent.
-__global__ __launch_bounds__(256) void latent_scores_kernel(const float *__restrict__ qa, LatentDims dm,
+__global__ __launch_bounds__(256) void latent_scores_kernel(const uint16_t *__restrict__ qa, LatentDims dm,
                                                             const uint16_t *__restrict__ cache, uint32_t cap,
                                                             const uint32_t *pos_dev, uint32_t keys_per_share,
                                                             float *__restrict__ part) {
@@ -529,46 +536,47 @@ __global__ __launch_bounds__(256) void latent_scores_kernel(const float *__restr
     const uint32_t nv = min(*pos_dev + 1, cap), k_begin = share * keys_per_share, k_end = min(nv, k_begin + keys_per_share);
     const float scale2 = 1.4426950408889634f * dm.scale;
     if (tid < 16) { ms[tid] = -1e30f; ls[tid] = 0.f; }
-    const float *qp = qa + (b * dm.heads + hc) * R + 8 * g;
+    const uint16_t *qp = qa + (b * dm.heads + hc) * 2 * R + 8 * g;
     const uint16_t *cb = cache + b * cap * R;
     const uint32_t per = ((R / 16) + 3) / 4;  // 16-wide column tiles of a wave (at most 16)
     float4_t acc[16];
 #pragma unroll
     for (int t = 0; t < 16; t++) acc[t] = float4_t{0.f, 0.f, 0.f, 0.f};
     for (uint32_t k0 = k_begin; k0 < k_end; k0 += kKeyTile) {
-        // transposed latents: two keys a dword
-        for (uint32_t i = tid; i < 256 * ((R / 8 + 7) / 8); i += 256) {  // 8 pieces x 32 key pairs a round
-            const uint32_t piece = (i & 7) + 8 * (i / 256), a = (i >> 3) & 31;
-            if (piece < R / 8) {
-                const uint4 x = *(const uint4 *)(cb + (uint64_t)min(k0 + 2 * a, k_end - 1) * R + 8 * piece);
-                const uint4 y = *(const uint4 *)(cb + (uint64_t)min(k0 + 2 * a + 1, k_end - 1) * R + 8 * piece);
-                const uint32_t xs[4] = {x.x, x.y, x.z, x.w}, ys[4] = {y.x, y.y, y.z, y.w};
-                uint32_t *dst = (uint32_t *)ct + piece * (8 * VLD / 2) + a;
-#pragma unroll
-                for (int e = 0; e < 4; e++) {
-                    dst[e * VLD] = __builtin_amdgcn_perm(ys[e], xs[e], 0x05040100u);
-                    dst[e * VLD + VLD / 2] = __builtin_amdgcn_perm(ys[e], xs[e], 0x07060302u);
-                }
-            }
-        }
-        // scores of keys k0 + 16 wave + c
+        // scores of keys k0 + 16 wave + c; eight steps' operands are on their way at once
         float4_t sc = {0.f, 0.f, 0.f, 0.f}, sc2 = {0.f, 0.f, 0.f, 0.f};
         const uint16_t *kp = cb + (uint64_t)min(k0 + 16 * wave + c, k_end - 1) * R + 8 * g;
-#pragma unroll 4
-        for (uint32_t s = 0; s < R / 32; s++) {
-            const float4 q0 = *(const float4 *)(qp + 32 * s), q1 = *(const float4 *)(qp + 32 * s + 4);
-            const float qv[8] = {q0.x, q0.y, q0.z, q0.w, q1.x, q1.y, q1.z, q1.w};
-            bf16x8_t qh, ql;
+        const uint32_t steps = R / 32;
+        for (uint32_t s0 = 0; s0 < steps; s0 += 8) {
+            bf16x8_t kf[8], qh[8], ql[8];
 #pragma unroll
-            for (int e = 0; e < 8; e++) {
-                __bf16 hi, lo;
-                split_bf16(qv[e], hi, lo);
-                qh[e] = hi;
-                ql[e] = lo;
+            for (int u = 0; u < 8; u++) {  // (a step behind the end re-reads the last one and is not used)
+                const uint32_t off = 32 * min(s0 + u, steps - 1);
+                kf[u] = *(const bf16x8_t *)(kp + off);
+                qh[u] = *(const bf16x8_t *)(qp + off);
+                ql[u] = *(const bf16x8_t *)(qp + R + off);
             }
-            const bf16x8_t kf = *(const bf16x8_t *)(kp + 32 * s);
-            sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh, kf, sc, 0, 0, 0);
-            sc2 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ql, kf, sc2, 0, 0, 0);
+            __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+            for (int u = 0; u < 8; u++)
+                if (s0 + u < steps) {
+                    sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh[u], kf[u], sc, 0, 0, 0);
+                    sc2 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ql[u], kf[u], sc2, 0, 0, 0);
+                }
+        }
+        // transposed latents: two keys a dword (8 pieces of 8 dims x 32 key pairs a round)
+#pragma unroll 4
+        for (uint32_t p0 = 0; p0 < R / 8; p0 += 8) {
+            const uint32_t piece = min(p0 + (tid & 7), R / 8 - 1), a = tid >> 3;
+            const uint4 x = *(const uint4 *)(cb + (uint64_t)min(k0 + 2 * a, k_end - 1) * R + 8 * piece);
+            const uint4 y = *(const uint4 *)(cb + (uint64_t)min(k0 + 2 * a + 1, k_end - 1) * R + 8 * piece);
+            const uint32_t xs[4] = {x.x, x.y, x.z, x.w}, ys[4] = {y.x, y.y, y.z, y.w};
+            uint32_t *dst = (uint32_t *)ct + piece * (8 * VLD / 2) + a;
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                dst[e * VLD] = __builtin_amdgcn_perm(ys[e], xs[e], 0x05040100u);
+                dst[e * VLD + VLD / 2] = __builtin_amdgcn_perm(ys[e], xs[e], 0x07060302u);
+            }
         }
         const uint32_t key = k0 + 16 * wave + c;
 #pragma unroll
@@ -629,42 +637,62 @@ __global__ __launch_bounds__(256) void latent_scores_kernel(const float *__restr
 }
 
 // One workgroup per (32 value dims, head, sequence): merges the shares, then W_uv rows against the result.
+// A wave's eight rows are requested before the merge, the shares' records sixteen at a time.
+template <int RP>  // pieces of 512 of the rank
 __global__ __launch_bounds__(256) void latent_expand_kernel(const float *__restrict__ part, const uint16_t *__restrict__ ukv,
                                                             LatentDims dm, uint32_t shares, float *__restrict__ out) {
     extern __shared__ float lds[];  // merged latent [rank]
-    __shared__ float ws[kMaxShares], lt_s;
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.y, R = dm.rank;
     const uint64_t b = blockIdx.z;
     const float *rec = part + (b * dm.heads + h) * shares * (R + 2);
-    if (wave == 0) {
-        const float m = lane < shares ? rec[lane * (R + 2)] : -1e30f, mm = wave_max(m);
-        const float w = lane < shares ? __builtin_amdgcn_exp2f(m - mm) : 0.f;
-        const float lt = wave_sum(lane < shares ? rec[lane * (R + 2) + 1] * w : 0.f);
-        if (lane < shares) ws[lane] = w;
-        if (lane == 0) lt_s = lt;
+    const uint32_t c0 = blockIdx.x * 32 + wave * 8;
+    uint4 w[8][RP];
+#pragma unroll
+    for (int i = 0; i < 8; i++)
+#pragma unroll
+        for (int k = 0; k < RP; k++)
+            w[i][k] = *(const uint4 *)(ukv + ((uint64_t)dm.heads * dm.d + h * dm.e + min(c0 + i, dm.e - 1)) * R + min(lane * 8 + 512 * k, R - 8));
+    // every wave finds the shares' weights for itself
+    const uint32_t sl = min(lane, shares - 1);
+    const float m = rec[sl * (R + 2)], l = rec[sl * (R + 2) + 1];
+    float a[2 * RP];
+#pragma unroll
+    for (int k = 0; k < 2 * RP; k++) a[k] = 0.f;
+    const float mm = wave_max(m), ws = lane < shares ? __builtin_amdgcn_exp2f(m - mm) : 0.f;
+    const float inv = 1.0f / wave_sum(l * ws);
+    for (uint32_t s0 = 0; s0 < shares; s0 += 16) {
+        float x[16][2 * RP];
+#pragma unroll
+        for (int s = 0; s < 16; s++)
+#pragma unroll
+            for (int k = 0; k < 2 * RP; k++) x[s][k] = rec[min(s0 + s, shares - 1) * (R + 2) + 2 + min(tid + 256 * k, R - 1)];
+#pragma unroll
+        for (int s = 0; s < 16; s++) {
+            const float wt = __shfl(ws, (int)(s0 + s), 64);  // (0 behind the last share)
+#pragma unroll
+            for (int k = 0; k < 2 * RP; k++) a[k] = fmaf(wt, x[s][k], a[k]);
+        }
     }
+#pragma unroll
+    for (int k = 0; k < 2 * RP; k++)
+        if (tid + 256 * k < R) lds[tid + 256 * k] = a[k] * inv;
     __syncthreads();
-    for (uint32_t r = tid; r < R; r += 256) {
-        float a = 0.f;
-        for (uint32_t s = 0; s < shares; s++) a = fmaf(ws[s], rec[s * (R + 2) + 2 + r], a);
-        lds[r] = a / lt_s;
-    }
-    __syncthreads();
-    const uint32_t c_end = min(dm.e, blockIdx.x * 32 + 32);
-    for (uint32_t cc = blockIdx.x * 32 + wave; cc < c_end; cc += 4) {
-        const uint16_t *w = ukv + ((uint64_t)dm.heads * dm.d + h * dm.e + cc) * R;
-        float a = 0.f;
-        for (uint32_t r = lane * 8; r < R; r += 512) {
-            const uint4 x = *(const uint4 *)(w + r);
-            const uint32_t xs[4] = {x.x, x.y, x.z, x.w};
+#pragma unroll
+    for (int i = 0; i < 8; i++) {
+        float v = 0.f;
+#pragma unroll
+        for (int k = 0; k < RP; k++) {
+            const uint32_t r = lane * 8 + 512 * k;
+            if (r >= R) continue;
+            const uint32_t xs[4] = {w[i][k].x, w[i][k].y, w[i][k].z, w[i][k].w};
 #pragma unroll
             for (int e = 0; e < 4; e++) {
-                a = fmaf(__uint_as_float(xs[e] << 16), lds[r + 2 * e], a);
-                a = fmaf(__uint_as_float(xs[e] & 0xffff0000u), lds[r + 2 * e + 1], a);
+                v = fmaf(__uint_as_float(xs[e] << 16), lds[r + 2 * e], v);
+                v = fmaf(__uint_as_float(xs[e] & 0xffff0000u), lds[r + 2 * e + 1], v);
             }
         }
-        a = wave_sum(a);
-        if (lane == 0) out[b * dm.heads * dm.e + h * dm.e + cc] = a;
+        v = wave_sum(v);
+        if (lane == 0 && c0 + i < dm.e) out[b * dm.heads * dm.e + h * dm.e + c0 + i] = v;
     }
 }
 
@@ -682,7 +710,8 @@ int launch_latent_decode(const float *q, const void *ukv, const LatentDims &dm, 
     const uint64_t want = latent_decode_scratch_bytes(dm, cache, batch);
     if (want && batch <= 16 && scratch && scratch_bytes >= want) {
         const uint16_t *w = (const uint16_t *)ukv, *cc = (const uint16_t *)cache.c;
-        float *qa = scratch, *part = scratch + batch * dm.heads * dm.rank;
+        uint16_t *qa = (uint16_t *)scratch;
+        float *part = scratch + batch * dm.heads * dm.rank;
         const uint32_t shares = latent_shares(cache.cap), bp = pad_batch(batch), R = dm.rank;
         const uint32_t per_share = (uint32_t)round_up(ceil_div(cache.cap, shares), kKeyTile);
         const dim3 agrid((unsigned)ceil_div(R, 128), dm.heads);
@@ -697,8 +726,9 @@ int launch_latent_decode(const float *q, const void *ukv, const LatentDims &dm, 
         const size_t slds = ((size_t)R * (kKeyTile + 8) + 2 * 16 * (kKeyTile + 8)) * 2 + (16 * (kKeyTile + 8) + 48) * 4;
         hipLaunchKernelGGL(latent_scores_kernel, dim3(shares, (unsigned)ceil_div(dm.heads, 16), (unsigned)batch), dim3(256),
                            slds, st, qa, dm, cc, cache.cap, pos_dev, per_share, part);
-        hipLaunchKernelGGL(latent_expand_kernel, dim3((unsigned)ceil_div(dm.e, 32), dm.heads, (unsigned)batch), dim3(256),
-                           (size_t)R * 4, st, part, w, dm, shares, out);
+        const dim3 egrid((unsigned)ceil_div(dm.e, 32), dm.heads, (unsigned)batch);
+        if (R <= 512) hipLaunchKernelGGL(latent_expand_kernel<1>, egrid, dim3(256), (size_t)R * 4, st, part, w, dm, shares, out);
+        else hipLaunchKernelGGL(latent_expand_kernel<2>, egrid, dim3(256), (size_t)R * 4, st, part, w, dm, shares, out);
         COEUS_HIP(hipGetLastError());
         return COEUS_OK;
     }
