@@ -227,17 +227,23 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaDims dm, DeltaOper
 // A reduction index of a matrix instruction is only a label: instruction i of a 16-wide step sums over
 // {4 g + i : g = lane / 16}, so a lane's operand pieces are 16 consecutive bytes, and an accumulator
 // tile (rows 4 g + i) is the next product's right operand as it stands.
+// The chunk operands lie in memory in that order, [16-row tile][16-wide step][lane][4]: a wave's load is
+// 1 KiB in a row (operand_index); V' as accumulator tiles, [16-row tile][16 columns][lane][4].
 constexpr uint32_t kChunk = 64;
 constexpr uint64_t kSegment = 4096;  // tokens whose chunk operands are in memory at once
 
+__device__ __forceinline__ uint32_t operand_index(uint32_t row, uint32_t k, uint32_t steps) {
+    return (((row >> 4) * steps + (k >> 4)) * 64 + ((k >> 2) & 3) * 16 + (row & 15)) * 4 + (k & 3);
+}
+
 struct ChunkBuf {
-    float *w, *vp, *p, *eg, *ed, *kt;
+    float *w, *vp, *p, *eg, *ed, *kt, *q;
     uint32_t chunks;  // per sequence
 };
 static uint32_t chunk_dim(uint32_t d) { return (uint32_t)round_up(d, 64); }
 static uint64_t chunk_floats(const DeltaDims &dm, uint64_t batch, uint64_t chunks) {
     const uint64_t dq = chunk_dim(dm.d);
-    return batch * chunks * (dm.heads * (kChunk * (dq + dm.e + kChunk) + 2 * kChunk) + (uint64_t)dm.kv_heads * dq * kChunk);
+    return batch * chunks * (dm.heads * (kChunk * (dq + round_up(dm.e, 16) + kChunk) + 2 * kChunk) + 2ull * dm.kv_heads * dq * kChunk);
 }
 
 __device__ __forceinline__ float4_t mfma4(const float4 &a, const float4_t &b, float4_t acc) {
@@ -257,9 +263,12 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaDims dm, DeltaOpe
     __shared__ float gs[kChunk], es[kChunk], bs[kChunk];
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
     const uint32_t chunk = blockIdx.x, h = blockIdx.y, H = dm.heads, KH = dm.kv_heads, hk = h / (H / KH);
-    const uint64_t b = blockIdx.z, first = t0 + (uint64_t)chunk * kChunk, left = seg - (uint64_t)chunk * kChunk;
+    const uint64_t b = blockIdx.z, tok0 = t0 + (uint64_t)chunk * kChunk, left = seg - (uint64_t)chunk * kChunk;
     const uint32_t live = left < kChunk ? (uint32_t)left : kChunk;  // tokens behind the end: beta = 0, k = q = v = 0
-    const uint64_t row0 = b * n + first, ci = ((b * H + h) * cb.chunks + chunk);
+    const uint64_t row0 = b * n + tok0, ci = ((b * H + h) * cb.chunks + chunk);
+    // Q and K^T in operand order are written once per query/key head, by the first of the heads that share it
+    const bool first = h % (H / KH) == 0;
+    const uint64_t ki = ((b * KH + hk) * cb.chunks + chunk) * DQ * kChunk;
     if (wave == 0) {
         float lg = lane < live ? op.lg[(row0 + lane) * H + h] : 0.f;
 #pragma unroll
@@ -297,6 +306,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaDims dm, DeltaOpe
             } else {
                 ra[m] = make_float4(0.f, 0.f, 0.f, 0.f);
                 if (r < live && q4 < dp) ra[m] = *(const float4 *)(op.q + ((row0 + r) * KH + hk) * dp + q4);
+                if (first) *(float4 *)(cb.q + ki + ((blk * NT + m) * 64 + lane) * 4) = ra[m];
             }
         }
         for (uint32_t t = 0; t < 4; t++) {
@@ -310,7 +320,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaDims dm, DeltaOpe
             for (int i = 0; i < 4; i++) {
                 const uint32_t ri = 16 * blk + 4 * g + i;
                 const float e = j <= ri ? expf(gs[ri] - gs[j]) * acc[i] : 0.f;
-                if (is_q) cb.p[(ci * kChunk + ri) * kChunk + j] = e;
+                if (is_q) cb.p[ci * kChunk * kChunk + operand_index(ri, j, 4)] = e;
                 else al[ri * ALD + j] = j < ri ? bs[ri] * e : 0.f;
             }
         }
@@ -360,26 +370,28 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaDims dm, DeltaOpe
             for (int j = 0; j < i; j++, k++) x[i] = mfma4(aa[k], x[j], x[i]);
             x[i] = mfma4(ta[i], x[i], float4_t{0.f, 0.f, 0.f, 0.f});
         }
-        if (is_w || col < dm.e) {
-            float *dst = is_w ? cb.w + ci * kChunk * DQ + col : cb.vp + ci * kChunk * dm.e + col;
-            const uint32_t ld = is_w ? DQ : dm.e;
 #pragma unroll
-            for (int i = 0; i < 4; i++)
+        for (int i = 0; i < 4; i++) {
+            if (is_w) {
 #pragma unroll
-                for (int k = 0; k < 4; k++) dst[(uint64_t)(16 * i + 4 * g + k) * ld] = x[i][k];
+                for (int k = 0; k < 4; k++) cb.w[ci * kChunk * DQ + operand_index(16 * i + 4 * g + k, col, NT)] = x[i][k];
+            } else {
+                *(float4_t *)(cb.vp + ci * kChunk * 16 * (tiles - NT) + ((i * (tiles - NT) + t - NT) * 64 + lane) * 4) = x[i];
+            }
         }
     }
-    if (h % (H / KH) == 0) {  // K^T once per query/key head
-        float *kt = cb.kt + ((b * KH + hk) * cb.chunks + chunk) * DQ * kChunk;
-        for (uint32_t i = tid; i < DQ * kChunk; i += 256) kt[i] = kl[(i % kChunk) * KLD + i / kChunk];
-    }
+    if (first)
+        for (uint32_t i = tid; i < DQ * kChunk; i += 256) {
+            const uint32_t dim = i % DQ, tk = i / DQ;
+            cb.kt[ki + operand_index(dim, tk, 4)] = kl[tk * KLD + dim];
+        }
 }
 
 // One workgroup of four waves per (16 columns of S, head, sequence).  Wave w keeps rows 16 QW w .. of the
 // state in accumulators, computes tokens 16 w .. of U and O, and hands both to the others through LDS.
 template <int QW>
-__global__ __launch_bounds__(256) void delta_carry_kernel(DeltaDims dm, const float *__restrict__ q, uint32_t dp, uint64_t n,
-                                                          uint64_t t0, uint64_t seg, ChunkBuf cb, float *state,
+__global__ __launch_bounds__(256) void delta_carry_kernel(DeltaDims dm, uint64_t n, uint64_t t0, uint64_t seg,
+                                                          ChunkBuf cb, float *state,
                                                           float *__restrict__ o, uint32_t blocks, uint32_t units) {
     constexpr uint32_t NT = 4 * QW, DQ = 16 * NT;
     __shared__ float4_t sl[2][NT][64], ul[2][4][64];
@@ -405,34 +417,29 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(DeltaDims dm, const fl
             const uint32_t r = 16 * (QW * wave + t) + 4 * g + i;
             s[t][i] = r < dm.d ? sp[(uint64_t)r * dm.e] : 0.f;
         }
-    const uint32_t tok = 16 * wave + c;  // this lane's row of the left operands
     float4 wa[NT], qa[NT], pa[4], ka[QW][4];
     float4 eg4, ed4[4];
-    float v4[4], egc;
+    float4_t v4;
+    float egc;
     // A chunk's operands are requested as soon as the registers of the chunk before are free: W, Q and V' while
     // P U and the state are computed, P, K^T and the decays behind them.
     auto fetch_wq = [&](uint32_t ch) {
-        const uint64_t ci = (b * H + h) * cb.chunks + ch;
-        const float *wp = cb.w + (ci * kChunk + tok) * DQ + 4 * g;
-        const uint64_t qrow = min((uint64_t)ch * kChunk + tok, seg - 1);  // (rows behind the end are not stored)
-        const float *qp = q + ((b * n + t0 + qrow) * KH + hk) * dp;
+        const uint64_t ci = (b * H + h) * cb.chunks + ch, ki = (b * KH + hk) * cb.chunks + ch;
+        const float4 *wp = (const float4 *)(cb.w + ci * kChunk * DQ) + wave * NT * 64 + lane;
+        const float4 *qp = (const float4 *)(cb.q + ki * kChunk * DQ) + wave * NT * 64 + lane;
 #pragma unroll
-        for (uint32_t m = 0; m < NT; m++) {
-            wa[m] = *(const float4 *)(wp + 16 * m);
-            qa[m] = *(const float4 *)(qp + min(16 * m + 4 * g, dp - 4));  // (the state is zero behind d)
-        }
-#pragma unroll
-        for (int i = 0; i < 4; i++) v4[i] = cb.vp[(ci * kChunk + 16 * wave + 4 * g + i) * dm.e + colc];
+        for (uint32_t m = 0; m < NT; m++) { wa[m] = wp[64 * m]; qa[m] = qp[64 * m]; }
+        v4 = *(const float4_t *)(cb.vp + ci * kChunk * 16 * blocks + ((wave * blocks + blk) * 64 + lane) * 4);
     };
     auto fetch_pk = [&](uint32_t ch) {
-        const uint64_t ci = (b * H + h) * cb.chunks + ch;
-        const float *pp = cb.p + (ci * kChunk + tok) * kChunk + 4 * g;
-        const float *kp = cb.kt + (((b * KH + hk) * cb.chunks + ch) * DQ + 16 * QW * wave + c) * kChunk + 4 * g;
+        const uint64_t ci = (b * H + h) * cb.chunks + ch, ki = (b * KH + hk) * cb.chunks + ch;
+        const float4 *pp = (const float4 *)(cb.p + ci * kChunk * kChunk) + wave * 4 * 64 + lane;
+        const float4 *kp = (const float4 *)(cb.kt + ki * kChunk * DQ) + QW * wave * 4 * 64 + lane;
 #pragma unroll
         for (int t = 0; t < 4; t++) {
-            pa[t] = *(const float4 *)(pp + 16 * t);
+            pa[t] = pp[64 * t];
 #pragma unroll
-            for (int u = 0; u < QW; u++) ka[u][t] = *(const float4 *)(kp + 16 * u * kChunk + 16 * t);
+            for (int u = 0; u < QW; u++) ka[u][t] = kp[(4 * u + t) * 64];
             ed4[t] = *(const float4 *)(cb.ed + ci * kChunk + 16 * t + 4 * g);
         }
         eg4 = *(const float4 *)(cb.eg + ci * kChunk + 16 * wave + 4 * g);
@@ -525,12 +532,13 @@ static int launch_chunks(const DeltaDims &dm, const DeltaOperands &op, const Del
         cb.p = take(hc * kChunk * kChunk);
         cb.eg = take(hc * kChunk);
         cb.ed = take(hc * kChunk);
+        cb.vp = take(hc * kChunk * round_up(dm.e, 16));
         cb.kt = take(batch * cb.chunks * dm.kv_heads * DQ * kChunk);
-        cb.vp = take(hc * kChunk * dm.e);  // last: its rows need no alignment
+        cb.q = take(batch * cb.chunks * dm.kv_heads * DQ * kChunk);
         hipLaunchKernelGGL((delta_chunk_kernel<4 * QW>), dim3(cb.chunks, dm.heads, (unsigned)batch), dim3(256), lds, st, dm,
                            op, dp, n, t0, seg, cb);
         const uint32_t blocks = (uint32_t)ceil_div(dm.e, 16), units = (uint32_t)(dm.heads * batch);
-        hipLaunchKernelGGL((delta_carry_kernel<QW>), dim3(blocks * units), dim3(256), 0, st, dm, op.q, dp, n, t0, seg, cb,
+        hipLaunchKernelGGL((delta_carry_kernel<QW>), dim3(blocks * units), dim3(256), 0, st, dm, n, t0, seg, cb,
                            state.s, o, blocks, units);
     }
     COEUS_HIP(hipGetLastError());

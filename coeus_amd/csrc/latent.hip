@@ -524,7 +524,7 @@ __global__ __launch_bounds__(256) void latent_scores_kernel(const uint16_t *__re
                                                             const uint16_t *__restrict__ cache, uint32_t cap,
                                                             const uint32_t *pos_dev, uint32_t keys_per_share,
                                                             float *__restrict__ part) {
-    constexpr uint32_t VLD = kKeyTile + 8, PLD = kKeyTile + 8;
+    constexpr uint32_t VLD = kKeyTile + 8, PLD = kKeyTile + 8;  // (16-byte rows; row stride 36 dwords)
     extern __shared__ __attribute__((aligned(16))) uint16_t lds16[];
     uint16_t *ct = lds16;                                    // latents of the tile, [rank][VLD]
     uint16_t *ph = ct + dm.rank * VLD, *pl = ph + 16 * PLD;  // weights, high and low parts, [16][PLD]
@@ -534,6 +534,7 @@ __global__ __launch_bounds__(256) void latent_scores_kernel(const uint16_t *__re
     const uint32_t share = blockIdx.x, h0 = blockIdx.y * 16, hc = min(h0 + c, dm.heads - 1);
     const uint64_t b = blockIdx.z;
     const uint32_t nv = min(*pos_dev + 1, cap), k_begin = share * keys_per_share, k_end = min(nv, k_begin + keys_per_share);
+    // (a share that no position has reached yet leaves an empty record)
     const float scale2 = 1.4426950408889634f * dm.scale;
     if (tid < 16) { ms[tid] = -1e30f; ls[tid] = 0.f; }
     const uint16_t *qp = qa + (b * dm.heads + hc) * 2 * R + 8 * g;
@@ -543,40 +544,48 @@ __global__ __launch_bounds__(256) void latent_scores_kernel(const uint16_t *__re
 #pragma unroll
     for (int t = 0; t < 16; t++) acc[t] = float4_t{0.f, 0.f, 0.f, 0.f};
     for (uint32_t k0 = k_begin; k0 < k_end; k0 += kKeyTile) {
-        // scores of keys k0 + 16 wave + c; eight steps' operands are on their way at once
+        // 512 of the rank a round.  Everything is requested at once, from addresses that do not depend on the
+        // position (slots that are not written yet hold finite values and are masked; a piece behind the end
+        // re-reads the last one and is not used): the tile as key pairs for the transposed copy (8 pieces of 8
+        // dims x 32 pairs a step), as right operands for keys k0 + 16 wave + c, and the absorbed queries.
         float4_t sc = {0.f, 0.f, 0.f, 0.f}, sc2 = {0.f, 0.f, 0.f, 0.f};
-        const uint16_t *kp = cb + (uint64_t)min(k0 + 16 * wave + c, k_end - 1) * R + 8 * g;
-        const uint32_t steps = R / 32;
-        for (uint32_t s0 = 0; s0 < steps; s0 += 8) {
-            bf16x8_t kf[8], qh[8], ql[8];
+        const uint16_t *kp = cb + (uint64_t)min(k0 + 16 * wave + c, cap - 1) * R + 8 * g;
+        const uint32_t a = tid >> 3, steps = R / 32;
+        const uint16_t *tx = cb + (uint64_t)min(k0 + 2 * a, cap - 1) * R, *ty = cb + (uint64_t)min(k0 + 2 * a + 1, cap - 1) * R;
+        for (uint32_t r0 = 0; r0 < R; r0 += 512) {
+            uint4 x[8], y[8];
+            bf16x8_t kf[16], qh[16], ql[16];
 #pragma unroll
-            for (int u = 0; u < 8; u++) {  // (a step behind the end re-reads the last one and is not used)
-                const uint32_t off = 32 * min(s0 + u, steps - 1);
+            for (int u = 0; u < 8; u++) {
+                const uint32_t off = min(r0 + 64 * u + 8 * (tid & 7), R - 8);
+                x[u] = *(const uint4 *)(tx + off);
+                y[u] = *(const uint4 *)(ty + off);
+            }
+#pragma unroll
+            for (int u = 0; u < 16; u++) {
+                const uint32_t off = min(r0 + 32 * u, R - 32);
                 kf[u] = *(const bf16x8_t *)(kp + off);
                 qh[u] = *(const bf16x8_t *)(qp + off);
                 ql[u] = *(const bf16x8_t *)(qp + R + off);
             }
             __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-            for (int u = 0; u < 8; u++)
-                if (s0 + u < steps) {
+            for (int u = 0; u < 8; u++) {
+                const uint32_t off = min(r0 + 64 * u + 8 * (tid & 7), R - 8);
+                const uint32_t xs[4] = {x[u].x, x[u].y, x[u].z, x[u].w}, ys[4] = {y[u].x, y[u].y, y[u].z, y[u].w};
+                uint32_t *dst = (uint32_t *)ct + off * (VLD / 2) + a;
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    dst[e * VLD] = __builtin_amdgcn_perm(ys[e], xs[e], 0x05040100u);
+                    dst[e * VLD + VLD / 2] = __builtin_amdgcn_perm(ys[e], xs[e], 0x07060302u);
+                }
+            }
+#pragma unroll
+            for (int u = 0; u < 16; u++)
+                if (r0 / 32 + u < steps) {
                     sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh[u], kf[u], sc, 0, 0, 0);
                     sc2 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ql[u], kf[u], sc2, 0, 0, 0);
                 }
-        }
-        // transposed latents: two keys a dword (8 pieces of 8 dims x 32 key pairs a round)
-#pragma unroll 4
-        for (uint32_t p0 = 0; p0 < R / 8; p0 += 8) {
-            const uint32_t piece = min(p0 + (tid & 7), R / 8 - 1), a = tid >> 3;
-            const uint4 x = *(const uint4 *)(cb + (uint64_t)min(k0 + 2 * a, k_end - 1) * R + 8 * piece);
-            const uint4 y = *(const uint4 *)(cb + (uint64_t)min(k0 + 2 * a + 1, k_end - 1) * R + 8 * piece);
-            const uint32_t xs[4] = {x.x, x.y, x.z, x.w}, ys[4] = {y.x, y.y, y.z, y.w};
-            uint32_t *dst = (uint32_t *)ct + piece * (8 * VLD / 2) + a;
-#pragma unroll
-            for (int e = 0; e < 4; e++) {
-                dst[e * VLD] = __builtin_amdgcn_perm(ys[e], xs[e], 0x05040100u);
-                dst[e * VLD + VLD / 2] = __builtin_amdgcn_perm(ys[e], xs[e], 0x07060302u);
-            }
         }
         const uint32_t key = k0 + 16 * wave + c;
 #pragma unroll

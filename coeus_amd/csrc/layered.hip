@@ -27,9 +27,10 @@ LayeredStack::~LayeredStack() {
 }
 
 // ---------------------------------------------------------------- state
-// Offsets are counted first (base null), then assigned: the recurrent part of every layer, then the rings
-// of cached latents (which need no clearing: positions not yet written are never read).
-int LayeredState::create(const LayeredStack &stack, bool bf16, uint64_t batch_, uint64_t max_ctx) {
+// Offsets are counted first, then assigned: the recurrent part of every layer, then the rings of cached
+// latents.  Those start as zeros and are not cleared again: a position that is not written yet has no weight,
+// but its slot may be read, so it has to hold finite values.
+int LayeredState::create(const LayeredStack &stack, bool bf16, uint64_t batch_, uint64_t max_ctx, hipStream_t st) {
     batch = batch_;
     layers.assign(stack.layers.size(), Layer{});
     uint64_t off = 0;
@@ -51,6 +52,7 @@ int LayeredState::create(const LayeredStack &stack, bool bf16, uint64_t batch_, 
         a[l] = take(batch * cap * m.kv_rank * (bf16 ? 2 : 4));
     }
     COEUS_TRY(mem.ensure(off ? off : 256));
+    COEUS_HIP(hipMemsetAsync(mem.p, 0, mem.bytes, st));
     for (size_t l = 0; l < layers.size(); l++) {
         char *p = (char *)mem.p;
         if (stack.layers[l].spec.mixer.kind == MixerKind::GatedDelta) layers[l].delta = DeltaState{(float *)(p + a[l]), (float *)(p + r[l])};
@@ -477,8 +479,7 @@ int layered_session_init(Session &s) {
     Model &m = *s.m;
     const LayeredStack &stack = *m.stack;
     const uint64_t B = s.batch, W = stack.cfg.width;
-    COEUS_TRY(s.state.create(stack, m.cfg.weight_dtype == COEUS_W_BF16, B, s.max_ctx));
-    COEUS_TRY(s.state.clear(m.stream));
+    COEUS_TRY(s.state.create(stack, m.cfg.weight_dtype == COEUS_W_BF16, B, s.max_ctx, m.stream));
     uint64_t in = 0, att = 0, ff = 0, q = 0, sc = 0;
     auto up = [](uint64_t &v, uint64_t x) { if (x > v) v = x; };
     for (size_t l = 0; l < stack.layers.size(); l++) {

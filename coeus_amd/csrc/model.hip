@@ -395,8 +395,7 @@ int model_forward(Model &m, const uint64_t *ids, uint64_t seq_len, float *logits
         // a sequence of its own: fresh state, dropped at the end
         LayeredState state;
         struct Drop { LayeredState &s; ~Drop() { s.release(); } } drop{state};
-        COEUS_TRY(state.create(*m.stack, c.weight_dtype == COEUS_W_BF16, 1, seq_len));
-        COEUS_TRY(state.clear(st));
+        COEUS_TRY(state.create(*m.stack, c.weight_dtype == COEUS_W_BF16, 1, seq_len, st));
         COEUS_TRY(layered_workspace(m, m.ws, 1, seq_len, 0));
         COEUS_TRY(m.ws.logits.ensure((all_rows ? seq_len : 1) * V * 4));
         COEUS_HIP(hipMemcpyAsync(m.ws.ids.p, ids, seq_len * 8, hipMemcpyHostToDevice, st));

@@ -55,8 +55,8 @@ struct LayeredState {
     std::vector<Layer> layers;
     DeviceBuf mem;
     uint64_t batch = 0, recurrent_bytes = 0;  // the recurrent part comes first in `mem` and starts at zero
-    int create(const LayeredStack &stack, bool bf16, uint64_t batch, uint64_t max_ctx);
-    int clear(hipStream_t st);  // start of a sequence
+    int create(const LayeredStack &stack, bool bf16, uint64_t batch, uint64_t max_ctx, hipStream_t st);
+    int clear(hipStream_t st);  // start of another sequence
     void release() { mem.release(); layers.clear(); }
 };
 
