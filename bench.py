@@ -2,6 +2,7 @@
 """Headline benchmark: decode throughput of the transformer forward path on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload NAME] [--batch B]
+    python bench.py --layered [SIZE,..] [--steps K] [--warmup W] [--batch B]
 
 Default workload (the 7B-shape configuration the headline target is stated on):
 7B-shape decoder, Q4_0 weights, f16 KV cache, batch 1, context filled to 4096.  A "step" is one
@@ -21,6 +22,10 @@ Prints ONE JSON line: whole-job tokens/s plus
                  250M f32 forward over 128 ids, 250M bf16, 250M Q8_0 at batch 1 and 8, the 1B-class
                  Q4_0 decoder at batch 4): throughput, ms per step, the roofline of each one's
                  dominant kernel and what its outputs were checked against.
+
+With --layered it measures layered decoders instead (three gated-delta-rule layers to one windowed
+latent-attention layer, a gated feed-forward in each) beside the bf16 transformer of the same width,
+depth, heads and feed-forward: one JSON line with prompt and decode throughput of both.
 """
 import argparse
 import json
@@ -340,6 +345,58 @@ def decode_workload(name, batches, K, W, use_graph, check):
     return res
 
 
+# ---------------------------------------------------------------- layered models
+# width, heads of 128, query/key heads of the delta rule, query latent, key/value latent, window,
+# feed-forward, layers
+LAYERED_SIZES = {"1024": (1024, 8, 4, 384, 256, 512, 2816, 12),
+                 "2048": (2048, 16, 8, 768, 512, 1024, 5632, 12),
+                 "4096": (4096, 32, 16, 1536, 512, 1024, 11008, 8)}
+
+
+def layered_pair(size, ctx, batch):
+    """(layered configuration, transformer configuration) of one size."""
+    from coeus_amd import LayeredConfig, Transformer250MConfig
+
+    W, H, KH, qr, kr, win, ff, L = LAYERED_SIZES[size]
+    mlp = {"kind": "dense", "ff": ff}
+    d = {"type": "delta", "mixer": dict(heads=H, kv_heads=KH, dim=128, vdim=128, conv=4), "mlp": mlp}
+    a = {"type": "latent_attention", "mlp": mlp,
+         "mixer": dict(heads=H, dim=128, vdim=128, q_rank=qr, kv_rank=kr, scale=128 ** -0.5, mask={"size": win})}
+    cfg = {"architecture": "Bofirax", "vocab": 32000, "width": W, "norm": {"eps": 1e-5},
+           "layers": [a if i % 4 == 3 else d for i in range(L)]}
+    peer = Transformer250MConfig(hidden_dim=W, num_layers=L, num_heads=H, head_dim=128, intermediate_dim=ff, vocab_size=32000,
+                                 max_seq_len=ctx, use_bias=False, activation="silu_gated", norm="rmsnorm", norm_scope="token",
+                                 weight_dtype="bf16", kv_dtype="bf16", max_batch=16)
+    return LayeredConfig(cfg, max_seq_len=ctx, max_batch=16), peer
+
+
+def layered_workload(size, B, K, W, ctx, use_graph, check):
+    """Both models of one size, measured alike: prompt pass, W warm-up steps, K timed greedy steps, the
+    decode matmuls and the mixers of a step replayed on their own."""
+    from coeus_amd import PLUGINS
+
+    out = {"size": size, "batch": B, "context": ctx}
+    for name, family, cfg in zip(("layered", "transformer"), ("layered_model", "transformer_model"), layered_pair(size, ctx, B)):
+        model = PLUGINS[family].create_builder().build(cfg, seed=0xC0E05)
+        rng = np.random.default_rng(0xC0E06)
+        sess, prompt, ids, dt, prefill_s, tok0, tok = run_decode(model, cfg, B, K, W, ctx, use_graph, rng, True)
+        leg = {"weights_gb": round(model.weight_bytes() / 1e9, 3), "hip_graph": sess.graph_enabled,
+               "prefill": {"tokens": int(prompt.size), "ms": round(prefill_s * 1e3, 2), "tok_s": round(prompt.size / prefill_s, 1)},
+               "decode": {"tok_s": round(B * K / dt, 1), "ms_per_step": round(dt * 1e3 / K, 4)}}
+        for key, timer in (("decode_matmuls", sess.time_decode_matmuls), ("decode_mixers", sess.time_decode_attention)):
+            ms, launches, nbytes = timer(20)
+            leg[key] = {"bound": "hbm", "us_per_call": round(ms * 1e3 / launches, 2), "calls_per_step": launches // 20,
+                        "bytes_per_call": nbytes // launches, "achieved": round(nbytes / ms / 1e6, 1), "peak": HBM_PEAK_GBS,
+                        "unit": "GB/s", "frac": round(nbytes / ms / 1e6 / HBM_PEAK_GBS, 4)}
+        if check:
+            leg["check"] = check_outputs(model, sess, prompt, ids, tok0, tok, W, K, ctx)
+        leg["outputs_checked"] = bool(check)
+        sess.close()
+        model.close()
+        out[name] = leg
+    return out
+
+
 def forward_workload(check, with_cpu):
     """The reference's own configuration: default Transformer250MConfig (f32 weights and cache,
     whole-slice LayerNorm), seeded weights, one forward over 128 uniform ids with the logits of
@@ -442,11 +499,30 @@ def main():
     ap.add_argument("--no-check", action="store_true", help="skip the output checks (profiling runs)")
     ap.add_argument("--no-other-workloads", action="store_true",
                     help="skip the other four benchmark configurations (default run of the 7B workload only)")
+    ap.add_argument("--layered", nargs="?", const=",".join(sorted(LAYERED_SIZES)), metavar="SIZE,..",
+                    help="layered decoders beside the transformer of the same size: " + ", ".join(sorted(LAYERED_SIZES)))
     a = ap.parse_args()
+    if a.layered and not set(a.layered.split(",")) <= set(LAYERED_SIZES):
+        ap.error(f"--layered takes sizes out of {', '.join(sorted(LAYERED_SIZES))}")
     if a.gpus != 1:
         print("bench.py measures ONE MI355X: this build has no multi-GPU path "
               "(pass --gpus 1).", file=sys.stderr)
         sys.exit(2)
+
+    if a.layered:
+        ctx = 4096
+        if a.steps + a.warmup + 1 >= ctx:
+            print("steps + warmup must stay below the context length", file=sys.stderr)
+            sys.exit(2)
+        sizes = [layered_workload(s, a.batch, a.steps, a.warmup, ctx, not a.no_graph, not a.no_check) for s in a.layered.split(",")]
+        last = sizes[-1]["layered"]["decode"]
+        print(json.dumps({
+            "metric": "layered decoder: decode tok/s @1 MI355X", "value": last["tok_s"], "unit": "tok/s", "n_gpus": 1,
+            "steps": a.steps, "warmup": a.warmup, "ms_per_step": last["ms_per_step"], "higher_is_better": True,
+            "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+            "config": {"model": f"layered {sizes[-1]['size']}", "global_batch": a.batch, "seq_len": ctx, "parallelism": "none"},
+            "sizes": sizes}))
+        return
 
     from coeus_amd import Transformer250MConfig, TransformerModelPlugin
 

@@ -45,6 +45,18 @@ class CLoadOptions(C.Structure):
     _fields_ = [("weight_dtype", C.c_uint32), ("max_seq_len", C.c_uint64), ("max_batch", C.c_uint64)]
 
 
+class CDeltaShape(C.Structure):
+    _fields_ = [(f, C.c_uint64) for f in ("heads", "kv_heads", "dim", "vdim", "conv", "in_ld")]
+
+
+class CDeltaWeights(C.Structure):
+    _fields_ = [(f, C.c_void_p) for f in ("conv_dev", "exp_a_dev", "dt_bias_dev", "norm_dev")] + [("eps", C.c_float)]
+
+
+class CLatentShape(C.Structure):
+    _fields_ = [(f, C.c_uint64) for f in ("heads", "dim", "vdim", "q_rank", "kv_rank", "window")] + [("scale", C.c_float)]
+
+
 # name -> (restype, argtypes); this table is also what the symbol-export test walks
 _u64, _u32, _f32 = C.c_uint64, C.c_uint32, C.c_float
 _vp, _cfgp = C.c_void_p, C.POINTER(CConfig)
@@ -137,6 +149,13 @@ SIGNATURES = {
                                             _vp]),
     "coeus_op_attention_decode_static": (C.c_int, [_vp, _vp, _vp, _u32, _u64, _u64, _u64, _u64, _u64, _u32, _u32,
                                                    _vp, _vp]),
+    "coeus_op_norm_residual": (C.c_int, [_vp, _u64, _u64, _vp, _vp, _f32, _vp, _vp]),
+    "coeus_op_delta_prompt": (C.c_int, [C.POINTER(CDeltaShape), C.POINTER(CDeltaWeights), _vp, _vp, _vp, _u64, _u64, _u64,
+                                        C.c_int, _vp, _vp]),
+    "coeus_op_delta_step": (C.c_int, [C.POINTER(CDeltaShape), C.POINTER(CDeltaWeights), _vp, _vp, _vp, _u64, _u64, _vp, _vp]),
+    "coeus_op_window_attention": (C.c_int, [C.POINTER(CLatentShape), _u32, _vp, _vp, _u64, _u64, _u64, _vp, _vp]),
+    "coeus_op_latent_decode": (C.c_int, [C.POINTER(CLatentShape), _u32, _vp, _vp, _vp, _f32, _vp, _vp, _u64, _u64, _u64, _vp,
+                                         _vp]),
 }
 
 _lib = None

@@ -710,4 +710,131 @@ int coeus_op_attention_decode_static(const float *qkv_dev, const void *k_cache_d
     COEUS_GUARD_END
 }
 
+// ---------------------------------------------------------------- mechanisms of layered models
+// Waits for the call's kernels, frees its buffers, and reports whichever failed first.
+static int finish_op(int rc, hipStream_t st, std::initializer_list<DeviceBuf *> bufs, const char *what) {
+    const hipError_t e = hipStreamSynchronize(st);
+    for (DeviceBuf *b : bufs) b->release();
+    if (rc == COEUS_OK && e != hipSuccess) rc = fail(COEUS_DEVICE_ERROR, "%s failed: %s", what, hipGetErrorString(e));
+    return rc;
+}
+
+int coeus_op_norm_residual(const float *y_dev, uint64_t rows, uint64_t hidden, const float *scale_dev, const float *ls_dev,
+                           float eps, float *h_dev, void *stream) {
+    COEUS_GUARD_BEGIN
+    if (!y_dev || !scale_dev || !h_dev) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    hipStream_t st = (hipStream_t)stream;
+    return finish_op(launch_norm_residual(y_dev, rows, hidden, scale_dev, ls_dev, eps, h_dev, st), st, {}, "norm");
+    COEUS_GUARD_END
+}
+
+static bool delta_args(const coeus_delta_shape *s, const coeus_delta_weights *w, DeltaDims &dm, DeltaParams &pr) {
+    if (!s || !w || !w->conv_dev || !w->exp_a_dev || !w->dt_bias_dev || !w->norm_dev) return false;
+    for (uint64_t v : {s->heads, s->kv_heads, s->dim, s->vdim, s->conv, s->in_ld})
+        if (v > 0x7fffffffull) return false;
+    dm = DeltaDims{(uint32_t)s->heads, (uint32_t)s->kv_heads, (uint32_t)s->dim, (uint32_t)s->vdim, (uint32_t)s->conv, (uint32_t)s->in_ld};
+    pr = DeltaParams{w->conv_dev, w->exp_a_dev, w->dt_bias_dev, w->norm_dev, w->eps};
+    return true;
+}
+
+int coeus_op_delta_prompt(const coeus_delta_shape *shape, const coeus_delta_weights *w, const float *proj_dev,
+                          float *state_dev, float *ring_dev, uint64_t batch, uint64_t n, uint64_t pos0, int chunked,
+                          float *out_dev, void *stream) {
+    COEUS_GUARD_BEGIN
+    DeltaDims dm;
+    DeltaParams pr;
+    if (!delta_args(shape, w, dm, pr) || !proj_dev || !state_dev || !ring_dev || !out_dev)
+        return fail(COEUS_INVALID_INPUT, "null pointer argument or size out of range");
+    if (batch == 0 || n == 0 || batch > 65535 || n > 0x7fffffffull)
+        return fail(COEUS_INVALID_INPUT, "delta rule: %llu x %llu rows out of range", (unsigned long long)batch, (unsigned long long)n);
+    hipStream_t st = (hipStream_t)stream;
+    const uint64_t rows = batch * n, qk = rows * dm.kv_heads * delta_padded_dim(dm.d) * 4;
+    DeviceBuf q, k, v, beta, lg, scratch;
+    const uint64_t sb = chunked ? delta_prompt_scratch_bytes(dm, batch, n) : 0;
+    int rc = q.ensure(qk);
+    if (rc == COEUS_OK) rc = k.ensure(qk);
+    if (rc == COEUS_OK) rc = v.ensure(rows * dm.heads * dm.e * 4);
+    if (rc == COEUS_OK) rc = beta.ensure(rows * dm.heads * 4);
+    if (rc == COEUS_OK) rc = lg.ensure(rows * dm.heads * 4);
+    if (rc == COEUS_OK && sb) rc = scratch.ensure(sb);
+    const DeltaOperands op{(float *)q.p, (float *)k.p, (float *)v.p, (float *)beta.p, (float *)lg.p};
+    const DeltaState state{state_dev, ring_dev};
+    if (rc == COEUS_OK) rc = launch_delta_prepare(proj_dev, dm, pr, state, batch, n, pos0, op, st);
+    if (rc == COEUS_OK) rc = launch_delta_ring(proj_dev, dm, state, batch, n, pos0, st);
+    if (rc == COEUS_OK) rc = launch_delta_prompt(dm, op, state, batch, n, out_dev, (float *)scratch.p, scratch.bytes, st);
+    if (rc == COEUS_OK) rc = launch_delta_gate(out_dev, proj_dev, dm, pr, rows, out_dev, nullptr, st);
+    return finish_op(rc, st, {&q, &k, &v, &beta, &lg, &scratch}, "delta rule");
+    COEUS_GUARD_END
+}
+
+static int upload_position(uint64_t pos, DeviceBuf &buf, hipStream_t st) {
+    if (pos >= 0x7fffffffull) return fail(COEUS_INVALID_INPUT, "position %llu out of range", (unsigned long long)pos);
+    const uint32_t p = (uint32_t)pos;
+    COEUS_TRY(buf.ensure(4));
+    COEUS_HIP(hipMemcpyAsync(buf.p, &p, 4, hipMemcpyHostToDevice, st));
+    COEUS_HIP(hipStreamSynchronize(st));
+    return COEUS_OK;
+}
+
+int coeus_op_delta_step(const coeus_delta_shape *shape, const coeus_delta_weights *w, const float *proj_dev,
+                        float *state_dev, float *ring_dev, uint64_t batch, uint64_t pos, float *out_dev, void *stream) {
+    COEUS_GUARD_BEGIN
+    DeltaDims dm;
+    DeltaParams pr;
+    if (!delta_args(shape, w, dm, pr) || !proj_dev || !state_dev || !ring_dev || !out_dev)
+        return fail(COEUS_INVALID_INPUT, "null pointer argument or size out of range");
+    hipStream_t st = (hipStream_t)stream;
+    DeviceBuf p;
+    int rc = upload_position(pos, p, st);
+    if (rc == COEUS_OK)
+        rc = launch_delta_step(proj_dev, dm, pr, DeltaState{state_dev, ring_dev}, batch, (const uint32_t *)p.p, out_dev, st);
+    return finish_op(rc, st, {&p}, "delta rule");
+    COEUS_GUARD_END
+}
+
+static int latent_args(const coeus_latent_shape *s, uint32_t kv_dtype, LatentDims &dm) {
+    if (!s) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    if (kv_dtype != COEUS_KV_BF16 && kv_dtype != COEUS_KV_F32)
+        return fail(COEUS_INVALID_INPUT, "latent attention: the tensors must be bf16 or f32");
+    for (uint64_t v : {s->heads, s->dim, s->vdim, s->q_rank, s->kv_rank, s->window})
+        if (v > 0x3fffffffull) return fail(COEUS_INVALID_INPUT, "latent attention: sizes out of range");
+    dm = LatentDims{(uint32_t)s->heads, (uint32_t)s->dim, (uint32_t)s->vdim, (uint32_t)s->q_rank, (uint32_t)s->kv_rank,
+                    (uint32_t)s->window, (uint32_t)round_up(s->q_rank + s->kv_rank, 4), s->scale};
+    return COEUS_OK;
+}
+
+int coeus_op_window_attention(const coeus_latent_shape *shape, uint32_t kv_dtype, const void *q_dev, const void *kv_dev,
+                              uint64_t batch, uint64_t n, uint64_t hist, float *out_dev, void *stream) {
+    COEUS_GUARD_BEGIN
+    LatentDims dm;
+    COEUS_TRY(latent_args(shape, kv_dtype, dm));
+    if (!q_dev || !kv_dev || !out_dev) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    hipStream_t st = (hipStream_t)stream;
+    const uint64_t q_ld = (uint64_t)dm.heads * dm.d, kv_ld = q_ld + (uint64_t)dm.heads * dm.e;
+    return finish_op(launch_window_attention(q_dev, q_ld, kv_dev, kv_ld, kv_dtype == COEUS_KV_BF16, dm, batch, n, hist, out_dev,
+                                             nullptr, st), st, {}, "window attention");
+    COEUS_GUARD_END
+}
+
+int coeus_op_latent_decode(const coeus_latent_shape *shape, uint32_t kv_dtype, const float *q_dev, const float *proj_dev,
+                           const float *scale_dev, float eps, const void *ukv_dev, void *cache_dev, uint64_t cap,
+                           uint64_t batch, uint64_t pos, float *out_dev, void *stream) {
+    COEUS_GUARD_BEGIN
+    LatentDims dm;
+    COEUS_TRY(latent_args(shape, kv_dtype, dm));
+    if (!q_dev || !proj_dev || !scale_dev || !ukv_dev || !cache_dev || !out_dev) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    if (cap == 0 || cap > 0x7fffffffull) return fail(COEUS_INVALID_INPUT, "latent attention: cache size out of range");
+    hipStream_t st = (hipStream_t)stream;
+    const LatentCache cache{cache_dev, (uint32_t)cap, kv_dtype == COEUS_KV_BF16};
+    DeviceBuf p, scratch;
+    int rc = upload_position(pos, p, st);
+    const uint64_t sb = latent_decode_scratch_bytes(dm, cache, batch);
+    if (rc == COEUS_OK && sb) rc = scratch.ensure(sb);
+    if (rc == COEUS_OK)
+        rc = launch_latent_decode(q_dev, ukv_dev, dm, LatentNew{proj_dev, scale_dev, eps}, cache, batch, (const uint32_t *)p.p,
+                                  out_dev, (float *)scratch.p, scratch.bytes, st);
+    return finish_op(rc, st, {&p, &scratch}, "latent attention");
+    COEUS_GUARD_END
+}
+
 }  // extern "C"

@@ -26,12 +26,27 @@ __device__ __forceinline__ void lat_store(void *p, uint64_t i, float v) {
 }
 
 static int check_dims(const LatentDims &dm, const LatentCache &cache) {
-    if (dm.heads == 0 || dm.heads > 65535 || dm.d == 0 || dm.d > 256 || dm.e == 0 || dm.e > 256 || dm.q_rank == 0 ||
+    if (dm.heads == 0 || dm.heads > 65534 || dm.d == 0 || dm.d > 256 || dm.e == 0 || dm.e > 256 || dm.q_rank == 0 ||
         dm.rank == 0 || dm.rank > 2048 || dm.in_ld < dm.q_rank + dm.rank)
         return fail(COEUS_INVALID_INPUT, "latent attention: sizes out of range");
     if (cache.cap == 0 || (dm.window && cache.cap > dm.window))
         return fail(COEUS_INVALID_INPUT, "latent attention: cache of %u positions for a window of %u", cache.cap, dm.window);
     return COEUS_OK;
+}
+
+// RMS norm of one row by a workgroup of 256: put(i, value) for every element.
+template <typename Put>
+__device__ __forceinline__ void norm_row_256(const float *__restrict__ x, uint32_t len, float eps,
+                                             const float *__restrict__ scale, float *sh, Put put) {
+    const uint32_t tid = threadIdx.x;
+    float s2 = 0.f;
+    for (uint32_t i = tid; i < len; i += 256) s2 = fmaf(x[i], x[i], s2);
+    s2 = wave_sum(s2);
+    __syncthreads();  // (sh may still be read for the row before)
+    if ((tid & 63) == 0) sh[tid >> 6] = s2;
+    __syncthreads();
+    const float rs = 1.0f / sqrtf(((sh[0] + sh[1]) + (sh[2] + sh[3])) / (float)len + eps);
+    for (uint32_t i = tid; i < len; i += 256) put(i, x[i] * rs * scale[i]);
 }
 
 // blockIdx.y + part0 0: the query latent, 1: the key/value latent.
@@ -46,24 +61,16 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(const float *__restric
     __shared__ float sh[4];
     const uint64_t row = blockIdx.x;
     const bool is_q = blockIdx.y + part0 == 0;
-    const uint32_t len = is_q ? dm.q_rank : dm.rank, tid = threadIdx.x;
     const float *x = proj + row * dm.in_ld + (is_q ? 0 : dm.q_rank);
-    float s2 = 0.f;
-    for (uint32_t i = tid; i < len; i += 256) s2 = fmaf(x[i], x[i], s2);
-    s2 = wave_sum(s2);
-    if ((tid & 63) == 0) sh[tid >> 6] = s2;
-    __syncthreads();
-    const float rs = 1.0f / sqrtf(((sh[0] + sh[1]) + (sh[2] + sh[3])) / (float)len + eps);
     if (is_q) {
-        for (uint32_t i = tid; i < len; i += 256) {
-            const float v = x[i] * rs * q_scale[i];
-            if (cq) cq[row * len + i] = v;
+        norm_row_256(x, dm.q_rank, eps, q_scale, sh, [&](uint32_t i, float v) {
+            if (cq) cq[row * dm.q_rank + i] = v;
             if (cq_lp) cq_lp[row * cq_ld + i] = f32_to_lp_bits(v, lp_bf16);
-        }
+        });
     } else {
         const uint64_t dst = pos_dev ? (row * cap + *pos_dev % cap) * dm.rank
                                      : ((row / n) * lat_rows + lat_off + row % n) * lat_ld;
-        for (uint32_t i = tid; i < len; i += 256) lat_store<BF16>(lat, dst + i, x[i] * rs * c_scale[i]);
+        norm_row_256(x, dm.rank, eps, c_scale, sh, [&](uint32_t i, float v) { lat_store<BF16>(lat, dst + i, v); });
     }
 }
 
@@ -468,11 +475,23 @@ static uint32_t latent_shares(uint32_t cap) {
 }
 
 // W_uk^T q as two bf16 numbers per element, [batch][heads][high, low][rank]: one workgroup per (128 columns of the rank, head) and every sequence, so
-// that the weights are read once.  Thread (g, r): column pair r, rows g, g + 4, ..
+// that the weights are read once.  Thread (g, r): column pair r, rows g, g + 4, ..  The workgroups behind the
+// last head (blockIdx.y == heads) normalise the new tokens' latents into the ring.
 template <int BP>
 __global__ __launch_bounds__(256) void latent_absorb_kernel(const float *__restrict__ q, const uint16_t *__restrict__ ukv,
-                                                            LatentDims dm, uint32_t batch, uint16_t *__restrict__ qa) {
+                                                            LatentDims dm, uint32_t batch, uint16_t *__restrict__ qa, LatentNew nw,
+                                                            uint16_t *__restrict__ cache, uint32_t cap,
+                                                            const uint32_t *pos_dev) {
     extern __shared__ float lds[];  // q [BP][d], partial sums [4][BP][128]
+    if (blockIdx.y == dm.heads) {
+        for (uint32_t b = blockIdx.x; b < batch; b += gridDim.x) {
+            __shared__ float sh[4];
+            const float *x = nw.proj + (uint64_t)b * dm.in_ld + dm.q_rank;
+            uint16_t *dst = cache + ((uint64_t)b * cap + *pos_dev % cap) * dm.rank;
+            norm_row_256(x, dm.rank, nw.eps, nw.scale, sh, [&](uint32_t i, float v) { dst[i] = f32_to_bf16_bits(v); });
+        }
+        return;
+    }
     const uint32_t tid = threadIdx.x, g = tid >> 6, rp = tid & 63, h = blockIdx.y, d = dm.d, R = dm.rank;
     const uint32_t r = blockIdx.x * 128 + 2 * rp, rc = min(r, R - 2);
     float *qs = lds, *red = lds + BP * d;
@@ -520,6 +539,7 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(const float *__restr
 // latents for 16 heads, the softmax of the tile runs over LDS, then a wave accumulates a quarter of the
 // rank.  Absorbed queries and weights enter the products as sums of two bf16 numbers each.
 // The share's record: maximum (base 2), sum, weighted latent.
+template <int PT>  // 16-wide column tiles of a wave: rank <= 64 PT
 __global__ __launch_bounds__(256) void latent_scores_kernel(const uint16_t *__restrict__ qa, LatentDims dm,
                                                             const uint16_t *__restrict__ cache, uint32_t cap,
                                                             const uint32_t *pos_dev, uint32_t keys_per_share,
@@ -539,12 +559,12 @@ __global__ __launch_bounds__(256) void latent_scores_kernel(const uint16_t *__re
     if (tid < 16) { ms[tid] = -1e30f; ls[tid] = 0.f; }
     const uint16_t *qp = qa + (b * dm.heads + hc) * 2 * R + 8 * g;
     const uint16_t *cb = cache + b * cap * R;
-    const uint32_t per = ((R / 16) + 3) / 4;  // 16-wide column tiles of a wave (at most 16)
-    float4_t acc[16];
+    constexpr uint32_t RD = PT == 4 ? 256 : 512;  // of the rank in a round
+    float4_t acc[PT];
 #pragma unroll
-    for (int t = 0; t < 16; t++) acc[t] = float4_t{0.f, 0.f, 0.f, 0.f};
+    for (int t = 0; t < PT; t++) acc[t] = float4_t{0.f, 0.f, 0.f, 0.f};
     for (uint32_t k0 = k_begin; k0 < k_end; k0 += kKeyTile) {
-        // 512 of the rank a round.  Everything is requested at once, from addresses that do not depend on the
+        // RD of the rank a round.  Everything is requested at once, from addresses that do not depend on the
         // position (slots that are not written yet hold finite values and are masked; a piece behind the end
         // re-reads the last one and is not used): the tile as key pairs for the transposed copy (8 pieces of 8
         // dims x 32 pairs a step), as right operands for keys k0 + 16 wave + c, and the absorbed queries.
@@ -552,17 +572,17 @@ __global__ __launch_bounds__(256) void latent_scores_kernel(const uint16_t *__re
         const uint16_t *kp = cb + (uint64_t)min(k0 + 16 * wave + c, cap - 1) * R + 8 * g;
         const uint32_t a = tid >> 3, steps = R / 32;
         const uint16_t *tx = cb + (uint64_t)min(k0 + 2 * a, cap - 1) * R, *ty = cb + (uint64_t)min(k0 + 2 * a + 1, cap - 1) * R;
-        for (uint32_t r0 = 0; r0 < R; r0 += 512) {
-            uint4 x[8], y[8];
-            bf16x8_t kf[16], qh[16], ql[16];
+        for (uint32_t r0 = 0; r0 < R; r0 += RD) {
+            uint4 x[RD / 64], y[RD / 64];
+            bf16x8_t kf[RD / 32], qh[RD / 32], ql[RD / 32];
 #pragma unroll
-            for (int u = 0; u < 8; u++) {
+            for (int u = 0; u < (int)RD / 64; u++) {
                 const uint32_t off = min(r0 + 64 * u + 8 * (tid & 7), R - 8);
                 x[u] = *(const uint4 *)(tx + off);
                 y[u] = *(const uint4 *)(ty + off);
             }
 #pragma unroll
-            for (int u = 0; u < 16; u++) {
+            for (int u = 0; u < (int)RD / 32; u++) {
                 const uint32_t off = min(r0 + 32 * u, R - 32);
                 kf[u] = *(const bf16x8_t *)(kp + off);
                 qh[u] = *(const bf16x8_t *)(qp + off);
@@ -570,7 +590,7 @@ __global__ __launch_bounds__(256) void latent_scores_kernel(const uint16_t *__re
             }
             __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-            for (int u = 0; u < 8; u++) {
+            for (int u = 0; u < (int)RD / 64; u++) {
                 const uint32_t off = min(r0 + 64 * u + 8 * (tid & 7), R - 8);
                 const uint32_t xs[4] = {x[u].x, x[u].y, x[u].z, x[u].w}, ys[4] = {y[u].x, y[u].y, y[u].z, y[u].w};
                 uint32_t *dst = (uint32_t *)ct + off * (VLD / 2) + a;
@@ -581,7 +601,7 @@ __global__ __launch_bounds__(256) void latent_scores_kernel(const uint16_t *__re
                 }
             }
 #pragma unroll
-            for (int u = 0; u < 16; u++)
+            for (int u = 0; u < (int)RD / 32; u++)
                 if (r0 / 32 + u < steps) {
                     sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh[u], kf[u], sc, 0, 0, 0);
                     sc2 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ql[u], kf[u], sc2, 0, 0, 0);
@@ -615,9 +635,9 @@ __global__ __launch_bounds__(256) void latent_scores_kernel(const uint16_t *__re
             pal[j] = *(const bf16x8_t *)(pl + c * PLD + 32 * j + 8 * g);
         }
 #pragma unroll
-        for (int t = 0; t < 16; t++) {
-            const uint32_t tile = wave * per + t;
-            if (t < (int)per && 16 * tile < R) {  // wave-uniform
+        for (int t = 0; t < PT; t++) {
+            const uint32_t tile = wave * PT + t;
+            if (16 * tile < R) {  // wave-uniform
 #pragma unroll
                 for (int i = 0; i < 4; i++) acc[t][i] *= cr[i];
 #pragma unroll
@@ -638,9 +658,9 @@ __global__ __launch_bounds__(256) void latent_scores_kernel(const uint16_t *__re
         float *rec = part + ((b * dm.heads + hh) * gridDim.x + share) * (R + 2);
         if (wave == 0 && c == 0) { rec[0] = ms[4 * g + i]; rec[1] = ls[4 * g + i]; }
 #pragma unroll
-        for (int t = 0; t < 16; t++) {
-            const uint32_t r = 16 * (wave * per + t) + c;
-            if (t < (int)per && r < R) rec[2 + r] = acc[t][i];
+        for (int t = 0; t < PT; t++) {
+            const uint32_t r = 16 * (wave * PT + t) + c;
+            if (r < R) rec[2 + r] = acc[t][i];
         }
     }
 }
@@ -711,36 +731,46 @@ uint64_t latent_decode_scratch_bytes(const LatentDims &dm, const LatentCache &ca
     return batch * dm.heads * (dm.rank + latent_shares(cache.cap) * (dm.rank + 2ull)) * 4;
 }
 
-int launch_latent_decode(const float *q, const void *ukv, const LatentDims &dm, const LatentCache &cache,
-                         uint64_t batch, const uint32_t *pos_dev, float *out, float *scratch, uint64_t scratch_bytes,
-                         hipStream_t st) {
+int launch_latent_decode(const float *q, const void *ukv, const LatentDims &dm, const LatentNew &nw,
+                         const LatentCache &cache, uint64_t batch, const uint32_t *pos_dev, float *out, float *scratch,
+                         uint64_t scratch_bytes, hipStream_t st) {
     COEUS_TRY(check_dims(dm, cache));
     if (batch == 0 || batch > 65535 || !pos_dev) return fail(COEUS_INVALID_INPUT, "latent attention: rows out of range");
     const uint64_t want = latent_decode_scratch_bytes(dm, cache, batch);
     if (want && batch <= 16 && scratch && scratch_bytes >= want) {
-        const uint16_t *w = (const uint16_t *)ukv, *cc = (const uint16_t *)cache.c;
+        const uint16_t *w = (const uint16_t *)ukv;
+        uint16_t *cc = (uint16_t *)cache.c;
         uint16_t *qa = (uint16_t *)scratch;
         float *part = scratch + batch * dm.heads * dm.rank;
         const uint32_t shares = latent_shares(cache.cap), bp = pad_batch(batch), R = dm.rank;
         const uint32_t per_share = (uint32_t)round_up(ceil_div(cache.cap, shares), kKeyTile);
-        const dim3 agrid((unsigned)ceil_div(R, 128), dm.heads);
+        const dim3 agrid((unsigned)ceil_div(R, 128), dm.heads + 1);
         const size_t alds = (bp * (size_t)dm.d + 4 * bp * 128) * 4;
 #define COEUS_LA(BPV) \
-    case BPV: hipLaunchKernelGGL(latent_absorb_kernel<BPV>, agrid, dim3(256), alds, st, q, w, dm, (uint32_t)batch, qa); break
+    case BPV: hipLaunchKernelGGL(latent_absorb_kernel<BPV>, agrid, dim3(256), alds, st, q, w, dm, (uint32_t)batch, qa, nw, cc, cache.cap, \
+                                 pos_dev); break
         switch (bp) { COEUS_LA(1); COEUS_LA(2); COEUS_LA(4); COEUS_LA(8); COEUS_LA(16); }
 #undef COEUS_LA
-        static const bool once = hipFuncSetAttribute((const void *)latent_scores_kernel,
-                                                     hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) == hipSuccess;
-        (void)once;
         const size_t slds = ((size_t)R * (kKeyTile + 8) + 2 * 16 * (kKeyTile + 8)) * 2 + (16 * (kKeyTile + 8) + 48) * 4;
-        hipLaunchKernelGGL(latent_scores_kernel, dim3(shares, (unsigned)ceil_div(dm.heads, 16), (unsigned)batch), dim3(256),
-                           slds, st, qa, dm, cc, cache.cap, pos_dev, per_share, part);
+        const dim3 sgrid(shares, (unsigned)ceil_div(dm.heads, 16), (unsigned)batch);
+#define COEUS_LS(PTV)                                                                                               \
+    do {                                                                                                            \
+        static const bool once = hipFuncSetAttribute((const void *)latent_scores_kernel<PTV>,                       \
+                                                     hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) == hipSuccess; \
+        (void)once;                                                                                                 \
+        hipLaunchKernelGGL(latent_scores_kernel<PTV>, sgrid, dim3(256), slds, st, qa, dm, cc, cache.cap, pos_dev, per_share, part); \
+    } while (0)
+        if (R <= 256) COEUS_LS(4);
+        else if (R <= 512) COEUS_LS(8);
+        else COEUS_LS(16);
+#undef COEUS_LS
         const dim3 egrid((unsigned)ceil_div(dm.e, 32), dm.heads, (unsigned)batch);
         if (R <= 512) hipLaunchKernelGGL(latent_expand_kernel<1>, egrid, dim3(256), (size_t)R * 4, st, part, w, dm, shares, out);
         else hipLaunchKernelGGL(latent_expand_kernel<2>, egrid, dim3(256), (size_t)R * 4, st, part, w, dm, shares, out);
         COEUS_HIP(hipGetLastError());
         return COEUS_OK;
     }
+    COEUS_TRY(launch_latent_norm(nw.proj, dm, nullptr, nw.scale, nw.eps, batch, 1, nullptr, nullptr, nullptr, 0, 0, 0, cache, pos_dev, st));
     const dim3 grid(dm.heads, (unsigned)batch);
     const size_t lds = 5 * (size_t)dm.rank * 4;
     if (cache.bf16)

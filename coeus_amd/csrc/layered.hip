@@ -580,9 +580,8 @@ int layered_decode(Session &s, hipStream_t st, int only, uint64_t *launches, uin
             const LatentDims dm = ly.latent_dims();
             float *cq = (float *)s.dmix.p, *q = cq + B * mx.q_rank;
             const bool fold = s.fuse && gemv_can_fuse_norm_dense(ly.uq, B);
-            if (rest)
-                COEUS_TRY(launch_latent_norm(proj, dm, ly.dq_norm, ly.dkv_norm, eps, B, 1, fold ? nullptr : cq, nullptr, nullptr,
-                                             0, 0, 0, sl.latent, pos, st));
+            if (rest && !fold)
+                COEUS_TRY(launch_latent_norm(proj, dm, ly.dq_norm, ly.dkv_norm, eps, B, 1, cq, nullptr, nullptr, 0, 0, 0, sl.latent, pos, st));
             if (fold && matmuls) {  // the query latent's norm rides on its expansion
                 Epilogue e;
                 e.out_f32 = q;
@@ -594,7 +593,8 @@ int layered_decode(Session &s, hipStream_t st, int only, uint64_t *launches, uin
                 COEUS_TRY(gemv(ly.uq, cq, q));
             }
             if (mixers) {
-                COEUS_TRY(launch_latent_decode(q, ly.ukv.data, dm, sl.latent, B, pos, att, (float *)s.dscratch.p, s.dscratch.bytes, st));
+                COEUS_TRY(launch_latent_decode(q, ly.ukv.data, dm, LatentNew{proj, ly.dkv_norm, eps}, sl.latent, B, pos, att,
+                                               (float *)s.dscratch.p, s.dscratch.bytes, st));
                 if (only == STEP_ATTENTION) {
                     const uint64_t nv = std::min<uint64_t>((uint64_t)s.host_pos[0] + 1, sl.latent.cap);
                     n_launch++;

@@ -85,11 +85,17 @@ int launch_latent_append(const void *lat, uint64_t lat_ld, uint64_t lat_rows, ui
 int launch_window_attention(const void *q, uint64_t q_ld, const void *kv, uint64_t kv_ld, bool bf16,
                             const LatentDims &dm, uint64_t batch, uint64_t n, uint64_t hist, float *out,
                             const LpOut *out_lp, hipStream_t st);
-// One new token per sequence against the cached latents (its own included): q [batch, heads * d] f32,
-// ukv [heads * d keys | heads * e values][rank] in the cache's type, out [batch, heads * e] f32.
-int launch_latent_decode(const float *q, const void *ukv, const LatentDims &dm, const LatentCache &cache,
-                         uint64_t batch, const uint32_t *pos_dev, float *out, float *scratch, uint64_t scratch_bytes,
-                         hipStream_t st);
+// One new token per sequence: its latent, normalised, goes into the ring, and its query is scored against
+// the cached latents (its own included).  q [batch, heads * d] f32, ukv [heads * d keys | heads * e
+// values][rank] in the cache's type, out [batch, heads * e] f32.
+struct LatentNew {
+    const float *proj;   // fused projection of the new tokens
+    const float *scale;  // [rank]
+    float eps;
+};
+int launch_latent_decode(const float *q, const void *ukv, const LatentDims &dm, const LatentNew &nw,
+                         const LatentCache &cache, uint64_t batch, const uint32_t *pos_dev, float *out, float *scratch,
+                         uint64_t scratch_bytes, hipStream_t st);
 uint64_t latent_decode_scratch_bytes(const LatentDims &dm, const LatentCache &cache, uint64_t batch);
 
 }  // namespace coeus

@@ -387,6 +387,53 @@ int coeus_op_attention_decode_static(const float *qkv_dev, const void *k_cache_d
                                      uint32_t kv_dtype, uint64_t batch, uint64_t num_heads,
                                      uint64_t head_dim, uint64_t max_ctx, uint64_t ctx, uint32_t nsplit,
                                      uint32_t merge, float *out_dev, void *stream);
+/* ---- mechanisms of the layered models (no counterpart in the reference); like the operators above, but
+ * each call allocates its scratch and synchronises `stream` before it returns ---------------------- */
+/* h[r, :] += y[r, :] / rms(y[r, :]) * scale (* ls, nullable): the norm behind a sublayer, in place. */
+int coeus_op_norm_residual(const float *y_dev, uint64_t rows, uint64_t hidden, const float *scale_dev,
+                           const float *ls_dev, float eps, float *h_dev, void *stream);
+/* The gated delta rule.  proj_dev rows of in_ld floats hold q | k (kv_heads x dim each) | v | gate
+ * (heads x vdim each) | step size | decay (heads each) as the projections give them.  conv_dev
+ * [conv][channels] over the q, k, v channels, exp_a_dev / dt_bias_dev [heads], norm_dev [vdim].
+ * state_dev [batch][heads][dim][vdim] and ring_dev [batch][conv][channels] (position p in slot
+ * p % conv) are read and moved on; zeros start a sequence.  out_dev [batch * n, heads * vdim]. */
+typedef struct coeus_delta_shape {
+    uint64_t heads, kv_heads, dim, vdim, conv, in_ld;
+} coeus_delta_shape;
+typedef struct coeus_delta_weights {
+    const float *conv_dev, *exp_a_dev, *dt_bias_dev, *norm_dev;
+    float eps;
+} coeus_delta_weights;
+/* n new tokens per sequence at positions pos0 ..: in chunks on the matrix cores when `chunked` is not
+ * zero and n is large enough for it, else token by token. */
+int coeus_op_delta_prompt(const coeus_delta_shape *shape, const coeus_delta_weights *w, const float *proj_dev,
+                          float *state_dev, float *ring_dev, uint64_t batch, uint64_t n, uint64_t pos0,
+                          int chunked, float *out_dev, void *stream);
+/* One new token per sequence at position pos (a decode step's launch). */
+int coeus_op_delta_step(const coeus_delta_shape *shape, const coeus_delta_weights *w, const float *proj_dev,
+                        float *state_dev, float *ring_dev, uint64_t batch, uint64_t pos, float *out_dev,
+                        void *stream);
+/* Latent attention.  Types of the tensors marked "kv": COEUS_KV_BF16 or COEUS_KV_F32.  window 0: every
+ * earlier position; else position i sees the `window` positions that end at i. */
+typedef struct coeus_latent_shape {
+    uint64_t heads, dim, vdim, q_rank, kv_rank, window;
+    float scale;
+} coeus_latent_shape;
+/* A prompt's attention on expanded keys and values: q_dev (kv) [batch * n, heads * dim], kv_dev (kv)
+ * [batch * (hist + n), heads * dim keys | heads * vdim values], the last n rows of a sequence being the
+ * queries' own.  out_dev f32 [batch * n, heads * vdim]. */
+int coeus_op_window_attention(const coeus_latent_shape *shape, uint32_t kv_dtype, const void *q_dev,
+                              const void *kv_dev, uint64_t batch, uint64_t n, uint64_t hist, float *out_dev,
+                              void *stream);
+/* A decode step's attention: proj_dev rows [q_rank | kv_rank] (padded to a multiple of 4) of the new
+ * tokens, whose normalised latent (scale_dev [kv_rank], eps) goes into the ring cache_dev (kv)
+ * [batch][cap][kv_rank] at slot pos % cap (cap <= window if there is one); q_dev f32
+ * [batch, heads * dim]; ukv_dev (kv) [heads * dim | heads * vdim][kv_rank]; out_dev f32
+ * [batch, heads * vdim]. */
+int coeus_op_latent_decode(const coeus_latent_shape *shape, uint32_t kv_dtype, const float *q_dev,
+                           const float *proj_dev, const float *scale_dev, float eps, const void *ukv_dev,
+                           void *cache_dev, uint64_t cap, uint64_t batch, uint64_t pos, float *out_dev,
+                           void *stream);
 /* Host-side sinusoidal table (MT:398-407), computed with the platform libm like the reference. */
 int coeus_positional_encoding(uint64_t max_seq_len, uint64_t hidden_dim, float *table_out);
 

@@ -1,5 +1,5 @@
 """The host logic of the library (errors, configuration and parameter layout, the .rustllm reader and
-writer with their error cases, the byte-pair tokenizer) built with AddressSanitizer and
+writer with their error cases, layered configurations and weight files, the byte-pair tokenizer) built with AddressSanitizer and
 UndefinedBehaviorSanitizer on the host pass and run through its own tests in a child process.
 Device code is not sanitized and not part of this build."""
 import os
@@ -23,7 +23,7 @@ def test_host_sources_clean_under_asan_and_ubsan():
                ASAN_OPTIONS="detect_leaks=0:verify_asan_link_order=0:abort_on_error=0:exitcode=99",
                UBSAN_OPTIONS="print_stacktrace=1:halt_on_error=1:exitcode=98")
     r = subprocess.run([sys.executable, "-m", "pytest", "-q", "-x", "-m", "not gpu", "-p", "no:cacheprovider",
-                        "tests/test_rustllm_file.py", "tests/test_tokenizer.py",
+                        "tests/test_rustllm_file.py", "tests/test_tokenizer.py", "tests/test_layered_host.py",
                         "tests/test_host_cpu.py::test_config_defaults_validate_and_counts",
                         "tests/test_host_cpu.py::test_default_init_and_positional_table_match_oracle_bitwise",
                         "tests/test_abi_layout.py::test_last_error_is_thread_local"],
