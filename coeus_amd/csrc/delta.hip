@@ -387,15 +387,18 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaDims dm, DeltaOpe
         }
 }
 
-// One workgroup of four waves per (16 columns of S, head, sequence).  Wave w keeps rows 16 QW w .. of the
-// state in accumulators, computes tokens 16 w .. of U and O, and hands both to the others through LDS.
+// One workgroup of eight waves per (16 columns of S, head, sequence).  Waves 0-3 carry the state: wave w keeps
+// rows 16 QW w .. of it in accumulators, computes tokens 16 w .. of U, and hands both to the others through
+// LDS.  Waves 4-7, one on each SIMD beside them, compute the outputs, which nobody waits for: they fill the
+// matrix cores while the state's waves exchange their pieces.
 template <int QW>
-__global__ __launch_bounds__(256) void delta_carry_kernel(DeltaDims dm, uint64_t n, uint64_t t0, uint64_t seg,
-                                                          ChunkBuf cb, float *state,
-                                                          float *__restrict__ o, uint32_t blocks, uint32_t units) {
+__global__ __launch_bounds__(512) void delta_carry_kernel(DeltaDims dm, uint64_t n, uint64_t t0, uint64_t seg,
+                                                          ChunkBuf cb, float *state, float *__restrict__ o,
+                                                          uint32_t blocks, uint32_t units) {
     constexpr uint32_t NT = 4 * QW, DQ = 16 * NT;
     __shared__ float4_t sl[2][NT][64], ul[2][4][64];
-    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
+    const uint32_t lane = threadIdx.x & 63, wave = (threadIdx.x >> 6) & 3, c = lane & 15, g = lane >> 4;
+    const bool carries = threadIdx.x < 256;
     const uint32_t H = dm.heads, KH = dm.kv_heads;
     // all column blocks of a head on one XCD (consecutive workgroups go round the 8 XCDs): its chunk
     // operands are fetched into one L2
@@ -408,98 +411,116 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(DeltaDims dm, uint64_t
     const uint32_t h = unit % H, hk = h / (H / KH);
     const uint64_t b = unit / H;
     const uint32_t col = blk * 16 + c, colc = min(col, dm.e - 1);
-    float *sp = state + ((b * H + h) * (uint64_t)dm.d) * dm.e + colc;
-    float4_t s[QW];
-#pragma unroll
-    for (int t = 0; t < QW; t++)
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const uint32_t r = 16 * (QW * wave + t) + 4 * g + i;
-            s[t][i] = r < dm.d ? sp[(uint64_t)r * dm.e] : 0.f;
-        }
-    float4 wa[NT], qa[NT], pa[4], ka[QW][4];
-    float4 eg4, ed4[4];
-    float4_t v4;
-    float egc;
-    // A chunk's operands are requested as soon as the registers of the chunk before are free: W, Q and V' while
-    // P U and the state are computed, P, K^T and the decays behind them.
-    auto fetch_wq = [&](uint32_t ch) {
-        const uint64_t ci = (b * H + h) * cb.chunks + ch, ki = (b * KH + hk) * cb.chunks + ch;
-        const float4 *wp = (const float4 *)(cb.w + ci * kChunk * DQ) + wave * NT * 64 + lane;
-        const float4 *qp = (const float4 *)(cb.q + ki * kChunk * DQ) + wave * NT * 64 + lane;
-#pragma unroll
-        for (uint32_t m = 0; m < NT; m++) { wa[m] = wp[64 * m]; qa[m] = qp[64 * m]; }
-        v4 = *(const float4_t *)(cb.vp + ci * kChunk * 16 * blocks + ((wave * blocks + blk) * 64 + lane) * 4);
-    };
-    auto fetch_pk = [&](uint32_t ch) {
-        const uint64_t ci = (b * H + h) * cb.chunks + ch, ki = (b * KH + hk) * cb.chunks + ch;
-        const float4 *pp = (const float4 *)(cb.p + ci * kChunk * kChunk) + wave * 4 * 64 + lane;
-        const float4 *kp = (const float4 *)(cb.kt + ki * kChunk * DQ) + QW * wave * 4 * 64 + lane;
-#pragma unroll
-        for (int t = 0; t < 4; t++) {
-            pa[t] = pp[64 * t];
-#pragma unroll
-            for (int u = 0; u < QW; u++) ka[u][t] = kp[(4 * u + t) * 64];
-            ed4[t] = *(const float4 *)(cb.ed + ci * kChunk + 16 * t + 4 * g);
-        }
-        eg4 = *(const float4 *)(cb.eg + ci * kChunk + 16 * wave + 4 * g);
-        egc = cb.eg[ci * kChunk + kChunk - 1];
-    };
     const uint32_t chunks = (uint32_t)((seg + kChunk - 1) / kChunk);
-    fetch_wq(0);
-    fetch_pk(0);
-    for (uint32_t ch = 0; ch < chunks; ch++) {
-        const uint32_t buf = ch & 1, next = ch + 1 < chunks ? ch + 1 : ch;
-#pragma unroll
-        for (int t = 0; t < QW; t++) sl[buf][QW * wave + t][lane] = s[t];
-        lds_barrier();
-        float4_t au = {0.f, 0.f, 0.f, 0.f}, ao = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (uint32_t m = 0; m < NT; m++) {
-            const float4_t sb = sl[buf][m][lane];
-            au = mfma4(wa[m], sb, au);
-            ao = mfma4(qa[m], sb, ao);
-        }
-        float4_t u;
-#pragma unroll
-        for (int i = 0; i < 4; i++) u[i] = v4[i] - au[i];
-        ul[buf][wave][lane] = u;
-        __builtin_amdgcn_sched_barrier(0);
-        fetch_wq(next);
-        __builtin_amdgcn_sched_barrier(0);
-        ao[0] *= eg4.x; ao[1] *= eg4.y; ao[2] *= eg4.z; ao[3] *= eg4.w;
-        lds_barrier();
-        float4_t ub[4];
-#pragma unroll
-        for (int t = 0; t < 4; t++) ub[t] = ul[buf][t][lane];
-#pragma unroll
-        for (int t = 0; t < 4; t++)
-            if (t <= (int)wave) ao = mfma4(pa[t], ub[t], ao);
-#pragma unroll
-        for (int t = 0; t < 4; t++) { ub[t][0] *= ed4[t].x; ub[t][1] *= ed4[t].y; ub[t][2] *= ed4[t].z; ub[t][3] *= ed4[t].w; }
-#pragma unroll
-        for (int w = 0; w < QW; w++) s[w] *= egc;
-#pragma unroll
-        for (int t = 0; t < 4; t++)
-#pragma unroll
-            for (int w = 0; w < QW; w++) s[w] = mfma4(ka[w][t], ub[t], s[w]);
-        __builtin_amdgcn_sched_barrier(0);
-        fetch_pk(next);
-        __builtin_amdgcn_sched_barrier(0);
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const uint64_t r = (uint64_t)ch * kChunk + 16 * wave + 4 * g + i;
-            if (r < seg && col < dm.e) o[((b * n + t0 + r) * H + h) * dm.e + col] = ao[i];
-        }
-    }
-    if (col < dm.e)
+    const uint64_t ci0 = (b * H + h) * cb.chunks, ki0 = (b * KH + hk) * cb.chunks;
+    // A chunk's operands are requested as soon as the registers of the chunk before are free.
+    if (carries) {
+        __builtin_amdgcn_s_setprio(2);  // the next chunk waits for these waves
+        float *sp = state + ((b * H + h) * (uint64_t)dm.d) * dm.e + colc;
+        float4_t s[QW];
 #pragma unroll
         for (int t = 0; t < QW; t++)
 #pragma unroll
             for (int i = 0; i < 4; i++) {
                 const uint32_t r = 16 * (QW * wave + t) + 4 * g + i;
-                if (r < dm.d) sp[(uint64_t)r * dm.e] = s[t][i];
+                s[t][i] = r < dm.d ? sp[(uint64_t)r * dm.e] : 0.f;
             }
+        float4 wa[NT], ka[QW][4], ed4[4];
+        float4_t v4;
+        float egc;
+        auto fetch_w = [&](uint32_t ch) {
+            const float4 *wp = (const float4 *)(cb.w + (ci0 + ch) * kChunk * DQ) + wave * NT * 64 + lane;
+#pragma unroll
+            for (uint32_t m = 0; m < NT; m++) wa[m] = wp[64 * m];
+            v4 = *(const float4_t *)(cb.vp + (ci0 + ch) * kChunk * 16 * blocks + ((wave * blocks + blk) * 64 + lane) * 4);
+        };
+        auto fetch_k = [&](uint32_t ch) {
+            const float4 *kp = (const float4 *)(cb.kt + (ki0 + ch) * kChunk * DQ) + QW * wave * 4 * 64 + lane;
+#pragma unroll
+            for (int t = 0; t < 4; t++) {
+#pragma unroll
+                for (int u = 0; u < QW; u++) ka[u][t] = kp[(4 * u + t) * 64];
+                ed4[t] = *(const float4 *)(cb.ed + (ci0 + ch) * kChunk + 16 * t + 4 * g);
+            }
+            egc = cb.eg[(ci0 + ch) * kChunk + kChunk - 1];
+        };
+        fetch_w(0);
+        fetch_k(0);
+        for (uint32_t ch = 0; ch < chunks; ch++) {
+            const uint32_t buf = ch & 1, next = ch + 1 < chunks ? ch + 1 : ch;
+#pragma unroll
+            for (int t = 0; t < QW; t++) sl[buf][QW * wave + t][lane] = s[t];
+            lds_barrier();
+            float4_t a0 = {0.f, 0.f, 0.f, 0.f}, a1 = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (uint32_t m = 0; m < NT; m += 2) {
+                a0 = mfma4(wa[m], sl[buf][m][lane], a0);
+                a1 = mfma4(wa[m + 1], sl[buf][m + 1][lane], a1);
+            }
+            ul[buf][wave][lane] = v4 - (a0 + a1);
+            __builtin_amdgcn_sched_barrier(0);
+            fetch_w(next);
+            __builtin_amdgcn_sched_barrier(0);
+            lds_barrier();
+#pragma unroll
+            for (int w = 0; w < QW; w++) s[w] *= egc;
+#pragma unroll
+            for (int t = 0; t < 4; t++) {
+                float4_t ub = ul[buf][t][lane];
+                ub[0] *= ed4[t].x; ub[1] *= ed4[t].y; ub[2] *= ed4[t].z; ub[3] *= ed4[t].w;
+#pragma unroll
+                for (int w = 0; w < QW; w++) s[w] = mfma4(ka[w][t], ub, s[w]);
+            }
+            __builtin_amdgcn_sched_barrier(0);
+            fetch_k(next);
+            __builtin_amdgcn_sched_barrier(0);
+        }
+        if (col < dm.e)
+#pragma unroll
+            for (int t = 0; t < QW; t++)
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const uint32_t r = 16 * (QW * wave + t) + 4 * g + i;
+                    if (r < dm.d) sp[(uint64_t)r * dm.e] = s[t][i];
+                }
+    } else {
+        constexpr uint32_t SPLIT = (3 * NT / 4) & ~1u;  // (even and below NT: every wave meets two barriers a chunk)
+        float4 qa[NT], pa[4], eg4;
+        auto fetch = [&](uint32_t ch) {
+            const float4 *qp = (const float4 *)(cb.q + (ki0 + ch) * kChunk * DQ) + wave * NT * 64 + lane;
+            const float4 *pp = (const float4 *)(cb.p + (ci0 + ch) * kChunk * kChunk) + wave * 4 * 64 + lane;
+#pragma unroll
+            for (uint32_t m = 0; m < NT; m++) qa[m] = qp[64 * m];
+#pragma unroll
+            for (int t = 0; t < 4; t++) pa[t] = pp[64 * t];
+            eg4 = *(const float4 *)(cb.eg + (ci0 + ch) * kChunk + 16 * wave + 4 * g);
+        };
+        fetch(0);
+        for (uint32_t ch = 0; ch < chunks; ch++) {
+            const uint32_t buf = ch & 1;
+            lds_barrier();  // S is there; it stays until the state's waves have passed this chunk's successor
+            float4_t a0 = {0.f, 0.f, 0.f, 0.f}, a1 = {0.f, 0.f, 0.f, 0.f}, ap = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (uint32_t m = 0; m < NT; m += 2) {
+                if (m == SPLIT) lds_barrier();  // U is there
+                a0 = mfma4(qa[m], sl[buf][m][lane], a0);
+                a1 = mfma4(qa[m + 1], sl[buf][m + 1][lane], a1);
+            }
+#pragma unroll
+            for (int t = 0; t < 4; t++)
+                if (t <= (int)wave) ap = mfma4(pa[t], ul[buf][t][lane], ap);
+            a0 += a1;
+            const float r[4] = {fmaf(eg4.x, a0[0], ap[0]), fmaf(eg4.y, a0[1], ap[1]), fmaf(eg4.z, a0[2], ap[2]), fmaf(eg4.w, a0[3], ap[3])};
+            __builtin_amdgcn_sched_barrier(0);
+            fetch(ch + 1 < chunks ? ch + 1 : ch);
+            __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const uint64_t row = (uint64_t)ch * kChunk + 16 * wave + 4 * g + i;
+                if (row < seg && col < dm.e) o[((b * n + t0 + row) * H + h) * dm.e + col] = r[i];
+            }
+        }
+    }
 }
 
 // A few dozen tokens are quicker one by one than through two launches of chunks.
@@ -538,7 +559,7 @@ static int launch_chunks(const DeltaDims &dm, const DeltaOperands &op, const Del
         hipLaunchKernelGGL((delta_chunk_kernel<4 * QW>), dim3(cb.chunks, dm.heads, (unsigned)batch), dim3(256), lds, st, dm,
                            op, dp, n, t0, seg, cb);
         const uint32_t blocks = (uint32_t)ceil_div(dm.e, 16), units = (uint32_t)(dm.heads * batch);
-        hipLaunchKernelGGL((delta_carry_kernel<QW>), dim3(blocks * units), dim3(256), 0, st, dm, n, t0, seg, cb,
+        hipLaunchKernelGGL((delta_carry_kernel<QW>), dim3(blocks * units), dim3(512), 0, st, dm, n, t0, seg, cb,
                            state.s, o, blocks, units);
     }
     COEUS_HIP(hipGetLastError());

@@ -34,7 +34,7 @@ static int check_dims(const LatentDims &dm, const LatentCache &cache) {
     return COEUS_OK;
 }
 
-// RMS norm of one row by a workgroup of 256: put(i, value) for every element.
+// RMS norm of one row by a workgroup of 256 (a decode step's few rows): put(i, value) for every element.
 template <typename Put>
 __device__ __forceinline__ void norm_row_256(const float *__restrict__ x, uint32_t len, float eps,
                                              const float *__restrict__ scale, float *sh, Put put) {
@@ -49,29 +49,41 @@ __device__ __forceinline__ void norm_row_256(const float *__restrict__ x, uint32
     for (uint32_t i = tid; i < len; i += 256) put(i, x[i] * rs * scale[i]);
 }
 
-// blockIdx.y + part0 0: the query latent, 1: the key/value latent.
+// One wave per (row, latent); part 0: the query latent, 1: the key/value latent, of 2 - part0 a row.  Up to
+// 1024 elements stay in registers between the sum and the store.
 template <bool BF16>
 __global__ __launch_bounds__(256) void latent_norm_kernel(const float *__restrict__ proj, LatentDims dm,
                                                           const float *__restrict__ q_scale,
-                                                          const float *__restrict__ c_scale, float eps, uint64_t n,
-                                                          float *cq, uint16_t *cq_lp, uint64_t cq_ld, bool lp_bf16,
+                                                          const float *__restrict__ c_scale, float eps, uint64_t rows,
+                                                          uint64_t n, float *cq, uint16_t *cq_lp, uint64_t cq_ld, bool lp_bf16,
                                                           void *lat, uint64_t lat_ld, uint64_t lat_rows,
                                                           uint64_t lat_off, uint32_t cap, const uint32_t *pos_dev,
                                                           uint32_t part0) {
-    __shared__ float sh[4];
-    const uint64_t row = blockIdx.x;
-    const bool is_q = blockIdx.y + part0 == 0;
-    const float *x = proj + row * dm.in_ld + (is_q ? 0 : dm.q_rank);
-    if (is_q) {
-        norm_row_256(x, dm.q_rank, eps, q_scale, sh, [&](uint32_t i, float v) {
-            if (cq) cq[row * dm.q_rank + i] = v;
-            if (cq_lp) cq_lp[row * cq_ld + i] = f32_to_lp_bits(v, lp_bf16);
-        });
-    } else {
-        const uint64_t dst = pos_dev ? (row * cap + *pos_dev % cap) * dm.rank
-                                     : ((row / n) * lat_rows + lat_off + row % n) * lat_ld;
-        norm_row_256(x, dm.rank, eps, c_scale, sh, [&](uint32_t i, float v) { lat_store<BF16>(lat, dst + i, v); });
+    const uint32_t lane = threadIdx.x & 63, parts = 2 - part0;
+    const uint64_t unit = (uint64_t)blockIdx.x * 4 + (threadIdx.x >> 6), row = unit / parts;
+    if (row >= rows) return;
+    const bool is_q = unit % parts + part0 == 0;
+    const uint32_t len = is_q ? dm.q_rank : dm.rank;
+    const float *x = proj + row * dm.in_ld + (is_q ? 0 : dm.q_rank), *scale = is_q ? q_scale : c_scale;
+    constexpr int U = 16;
+    float v[U], s2 = 0.f;
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+        v[u] = lane + 64 * u < len ? x[lane + 64 * u] : 0.f;
+        s2 = fmaf(v[u], v[u], s2);
     }
+    for (uint32_t i = lane + 64 * U; i < len; i += 64) s2 = fmaf(x[i], x[i], s2);
+    const float rs = 1.0f / sqrtf(wave_sum(s2) / (float)len + eps);
+    const uint64_t dst = pos_dev ? (row * cap + *pos_dev % cap) * dm.rank : ((row / n) * lat_rows + lat_off + row % n) * lat_ld;
+    auto put = [&](uint32_t i, float y) {
+        if (!is_q) lat_store<BF16>(lat, dst + i, y);
+        if (is_q && cq) cq[row * dm.q_rank + i] = y;
+        if (is_q && cq_lp) cq_lp[row * cq_ld + i] = f32_to_lp_bits(y, lp_bf16);
+    };
+#pragma unroll
+    for (int u = 0; u < U; u++)
+        if (lane + 64 * u < len) put(lane + 64 * u, v[u] * rs * scale[lane + 64 * u]);
+    for (uint32_t i = lane + 64 * U; i < len; i += 64) put(i, x[i] * rs * scale[i]);
 }
 
 int launch_latent_norm(const float *proj, const LatentDims &dm, const float *q_scale, const float *c_scale, float eps,
@@ -82,16 +94,17 @@ int launch_latent_norm(const float *proj, const LatentDims &dm, const float *q_s
     if (batch == 0 || n == 0 || batch * n > 0x7fffffffull || (pos_dev && n != 1))
         return fail(COEUS_INVALID_INPUT, "latent attention: rows out of range");
     const uint32_t part0 = cq || cq_lp ? 0 : 1;  // no place for the query latent: its consumer normalises it
-    const dim3 grid((unsigned)(batch * n), 2 - part0);
+    const uint64_t rows = batch * n;
+    const dim3 grid((unsigned)ceil_div(rows * (2 - part0), 4));
     uint16_t *lp = cq_lp ? (uint16_t *)cq_lp->p : nullptr;
     const uint64_t ld = cq_lp ? cq_lp->ld : 0;
     const bool lp_bf = cq_lp && cq_lp->bf16;
     void *dst = pos_dev ? cache.c : lat;
     if (cache.bf16)
-        hipLaunchKernelGGL(latent_norm_kernel<true>, grid, dim3(256), 0, st, proj, dm, q_scale, c_scale, eps, n, cq, lp, ld,
+        hipLaunchKernelGGL(latent_norm_kernel<true>, grid, dim3(256), 0, st, proj, dm, q_scale, c_scale, eps, rows, n, cq, lp, ld,
                            lp_bf, dst, lat_ld, lat_rows, lat_off, cache.cap, pos_dev, part0);
     else
-        hipLaunchKernelGGL(latent_norm_kernel<false>, grid, dim3(256), 0, st, proj, dm, q_scale, c_scale, eps, n, cq, lp, ld,
+        hipLaunchKernelGGL(latent_norm_kernel<false>, grid, dim3(256), 0, st, proj, dm, q_scale, c_scale, eps, rows, n, cq, lp, ld,
                            lp_bf, dst, lat_ld, lat_rows, lat_off, cache.cap, pos_dev, part0);
     COEUS_HIP(hipGetLastError());
     return COEUS_OK;
