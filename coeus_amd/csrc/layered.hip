@@ -6,7 +6,6 @@
 #include "model.hpp"
 
 #include <cmath>
-#include <functional>
 
 namespace coeus {
 

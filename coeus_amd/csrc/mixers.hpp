@@ -20,7 +20,7 @@ struct DeltaDims {
     __host__ __device__ uint32_t decay_off() const { return beta_off() + heads; }
 };
 struct DeltaParams {
-    const float *conv;     // [taps][channels], the last tap is the current token's
+    const float *conv;     // [taps][channels], tap taps - 1 meets the newest input
     const float *exp_a;    // [heads] exp(A_log)
     const float *dt_bias;  // [heads]
     const float *norm;     // [e]

@@ -280,7 +280,9 @@ int coeus_session_time_decode_matmuls(coeus_session *s, uint64_t reps, float *ms
                                       uint64_t *launches_out, uint64_t *bytes_out);
 /* The same for the attention launches of one step (one per layer) over the positions cached so
  * far: *bytes_out = keys and values of every cached position of every (sequence, head) plus the
- * query and output rows.  The kernel that dominates a step at batch 16. */
+ * query and output rows.  The kernel that dominates a step at batch 16.  On a layered model: the mixers'
+ * launches behind the projections, with the bytes of their states, rings, cached latents and expansion
+ * weights; recurrent states move on, so reset the session afterwards. */
 int coeus_session_time_decode_attention(coeus_session *s, uint64_t reps, float *ms_out,
                                         uint64_t *launches_out, uint64_t *bytes_out);
 uint64_t coeus_session_position(const coeus_session *s);
