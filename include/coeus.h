@@ -429,7 +429,8 @@ int coeus_op_window_attention(const coeus_latent_shape *shape, uint32_t kv_dtype
                               void *stream);
 /* A decode step's attention: proj_dev rows [q_rank | kv_rank] (padded to a multiple of 4) of the new
  * tokens, whose normalised latent (scale_dev [kv_rank], eps) goes into the ring cache_dev (kv)
- * [batch][cap][kv_rank] at slot pos % cap (cap <= window if there is one); q_dev f32
+ * [batch][cap][kv_rank] at slot pos % cap (cap <= window if there is one; slots not written yet must
+ * hold finite values); q_dev f32
  * [batch, heads * dim]; ukv_dev (kv) [heads * dim | heads * vdim][kv_rank]; out_dev f32
  * [batch, heads * vdim]. */
 int coeus_op_latent_decode(const coeus_latent_shape *shape, uint32_t kv_dtype, const float *q_dev,
