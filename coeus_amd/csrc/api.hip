@@ -811,7 +811,7 @@ int coeus_op_window_attention(const coeus_latent_shape *shape, uint32_t kv_dtype
     if (!q_dev || !kv_dev || !out_dev) return fail(COEUS_INVALID_INPUT, "null pointer argument");
     hipStream_t st = (hipStream_t)stream;
     const uint64_t q_ld = (uint64_t)dm.heads * dm.d, kv_ld = q_ld + (uint64_t)dm.heads * dm.e;
-    return finish_op(launch_window_attention(q_dev, q_ld, kv_dev, kv_ld, kv_dtype == COEUS_KV_BF16, dm, batch, n, hist, out_dev,
+    return finish_op(launch_window_attention(q_dev, q_ld, kv_dev, kv_ld, kv_dtype == COEUS_KV_BF16, dm.window_shape(), batch, n, hist, out_dev,
                                              nullptr, st), st, {}, "window attention");
     COEUS_GUARD_END
 }
@@ -825,7 +825,7 @@ int coeus_op_latent_decode(const coeus_latent_shape *shape, uint32_t kv_dtype, c
     if (!q_dev || !proj_dev || !scale_dev || !ukv_dev || !cache_dev || !out_dev) return fail(COEUS_INVALID_INPUT, "null pointer argument");
     if (cap == 0 || cap > 0x7fffffffull) return fail(COEUS_INVALID_INPUT, "latent attention: cache size out of range");
     hipStream_t st = (hipStream_t)stream;
-    const LatentCache cache{cache_dev, (uint32_t)cap, kv_dtype == COEUS_KV_BF16};
+    const RowRing cache{cache_dev, (uint32_t)cap, kv_dtype == COEUS_KV_BF16};
     DeviceBuf p, scratch;
     int rc = upload_position(pos, p, st);
     const uint64_t sb = latent_decode_scratch_bytes(dm, cache, batch);

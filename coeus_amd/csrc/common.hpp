@@ -149,10 +149,14 @@ struct LpOut {
     bool bf16 = false;
 };
 
+// Pairs of weight rows (gate, up) that become one output.
+static constexpr bool epi_gated(uint32_t act) { return act == COEUS_EPI_SILU_GATE || act == COEUS_EPI_CLAMP_GATE; }
+
 struct Epilogue {
     const float *bias = nullptr;     // [n]
     const float *residual = nullptr; // [rows, n_eff]
     uint32_t act = COEUS_EPI_NONE;   // COEUS_EPI_*
+    float limit = 0.f;               // COEUS_EPI_CLAMP_GATE, COEUS_EPI_SOFTCAP
     float *out_f32 = nullptr;        // [rows, n_eff] (nullable if out_xq set)
     __half *out_xq = nullptr;        // xq format with bp_out (decode chaining)
     uint32_t bp_out = 0;
@@ -177,7 +181,7 @@ struct Epilogue {
 struct NormFuse {
     const float *h = nullptr;      // [batch, k] f32 residual stream
     const float *scale = nullptr;  // [k]
-    const float *bias = nullptr;   // [k] (LayerNorm only)
+    const float *bias = nullptr;   // [k] (LayerNorm only; dense weights: nullable)
     float eps = 0.f;
     uint32_t kind = COEUS_NORM_LAYERNORM;
     // [batch][ceil(k/16)] {sum, M2} records of h written by its producer (Epilogue::stats_out or
@@ -195,6 +199,12 @@ struct NormFuse {
     // rows to h_out (not h: every workgroup reads h).
     const float *y = nullptr, *ls = nullptr;
     float *h_out = nullptr;
+    // Dense weights only, hyper-connections: h holds `streams` rows per sequence, y (nullable) the output of
+    // the sublayer before, whose mix [streams][streams], out [streams] and mult give the new streams (stored
+    // to h_out, not h); the matmul multiplies the layer norm of their sum weighted by in [streams].
+    const float *mix = nullptr, *out = nullptr, *in = nullptr;
+    float mult = 0.f;
+    uint32_t streams = 0;
 };
 // True when launch_gemv can take `nf` for this weight and batch (quantised weights whose whole
 // activation block fits in LDS).
@@ -204,6 +214,8 @@ bool gemv_can_fuse_norm(const Weight &w, uint64_t batch);
 bool gemv_can_fuse_norm_dense(const Weight &w, uint64_t batch);
 // ... and for the norm behind a sublayer (NormFuse::y): two rows per sequence have to fit.
 bool gemv_can_fuse_post_norm(const Weight &w, uint64_t batch);
+// ... and for hyper-connections (NormFuse::streams).
+bool gemv_can_fuse_hyper(const Weight &w, uint64_t batch, uint64_t streams);
 // The same normalisation as a launch of its own (batches too large for the folded form):
 // nf.h rows -> xq, row statistics merged from nf.stats.  Padding rows of xq are not written.
 int launch_norm_from_stats(const NormFuse &nf, uint64_t batch, uint64_t k, uint64_t k_pad, __half *xq,
@@ -263,14 +275,27 @@ size_t norm_sequence_scratch_bytes();
 // h += RMSNorm(y; scale, eps) * ls (nullable: 1) row by row; h_lp (nullable) receives 16-bit rows of the new h
 int launch_norm_residual(const float *y, uint64_t rows, uint64_t hidden, const float *scale, const float *ls,
                          float eps, float *h, hipStream_t st, const LpOut *h_lp = nullptr);
+// One step of hyper-connections on rows of `streams` streams x [rows][streams][hidden], in place, in front of
+// the next sublayer: x_t <- sum_s mix[s][t] x_s + mult out[t] y with the output y of the sublayer before (null:
+// the streams stay), then u = sum_t in[t] x_t (in null: their plain sum), and its layer norm with weight norm
+// (nullable: u itself) as f32 rows (u) and / or 16-bit rows (u_lp).
+constexpr uint32_t kMaxHyperStreams = 8;
+struct HyperStep {
+    uint32_t streams = 0;
+    const float *y = nullptr, *mix = nullptr, *out = nullptr;
+    float mult = 0.f;
+    const float *in = nullptr, *norm = nullptr;
+    float eps = 0.f;
+};
+int launch_hyper(float *x, uint64_t rows, uint64_t hidden, const HyperStep &h, float *u, const LpOut *u_lp, hipStream_t st);
 // dst[i, :] = src[rows_dev[i], :] for i < count (row numbers are checked by the caller)
 int launch_gather_rows(const float *src, const uint64_t *rows_dev, uint64_t count, uint64_t hidden, float *dst,
                        hipStream_t st);
-// pe nullable: no positional term
+// pe nullable: no positional term; the table's values times `scale`, `copies` rows of x per id
 int launch_embed(const void *table, bool table_bf16, const float *pe, const uint64_t *ids,
                  uint64_t rows, uint64_t rows_per_seq, uint64_t pos0, const uint32_t *pos_dev,
                  uint64_t hidden, float *x, float2 *stats, hipStream_t st, const float *g_scale = nullptr,
-                 float *g_out = nullptr);
+                 float *g_out = nullptr, float scale = 1.f, uint32_t copies = 1);
 // g[row][k] = h[row][k] * scale[k] (NormFuse::g for rows that no epilogue produced)
 int launch_prescale(const float *h, const float *scale, uint64_t rows, uint64_t k, float *g, hipStream_t st);
 // `advance` (nullable; rows == 1 only): {position, step} counters that the kernel increments

@@ -246,13 +246,6 @@ static uint64_t chunk_floats(const DeltaDims &dm, uint64_t batch, uint64_t chunk
     return batch * chunks * (dm.heads * (kChunk * (dq + round_up(dm.e, 16) + kChunk) + 2 * kChunk) + 2ull * dm.kv_heads * dq * kChunk);
 }
 
-__device__ __forceinline__ float4_t mfma4(const float4 &a, const float4_t &b, float4_t acc) {
-    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b[0], acc, 0, 0, 0);
-    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b[1], acc, 0, 0, 0);
-    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b[2], acc, 0, 0, 0);
-    return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b[3], acc, 0, 0, 0);
-}
-
 // One workgroup of 256 per (chunk, head, sequence).  dp: row length of the prepared q and k.
 template <int NT>  // 16-wide steps of the padded query/key size
 __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaDims dm, DeltaOperands op, uint32_t dp, uint64_t n,

@@ -85,6 +85,18 @@ __device__ __forceinline__ float wave_max(float v) {
     return fmaxf(__uint_as_float(r[0]), __uint_as_float(r[1]));
 }
 
+// f32 product of 16 x 16 tiles over 16 of k in four instructions.  A reduction index is only a label:
+// instruction i sums over {4 g + i : g = lane / 16}, so a lane's operand pieces are four consecutive k.
+__device__ __forceinline__ float4_t mfma4(const float4_t &a, const float4_t &b, float4_t acc) {
+    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[0], b[0], acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[1], b[1], acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[2], b[2], acc, 0, 0, 0);
+    return __builtin_amdgcn_mfma_f32_16x16x4f32(a[3], b[3], acc, 0, 0, 0);
+}
+__device__ __forceinline__ float4_t mfma4(const float4 &a, const float4_t &b, float4_t acc) {
+    return mfma4(float4_t{a.x, a.y, a.z, a.w}, b, acc);
+}
+
 // Which (query tile, head) a workgroup of a prefill grid (x = query tiles, y = heads) works on.
 // Causal work grows with the query tile: the last (longest) tiles are dispatched first, so that
 // the short ones fill in behind them instead of the long ones forming the tail.  The hardware
@@ -116,6 +128,22 @@ __device__ __forceinline__ uint16_t f32_to_bf16_bits(float x) {
     return (uint16_t)(u >> 16);
 }
 
+// Elements of a buffer whose type is a launch parameter: bf16 or f32.
+template <bool BF16>
+__device__ __forceinline__ float elem_load(const void *p, uint64_t i) {
+    return BF16 ? bf16_bits_to_f32(((const uint16_t *)p)[i]) : ((const float *)p)[i];
+}
+template <bool BF16>
+__device__ __forceinline__ void elem_store(void *p, uint64_t i, float v) {
+    if (BF16) ((uint16_t *)p)[i] = f32_to_bf16_bits(v);
+    else ((float *)p)[i] = v;
+}
+// a = hi + lo to 16 bits of mantissa
+__device__ __forceinline__ void split_bf16(float a, __bf16 &hi, __bf16 &lo) {
+    hi = (__bf16)a;
+    lo = (__bf16)(a - (float)hi);
+}
+
 // math::gelu (MT:94-99)
 __device__ __forceinline__ float gelu_tanh(float x) {
     const float c0 = 0.7978845608028654f, c1 = 0.044715f;
@@ -133,6 +161,17 @@ __device__ __forceinline__ float fast_gelu(float x) {
     return x * fast_sigmoid(2.0f * c0 * x * (1.0f + c1 * x * x));
 }
 
+// Clamped gate: g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit).
+__device__ __forceinline__ float clamped_gate(float gate, float up, float limit) {
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    return g * fast_sigmoid(1.702f * g) * (u + 1.0f);
+}
+// cap tanh(x / cap) = cap (1 - 2 / (1 + e^(2 x / cap))): a rounding of the cap's size in the worst case
+__device__ __forceinline__ float soft_cap(float x, float cap) {
+    const float t = __builtin_amdgcn_exp2f(2.8853900817779268f * (x / cap));
+    return fmaf(-2.0f * cap, __builtin_amdgcn_rcpf(1.0f + t), cap);
+}
+
 // Position of element (b, k) in the xq interchange format ([k_pad/8][bp][8] f16).
 __device__ __forceinline__ uint64_t xq_index(uint64_t k, uint32_t b, uint32_t bp) {
     return ((k >> 3) * bp + b) * 8 + (k & 7);
@@ -144,6 +183,7 @@ struct EpiArgs {
     float *out_f32;
     __half *out_xq;
     uint32_t act, bp_out;
+    float limit;
     uint64_t n;      // weight rows (outputs before gating)
     uint64_t n_eff;  // outputs written per activation row (n, or n/2 when gated)
     // fused q|k|v projection of a decode step: columns >= kv_inner go straight into the cache
@@ -211,6 +251,7 @@ __device__ __forceinline__ float epi_store(const EpiArgs &e, uint64_t row, uint6
         return v;
     }
     if (e.act == COEUS_EPI_GELU) v = gelu_tanh(v);
+    if (e.act == COEUS_EPI_SOFTCAP) v = soft_cap(v, e.limit);
     if (e.residual) v += preloaded ? res : e.residual[row * e.n_eff + j];
     if (e.out_f32) e.out_f32[row * e.n_eff + j] = v;
     if (e.out_xq) e.out_xq[xq_index(j, (uint32_t)row, e.bp_out)] = __float2half_rn(v);
@@ -221,7 +262,7 @@ __device__ __forceinline__ float epi_store(const EpiArgs &e, uint64_t row, uint6
 __device__ __forceinline__ void epi_store_gated(const EpiArgs &e, uint64_t row, uint64_t m, float g,
                                                 float u) {
     if (e.bias) { g += e.bias[2 * m]; u += e.bias[2 * m + 1]; }
-    float v = silu(g) * u;
+    float v = e.act == COEUS_EPI_CLAMP_GATE ? clamped_gate(g, u, e.limit) : silu(g) * u;
     if (e.residual) v += e.residual[row * e.n_eff + m];
     if (e.out_f32) e.out_f32[row * e.n_eff + m] = v;
     if (e.out_xq) e.out_xq[xq_index(m, (uint32_t)row, e.bp_out)] = __float2half_rn(v);
@@ -235,9 +276,10 @@ static inline EpiArgs make_epi(const Epilogue &ep, uint64_t n) {
     e.out_f32 = ep.out_f32;
     e.out_xq = ep.out_xq;
     e.act = ep.act;
+    e.limit = ep.limit;
     e.bp_out = ep.bp_out;
     e.n = n;
-    e.n_eff = ep.act == COEUS_EPI_SILU_GATE ? n / 2 : n;
+    e.n_eff = epi_gated(ep.act) ? n / 2 : n;
     e.kv_k = ep.kv_k;
     e.kv_v = ep.kv_v;
     e.kv_pos = ep.kv_pos;

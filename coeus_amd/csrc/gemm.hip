@@ -106,7 +106,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const float *__restrict__
     }
     // accumulator i of lane l: row 8*(i/4) + 4*(l/32) + i%4, column l%32
     const uint64_t col = n0 + wn + (lane & 31);
-    const bool gated = e.act == COEUS_EPI_SILU_GATE;
+    const bool gated = epi_gated(e.act);
 #pragma unroll
     for (int i = 0; i < 16; i++) {
         const uint64_t row = m0 + wm + 8 * (i >> 2) + 4 * (lane >> 5) + (i & 3);
@@ -191,7 +191,7 @@ __global__ __launch_bounds__(256) void gemm_f32_small_kernel(const float *__rest
     __syncthreads();
     // wave v finishes accumulator elements 4v..4v+3: rows 8v + 4 (l / 32) + 0..3, column l % 32
     const uint64_t col = n0 + (lane & 31);
-    const bool gated = e.act == COEUS_EPI_SILU_GATE;
+    const bool gated = epi_gated(e.act);
 #pragma unroll
     for (int q = 0; q < 4; q++) {
         const int i = 4 * wave + q;
@@ -242,7 +242,7 @@ static int launch_gemm_f32(const Weight &w, const float *a, uint64_t m, const Ep
         plain = make_epi(pe, w.n);
     }
     const EpiArgs &ke = splits > 1 ? plain : e;
-    const uint64_t groups = ceil_div(w.n, e.act == COEUS_EPI_SILU_GATE ? 8 : 4);
+    const uint64_t groups = ceil_div(w.n, epi_gated(e.act) ? 8 : 4);
     if (scr.ev_begin) COEUS_HIP(hipEventRecord(scr.ev_begin, st));
     for (uint32_t rep = 0; rep < (scr.repeat ? scr.repeat : 1); rep++) {
         if (small && (w.k & 3) == 0)
@@ -341,7 +341,7 @@ __global__ __launch_bounds__(256) void gemm_h_kernel(const uint16_t *__restrict_
                 }
         }
     }
-    const bool gated = e.act == COEUS_EPI_SILU_GATE;
+    const bool gated = epi_gated(e.act);
 #pragma unroll
     for (int x = 0; x < 2; x++)
 #pragma unroll
@@ -418,6 +418,9 @@ __device__ __forceinline__ void epi_row4(const EpiArgs &e, bool vec4, const KvCo
         if (e.act == COEUS_EPI_GELU)
 #pragma unroll
             for (int q = 0; q < 4; q++) v[q] = gelu_tanh(v[q]);
+        if (e.act == COEUS_EPI_SOFTCAP)
+#pragma unroll
+            for (int q = 0; q < 4; q++) v[q] = soft_cap(v[q], e.limit);
         if (e.residual) {
             const float4 r4 = *(const float4 *)(e.residual + row * e.n_eff + col);
             v[0] += r4.x; v[1] += r4.y; v[2] += r4.z; v[3] += r4.w;
@@ -437,7 +440,7 @@ __device__ __forceinline__ void epi_row4_gated(const EpiArgs &e, bool vec4, uint
     if (vec4 && !e.bias && !e.residual && raw + 7 < n) {
         float o[4];
 #pragma unroll
-        for (int q = 0; q < 4; q++) o[q] = silu(gv[q]) * uv[q];
+        for (int q = 0; q < 4; q++) o[q] = e.act == COEUS_EPI_CLAMP_GATE ? clamped_gate(gv[q], uv[q], e.limit) : silu(gv[q]) * uv[q];
         epi_store4(e, row, ocol, o);
     } else {
 #pragma unroll
@@ -450,7 +453,7 @@ __device__ __forceinline__ void epi_row4_gated(const EpiArgs &e, bool vec4, uint
 // over its share of k) in split order and runs the epilogue.  One thread per 4 outputs of a row.
 __global__ __launch_bounds__(256) void gemm_split_reduce_kernel(const float *__restrict__ part, uint32_t splits,
                                                                 uint64_t m, uint64_t n, EpiArgs e) {
-    const bool gated = e.act == COEUS_EPI_SILU_GATE;
+    const bool gated = epi_gated(e.act);
     const bool vec4 = epi_vec4(e);
     const uint64_t raw_per_thread = gated ? 8 : 4;
     const uint64_t groups = (n + raw_per_thread - 1) / raw_per_thread;  // per row
@@ -505,7 +508,7 @@ __device__ __forceinline__ void h256_tile_of(uint32_t bid, uint32_t tiles_m, uin
 __global__ __launch_bounds__(256) void gemm_tail_reduce_kernel(const float *__restrict__ part, uint32_t splits,
                                                                uint32_t full_tiles, uint32_t tiles_m,
                                                                uint32_t tiles_n, uint64_t m, uint64_t n, EpiArgs e) {
-    const bool gated = e.act == COEUS_EPI_SILU_GATE;
+    const bool gated = epi_gated(e.act);
     const bool vec4 = epi_vec4(e);
     const uint32_t rpt = gated ? 8 : 4, gpr = 256 / rpt;  // raw columns per thread, threads per tile row
     const uint32_t j = blockIdx.x >> 6, within = (blockIdx.x & 63) * 256 + threadIdx.x;
@@ -727,7 +730,7 @@ __global__ __launch_bounds__(512) void gemm_h256_kernel(const uint16_t *a, const
         e = pe;
         em = TM; en = TN; em0 = 0; en0 = 0;
     }
-    const bool gated = e.act == COEUS_EPI_SILU_GATE;
+    const bool gated = epi_gated(e.act);
     const bool vec4 = epi_vec4(e);
     auto strip_out = [&](const float16_t (&t)[2], uint32_t x) {
 #pragma unroll
@@ -1102,9 +1105,9 @@ __device__ __forceinline__ void k64_strip_kv(const float *strip, uint32_t lane, 
     }
 }
 
-// SiLU-gated pairs without bias or residual: weight rows (2c, 2c+1) = (gate_c, up_c); a lane
+// Gated pairs without bias or residual: weight rows (2c, 2c+1) = (gate_c, up_c); a lane
 // takes 4 outputs = 8 strip columns of rows lane / 16, + 4, ...
-template <bool LP, bool BF16OUT = false>
+template <bool CLAMP, bool LP, bool BF16OUT = false>
 __device__ __forceinline__ void k64_strip_gated(const float *strip, uint32_t lane, const EpiArgs &e, uint64_t row0,
                                                 uint64_t col0, uint64_t em) {
     const uint32_t o4 = (lane & 15) * 4, r0 = lane >> 4;
@@ -1115,7 +1118,14 @@ __device__ __forceinline__ void k64_strip_gated(const float *strip, uint32_t lan
         const uint64_t row = row0 + r;
         const float4 p0 = *(const float4 *)(strip + r * K64_TS + 2 * o4);
         const float4 p1 = *(const float4 *)(strip + r * K64_TS + 2 * o4 + 4);
-        const float v[4] = {k64_silu(p0.x) * p0.y, k64_silu(p0.z) * p0.w, k64_silu(p1.x) * p1.y, k64_silu(p1.z) * p1.w};
+        float v[4];
+        if (CLAMP) {
+            v[0] = clamped_gate(p0.x, p0.y, e.limit); v[1] = clamped_gate(p0.z, p0.w, e.limit);
+            v[2] = clamped_gate(p1.x, p1.y, e.limit); v[3] = clamped_gate(p1.z, p1.w, e.limit);
+        } else {
+            v[0] = k64_silu(p0.x) * p0.y; v[1] = k64_silu(p0.z) * p0.w;
+            v[2] = k64_silu(p1.x) * p1.y; v[3] = k64_silu(p1.z) * p1.w;
+        }
         if (row < em) {
             if (LP) *(uint2 *)(e.out_lp + row * e.lp_ld + ocol) = k64_pack4<BF16OUT>(v);
             else *(float4 *)(e.out_f32 + row * e.n_eff + ocol) = make_float4(v[0], v[1], v[2], v[3]);
@@ -1131,7 +1141,8 @@ __device__ __forceinline__ uint32_t k64_epilogue_kind(const EpiArgs &e, bool vec
     bits = (e.bias ? 1u : 0u) | (e.residual ? 2u : 0u) | (e.act == COEUS_EPI_GELU ? 4u : 0u) | (e.out_lp ? 8u : 0u);
     const bool one_out = (e.out_f32 != nullptr) != (e.out_lp != nullptr);
     if (!vec4 || col0 + 128 > en || (en & 3)) return K64_GENERIC;
-    if (e.act == COEUS_EPI_SILU_GATE) return (!e.bias && !e.residual && one_out) ? K64_GATED : K64_GENERIC;
+    if (e.act == COEUS_EPI_SOFTCAP) return K64_GENERIC;
+    if (epi_gated(e.act)) return (!e.bias && !e.residual && one_out) ? K64_GATED : K64_GENERIC;
     if (e.kv_k) {
         if (!e.kv_rows_per_seq || (e.kv_inner & 127)) return K64_GENERIC;
         if (col0 >= e.kv_inner) return K64_KV;
@@ -1181,9 +1192,17 @@ __device__ __forceinline__ void k64_strip_out(const float *strip, uint32_t lane,
             else k64_strip_kv<false, COEUS_KV_F32>(strip, lane, e, row0, col0, em, en);
         }
     } else if (kind == K64_GATED) {
-        if (!e.out_lp) k64_strip_gated<false>(strip, lane, e, row0, col0, em);
-        else if (e.lp_bf16) k64_strip_gated<true, true>(strip, lane, e, row0, col0, em);
-        else k64_strip_gated<true, false>(strip, lane, e, row0, col0, em);
+        const bool clamp = e.act == COEUS_EPI_CLAMP_GATE;
+        if (!e.out_lp) {
+            if (clamp) k64_strip_gated<true, false>(strip, lane, e, row0, col0, em);
+            else k64_strip_gated<false, false>(strip, lane, e, row0, col0, em);
+        } else if (e.lp_bf16) {
+            if (clamp) k64_strip_gated<true, true, true>(strip, lane, e, row0, col0, em);
+            else k64_strip_gated<false, true, true>(strip, lane, e, row0, col0, em);
+        } else {
+            if (clamp) k64_strip_gated<true, true, false>(strip, lane, e, row0, col0, em);
+            else k64_strip_gated<false, true, false>(strip, lane, e, row0, col0, em);
+        }
     } else {
         k64_strip_generic(strip, lane, e, gated, vec4, row0, col0, em, en);
     }
@@ -1314,7 +1333,7 @@ __global__ __launch_bounds__(256) void gemm_h256k64_kernel(const uint16_t *a, co
         e = pe;
         em = TM; en = TN; em0 = 0; en0 = 0;
     }
-    const bool gated = e.act == COEUS_EPI_SILU_GATE;
+    const bool gated = epi_gated(e.act);
     const bool vec4 = epi_vec4(e);
     uint32_t bits;
     const uint32_t kind = k64_epilogue_kind(e, vec4, en0 + wn, en, bits);
@@ -1404,9 +1423,11 @@ int launch_gemm(const Weight &w, const void *a_in, uint64_t m, const Epilogue &e
                 hipStream_t st, bool a_staged) {
     const float *a = (const float *)a_in;
     if (m == 0) return fail(COEUS_INVALID_INPUT, "matmul with zero rows");
-    if (ep.act == COEUS_EPI_SILU_GATE && (w.n & 1))
+    if (epi_gated(ep.act) && (w.n & 1))
         return fail(COEUS_INVALID_INPUT, "gated epilogue needs an even number of weight rows");
     if (ep.out_xq) return fail(COEUS_INVALID_INPUT, "prefill matmul has no xq output");
+    if (ep.act >= COEUS_EPI_CLAMP_GATE && w.dtype >= COEUS_W_Q8_0)
+        return fail(COEUS_INVALID_INPUT, "epilogue %u takes f32 or bf16 weights", ep.act);
     if (w.dtype == COEUS_W_F32) {
         if (a_staged) return fail(COEUS_INVALID_INPUT, "f32 weights take f32 activations");
         return launch_gemm_f32(w, a, m, ep, scr, st);
@@ -1432,7 +1453,7 @@ int launch_gemm(const Weight &w, const void *a_in, uint64_t m, const Epilogue &e
             uint32_t splits = 1;
             COEUS_TRY(launch_gemm_qskinny(w, ap, lda, m, e, scr.partials, scr.partials_bytes, &splits, st));
             if (splits > 1) {
-                const uint64_t groups = ceil_div(w.n, e.act == COEUS_EPI_SILU_GATE ? 8 : 4);
+                const uint64_t groups = ceil_div(w.n, epi_gated(e.act) ? 8 : 4);
                 hipLaunchKernelGGL(gemm_split_reduce_kernel, dim3((unsigned)ceil_div(m * groups, 256)), dim3(256), 0, st,
                                    (const float *)scr.partials, splits, m, w.n, e);
             }
@@ -1489,7 +1510,7 @@ int launch_gemm(const Weight &w, const void *a_in, uint64_t m, const Epilogue &e
             plain = make_epi(pe, w.n);
         }
         const EpiArgs &ke = splits > 1 ? plain : e;
-        const uint64_t groups = ceil_div(w.n, e.act == COEUS_EPI_SILU_GATE ? 8 : 4);
+        const uint64_t groups = ceil_div(w.n, epi_gated(e.act) ? 8 : 4);
         if (scr.ev_begin) COEUS_HIP(hipEventRecord(scr.ev_begin, st));
         for (uint32_t rep = 0; rep < (scr.repeat ? scr.repeat : 1); rep++) {
             if (w.k % UK == 0 && bf)

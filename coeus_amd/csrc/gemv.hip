@@ -998,10 +998,18 @@ static int launch_gemv_quant(const Weight &w, const __half *xq, uint64_t batch, 
 // NORM = 3: the norm of the sublayer before stands behind it.  x is the residual stream h, y the
 // sublayer's bare output: the workgroup stages h + y / rms(y) * scale (* ls), and the first one stores
 // these rows as the new residual stream.  LDS: y rows (then the sums), [2][k] scales, h rows behind them.
+// NORM = 4: hyper-connections.  x holds `streams` rows per batch entry, y the output of the sublayer before
+// (null: none yet).  The workgroup stages the layer norm of sum_t in[t] x'_t, x'_t = sum_s mix[s][t] x_s +
+// mult out[t] y, and the first one stores the x'_t.  What a sum over t needs of the old streams is one
+// coefficient per stream, so only that workgroup forms the new ones.
 struct PostNorm {
     const float *y, *ls;
     float *h_out;
+    const float *mix, *out, *in;
+    float mult;
+    uint32_t streams;
 };
+constexpr int kFusedStreams = 4;
 template <bool BF16, int BP, int NORM>
 __global__ __launch_bounds__(1024) void gemv_dense_kernel(const void *__restrict__ wdata,
                                                           const float *__restrict__ x, uint64_t k,
@@ -1046,9 +1054,49 @@ __global__ __launch_bounds__(1024) void gemv_dense_kernel(const void *__restrict
         float ps[BP];
 #pragma unroll
         for (int b = 0; b < BP; b++) ps[b] = 0.f;
+        constexpr int NS = NORM == 4 ? kFusedStreams : 1;
+        float cs[NS], cy = 0.f;  // NORM == 4: what x_s and y contribute to the weighted sum of the new streams
+        const uint32_t S = NORM == 4 ? post.streams : 1;
+        if (NORM == 4) {
+#pragma unroll
+            for (int s = 0; s < NS; s++) {
+                cs[s] = 0.f;
+                if (s >= (int)S) continue;
+                if (!post.y) { cs[s] = post.in[s]; continue; }
+                for (uint32_t u = 0; u < S; u++) cs[s] = fmaf(post.mix[s * S + u], post.in[u], cs[s]);
+                cy = fmaf(post.mult * post.out[s], post.in[s], cy);
+            }
+        }
         for (uint64_t i = threadIdx.x; i < k; i += blockDim.x) {
             gs[i] = nscale[i];
-            if (NORM == 1) bs[i] = nbias[i];
+            if (NORM == 1) bs[i] = nbias ? nbias[i] : 0.f;
+            if (NORM == 4) {
+#pragma unroll
+                for (int b = 0; b < BP; b++)
+                    if (b < (int)batch) {
+                        float xv[NS];
+#pragma unroll
+                        for (int s = 0; s < NS; s++) xv[s] = s < (int)S ? x[((uint64_t)b * S + s) * k + i] : 0.f;
+                        const float yv = post.y ? post.y[(uint64_t)b * k + i] : 0.f;
+                        float v = cy * yv;
+#pragma unroll
+                        for (int s = 0; s < NS; s++) v = fmaf(cs[s], xv[s], v);
+                        xn[(uint64_t)b * k + i] = v;
+                        ps[b] += v;
+                        if (blockIdx.x == 0 && post.y) {
+#pragma unroll
+                            for (int u = 0; u < NS; u++)
+                                if (u < (int)S) {
+                                    float nv = post.mult * post.out[u] * yv;
+#pragma unroll
+                                    for (int s = 0; s < NS; s++)
+                                        if (s < (int)S) nv = fmaf(post.mix[s * S + u], xv[s], nv);
+                                    post.h_out[((uint64_t)b * S + u) * k + i] = nv;
+                                }
+                        }
+                    }
+                continue;
+            }
             if (NORM == 3) bs[i] = post.ls ? post.ls[i] : 1.0f;
 #pragma unroll
             for (int b = 0; b < BP; b++)
@@ -1072,7 +1120,7 @@ __global__ __launch_bounds__(1024) void gemv_dense_kernel(const void *__restrict
                 for (uint32_t w = 0; w < nwaves; w++) tot += red[w * BP + lane];
             return tot;
         };
-        if (NORM == 1) {
+        if (NORM == 1 || NORM == 4) {
             const float tot = finish(ps);
             if (wave == 0 && lane < BP) stat[lane] = tot / (float)k;
             __syncthreads();
@@ -1165,7 +1213,7 @@ __global__ __launch_bounds__(1024) void gemv_dense_kernel(const void *__restrict
     }
 #pragma unroll
     for (int b = 0; b < BP; b++) acc[b] = wave_sum(acc[b]);
-    if (e.act == COEUS_EPI_SILU_GATE) {
+    if (epi_gated(e.act)) {
         // pair (gate_m, up_m) = rows (2m, 2m+1) live in neighbouring waves: go through LDS
         __shared__ float pair[16][16];
         if (lane == 0)
@@ -1199,32 +1247,40 @@ bool gemv_can_fuse_post_norm(const Weight &w, uint64_t batch) {
     return gemv_dense_post_lds(w.k, pad_batch(batch)) <= kDenseNormLdsLimit;
 }
 
+bool gemv_can_fuse_hyper(const Weight &w, uint64_t batch, uint64_t streams) {
+    return streams >= 1 && streams <= kFusedStreams && gemv_can_fuse_norm_dense(w, batch);
+}
+
 template <bool BF16>
 static int launch_gemv_dense(const Weight &w, const float *x, uint64_t batch, const EpiArgs &e,
                              hipStream_t st, const NormFuse *nf) {
     const uint32_t bp = pad_batch(batch), b = (uint32_t)batch;
-    const bool post_norm = nf && nf->y;
+    const bool hyper = nf && nf->streams, post_norm = nf && nf->y && !hyper;
+    if (hyper && (!gemv_can_fuse_hyper(w, batch, nf->streams) || !nf->in || nf->kind != COEUS_NORM_LAYERNORM || nf->ld ||
+                  (nf->y && (!nf->mix || !nf->out || !nf->h_out || nf->h_out == nf->h))))
+        return fail(COEUS_INVALID_INPUT, "folded hyper-connections: bad arguments or too many streams");
     if (nf && !(post_norm ? gemv_can_fuse_post_norm(w, batch) : gemv_can_fuse_norm_dense(w, batch)))
         return fail(COEUS_INVALID_INPUT, "norm fusion needs the normalised activations to fit in LDS");
     if (post_norm && (!nf->h || !nf->scale || !nf->h_out || nf->h_out == nf->h || nf->kind != COEUS_NORM_RMSNORM))
         return fail(COEUS_INVALID_INPUT, "a norm behind the previous sublayer needs its output, the residual rows and "
                                          "a place for the new ones");
-    if (nf && !post_norm && (!nf->h || !nf->scale || (nf->kind == COEUS_NORM_LAYERNORM && !nf->bias)))
+    if (nf && !post_norm && (!nf->h || !nf->scale))
         return fail(COEUS_INVALID_INPUT, "null pointer argument");
     // plain: 4 rows per workgroup; folded norm: 16, so that the block is normalised once per 16 rows
     const uint32_t waves = nf ? 16 : 4;
     const dim3 grid((unsigned)ceil_div(w.n, waves)), block(waves * 64);
     const size_t lds = !nf ? 0 : post_norm ? gemv_dense_post_lds(w.k, bp) : gemv_dense_norm_lds(w.k, bp);
-    const int norm = !nf ? 0 : post_norm ? 3 : nf->kind == COEUS_NORM_RMSNORM ? 2 : 1;
+    const int norm = !nf ? 0 : hyper ? 4 : post_norm ? 3 : nf->kind == COEUS_NORM_RMSNORM ? 2 : 1;
     const uint64_t ldx = nf && nf->ld ? nf->ld : w.k;
-    const PostNorm post = post_norm ? PostNorm{nf->y, nf->ls, nf->h_out} : PostNorm{nullptr, nullptr, nullptr};
+    PostNorm post{};
+    if (post_norm || hyper) post = PostNorm{nf->y, nf->ls, nf->h_out, nf->mix, nf->out, nf->in, nf->mult, nf->streams};
     const float *xin = nf ? nf->h : x;
     const float *ns = nf ? nf->scale : nullptr, *nb = nf ? nf->bias : nullptr;
     const float eps = nf ? nf->eps : 0.f;
 #define COEUS_GEMVD2(BPV, NV) \
     hipLaunchKernelGGL((gemv_dense_kernel<BF16, BPV, NV>), grid, block, lds, st, w.data, xin, w.k, b, e, ns, nb, eps, ldx, post)
 #define COEUS_GEMVD(BPV) \
-    do { if (norm == 0) COEUS_GEMVD2(BPV, 0); else if (norm == 1) COEUS_GEMVD2(BPV, 1); else if (norm == 2) COEUS_GEMVD2(BPV, 2); else COEUS_GEMVD2(BPV, 3); } while (0)
+    do { if (norm == 0) COEUS_GEMVD2(BPV, 0); else if (norm == 1) COEUS_GEMVD2(BPV, 1); else if (norm == 2) COEUS_GEMVD2(BPV, 2); else if (norm == 3) COEUS_GEMVD2(BPV, 3); else COEUS_GEMVD2(BPV, 4); } while (0)
     switch (bp) {
         case 1: COEUS_GEMVD(1); break;
         case 2: COEUS_GEMVD(2); break;
@@ -1243,7 +1299,9 @@ int launch_gemv(const Weight &w, const void *x, uint64_t batch, const Epilogue &
     if (batch == 0 || batch > 16)
         return fail(COEUS_INVALID_INPUT, "decode matmul batch %llu out of range [1, 16]",
                     (unsigned long long)batch);
-    if (ep.act == COEUS_EPI_SILU_GATE && (w.n & 1))
+    if (ep.act >= COEUS_EPI_CLAMP_GATE && w.dtype >= COEUS_W_Q8_0)
+        return fail(COEUS_INVALID_INPUT, "epilogue %u takes f32 or bf16 weights", ep.act);
+    if (epi_gated(ep.act) && (w.n & 1))
         return fail(COEUS_INVALID_INPUT, "gated epilogue needs an even number of weight rows");
     const EpiArgs e = make_epi(ep, w.n);
     if (e.g_out && (w.dtype < COEUS_W_Q8_0 || pad_batch(batch) > 4 || !e.g_scale || e.act == COEUS_EPI_SILU_GATE || e.kv_k))

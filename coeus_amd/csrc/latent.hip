@@ -1,9 +1,7 @@
-// Attention through low-rank latents with an optional sliding window.
+// Attention through low-rank latents with an optional sliding window: the latents' norms and a decode step
+// (a prompt's latents are expanded by a matmul and attended to in window.hip).
 //
 //   latent_norm_kernel        RMS norms of the query latent and of the key/value latent
-//   latent_gather / append    cached latents in front of a prompt's portion / its own into the ring
-//   window_prefill_kernel     prompt, bf16: expanded keys and values on the matrix cores
-//   window_attn_kernel        prompt: one wave per (row, head), any size and type
 // Decode takes the query into latent space (W_uk^T q), scores it against the cached latents, which all
 // heads share, and expands the weighted latent by W_uv:
 //   latent_absorb_kernel      W_uk^T q of every head; the new token's latent, normalised, into the ring
@@ -15,17 +13,8 @@
 
 namespace coeus {
 
-template <bool BF16>
-__device__ __forceinline__ float lat_load(const void *p, uint64_t i) {
-    return BF16 ? bf16_bits_to_f32(((const uint16_t *)p)[i]) : ((const float *)p)[i];
-}
-template <bool BF16>
-__device__ __forceinline__ void lat_store(void *p, uint64_t i, float v) {
-    if (BF16) ((uint16_t *)p)[i] = f32_to_bf16_bits(v);
-    else ((float *)p)[i] = v;
-}
 
-static int check_dims(const LatentDims &dm, const LatentCache &cache) {
+static int check_dims(const LatentDims &dm, const RowRing &cache) {
     if (dm.heads == 0 || dm.heads > 65534 || dm.d == 0 || dm.d > 256 || dm.e == 0 || dm.e > 256 || dm.q_rank == 0 ||
         dm.rank == 0 || dm.rank > 2048 || dm.in_ld < dm.q_rank + dm.rank)
         return fail(COEUS_INVALID_INPUT, "latent attention: sizes out of range");
@@ -76,7 +65,7 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(const float *__restric
     const float rs = 1.0f / sqrtf(wave_sum(s2) / (float)len + eps);
     const uint64_t dst = pos_dev ? (row * cap + *pos_dev % cap) * dm.rank : ((row / n) * lat_rows + lat_off + row % n) * lat_ld;
     auto put = [&](uint32_t i, float y) {
-        if (!is_q) lat_store<BF16>(lat, dst + i, y);
+        if (!is_q) elem_store<BF16>(lat, dst + i, y);
         if (is_q && cq) cq[row * dm.q_rank + i] = y;
         if (is_q && cq_lp) cq_lp[row * cq_ld + i] = f32_to_lp_bits(y, lp_bf16);
     };
@@ -88,7 +77,7 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(const float *__restric
 
 int launch_latent_norm(const float *proj, const LatentDims &dm, const float *q_scale, const float *c_scale, float eps,
                        uint64_t batch, uint64_t n, float *cq, const LpOut *cq_lp, void *lat, uint64_t lat_ld,
-                       uint64_t lat_rows, uint64_t lat_off, const LatentCache &cache, const uint32_t *pos_dev,
+                       uint64_t lat_rows, uint64_t lat_off, const RowRing &cache, const uint32_t *pos_dev,
                        hipStream_t st) {
     COEUS_TRY(check_dims(dm, cache));
     if (batch == 0 || n == 0 || batch * n > 0x7fffffffull || (pos_dev && n != 1))
@@ -110,315 +99,6 @@ int launch_latent_norm(const float *proj, const LatentDims &dm, const float *q_s
     return COEUS_OK;
 }
 
-// Rows of `rank` elements between the ring and a contiguous buffer: blockIdx.x counts `cnt` positions
-// from pos_first, whose buffer row is row_first.
-template <typename T, bool TO_RING>
-__global__ __launch_bounds__(64) void latent_copy_kernel(T *ring, uint32_t cap, uint32_t rank, T *buf, uint64_t ld,
-                                                         uint64_t rows_per_seq, uint64_t pos_first, uint64_t row_first) {
-    const uint64_t i = blockIdx.x, b = blockIdx.y;
-    T *r = ring + (b * cap + (pos_first + i) % cap) * rank, *l = buf + (b * rows_per_seq + row_first + i) * ld;
-    for (uint32_t t = threadIdx.x; t < rank; t += 64) {
-        if (TO_RING) r[t] = l[t];
-        else l[t] = r[t];
-    }
-}
-
-template <bool TO_RING>
-static int latent_copy(const LatentCache &cache, uint32_t rank, uint64_t batch, uint64_t cnt, uint64_t pos_first, void *buf,
-                       uint64_t ld, uint64_t rows_per_seq, uint64_t row_first, hipStream_t st) {
-    if (cnt == 0) return COEUS_OK;
-    if (cnt > cache.cap || batch == 0 || batch > 65535) return fail(COEUS_INVALID_INPUT, "latent attention: rows out of range");
-    const dim3 grid((unsigned)cnt, (unsigned)batch);
-    if (cache.bf16)
-        hipLaunchKernelGGL((latent_copy_kernel<uint16_t, TO_RING>), grid, dim3(64), 0, st, (uint16_t *)cache.c, cache.cap, rank,
-                           (uint16_t *)buf, ld, rows_per_seq, pos_first, row_first);
-    else
-        hipLaunchKernelGGL((latent_copy_kernel<float, TO_RING>), grid, dim3(64), 0, st, (float *)cache.c, cache.cap, rank,
-                           (float *)buf, ld, rows_per_seq, pos_first, row_first);
-    COEUS_HIP(hipGetLastError());
-    return COEUS_OK;
-}
-
-int launch_latent_gather(const LatentCache &cache, uint32_t rank, uint64_t batch, uint64_t hist, uint64_t pos0,
-                         void *lat, uint64_t lat_ld, uint64_t lat_rows, hipStream_t st) {
-    if (hist > pos0) return fail(COEUS_INVALID_INPUT, "latent attention: rows out of range");
-    return latent_copy<false>(cache, rank, batch, hist, pos0 - hist, lat, lat_ld, lat_rows, 0, st);
-}
-
-int launch_latent_append(const void *lat, uint64_t lat_ld, uint64_t lat_rows, uint64_t hist, const LatentCache &cache,
-                         uint32_t rank, uint64_t batch, uint64_t n, uint64_t pos0, hipStream_t st) {
-    const uint64_t cnt = n < cache.cap ? n : cache.cap;
-    return latent_copy<true>(cache, rank, batch, cnt, pos0 + n - cnt, (void *)lat, lat_ld, lat_rows, hist + n - cnt, st);
-}
-
-// ---------------------------------------------------------------- prompt attention, any size and type
-// Row i of a sequence is key hist + i and sees keys lo .. hist + i, lo = max(0, hist + i - window + 1).
-template <bool BF16>
-__global__ __launch_bounds__(256) void window_attn_kernel(const void *__restrict__ q, uint64_t q_ld,
-                                                          const void *__restrict__ kv, uint64_t kv_ld, LatentDims dm,
-                                                          uint32_t n, uint32_t hist, float *__restrict__ out,
-                                                          uint16_t *__restrict__ out_lp, uint64_t lp_ld, bool lp_bf16) {
-    extern __shared__ float lds[];  // per wave: q[d] + p[64]
-    const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    const uint32_t i = blockIdx.x * 4 + wave, h = blockIdx.y;
-    const uint64_t b = blockIdx.z;
-    if (i >= n) return;
-    float *qs = lds + wave * (dm.d + 64), *ps = qs + dm.d;
-    const uint64_t row = b * n + i, k0 = b * (hist + n);
-    for (uint32_t t = lane; t < dm.d; t += 64) qs[t] = lat_load<BF16>(q, row * q_ld + h * dm.d + t);
-    const uint32_t end = hist + i + 1, lo = dm.window && end > dm.window ? end - dm.window : 0;
-    const uint32_t voff = dm.heads * dm.d + h * dm.e;
-    float m = -INFINITY, l = 0.f, acc[4] = {0.f, 0.f, 0.f, 0.f};
-    for (uint32_t j0 = lo; j0 < end; j0 += 64) {
-        const uint32_t j = j0 + lane;
-        float s = -INFINITY;
-        if (j < end) {
-            float dot = 0.f;
-            const uint64_t kr = (k0 + j) * kv_ld + h * dm.d;
-            for (uint32_t t = 0; t < dm.d; t++) dot = fmaf(qs[t], lat_load<BF16>(kv, kr + t), dot);
-            s = dot * dm.scale;
-        }
-        const float m_new = fmaxf(m, wave_max(s));
-        const float p = j < end ? expf(s - m_new) : 0.f, corr = expf(m - m_new);
-        l = l * corr + wave_sum(p);
-        m = m_new;
-        ps[lane] = p;
-#pragma unroll
-        for (int t = 0; t < 4; t++) acc[t] *= corr;
-        const uint32_t cnt = min(64u, end - j0);
-        for (uint32_t jj = 0; jj < cnt; jj++) {
-            const float pj = ps[jj];
-            const uint64_t vr = (k0 + j0 + jj) * kv_ld + voff;
-#pragma unroll
-            for (int t = 0; t < 4; t++)
-                if (lane + 64 * t < dm.e) acc[t] = fmaf(pj, lat_load<BF16>(kv, vr + lane + 64 * t), acc[t]);
-        }
-    }
-    const float inv = 1.0f / l;
-#pragma unroll
-    for (int t = 0; t < 4; t++) {
-        const uint32_t c = lane + 64 * t;
-        if (c >= dm.e) continue;
-        if (out) out[row * dm.heads * dm.e + h * dm.e + c] = acc[t] * inv;
-        if (out_lp) out_lp[row * lp_ld + h * dm.e + c] = f32_to_lp_bits(acc[t] * inv, lp_bf16);
-    }
-}
-
-// ---------------------------------------------------------------- prompt attention on the matrix cores
-// The scheme of attn_prefill_kernel (scores and outputs transposed, so that a query stays in its lanes and
-// the weights never leave registers) with key and value sizes of their own, rounded up to DK and DV (a
-// piece behind the end re-reads the last one: its query dims are zero / its outputs are not stored), and a
-// lower edge.  The f32 weights enter the product with V as a sum of two bf16 numbers.
-__device__ __forceinline__ void split_bf16(float a, __bf16 &hi, __bf16 &lo) {
-    hi = (__bf16)a;
-    lo = (__bf16)(a - (float)hi);
-}
-
-template <int DK, int DV>
-__global__ __launch_bounds__(256) void window_prefill_kernel(const uint16_t *__restrict__ q, uint64_t q_ld,
-                                                             const uint16_t *__restrict__ kv, uint64_t kv_ld,
-                                                             LatentDims dm, uint32_t n, uint32_t hist,
-                                                             float *__restrict__ out, uint16_t *__restrict__ out_lp,
-                                                             uint64_t lp_ld, bool lp_bf16) {
-    constexpr int KT = 32, KLD = DK + 8, VLD = 36, NKS = DK / 16, NDT = DV / 32, KP = DK / 64, VP = (DV + 127) / 128;
-    extern __shared__ __attribute__((aligned(16))) uint16_t lds16[];
-    uint16_t *const ks = lds16, *const vt = lds16 + 2 * KT * KLD;  // [2][key][dim], [2][dim][key]
-    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, qi = lane & 31, hf = lane >> 5;
-    uint32_t qt, h;
-    prefill_tile_of_block(qt, h);
-    const uint64_t b = blockIdx.z;
-    const uint32_t r0 = qt * 128 + wave * 32, r = r0 + qi, rc = min(r, n - 1);
-    const uint32_t qkey = hist + rc, W = dm.window ? dm.window : 0xffffffffu;  // row rc is key qkey, sees (qkey - W, qkey]
-    const float scale2 = 1.4426950408889634f * dm.scale;
-    bf16x8_t qf[NKS];
-    {
-        const uint16_t *qp = q + (b * n + rc) * q_ld + h * dm.d;
-#pragma unroll
-        for (int s = 0; s < NKS; s++) {
-            union { uint4 u; bf16x8_t v; } cv;
-            const uint32_t d0 = 16 * s + 8 * hf;
-            cv.u = *(const uint4 *)(qp + min(d0, dm.d - 8));
-            if (d0 >= dm.d) cv.u = make_uint4(0, 0, 0, 0);
-            qf[s] = cv.v;
-        }
-    }
-    const uint16_t *kb = kv + b * (hist + n) * kv_ld + h * dm.d;
-    const uint16_t *vb = kv + b * (hist + n) * kv_ld + dm.heads * dm.d + h * dm.e;
-    const uint32_t first_q = hist + qt * 128, kmax = hist + min(n, qt * 128 + 128) - 1;
-    const uint32_t t_begin = (first_q >= W ? first_q - W + 1 : 0) / KT, t_end = kmax / KT + 1;
-    const uint32_t wave_lo = hist + min(r0, n - 1), wave_hi = hist + min(r0 + 31, n - 1);
-    const bool wave_live = r0 < n;
-
-    const uint32_t kkey = tid >> 3, kpc = tid & 7, va = tid & 15, vdp = tid >> 4;
-    uint4 rk0, rk1, rk2, rk3, rv0, rv1, rv2, rv3;  // (named: arrays captured by the lambdas end up in scratch memory)
-    rk0 = rk1 = rk2 = rk3 = rv0 = rv1 = rv2 = rv3 = make_uint4(0, 0, 0, 0);
-    auto kload = [&](uint64_t krow, uint32_t u, uint4 &x) { x = *(const uint4 *)(kb + krow + min(8 * (kpc + 8 * u), dm.d - 8)); };
-    auto vload = [&](uint32_t t, uint32_t u, uint4 &x, uint4 &y) {
-        const uint32_t d0 = min(8 * (vdp + 16 * u), dm.e - 8);
-        x = *(const uint4 *)(vb + (uint64_t)min(t * KT + 2 * va, kmax) * kv_ld + d0);
-        y = *(const uint4 *)(vb + (uint64_t)min(t * KT + 2 * va + 1, kmax) * kv_ld + d0);
-    };
-    auto gload = [&](uint32_t t) {
-        const uint64_t krow = (uint64_t)min(t * KT + kkey, kmax) * kv_ld;
-        kload(krow, 0, rk0);
-        if (KP > 1) kload(krow, 1, rk1);
-        if (KP > 2) { kload(krow, 2, rk2); kload(krow, 3, rk3); }
-        if (DV >= 128 || vdp < DV / 8) vload(t, 0, rv0, rv1);
-        if (VP > 1) vload(t, 1, rv2, rv3);
-    };
-    auto kstore = [&](uint32_t buf, uint32_t u, const uint4 &x) { *(uint4 *)(ks + buf * KT * KLD + kkey * KLD + 8 * (kpc + 8 * u)) = x; };
-    auto vstore = [&](uint32_t buf, uint32_t u, const uint4 &x, const uint4 &y) {
-        uint32_t *dst = (uint32_t *)(vt + buf * DV * VLD) + (vdp + 16 * u) * (8 * VLD / 2) + va;
-        const uint32_t a[4] = {x.x, x.y, x.z, x.w}, c[4] = {y.x, y.y, y.z, y.w};
-#pragma unroll
-        for (int e = 0; e < 4; e++) {
-            dst[e * VLD] = __builtin_amdgcn_perm(c[e], a[e], 0x05040100u);
-            dst[e * VLD + VLD / 2] = __builtin_amdgcn_perm(c[e], a[e], 0x07060302u);
-        }
-    };
-    auto lstore = [&](uint32_t buf) {
-        kstore(buf, 0, rk0);
-        if (KP > 1) kstore(buf, 1, rk1);
-        if (KP > 2) { kstore(buf, 2, rk2); kstore(buf, 3, rk3); }
-        if (DV >= 128 || vdp < DV / 8) vstore(buf, 0, rv0, rv1);
-        if (VP > 1) vstore(buf, 1, rv2, rv3);
-    };
-    float16_t o[NDT];
-#pragma unroll
-    for (int d = 0; d < NDT; d++)
-#pragma unroll
-        for (int i = 0; i < 16; i++) o[d][i] = 0.f;
-    float m = -1e30f, l = 0.f;  // (finite: a tile may hold no key that this query sees)
-
-    gload(t_begin);
-    lstore(t_begin & 1);
-    gload(min(t_begin + 1, t_end - 1));
-    for (uint32_t t = t_begin; t < t_end; t++) {
-        __syncthreads();
-        lstore((t + 1) & 1);
-        gload(min(t + 2, t_end - 1));
-        const uint32_t k0 = t * KT;
-        if (!wave_live || k0 > wave_hi || (wave_lo >= W && k0 + KT - 1 <= wave_lo - W)) continue;  // wave-uniform
-        const uint16_t *kt_ = ks + (t & 1) * KT * KLD, *vt_ = vt + (t & 1) * DV * VLD;
-        float16_t sc;
-#pragma unroll
-        for (int i = 0; i < 16; i++) sc[i] = 0.f;
-#pragma unroll
-        for (int s = 0; s < NKS; s++)
-            sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8_t *)(kt_ + qi * KLD + 16 * s + 8 * hf), qf[s], sc, 0, 0, 0);
-        float tmax = -INFINITY;
-#pragma unroll
-        for (int i = 0; i < 16; i++) sc[i] *= scale2;
-        if (k0 + KT - 1 > wave_lo || (wave_hi >= W && k0 <= wave_hi - W)) {  // an edge crosses the tile
-#pragma unroll
-            for (int i = 0; i < 16; i++) {
-                const uint32_t key = k0 + 4 * hf + 8 * (i >> 2) + (i & 3);
-                sc[i] = key > qkey || qkey - key >= W ? -INFINITY : sc[i];
-            }
-        }
-#pragma unroll
-        for (int i = 0; i < 16; i++) tmax = fmaxf(tmax, sc[i]);
-        const float m_new = fmaxf(m, both_halves_max(tmax));
-        float psum = 0.f, pv[16];
-#pragma unroll
-        for (int i = 0; i < 16; i++) {
-            pv[i] = __builtin_amdgcn_exp2f(sc[i] - m_new);  // 2^(-inf) = 0 for keys that are not seen
-            psum += pv[i];
-        }
-        if (__builtin_amdgcn_ballot_w64(m_new != m) != 0) {
-            const float corr = __builtin_amdgcn_exp2f(m - m_new);
-            l *= corr;
-#pragma unroll
-            for (int d = 0; d < NDT; d++)
-#pragma unroll
-                for (int i = 0; i < 16; i++) o[d][i] *= corr;
-        }
-        l += psum;
-        m = m_new;
-        bf16x8_t ph[2], pl[2];
-#pragma unroll
-        for (int j = 0; j < 2; j++)
-#pragma unroll
-            for (int e = 0; e < 8; e++) {
-                __bf16 hi, lo;
-                split_bf16(pv[8 * j + e], hi, lo);
-                ph[j][e] = hi;
-                pl[j][e] = lo;
-            }
-#pragma unroll
-        for (int d = 0; d < NDT; d++)
-#pragma unroll
-            for (int j = 0; j < 2; j++) {
-                const uint16_t *vp = vt_ + (d * 32 + qi) * VLD + 16 * j + 4 * hf;
-                const uint2 v0 = *(const uint2 *)vp, v1 = *(const uint2 *)(vp + 8);
-                union { uint4 u; bf16x8_t v; } vf;
-                vf.u = make_uint4(v0.x, v0.y, v1.x, v1.y);
-                o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf.v, pl[j], o[d], 0, 0, 0);
-                o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf.v, ph[j], o[d], 0, 0, 0);
-            }
-    }
-    if (r >= n) return;
-    const float inv = 1.0f / xor32_sum(l);
-    const uint64_t row = b * n + r;
-#pragma unroll
-    for (int d = 0; d < NDT; d++)
-#pragma unroll
-        for (int gq = 0; gq < 4; gq++) {
-            const uint32_t c0 = d * 32 + 8 * gq + 4 * hf;  // e % 8 == 0: four columns are all in or all out
-            if (c0 >= dm.e) continue;
-            const float v[4] = {o[d][4 * gq] * inv, o[d][4 * gq + 1] * inv, o[d][4 * gq + 2] * inv, o[d][4 * gq + 3] * inv};
-            if (out) *(float4 *)(out + row * dm.heads * dm.e + h * dm.e + c0) = make_float4(v[0], v[1], v[2], v[3]);
-            if (out_lp) {
-                uint2 p;
-                p.x = (uint32_t)f32_to_lp_bits(v[0], lp_bf16) | ((uint32_t)f32_to_lp_bits(v[1], lp_bf16) << 16);
-                p.y = (uint32_t)f32_to_lp_bits(v[2], lp_bf16) | ((uint32_t)f32_to_lp_bits(v[3], lp_bf16) << 16);
-                *(uint2 *)(out_lp + row * lp_ld + h * dm.e + c0) = p;
-            }
-        }
-}
-
-int launch_window_attention(const void *q, uint64_t q_ld, const void *kv, uint64_t kv_ld, bool bf16,
-                            const LatentDims &dm, uint64_t batch, uint64_t n, uint64_t hist, float *out,
-                            const LpOut *out_lp, hipStream_t st) {
-    if (batch == 0 || batch > 65535 || n == 0 || hist + n > 0x7fffffffull || dm.heads == 0 || dm.heads > 65535 ||
-        dm.d == 0 || dm.d > 256 || dm.e == 0 || dm.e > 256)
-        return fail(COEUS_INVALID_INPUT, "window attention: sizes out of range");
-    uint16_t *lp = out_lp ? (uint16_t *)out_lp->p : nullptr;
-    const uint64_t lp_ld = out_lp ? out_lp->ld : 0;
-    const bool lp_bf = out_lp && out_lp->bf16;
-    // the matrix-core kernel moves 8 dims at a time
-    if (bf16 && dm.d % 8 == 0 && dm.e % 8 == 0 && q_ld % 8 == 0 && kv_ld % 8 == 0 && lp_ld % 4 == 0) {
-        const dim3 pgrid((unsigned)ceil_div(n, 128), dm.heads, (unsigned)batch);
-#define COEUS_WP(DKV, DVV)                                                                                           \
-    do {                                                                                                             \
-        static const bool once = hipFuncSetAttribute((const void *)window_prefill_kernel<DKV, DVV>,                  \
-                                                     hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024) == hipSuccess; \
-        (void)once;                                                                                                  \
-        hipLaunchKernelGGL((window_prefill_kernel<DKV, DVV>), pgrid, dim3(256), (2 * 32 * (DKV + 8) + 2 * DVV * 36) * 2, st, \
-                           (const uint16_t *)q, q_ld, (const uint16_t *)kv, kv_ld, dm, (uint32_t)n, (uint32_t)hist, out, lp, \
-                           lp_ld, lp_bf);                                                                            \
-    } while (0)
-#define COEUS_WPV(DKV) do { if (dm.e <= 64) COEUS_WP(DKV, 64); else if (dm.e <= 128) COEUS_WP(DKV, 128); else COEUS_WP(DKV, 256); } while (0)
-        if (dm.d <= 64) COEUS_WPV(64);
-        else if (dm.d <= 128) COEUS_WPV(128);
-        else COEUS_WPV(256);
-#undef COEUS_WPV
-#undef COEUS_WP
-        COEUS_HIP(hipGetLastError());
-        return COEUS_OK;
-    }
-    const dim3 grid((unsigned)ceil_div(n, 4), dm.heads, (unsigned)batch);
-    const size_t lds = 4 * (dm.d + 64) * sizeof(float);
-    if (bf16)
-        hipLaunchKernelGGL(window_attn_kernel<true>, grid, dim3(256), lds, st, q, q_ld, kv, kv_ld, dm, (uint32_t)n,
-                           (uint32_t)hist, out, lp, lp_ld, lp_bf);
-    else
-        hipLaunchKernelGGL(window_attn_kernel<false>, grid, dim3(256), lds, st, q, q_ld, kv, kv_ld, dm, (uint32_t)n,
-                           (uint32_t)hist, out, lp, lp_ld, lp_bf);
-    COEUS_HIP(hipGetLastError());
-    return COEUS_OK;
-}
-
 // ---------------------------------------------------------------- decode
 // One workgroup per (head, sequence).  The ring never holds more than the visible positions (cap <=
 // window), and a softmax does not care about their order: slots 0 .. min(pos + 1, cap) - 1 are the keys.
@@ -435,7 +115,7 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const float *__restr
     const uint64_t uk = (uint64_t)h * dm.d * R, uv = ((uint64_t)dm.heads * dm.d + h * dm.e) * R;
     for (uint32_t r = tid; r < R; r += 256) {
         float a = 0.f;
-        for (uint32_t t = 0; t < dm.d; t++) a = fmaf(qh[t], lat_load<BF16>(ukv, uk + (uint64_t)t * R + r), a);
+        for (uint32_t t = 0; t < dm.d; t++) a = fmaf(qh[t], elem_load<BF16>(ukv, uk + (uint64_t)t * R + r), a);
         qa[r] = a;
     }
     __syncthreads();
@@ -447,14 +127,14 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const float *__restr
     for (uint32_t j = wave; j < nv; j += 4) {
         const uint64_t cr = (b * cap + j) * R;
         float dot = 0.f;
-        for (uint32_t r = lane; r < R; r += 64) dot = fmaf(qa[r], lat_load<BF16>(cache, cr + r), dot);
+        for (uint32_t r = lane; r < R; r += 64) dot = fmaf(qa[r], elem_load<BF16>(cache, cr + r), dot);
         const float s = wave_sum(dot) * dm.scale;
         const float m_new = fmaxf(m, s), corr = expf(m - m_new), p = expf(s - m_new);
         l = l * corr + p;
         m = m_new;
 #pragma unroll
         for (int u = 0; u < U; u++)
-            if (lane + 64 * u < R) acc[u] = fmaf(p, lat_load<BF16>(cache, cr + lane + 64 * u), acc[u] * corr);
+            if (lane + 64 * u < R) acc[u] = fmaf(p, elem_load<BF16>(cache, cr + lane + 64 * u), acc[u] * corr);
     }
     if (lane == 0) { sm[wave] = m; sl[wave] = l; }
 #pragma unroll
@@ -470,7 +150,7 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const float *__restr
     __syncthreads();
     for (uint32_t c = wave; c < dm.e; c += 4) {
         float a = 0.f;
-        for (uint32_t r = lane; r < R; r += 64) a = fmaf(qa[r], lat_load<BF16>(ukv, uv + (uint64_t)c * R + r), a);
+        for (uint32_t r = lane; r < R; r += 64) a = fmaf(qa[r], elem_load<BF16>(ukv, uv + (uint64_t)c * R + r), a);
         a = wave_sum(a);
         if (lane == 0) out[b * dm.heads * dm.e + h * dm.e + c] = a;
     }
@@ -738,14 +418,14 @@ __global__ __launch_bounds__(256) void latent_expand_kernel(const float *__restr
     }
 }
 
-uint64_t latent_decode_scratch_bytes(const LatentDims &dm, const LatentCache &cache, uint64_t batch) {
+uint64_t latent_decode_scratch_bytes(const LatentDims &dm, const RowRing &cache, uint64_t batch) {
     if (!latent_decode_fast(dm, cache.bf16)) return 0;
     // absorbed queries, then a record per (sequence, head, share)
     return batch * dm.heads * (dm.rank + latent_shares(cache.cap) * (dm.rank + 2ull)) * 4;
 }
 
 int launch_latent_decode(const float *q, const void *ukv, const LatentDims &dm, const LatentNew &nw,
-                         const LatentCache &cache, uint64_t batch, const uint32_t *pos_dev, float *out, float *scratch,
+                         const RowRing &cache, uint64_t batch, const uint32_t *pos_dev, float *out, float *scratch,
                          uint64_t scratch_bytes, hipStream_t st) {
     COEUS_TRY(check_dims(dm, cache));
     if (batch == 0 || batch > 65535 || !pos_dev) return fail(COEUS_INVALID_INPUT, "latent attention: rows out of range");

@@ -78,7 +78,7 @@ void Workspace::release() {
     h.release(); x.release(); qkv.release(); att.release(); ff.release(); ids.release();
     a_lp.release(); b_lp.release(); w_lp.release(); logits.release(); xq.release(); norm_part.release();
     gemm_part.release();
-    mix.release(); lat.release(); q_lp.release(); kv_lp.release();
+    mix.release(); lat.release(); q_lp.release(); kv_lp.release(); streams.release();
     rows = 0;
 }
 
@@ -338,8 +338,7 @@ static int logits_gemv(Model &m, Workspace &ws, const float *x_rows, uint64_t co
                        hipStream_t st) {
     for (uint64_t r0 = 0; r0 < count; r0 += 16) {
         const uint64_t b = count - r0 < 16 ? count - r0 : 16;
-        Epilogue e;
-        e.out_f32 = logits + r0 * m.cfg.vocab_size;
+        const Epilogue e = m.logits_epilogue(logits + r0 * m.cfg.vocab_size);
         const void *xin = x_rows + r0 * m.cfg.hidden_dim;
         if (m.out.dtype >= COEUS_W_Q8_0) {
             COEUS_TRY(ws.xq.ensure(m.out.k_pad * 16 * 2));
@@ -370,8 +369,7 @@ static int finish_forward(Model &m, uint64_t seq_len, float *logits_out, bool al
     COEUS_TRY(launch_norm(c.norm, c.norm_scope, h, seq_len, H, m.fin_s, m.fin_b, c.layer_norm_eps, x,
                           nullptr, 0, st, nullptr, (double *)m.ws.norm_part.p));
     if (all_rows) {
-        Epilogue e;
-        e.out_f32 = logits;
+        const Epilogue e = m.logits_epilogue(logits);
         COEUS_TRY(launch_gemm(m.out, x, seq_len, e, m.ws.gs, st));
     } else {
         COEUS_TRY(logits_gemv(m, m.ws, x + (seq_len - 1) * H, 1, logits, st));
@@ -606,7 +604,7 @@ static int enqueue_decode_step(Session &s, hipStream_t st, int only = STEP_ALL,
     if (m.stack) {
         if (!matmuls_only)
             COEUS_TRY(launch_embed(m.embed, m.embed_bf16, nullptr, (const uint64_t *)s.dids.p, B, 1, 0, pos_dev, H, h,
-                                   nullptr, st));
+                                   nullptr, st, nullptr, nullptr, m.embed_scale, m.streams()));
         return layered_decode(s, st, only, launches, bytes);
     }
     if (!matmuls_only)

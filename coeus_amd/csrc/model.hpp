@@ -28,29 +28,41 @@ struct LayerWeights {
     const float *b_qkv = nullptr, *b_o = nullptr, *b_up = nullptr, *b_down = nullptr;
 };
 
-// One layer of a layered model on the device.
+// What stands around one sublayer of a layered model: its norm, then either the per-channel scale of a norm
+// behind it, or the hyper-connections' weights.
+struct Around {
+    const float *norm = nullptr, *ls = nullptr;
+    const float *in = nullptr, *out = nullptr, *mix = nullptr;
+};
+// One layer of a layered model on the device (one that uses another's tensors holds none).
 struct LayeredLayer {
     LayerSpec spec;
     Weight in, o, up, down;  // fused input projection, output projection; up: interleaved (gate, up) rows
     Weight uq, ukv;          // latent attention: query expansion; key and value expansions, one behind the other
     DeltaParams delta{};
     const float *dq_norm = nullptr, *dkv_norm = nullptr;
-    const float *norm1 = nullptr, *ls1 = nullptr, *norm2 = nullptr, *ls2 = nullptr;
+    MemoryParams memory{};
+    const float *wqk = nullptr;  // shared keys and values: query norm weight * key norm weight
+    Around around_mixer, around_ff;
     DeltaDims delta_dims() const;
     LatentDims latent_dims() const;
+    MemoryDims memory_dims() const;
+    SharedKvDims shared_dims() const;
 };
 struct LayeredStack {
     LayeredConfig cfg;
     std::vector<LayeredLayer> layers;
     float *small = nullptr;  // every f32 vector of every layer
     ~LayeredStack();
+    const LayeredLayer &weights(size_t l) const { return layers[cfg.layers[l].source]; }
 };
 // What the sequences of a session carry from token to token, layer by layer: matrix states and
-// convolution rings of recurrent layers, rings of cached latents of attention layers.
+// convolution rings of recurrent layers, rings of cached rows of attention layers.
 struct LayeredState {
     struct Layer {
         DeltaState delta{};
-        LatentCache latent{};
+        MemoryState memory{};
+        RowRing ring{};  // latents, or keys that are also the values
     };
     std::vector<Layer> layers;
     DeviceBuf mem;
@@ -66,7 +78,8 @@ struct Model;
 struct Workspace {
     uint64_t rows = 0;
     DeviceBuf h, x, qkv, att, ff, ids, a_lp, b_lp, w_lp, logits, xq, norm_part, gemm_part;
-    DeviceBuf mix, lat, q_lp, kv_lp;  // layered models: mixer operands, latents, 16-bit queries / keys and values
+    DeviceBuf mix, lat, q_lp, kv_lp;  // layered models: mixer operands, cached and new rows, queries / keys and values
+    DeviceBuf streams;                // hyper-connections: [rows][streams][hidden]
     GemmScratch gs;
     int ensure(const Model &m, uint64_t rows_needed, uint64_t logit_rows);
     void release();
@@ -96,8 +109,16 @@ struct Model {
     // HBM that resident f16 copies of quantised weights may still take (prefill matmul operands)
     static constexpr uint64_t kExpandBudget = 64ull << 30;
     uint64_t expand_budget = kExpandBudget;
+    float embed_scale = 1.f, logit_softcap = 0.f;
     std::unique_ptr<LayeredStack> stack;  // set: the blocks are the stack's layers, not `layers`
     ~Model();
+    uint32_t streams() const { return stack && stack->cfg.streams ? (uint32_t)stack->cfg.streams : 1; }
+    Epilogue logits_epilogue(float *dst) const {
+        Epilogue e;
+        e.out_f32 = dst;
+        if (logit_softcap > 0.f) { e.act = COEUS_EPI_SOFTCAP; e.limit = logit_softcap; }
+        return e;
+    }
 };
 
 struct Session {

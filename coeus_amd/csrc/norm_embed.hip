@@ -7,6 +7,7 @@
 //                         scale/bias indexed i % hidden.
 //   embed_kernel          x[s,:] = E[id_s,:] + PE[pos0+s,:]  (MT:812-835)
 //   norm_residual_kernel  h += RMSNorm(y) * layer_scale: norms that stand behind a sublayer
+//   hyper_kernel          hyper-connections: the sublayer's output into the streams, the next one's input
 #include "device_utils.hpp"
 
 namespace coeus {
@@ -84,7 +85,7 @@ __global__ __launch_bounds__(256) void norm_token_kernel(const float *__restrict
             const float4 sc = *(const float4 *)(scale + 4 * i);
             float o[4] = {sc.x * (v[u].x - mean) * rs, sc.y * (v[u].y - mean) * rs,
                           sc.z * (v[u].z - mean) * rs, sc.w * (v[u].w - mean) * rs};
-            if (!RMS) {
+            if (!RMS && bias) {
                 const float4 bi = *(const float4 *)(bias + 4 * i);
                 o[0] += bi.x; o[1] += bi.y; o[2] += bi.z; o[3] += bi.w;
             }
@@ -117,7 +118,7 @@ __global__ __launch_bounds__(256) void norm_token_kernel(const float *__restrict
     const float sd = sqrtf(var + eps);
     for (uint64_t i = threadIdx.x; i < hidden; i += blockDim.x) {
         float v = scale[i] * (xr[i] - mean) / sd;
-        if (!RMS) v += bias[i];
+        if (!RMS && bias) v += bias[i];
         if (y) y[row * hidden + i] = v;
         if (y_xq) y_xq[xq_index(i, (uint32_t)row, bp)] = __float2half_rn(v);
         if (y_lp) y_lp[row * lp_ld + i] = f32_to_lp_bits(v, lp_bf16);
@@ -167,7 +168,7 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(const float *__restrict_
         const float4 sc = *(const float4 *)(scale + 4 * i);
         float o[4] = {sc.x * (v[u].x - mean) * rs, sc.y * (v[u].y - mean) * rs,
                       sc.z * (v[u].z - mean) * rs, sc.w * (v[u].w - mean) * rs};
-        if (!RMS) {
+        if (!RMS && bias) {
             const float4 bi = *(const float4 *)(bias + 4 * i);
             o[0] += bi.x; o[1] += bi.y; o[2] += bi.z; o[3] += bi.w;
         }
@@ -391,6 +392,158 @@ int launch_norm_residual(const float *y, uint64_t rows, uint64_t hidden, const f
     return COEUS_OK;
 }
 
+// Hyper-connections (launch_hyper).  One workgroup per row of up to 4 * blockDim.x * VM elements (a multiple of
+// 4): the streams pass through registers 16 bytes at a time, the weighted sum stays there for the norm.
+// SMAX >= streams.  out may be h.y itself (a thread reads y where it writes out).
+template <int SMAX, int VM>
+__global__ __launch_bounds__(256) void hyper_kernel(float *__restrict__ x, uint32_t hidden, HyperStep h, float *out,
+                                                    uint16_t *__restrict__ out_lp, uint64_t lp_ld, bool lp_bf16) {
+    __shared__ float sh[16];
+    const uint64_t row = blockIdx.x;
+    const uint32_t n4 = hidden / 4, S = h.streams;
+    float *xr = x + row * S * hidden;
+    float4 v[VM];
+    float s1 = 0.f;
+#pragma unroll
+    for (int u = 0; u < VM; u++) {
+        const uint32_t i = threadIdx.x + blockDim.x * u;
+        v[u] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (i >= n4) continue;
+        float4 a[SMAX];
+#pragma unroll
+        for (int s = 0; s < SMAX; s++)
+            if (s < (int)S) a[s] = *(const float4 *)(xr + (uint64_t)s * hidden + 4 * i);
+        if (h.y) {
+            const float4 y = *(const float4 *)(h.y + row * hidden + 4 * i);
+#pragma unroll
+            for (int t = 0; t < SMAX; t++) {
+                if (t >= (int)S) continue;
+                const float o = h.mult * h.out[t], w = h.in ? h.in[t] : 1.0f;
+                float4 b = make_float4(o * y.x, o * y.y, o * y.z, o * y.w);
+#pragma unroll
+                for (int s = 0; s < SMAX; s++) {
+                    if (s >= (int)S) continue;
+                    const float m = h.mix[s * S + t];
+                    b.x = fmaf(m, a[s].x, b.x); b.y = fmaf(m, a[s].y, b.y);
+                    b.z = fmaf(m, a[s].z, b.z); b.w = fmaf(m, a[s].w, b.w);
+                }
+                *(float4 *)(xr + (uint64_t)t * hidden + 4 * i) = b;
+                v[u].x = fmaf(w, b.x, v[u].x); v[u].y = fmaf(w, b.y, v[u].y);
+                v[u].z = fmaf(w, b.z, v[u].z); v[u].w = fmaf(w, b.w, v[u].w);
+            }
+        } else {
+#pragma unroll
+            for (int t = 0; t < SMAX; t++) {
+                if (t >= (int)S) continue;
+                const float w = h.in ? h.in[t] : 1.0f;
+                v[u].x = fmaf(w, a[t].x, v[u].x); v[u].y = fmaf(w, a[t].y, v[u].y);
+                v[u].z = fmaf(w, a[t].z, v[u].z); v[u].w = fmaf(w, a[t].w, v[u].w);
+            }
+        }
+        s1 += (v[u].x + v[u].y) + (v[u].z + v[u].w);
+    }
+    float mean = 0.f, rs = 1.0f;
+    if (h.norm) {
+        mean = block_sum(s1, sh) / (float)hidden;
+        float s2 = 0.f;
+#pragma unroll
+        for (int u = 0; u < VM; u++) {
+            if (threadIdx.x + blockDim.x * u >= n4) continue;
+            const float d0 = v[u].x - mean, d1 = v[u].y - mean, d2 = v[u].z - mean, d3 = v[u].w - mean;
+            s2 = fmaf(d0, d0, s2); s2 = fmaf(d1, d1, s2); s2 = fmaf(d2, d2, s2); s2 = fmaf(d3, d3, s2);
+        }
+        rs = 1.0f / sqrtf(block_sum(s2, sh) / (float)hidden + h.eps);
+    }
+#pragma unroll
+    for (int u = 0; u < VM; u++) {
+        const uint32_t i = threadIdx.x + blockDim.x * u;
+        if (i >= n4) continue;
+        const float4 sc = h.norm ? *(const float4 *)(h.norm + 4 * i) : make_float4(1.f, 1.f, 1.f, 1.f);
+        const float4 o = make_float4((v[u].x - mean) * rs * sc.x, (v[u].y - mean) * rs * sc.y, (v[u].z - mean) * rs * sc.z,
+                                     (v[u].w - mean) * rs * sc.w);
+        if (out) *(float4 *)(out + row * hidden + 4 * i) = o;
+        if (out_lp) {
+            uint2 p;
+            p.x = (uint32_t)f32_to_lp_bits(o.x, lp_bf16) | ((uint32_t)f32_to_lp_bits(o.y, lp_bf16) << 16);
+            p.y = (uint32_t)f32_to_lp_bits(o.z, lp_bf16) | ((uint32_t)f32_to_lp_bits(o.w, lp_bf16) << 16);
+            *(uint2 *)(out_lp + row * lp_ld + 4 * i) = p;
+        }
+    }
+}
+
+// The same for any width whose row fits in LDS.
+__global__ __launch_bounds__(256) void hyper_any_kernel(float *__restrict__ x, uint32_t hidden, HyperStep h, float *out,
+                                                        uint16_t *__restrict__ out_lp, uint64_t lp_ld, bool lp_bf16) {
+    extern __shared__ float lds_row[];
+    __shared__ float sh[16];
+    const uint64_t row = blockIdx.x;
+    const uint32_t S = h.streams;
+    float *xr = x + row * S * hidden;
+    float s1 = 0.f;
+    for (uint32_t i = threadIdx.x; i < hidden; i += blockDim.x) {
+        float a[kMaxHyperStreams], v = 0.f;
+#pragma unroll
+        for (int s = 0; s < (int)kMaxHyperStreams; s++) a[s] = s < (int)S ? xr[(uint64_t)s * hidden + i] : 0.f;
+        const float y = h.y ? h.y[row * hidden + i] : 0.f;
+#pragma unroll
+        for (int t = 0; t < (int)kMaxHyperStreams; t++) {
+            if (t >= (int)S) continue;
+            float b = a[t];
+            if (h.y) {
+                b = h.mult * h.out[t] * y;
+#pragma unroll
+                for (int s = 0; s < (int)kMaxHyperStreams; s++)
+                    if (s < (int)S) b = fmaf(h.mix[s * S + t], a[s], b);
+                xr[(uint64_t)t * hidden + i] = b;
+            }
+            v = fmaf(h.in ? h.in[t] : 1.0f, b, v);
+        }
+        lds_row[i] = v;
+        s1 += v;
+    }
+    float mean = 0.f, rs = 1.0f;
+    if (h.norm) {
+        mean = block_sum(s1, sh) / (float)hidden;
+        float s2 = 0.f;
+        for (uint32_t i = threadIdx.x; i < hidden; i += blockDim.x) s2 = fmaf(lds_row[i] - mean, lds_row[i] - mean, s2);
+        rs = 1.0f / sqrtf(block_sum(s2, sh) / (float)hidden + h.eps);
+    }
+    for (uint32_t i = threadIdx.x; i < hidden; i += blockDim.x) {
+        const float o = (lds_row[i] - mean) * rs * (h.norm ? h.norm[i] : 1.0f);
+        if (out) out[row * hidden + i] = o;
+        if (out_lp) out_lp[row * lp_ld + i] = f32_to_lp_bits(o, lp_bf16);
+    }
+}
+
+int launch_hyper(float *x, uint64_t rows, uint64_t hidden, const HyperStep &h, float *u, const LpOut *u_lp, hipStream_t st) {
+    if (rows == 0 || rows > 0x7fffffffull || hidden == 0 || hidden > 32768 || h.streams == 0 || h.streams > kMaxHyperStreams ||
+        (h.y && (!h.mix || !h.out)) || (!u && !u_lp))
+        return fail(COEUS_INVALID_INPUT, "hyper-connections: bad shape or arguments");
+    uint16_t *lp = u_lp ? (uint16_t *)u_lp->p : nullptr;
+    const uint64_t ld = u_lp ? u_lp->ld : 0;
+    const bool bf = u_lp && u_lp->bf16;
+    const dim3 grid((unsigned)rows);
+    if ((hidden & 3) == 0 && hidden <= 8192 && (ld & 3) == 0) {
+        const uint64_t n4 = hidden / 4, threads = std::min<uint64_t>(256, round_up(n4, 64)), vm = ceil_div(n4, threads);
+#define COEUS_HY2(SV, VV) \
+    hipLaunchKernelGGL((hyper_kernel<SV, VV>), grid, dim3((unsigned)threads), 0, st, x, (uint32_t)hidden, h, u, lp, ld, bf)
+#define COEUS_HY(SV) do { if (vm <= 2) COEUS_HY2(SV, 2); else if (vm <= 4) COEUS_HY2(SV, 4); else COEUS_HY2(SV, 8); } while (0)
+        if (h.streams <= 2) COEUS_HY(2);
+        else if (h.streams == 3) COEUS_HY(3);
+        else if (h.streams == 4) COEUS_HY(4);
+        else COEUS_HY(8);
+#undef COEUS_HY
+#undef COEUS_HY2
+    } else {
+        static const bool once = hipFuncSetAttribute((const void *)hyper_any_kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                                     128 * 1024) == hipSuccess;
+        (void)once;
+        hipLaunchKernelGGL(hyper_any_kernel, grid, dim3(256), hidden * 4, st, x, (uint32_t)hidden, h, u, lp, ld, bf);
+    }
+    COEUS_HIP(hipGetLastError());
+    return COEUS_OK;
+}
+
 // dst[i, :] = src[rows[i], :]
 __global__ __launch_bounds__(256) void gather_rows_kernel(const float *__restrict__ src, const uint64_t *__restrict__ rows,
                                                           uint64_t hidden, float *__restrict__ dst) {
@@ -414,7 +567,8 @@ __global__ __launch_bounds__(1024) void embed_kernel(const void *__restrict__ ta
                                                      const uint64_t *__restrict__ ids, uint64_t pos0,
                                                      const uint32_t *pos_dev, uint32_t rows_per_seq,
                                                      uint64_t hidden, float *x, float2 *stats,
-                                                     const float *__restrict__ g_scale, float *g_out) {
+                                                     const float *__restrict__ g_scale, float *g_out,
+                                                     float scale, uint32_t copies) {
     const uint64_t row = blockIdx.x;
     const uint64_t id = ids[row];
     const uint64_t pos = (pos_dev ? (uint64_t)*pos_dev : pos0) + row % rows_per_seq;
@@ -432,7 +586,7 @@ __global__ __launch_bounds__(1024) void embed_kernel(const void *__restrict__ ta
             if (i < hidden) {
                 const float ev = BF16 ? bf16_bits_to_f32(((const uint16_t *)table)[id * hidden + i])
                                       : ((const float *)table)[id * hidden + i];
-                v[u] = pe ? ev + pe[pos * hidden + i] : ev;
+                v[u] = pe ? ev + pe[pos * hidden + i] : ev * scale;
             }
         }
 #pragma unroll
@@ -440,7 +594,8 @@ __global__ __launch_bounds__(1024) void embed_kernel(const void *__restrict__ ta
             const uint64_t i0 = g0 + (uint64_t)u * blockDim.x, i = i0 + (threadIdx.x & 15);
             if (i0 >= hidden) break;  // the same for the 16 lanes of a group
             const bool live = i < hidden;
-            if (live) x[row * hidden + i] = v[u];
+            if (live)
+                for (uint32_t c = 0; c < copies; c++) x[(row * copies + c) * hidden + i] = v[u];
             if (live && g_out) g_out[row * hidden + i] = v[u] * g_scale[i];
             if (stats) {
                 const uint64_t left = hidden - i0;
@@ -453,18 +608,21 @@ __global__ __launch_bounds__(1024) void embed_kernel(const void *__restrict__ ta
 
 int launch_embed(const void *table, bool table_bf16, const float *pe, const uint64_t *ids,
                  uint64_t rows, uint64_t rows_per_seq, uint64_t pos0, const uint32_t *pos_dev,
-                 uint64_t hidden, float *x, float2 *stats, hipStream_t st, const float *g_scale, float *g_out) {
+                 uint64_t hidden, float *x, float2 *stats, hipStream_t st, const float *g_scale, float *g_out, float scale,
+                 uint32_t copies) {
     if (rows == 0) return fail(COEUS_INVALID_INPUT, "empty embedding input");
     if (g_out && !g_scale) return fail(COEUS_INVALID_INPUT, "pre-scaled rows need the scale");
+    if (copies == 0 || ((stats || g_out) && copies != 1) || (pe && scale != 1.f))
+        return fail(COEUS_INVALID_INPUT, "embedding: bad combination of arguments");
     // one lane per element up to 1024 (whole groups of 16); few rows (a decode step) are bound
     // by latency, many rows (a prompt) by the number of workgroups, which 256 lanes serve better
     const unsigned threads = rows > 64 ? 256u : (unsigned)std::min<uint64_t>(1024, round_up(hidden, 64));
     if (table_bf16)
         hipLaunchKernelGGL(embed_kernel<true>, dim3((unsigned)rows), dim3(threads), 0, st, table, pe, ids,
-                           pos0, pos_dev, (uint32_t)rows_per_seq, hidden, x, stats, g_scale, g_out);
+                           pos0, pos_dev, (uint32_t)rows_per_seq, hidden, x, stats, g_scale, g_out, scale, copies);
     else
         hipLaunchKernelGGL(embed_kernel<false>, dim3((unsigned)rows), dim3(threads), 0, st, table, pe, ids,
-                           pos0, pos_dev, (uint32_t)rows_per_seq, hidden, x, stats, g_scale, g_out);
+                           pos0, pos_dev, (uint32_t)rows_per_seq, hidden, x, stats, g_scale, g_out, scale, copies);
     COEUS_HIP(hipGetLastError());
     return COEUS_OK;
 }

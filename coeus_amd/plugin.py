@@ -344,7 +344,8 @@ class LayeredModelPlugin:
         return (0, 1, 0)
 
     def capabilities(self):
-        return ("model_building", "gated_delta_rule", "latent_attention", "sliding_window")
+        return ("model_building", "gated_delta_rule", "latent_attention", "sliding_window", "matrix_memory",
+                "shared_key_value_attention", "hyper_connections")
 
     def create_builder(self):
         return LayeredModelBuilder()

@@ -310,7 +310,11 @@ int coeus_weight_dequantize(const coeus_weight *w, float *host_out);
 uint64_t coeus_weight_bytes(const coeus_weight *w);
 void coeus_weight_destroy(coeus_weight *w);
 
-enum { COEUS_EPI_NONE = 0, COEUS_EPI_GELU = 1, COEUS_EPI_SILU_GATE = 2 };
+enum { COEUS_EPI_NONE = 0, COEUS_EPI_GELU = 1, COEUS_EPI_SILU_GATE = 2,
+       /* with a limit of their own (coeus_op_matmul_limited), f32 and bf16 weights only: the clamped gate
+        * g sigmoid(1.702 g) (u + 1) of g = min(gate_j, limit), u = clamp(up_j, -limit, limit), rows interleaved
+        * like COEUS_EPI_SILU_GATE's; and limit * tanh(y / limit) */
+       COEUS_EPI_CLAMP_GATE = 3, COEUS_EPI_SOFTCAP = 4 };
 
 /* y[b, :] = epilogue(x[b, :] . W + bias) (+ residual[b, :]) for b < batch <= 16: the decode
  * matmul (MT:50-74 with m = batch).  x_dev [batch, k_in] f32, y_dev [batch, n_out] f32.
