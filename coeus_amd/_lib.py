@@ -15,7 +15,7 @@ NORM_LAYERNORM, NORM_RMSNORM = 0, 1
 SCOPE_SEQUENCE, SCOPE_TOKEN = 0, 1
 W_F32, W_BF16, W_Q8_0, W_Q4_0 = 0, 1, 2, 3
 KV_F32, KV_F16, KV_BF16 = 0, 1, 2
-EPI_NONE, EPI_GELU, EPI_SILU_GATE = 0, 1, 2
+EPI_NONE, EPI_GELU, EPI_SILU_GATE, EPI_CLAMP_GATE, EPI_SOFTCAP = 0, 1, 2, 3, 4
 MERGE_IN_KERNEL, MERGE_SEPARATE = 0, 1
 
 
@@ -55,6 +55,24 @@ class CDeltaWeights(C.Structure):
 
 class CLatentShape(C.Structure):
     _fields_ = [(f, C.c_uint64) for f in ("heads", "dim", "vdim", "q_rank", "kv_rank", "window")] + [("scale", C.c_float)]
+
+
+class CHyperStep(C.Structure):
+    _fields_ = ([("streams", C.c_uint64)] + [(f, C.c_void_p) for f in ("y_dev", "mix_dev", "out_dev", "in_dev", "norm_dev")] +
+                [("mult", C.c_float), ("eps", C.c_float)])
+
+
+class CMemoryShape(C.Structure):
+    _fields_ = [(f, C.c_uint64) for f in ("heads", "dim", "vdim", "in_ld")] + [("gate_cap", C.c_float)]
+
+
+class CMemoryWeights(C.Structure):
+    _fields_ = [(f, C.c_void_p) for f in ("in_bias_dev", "forget_bias_dev", "norm_dev")] + [("eps", C.c_float)]
+
+
+class CSharedKvShape(C.Structure):
+    _fields_ = ([(f, C.c_uint64) for f in ("heads", "kv_heads", "dim", "window", "in_ld")] +
+                [("scale", C.c_float), ("slope_range", C.c_float)])
 
 
 # name -> (restype, argtypes); this table is also what the symbol-export test walks
@@ -141,6 +159,7 @@ SIGNATURES = {
     "coeus_op_norm_gemv": (C.c_int, [_vp, _vp, _u64, _u32, _vp, _vp, _f32, _vp, _vp, _u32, _vp, C.POINTER(C.c_int),
                                      _vp]),
     "coeus_op_gemm": (C.c_int, [_vp, _vp, _u64, _vp, _vp, _u32, _vp, _vp]),
+    "coeus_op_matmul_limited": (C.c_int, [_vp, _vp, _u64, C.c_int, _u32, _f32, _vp, _vp]),
     "coeus_op_gemm_timed": (C.c_int, [_vp, _vp, _u64, _u32, _vp, _u32, _vp, _vp]),
     "coeus_op_norm": (C.c_int, [_u32, _u32, _vp, _u64, _u64, _vp, _vp, _f32, _vp, _vp]),
     "coeus_op_embed": (C.c_int, [_vp, _vp, _vp, _u64, _u64, _u64, _vp, _vp]),
@@ -156,6 +175,15 @@ SIGNATURES = {
     "coeus_op_window_attention": (C.c_int, [C.POINTER(CLatentShape), _u32, _vp, _vp, _u64, _u64, _u64, _vp, _vp]),
     "coeus_op_latent_decode": (C.c_int, [C.POINTER(CLatentShape), _u32, _vp, _vp, _vp, _f32, _vp, _vp, _u64, _u64, _u64, _vp,
                                          _vp]),
+    "coeus_op_hyper": (C.c_int, [C.POINTER(CHyperStep), _vp, _u64, _u64, _vp, _vp]),
+    "coeus_op_hyper_gemv": (C.c_int, [_vp, C.POINTER(CHyperStep), _vp, _u64, _vp, _u32, _f32, _vp, _vp]),
+    "coeus_op_memory_prompt": (C.c_int, [C.POINTER(CMemoryShape), C.POINTER(CMemoryWeights), _vp, _vp, _vp, _vp, _u64, _u64,
+                                         C.c_int, _vp, _vp]),
+    "coeus_op_memory_step": (C.c_int, [C.POINTER(CMemoryShape), C.POINTER(CMemoryWeights), _vp, _vp, _vp, _vp, _u64, _vp, _vp]),
+    "coeus_shared_kv_row_len": (_u64, [_u64, _u64]),
+    "coeus_op_shared_kv_prompt": (C.c_int, [C.POINTER(CSharedKvShape), _u32, _vp, _vp, _f32, _vp, _u64, _u64, _u64, _u64, _vp,
+                                            _vp]),
+    "coeus_op_shared_kv_decode": (C.c_int, [C.POINTER(CSharedKvShape), _u32, _vp, _vp, _f32, _vp, _u64, _u64, _u64, _vp, _vp]),
 }
 
 _lib = None

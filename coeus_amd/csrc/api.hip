@@ -461,19 +461,14 @@ int coeus_op_norm_gemv(const coeus_weight *w, const float *h_dev, uint64_t batch
     COEUS_GUARD_END
 }
 
-int coeus_op_gemm(const coeus_weight *w, const float *a_dev, uint64_t m, const float *bias_dev,
-                  const float *residual_dev, uint32_t epilogue, float *c_dev, void *stream) {
-    COEUS_GUARD_BEGIN
-    if (!w || !a_dev || !c_dev) return fail(COEUS_INVALID_INPUT, "null pointer argument");
-    if (epilogue > COEUS_EPI_SILU_GATE) return fail(COEUS_INVALID_INPUT, "unknown epilogue %u", epilogue);
-    hipStream_t st = (hipStream_t)stream;
-    const Epilogue e = make_user_epilogue(bias_dev, residual_dev, epilogue, c_dev);
+// Staging and split buffers live as long as the call.
+static int run_gemm(const Weight &w, const float *a_dev, uint64_t m, const Epilogue &e, hipStream_t st) {
     GemmScratch scr;
     DeviceBuf a_lp, w_lp, part;
-    if (w->w.dtype != COEUS_W_F32) {
-        COEUS_TRY(a_lp.ensure(m * gemm_ld(w->w.k) * 2));
-        if (w->w.dtype >= COEUS_W_Q8_0) {
-            int rc = w_lp.ensure(w->w.n * gemm_ld(w->w.k) * 2);
+    if (w.dtype != COEUS_W_F32) {
+        COEUS_TRY(a_lp.ensure(m * gemm_ld(w.k) * 2));
+        if (w.dtype >= COEUS_W_Q8_0) {
+            int rc = w_lp.ensure(w.n * gemm_ld(w.k) * 2);
             if (rc != COEUS_OK) { a_lp.release(); return rc; }
         }
         scr.a_lp = a_lp.p; scr.a_lp_bytes = a_lp.bytes;
@@ -481,10 +476,10 @@ int coeus_op_gemm(const coeus_weight *w, const float *a_dev, uint64_t m, const f
     }
     // (a launch of few tiles is split along k when it has room for the partial products; without
     // the room it runs unsplit)
-    if (const uint64_t pb = gemm_split_scratch_bytes(w->w, m))
+    if (const uint64_t pb = gemm_split_scratch_bytes(w, m))
         if (part.ensure(pb) != COEUS_OK) part.release();
     scr.partials = (float *)part.p; scr.partials_bytes = part.bytes;
-    int rc = launch_gemm(w->w, a_dev, m, e, scr, st);
+    int rc = launch_gemm(w, a_dev, m, e, scr, st);
     if (a_lp.p || w_lp.p || part.p) {
         // the staging buffers die with this call: wait for the kernels that read them
         hipError_t se = hipStreamSynchronize(st);
@@ -494,6 +489,35 @@ int coeus_op_gemm(const coeus_weight *w, const float *a_dev, uint64_t m, const f
         if (rc == COEUS_OK && se != hipSuccess) rc = fail(COEUS_DEVICE_ERROR, "matmul failed: %s", hipGetErrorString(se));
     }
     return rc;
+}
+
+int coeus_op_gemm(const coeus_weight *w, const float *a_dev, uint64_t m, const float *bias_dev,
+                  const float *residual_dev, uint32_t epilogue, float *c_dev, void *stream) {
+    COEUS_GUARD_BEGIN
+    if (!w || !a_dev || !c_dev) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    if (epilogue > COEUS_EPI_SILU_GATE) return fail(COEUS_INVALID_INPUT, "unknown epilogue %u", epilogue);
+    return run_gemm(w->w, a_dev, m, make_user_epilogue(bias_dev, residual_dev, epilogue, c_dev), (hipStream_t)stream);
+    COEUS_GUARD_END
+}
+
+static int limited_epilogue(uint32_t epilogue, float limit, float *y, Epilogue &e) {
+    if (epilogue != COEUS_EPI_NONE && epilogue != COEUS_EPI_CLAMP_GATE && epilogue != COEUS_EPI_SOFTCAP)
+        return fail(COEUS_INVALID_INPUT, "epilogue %u has no limit", epilogue);
+    if (epilogue != COEUS_EPI_NONE && !(limit > 0.f)) return fail(COEUS_INVALID_INPUT, "an epilogue's limit must be positive");
+    e = make_user_epilogue(nullptr, nullptr, epilogue, y);
+    e.limit = limit;
+    return COEUS_OK;
+}
+
+int coeus_op_matmul_limited(const coeus_weight *w, const float *x_dev, uint64_t rows, int prompt, uint32_t epilogue, float limit,
+                            float *y_dev, void *stream) {
+    COEUS_GUARD_BEGIN
+    if (!w || !x_dev || !y_dev) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    if (w->w.dtype >= COEUS_W_Q8_0) return fail(COEUS_INVALID_INPUT, "an epilogue with a limit takes f32 or bf16 weights");
+    Epilogue e;
+    COEUS_TRY(limited_epilogue(epilogue, limit, y_dev, e));
+    if (prompt) return run_gemm(w->w, x_dev, rows, e, (hipStream_t)stream);
+    return launch_gemv(w->w, x_dev, rows, e, (hipStream_t)stream);
     COEUS_GUARD_END
 }
 
@@ -834,6 +858,167 @@ int coeus_op_latent_decode(const coeus_latent_shape *shape, uint32_t kv_dtype, c
         rc = launch_latent_decode(q_dev, ukv_dev, dm, LatentNew{proj_dev, scale_dev, eps}, cache, batch, (const uint32_t *)p.p,
                                   out_dev, (float *)scratch.p, scratch.bytes, st);
     return finish_op(rc, st, {&p, &scratch}, "latent attention");
+    COEUS_GUARD_END
+}
+
+// ---- hyper-connections, matrix memory, attention whose values are its keys
+static int hyper_args(const coeus_hyper_step *h, HyperStep &out) {
+    if (!h) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    if (h->streams == 0 || h->streams > kMaxHyperStreams) return fail(COEUS_INVALID_INPUT, "hyper-connections: 1 to %u streams", kMaxHyperStreams);
+    if (h->y_dev && (!h->mix_dev || !h->out_dev)) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    out.streams = (uint32_t)h->streams;
+    out.y = h->y_dev; out.mix = h->mix_dev; out.out = h->out_dev;
+    out.in = h->in_dev; out.norm = h->norm_dev;
+    out.mult = h->mult; out.eps = h->eps;
+    return COEUS_OK;
+}
+
+int coeus_op_hyper(const coeus_hyper_step *step, float *x_dev, uint64_t rows, uint64_t hidden, float *u_dev, void *stream) {
+    COEUS_GUARD_BEGIN
+    HyperStep h;
+    COEUS_TRY(hyper_args(step, h));
+    if (!x_dev || !u_dev) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    hipStream_t st = (hipStream_t)stream;
+    return finish_op(launch_hyper(x_dev, rows, hidden, h, u_dev, nullptr, st), st, {}, "hyper-connections");
+    COEUS_GUARD_END
+}
+
+int coeus_op_hyper_gemv(const coeus_weight *w, const coeus_hyper_step *step, const float *x_dev, uint64_t batch, float *x_new_dev,
+                        uint32_t epilogue, float limit, float *y_dev, void *stream) {
+    COEUS_GUARD_BEGIN
+    HyperStep h;
+    COEUS_TRY(hyper_args(step, h));
+    if (!w || !x_dev || !y_dev || !h.in || !h.norm || (h.y && !x_new_dev)) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    if (w->w.dtype >= COEUS_W_Q8_0 || !gemv_can_fuse_hyper(w->w, batch, h.streams))
+        return fail(COEUS_INVALID_INPUT, "folded hyper-connections: weight type, width, batch or streams out of range");
+    Epilogue e;
+    COEUS_TRY(limited_epilogue(epilogue, limit, y_dev, e));
+    NormFuse nf;
+    nf.h = x_dev; nf.h_out = x_new_dev; nf.kind = COEUS_NORM_LAYERNORM; nf.eps = h.eps;
+    nf.scale = h.norm; nf.in = h.in; nf.streams = h.streams; nf.mult = h.mult;
+    nf.y = h.y; nf.mix = h.mix; nf.out = h.out;
+    hipStream_t st = (hipStream_t)stream;
+    return finish_op(launch_gemv(w->w, nullptr, batch, e, st, &nf), st, {}, "hyper-connections");
+    COEUS_GUARD_END
+}
+
+static bool memory_args(const coeus_memory_shape *s, const coeus_memory_weights *w, MemoryDims &dm, MemoryParams &pr) {
+    if (!s || !w || !w->in_bias_dev || !w->forget_bias_dev || !w->norm_dev) return false;
+    for (uint64_t v : {s->heads, s->dim, s->vdim, s->in_ld})
+        if (v > 0x7fffffffull) return false;
+    dm = MemoryDims{(uint32_t)s->heads, (uint32_t)s->dim, (uint32_t)s->vdim, (uint32_t)s->in_ld, s->gate_cap};
+    pr = MemoryParams{w->in_bias_dev, w->forget_bias_dev, w->norm_dev, w->eps};
+    return true;
+}
+
+int coeus_op_memory_prompt(const coeus_memory_shape *shape, const coeus_memory_weights *w, const float *proj_dev, float *state_dev,
+                           float *norm_state_dev, float *max_dev, uint64_t batch, uint64_t n, int chunked, float *out_dev,
+                           void *stream) {
+    COEUS_GUARD_BEGIN
+    MemoryDims dm;
+    MemoryParams pr;
+    if (!memory_args(shape, w, dm, pr) || !proj_dev || !state_dev || !norm_state_dev || !max_dev || !out_dev)
+        return fail(COEUS_INVALID_INPUT, "null pointer argument or size out of range");
+    if (batch == 0 || n == 0 || batch > 65535 || n > 0x7fffffffull)
+        return fail(COEUS_INVALID_INPUT, "matrix memory: %llu x %llu rows out of range", (unsigned long long)batch, (unsigned long long)n);
+    hipStream_t st = (hipStream_t)stream;
+    DeviceBuf scratch;
+    int rc = scratch.ensure(memory_prompt_scratch_bytes(dm, batch, n, chunked != 0));
+    if (rc == COEUS_OK)
+        rc = launch_memory_prompt(proj_dev, dm, pr, MemoryState{state_dev, norm_state_dev, max_dev}, batch, n, out_dev, nullptr,
+                                  (float *)scratch.p, scratch.bytes, st, chunked != 0);
+    return finish_op(rc, st, {&scratch}, "matrix memory");
+    COEUS_GUARD_END
+}
+
+int coeus_op_memory_step(const coeus_memory_shape *shape, const coeus_memory_weights *w, const float *proj_dev, float *state_dev,
+                         float *norm_state_dev, float *max_dev, uint64_t batch, float *out_dev, void *stream) {
+    COEUS_GUARD_BEGIN
+    MemoryDims dm;
+    MemoryParams pr;
+    if (!memory_args(shape, w, dm, pr) || !proj_dev || !state_dev || !norm_state_dev || !max_dev || !out_dev)
+        return fail(COEUS_INVALID_INPUT, "null pointer argument or size out of range");
+    hipStream_t st = (hipStream_t)stream;
+    return finish_op(launch_memory_step(proj_dev, dm, pr, MemoryState{state_dev, norm_state_dev, max_dev}, batch, out_dev, st), st, {},
+                     "matrix memory");
+    COEUS_GUARD_END
+}
+
+static int shared_kv_args(const coeus_shared_kv_shape *s, uint32_t kv_dtype, SharedKvDims &dm) {
+    if (!s) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    if (kv_dtype != COEUS_KV_BF16 && kv_dtype != COEUS_KV_F32)
+        return fail(COEUS_INVALID_INPUT, "shared keys and values: the ring must be bf16 or f32");
+    for (uint64_t v : {s->heads, s->kv_heads, s->dim, s->window, s->in_ld})
+        if (v > 0x3fffffffull) return fail(COEUS_INVALID_INPUT, "shared keys and values: sizes out of range");
+    if (!s->kv_heads || (s->heads + s->kv_heads) * s->dim > (1u << 24))
+        return fail(COEUS_INVALID_INPUT, "shared keys and values: sizes out of range");
+    dm = SharedKvDims{(uint32_t)s->heads, (uint32_t)s->kv_heads, (uint32_t)s->dim, (uint32_t)s->window, (uint32_t)s->in_ld, s->scale,
+                      s->slope_range};
+    return COEUS_OK;
+}
+
+uint64_t coeus_shared_kv_row_len(uint64_t kv_heads, uint64_t dim) {
+    if (kv_heads > (1u << 20) || dim > (1u << 20) || kv_heads * dim > (1u << 24)) return 0;
+    SharedKvDims dm{};
+    dm.kv_heads = (uint32_t)kv_heads;
+    dm.d = (uint32_t)dim;
+    return dm.row_len();
+}
+
+int coeus_op_shared_kv_prompt(const coeus_shared_kv_shape *shape, uint32_t kv_dtype, const float *proj_dev, const float *wqk_dev,
+                              float eps, void *ring_dev, uint64_t cap, uint64_t batch, uint64_t n, uint64_t pos0, float *out_dev,
+                              void *stream) {
+    COEUS_GUARD_BEGIN
+    SharedKvDims dm;
+    COEUS_TRY(shared_kv_args(shape, kv_dtype, dm));
+    if (!proj_dev || !wqk_dev || !ring_dev || !out_dev) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    const uint64_t hist = dm.window && dm.window - 1 < pos0 ? dm.window - 1 : pos0, krows = hist + n, rl = dm.row_len();
+    // (a ring shorter than the window holds the whole context)
+    if (cap == 0 || cap > 0x7fffffffull || batch == 0 || batch > 65535 || n == 0 || n > 0x3fffffffull || pos0 > 0x3fffffffull ||
+        (dm.window && cap > dm.window) || ((!dm.window || cap < dm.window) && pos0 + n > cap))
+        return fail(COEUS_INVALID_INPUT, "shared keys and values: rows or ring out of range");
+    hipStream_t st = (hipStream_t)stream;
+    const bool bf16 = kv_dtype == COEUS_KV_BF16;
+    const uint64_t es = bf16 ? 2 : 4;
+    const RowRing ring{ring_dev, (uint32_t)cap, bf16};
+    DeviceBuf q, kv;
+    int rc = q.ensure(batch * n * dm.heads * dm.d * es);
+    if (rc == COEUS_OK) rc = kv.ensure(batch * krows * rl * es);
+    if (rc == COEUS_OK) rc = launch_ring_gather(ring, (uint32_t)rl, batch, hist, pos0, kv.p, rl, krows, st);
+    if (rc == COEUS_OK) rc = launch_shared_kv_prepare(proj_dev, dm, wqk_dev, eps, batch, n, bf16, q.p, kv.p, krows, hist, st);
+    if (rc == COEUS_OK) rc = launch_ring_append(kv.p, rl, krows, hist, ring, (uint32_t)rl, batch, n, pos0, st);
+    if (rc == COEUS_OK)
+        rc = launch_window_attention(q.p, (uint64_t)dm.heads * dm.d, kv.p, rl, bf16, dm.window_shape(proj_dev + dm.gate_off()), batch, n,
+                                     hist, out_dev, nullptr, st);
+    return finish_op(rc, st, {&q, &kv}, "shared keys and values");
+    COEUS_GUARD_END
+}
+
+int coeus_op_shared_kv_decode(const coeus_shared_kv_shape *shape, uint32_t kv_dtype, const float *proj_dev, const float *wqk_dev,
+                              float eps, void *ring_dev, uint64_t cap, uint64_t batch, uint64_t pos, float *out_dev, void *stream) {
+    COEUS_GUARD_BEGIN
+    SharedKvDims dm;
+    COEUS_TRY(shared_kv_args(shape, kv_dtype, dm));
+    if (!proj_dev || !wqk_dev || !ring_dev || !out_dev) return fail(COEUS_INVALID_INPUT, "null pointer argument");
+    if (cap == 0 || cap > 0x7fffffffull || batch == 0 || batch > 65535 || (dm.window && cap > dm.window) ||
+        ((!dm.window || cap < dm.window) && pos >= cap))
+        return fail(COEUS_INVALID_INPUT, "shared keys and values: batch, position or ring out of range");
+    if (dm.heads == 0 || dm.heads % dm.kv_heads || dm.d == 0 || dm.d > 256)
+        return fail(COEUS_INVALID_INPUT, "shared keys and values: sizes out of range");
+    hipStream_t st = (hipStream_t)stream;
+    const RowRing ring{ring_dev, (uint32_t)cap, kv_dtype == COEUS_KV_BF16};
+    const uint64_t counters = shared_kv_decode_counters(dm, batch);
+    DeviceBuf p, scratch, cnt;
+    int rc = upload_position(pos, p, st);
+    if (rc == COEUS_OK) rc = scratch.ensure(shared_kv_decode_scratch_bytes(dm, ring, batch));
+    if (rc == COEUS_OK) rc = cnt.ensure(counters * 4);
+    if (rc == COEUS_OK) {
+        hipLaunchKernelGGL(clear_u32_kernel, dim3((unsigned)ceil_div(counters, 256)), dim3(256), 0, st, (uint32_t *)cnt.p,
+                           (uint32_t)counters);
+        rc = launch_shared_kv_decode(proj_dev, dm, wqk_dev, eps, ring, batch, (const uint32_t *)p.p, out_dev, (float *)scratch.p,
+                                     scratch.bytes, (uint32_t *)cnt.p, counters, st);
+    }
+    return finish_op(rc, st, {&p, &scratch, &cnt}, "shared keys and values");
     COEUS_GUARD_END
 }
 

@@ -197,12 +197,13 @@ int coeus_model_create(const coeus_config *cfg, const float *params, uint64_t n_
  * fixed init, MT:604-611); exists so multi-GB configurations need no host-side buffer. */
 int coeus_model_create_seeded(const coeus_config *cfg, uint64_t seed, coeus_model **out);
 /* ---- layered models (no counterpart in the reference) --------------------------------------
- * Decoders whose layers name their own token mixer: a gated delta rule with short convolutions, or
- * attention through low-rank latents in a sliding window.  A folder holds config.json (its
- * "architecture" selects the design from the library's registry: "Bofirax") and model.safetensors
- * (BF16 or F32).  The handle is a coeus_model like any other: coeus_model_forward*, sessions,
+ * Decoders whose layers name their own token mixer: "Bofirax" has a gated delta rule with short
+ * convolutions and attention through low-rank latents in a sliding window; "Zekilix" matrix memories and
+ * windowed attention whose values are its keys, between several residual streams, in layers that may share
+ * tensors.  A folder holds config.json (its "architecture" selects the design from the library's registry)
+ * and model.safetensors (BF16 or F32).  The handle is a coeus_model like any other: coeus_model_forward*, sessions,
  * generation and sampling work on it; coeus_model_config reports width, depth, vocabulary, storage
- * types and limits.  Weight storage COEUS_W_BF16 (16-bit matrix products, bf16 latents in the cache;
+ * types and limits.  Weight storage COEUS_W_BF16 (16-bit matrix products, bf16 latents or keys in the cache;
  * norms, recurrences, scores and the residual stream in f32) or COEUS_W_F32 (everything in f32). */
 typedef struct coeus_load_options {
     uint32_t weight_dtype; /* COEUS_W_BF16 or COEUS_W_F32 */
@@ -339,6 +340,10 @@ int coeus_op_norm_gemv(const coeus_weight *w, const float *h_dev, uint64_t batch
 /* C[m, n_out] = epilogue(A[m, k_in] . W + bias) (+ residual): the prefill matmul. */
 int coeus_op_gemm(const coeus_weight *w, const float *a_dev, uint64_t m, const float *bias_dev,
                   const float *residual_dev, uint32_t epilogue, float *c_dev, void *stream);
+/* The matmul with an epilogue that has a limit: COEUS_EPI_CLAMP_GATE, COEUS_EPI_SOFTCAP (or COEUS_EPI_NONE), f32
+ * and bf16 weights.  prompt 0: the decode matmul (rows <= 16), else the prefill matmul. */
+int coeus_op_matmul_limited(const coeus_weight *w, const float *x_dev, uint64_t rows, int prompt, uint32_t epilogue,
+                            float limit, float *y_dev, void *stream);
 /* Measurement variant of coeus_op_gemm (no reference counterpart; used by the benchmark's
  * matrix-core roofline): runs the staging conversions and one untimed matmul, then launches the
  * matmul kernel `reps` times between two events on `stream` and returns the elapsed
@@ -441,6 +446,68 @@ int coeus_op_latent_decode(const coeus_latent_shape *shape, uint32_t kv_dtype, c
                            const float *proj_dev, const float *scale_dev, float eps, const void *ukv_dev,
                            void *cache_dev, uint64_t cap, uint64_t batch, uint64_t pos, float *out_dev,
                            void *stream);
+/* Hyper-connections: rows of `streams` streams of `hidden` f32 elements.  A step takes the output y of the sublayer
+ * before into them, x_t <- sum_s mix[s][t] x_s + mult * out[t] * y (y_dev null: they stay), and forms what the
+ * next sublayer reads: u = sum_t in[t] x_t (in_dev null: all ones), then u's layer norm with weight norm_dev (null:
+ * u itself).  mix_dev [streams][streams], from first; out_dev, in_dev [streams]; at most 8 streams. */
+typedef struct coeus_hyper_step {
+    uint64_t streams;
+    const float *y_dev, *mix_dev, *out_dev, *in_dev, *norm_dev;
+    float mult, eps;
+} coeus_hyper_step;
+/* In place on x_dev [rows][streams][hidden]; u_dev [rows][hidden] (may be y_dev). */
+int coeus_op_hyper(const coeus_hyper_step *step, float *x_dev, uint64_t rows, uint64_t hidden, float *u_dev,
+                   void *stream);
+/* The same folded into the decode matmul that reads u, as decode steps run it (f32 and bf16 weights, at most 4
+ * streams): y_dev [batch][n_out] = epilogue(u . W), the new streams (if y_dev of the step is set) to
+ * x_new_dev, which must not be x_dev. */
+int coeus_op_hyper_gemv(const coeus_weight *w, const coeus_hyper_step *step, const float *x_dev, uint64_t batch,
+                        float *x_new_dev, uint32_t epilogue, float limit, float *y_dev, void *stream);
+/* Matrix memory.  proj_dev rows of in_ld floats hold q | k (heads x dim each) | v | gate (heads x vdim each) |
+ * input gate | forget gate (heads each) as the projections give them.  With c(z) = gate_cap tanh(z / gate_cap), per
+ * head i = c(input + in_bias), f = logsigmoid(c(forget + forget_bias)), q / sqrt(dim):
+ *   m' = max(f + m, i);  S <- e^(f + m - m') S + e^(i - m') k v^T;  n alike with k alone;  m <- m'
+ *   o = S^T q / (max(|n . q|, e^-m) + 1e-6);  out = o / rms(o) * norm * sigmoid(gate), norm_dev [heads * vdim].
+ * state_dev [batch][heads][dim][vdim], norm_state_dev [batch][heads][dim] and max_dev [batch][heads] hold S, n and
+ * m and are moved on; zeros start a sequence.  dim <= 512, vdim <= 1024. */
+typedef struct coeus_memory_shape {
+    uint64_t heads, dim, vdim, in_ld;
+    float gate_cap;
+} coeus_memory_shape;
+typedef struct coeus_memory_weights {
+    const float *in_bias_dev, *forget_bias_dev, *norm_dev;
+    float eps;
+} coeus_memory_weights;
+/* n new tokens per sequence: in chunks on the matrix cores when `chunked` is not zero and n and the sizes allow
+ * it, else token by token.  out_dev [batch * n, heads * vdim]. */
+int coeus_op_memory_prompt(const coeus_memory_shape *shape, const coeus_memory_weights *w, const float *proj_dev,
+                           float *state_dev, float *norm_state_dev, float *max_dev, uint64_t batch, uint64_t n,
+                           int chunked, float *out_dev, void *stream);
+/* One new token per sequence (a decode step's launch). */
+int coeus_op_memory_step(const coeus_memory_shape *shape, const coeus_memory_weights *w, const float *proj_dev,
+                         float *state_dev, float *norm_state_dev, float *max_dev, uint64_t batch, float *out_dev,
+                         void *stream);
+/* Attention whose values are its keys.  proj_dev rows of in_ld floats hold q (heads x dim) | k (kv_heads x dim) |
+ * gate (heads x dim).  q and k are RMS-normalised over all heads at once for the scores; wqk_dev [heads * dim] =
+ * the query norm's weight times the key norm's weight of the head it looks at.  score = (q . k) scale -
+ * slope(h) distance, slope(h) = 2^(-slope_range (h + 1) / heads) (slope_range 0: none); the values are k as
+ * projected; the outputs meet sigmoid(gate).  window as for latent attention. */
+typedef struct coeus_shared_kv_shape {
+    uint64_t heads, kv_heads, dim, window, in_ld;
+    float scale, slope_range;
+} coeus_shared_kv_shape;
+/* Elements of a cached row: the keys of all heads, and their inverse root mean square (an f32). */
+uint64_t coeus_shared_kv_row_len(uint64_t kv_heads, uint64_t dim);
+/* n new tokens per sequence at positions pos0 ..; ring_dev (kv_dtype) [batch][cap][row], position p in slot p % cap, is
+ * read and moved on (cap = window, or less where it holds the whole context; slots not written yet must hold
+ * finite values).  out_dev f32 [batch * n, heads * dim]. */
+int coeus_op_shared_kv_prompt(const coeus_shared_kv_shape *shape, uint32_t kv_dtype, const float *proj_dev,
+                              const float *wqk_dev, float eps, void *ring_dev, uint64_t cap, uint64_t batch,
+                              uint64_t n, uint64_t pos0, float *out_dev, void *stream);
+/* One new token per sequence at position pos. */
+int coeus_op_shared_kv_decode(const coeus_shared_kv_shape *shape, uint32_t kv_dtype, const float *proj_dev,
+                              const float *wqk_dev, float eps, void *ring_dev, uint64_t cap, uint64_t batch,
+                              uint64_t pos, float *out_dev, void *stream);
 /* Host-side sinusoidal table (MT:398-407), computed with the platform libm like the reference. */
 int coeus_positional_encoding(uint64_t max_seq_len, uint64_t hidden_dim, float *table_out);
 

@@ -192,13 +192,20 @@ def hyper_write(xs, mix, out, y, mult):
 HYPER_MIXERS = {"mlstm": memory_mixer, "attention": shared_kv_attention_mixer}
 
 
+def tensors_of(cfg, i):
+    """The layer whose tensors layer i uses."""
+    while cfg["layers"][i].get("weights_of") is not None:
+        i = cfg["layers"][i]["weights_of"]
+    return i
+
+
 def forward_hyper(cfg, W, tokens, dtype, layers_out):
     eps, mult = dtype(cfg["norm"]["eps"]), dtype(cfg["residual_mult"])
     x = W["embed"][np.asarray(tokens, dtype=np.int64)] * dtype(cfg["embedding"]["scale"])
     xs = np.stack([x] * cfg["streams"])
     for i, layer in enumerate(cfg["layers"]):
-        p = f"l{layer.get('weights_of', i)}"
-        subs = [(".hc1", ".norm1", lambda u: HYPER_MIXERS[layer["type"]](u, W, p + ".mix", layer["mixer"], eps))]
+        p = f"l{tensors_of(cfg, i)}"
+        subs = [(".hc1", ".norm1", lambda u: HYPER_MIXERS[layer["type"].split("_")[0]](u, W, p + ".mix", layer["mixer"], eps))]
         if layer["mlp"] is not None:
             subs.append((".hc2", ".norm2", lambda u: clamped_ff(u, W, p + ".mlp", layer["mlp"]["limit"])))
         for hc, norm, f in subs:

@@ -192,3 +192,21 @@ def test_rust_extern_declarations_match_the_header():
         for ret, params, f in variants:
             assert ret == c_ret, (f, name, ret, c_ret)
             assert params == c_params, (f, name, params, c_params)
+
+
+def test_layered_structs_match_the_header(tmp_path):
+    pairs = [(_lib.CLoadOptions, "coeus_load_options"), (_lib.CDeltaShape, "coeus_delta_shape"), (_lib.CDeltaWeights, "coeus_delta_weights"),
+             (_lib.CLatentShape, "coeus_latent_shape"), (_lib.CHyperStep, "coeus_hyper_step"), (_lib.CMemoryShape, "coeus_memory_shape"),
+             (_lib.CMemoryWeights, "coeus_memory_weights"), (_lib.CSharedKvShape, "coeus_shared_kv_shape")]
+    lines = ['#include <stddef.h>', '#include <stdio.h>', '#include "coeus.h"', 'int main(void) {']
+    for cls, name in pairs:
+        lines.append(f'  printf("{name} %zu\\n", sizeof({name}));')
+        lines += [f'  printf("{name}.{f} %zu\\n", offsetof({name}, {f}));' for f, _ in cls._fields_]
+    src, exe = tmp_path / "layout.c", tmp_path / "layout"
+    src.write_text("\n".join(lines + ['  return 0;', '}']))
+    subprocess.check_call(["gcc", "-std=c11", "-I", os.path.join(ROOT, "include"), str(src), "-o", str(exe)])
+    lay = dict(line.split() for line in subprocess.check_output([str(exe)], text=True).splitlines())
+    for cls, name in pairs:
+        assert C.sizeof(cls) == int(lay[name]), name
+        for f, _ in cls._fields_:
+            assert getattr(cls, f).offset == int(lay[f"{name}.{f}"]), (name, f)

@@ -10,7 +10,8 @@ from coeus_amd import BasicGenerationConfig, LayeredConfig, PLUGINS, ProcessingE
 from coeus_amd.device import DeviceArray
 from coeus_amd.plugin import _check
 from gpu_util import dev
-from layered_util import CONFIGS, bf16_round, config, delta, latent, weights, write_folder
+from layered_util import (BOFIRAX, CONFIGS, ZEKILIX, bf16_round, config, delta, hyper_config, latent, memory, shared_kv, weights,
+                          write_folder)
 from oracle import layered as L
 
 pytestmark = pytest.mark.gpu
@@ -328,10 +329,10 @@ def test_prompt_layers_and_logits(folder, name, dtype):
     assert max(rows) < 2.5 * LIMIT[dtype] and off(got[0], want) < LIMIT[dtype]
     assert off(m.forward(ids), want[-1]) < 2.5 * LIMIT[dtype]
     assert off(m.forward_all(ids[:70]), want[:70]) < LIMIT[dtype]
-    assert m.num_parameters() == sum(a.size for a in w.values()) and m.name() == "Bofirax"
+    assert m.num_parameters() == sum(a.size for a in w.values()) and m.name() == cfg["architecture"]
 
 
-@pytest.mark.parametrize("name", sorted(CONFIGS))
+@pytest.mark.parametrize("name", BOFIRAX)
 def test_the_limit_would_show_a_mistake(folder, name):
     """Mistakes planted in the oracle move its logits well beyond the limits of these tests."""
     _, cfg, w = folder(name)
@@ -350,6 +351,41 @@ def test_the_limit_would_show_a_mistake(folder, name):
         without = dict(w)
         without[f"l{i}.ls1"] = np.ones_like(w[f"l{i}.ls1"])
         assert off(L.forward(cfg, without, ids), right) > LIMIT["bf16"]
+
+
+@pytest.mark.parametrize("name", ZEKILIX)
+def test_the_limit_would_show_a_mistake_in_these(folder, name):
+    _, cfg, w = folder(name)
+    ids = tokens(cfg, 150)
+    right = L.forward(cfg, w, ids)
+
+    def moved(change=None, w2=None, at=slice(None), by=20 * LIMIT["f32"]):
+        c = json.loads(json.dumps(cfg))
+        if change:
+            change(c)
+        assert off(L.forward(c, w2 or w, ids)[at], right[at]) > by
+
+    moved(lambda c: c.update(residual_mult=1.01 * c["residual_mult"]))
+    moved(lambda c: c.update(logit_softcap=1.01 * c["logit_softcap"]))
+    moved(lambda c: c["embedding"].update(scale=1.01 * c["embedding"]["scale"]))
+    for i, layer in enumerate(cfg["layers"]):
+        m, p = layer["mixer"], f"l{L.tensors_of(cfg, i)}."
+        if "mask" in m:
+            moved(lambda c: c["layers"][i]["mixer"]["mask"].update(size=m["mask"]["size"] + 1), at=slice(100, None))
+        if "kv_heads" in m:
+            moved(lambda c: c["layers"][i]["mixer"].update(scale=1.02 * m["scale"]) if m.get("mask") != {"size": 1} else
+                  c.update(residual_mult=0.5 * c["residual_mult"]))
+        if "gate_cap" in m:
+            moved(lambda c: c["layers"][i]["mixer"].update(gate_cap=1.1 * m["gate_cap"]))
+        if layer["mlp"]:
+            moved(lambda c: c["layers"][i]["mlp"].update(limit=1.1 * layer["mlp"]["limit"]))
+        if cfg["streams"] > 1:
+            hc = p + ("hc2" if layer["mlp"] else "hc1")
+            moved(w2={**w, hc + ".mix": w[hc + ".mix"].T})
+            if i < len(cfg["layers"]) - 1:  # (behind the last one only their sum counts)
+                moved(w2={**w, hc + ".out": w[hc + ".out"][::-1]})
+            if i or layer["mlp"]:  # (the streams are equal in front of the first sublayer)
+                moved(w2={**w, hc + ".in": w[hc + ".in"][::-1]})
 
 
 @pytest.mark.parametrize("dtype", ["f32", "bf16"])
@@ -374,7 +410,7 @@ def test_decoding_and_portions(folder, name, dtype):
 
 
 @pytest.mark.parametrize("dtype", ["f32", "bf16"])
-@pytest.mark.parametrize("name", ["mixed", "odd", "wide"])
+@pytest.mark.parametrize("name", ["mixed", "odd", "wide", "hyper", "hyper_odd", "hyper_wide"])
 def test_batches_and_reused_sessions(folder, name, dtype):
     path, cfg, w = folder(name)
     m = load_model(path, weight_dtype=dtype, max_batch=3)
@@ -409,10 +445,11 @@ def oracle_greedy(cfg, w, ids, n):
     return out, margin
 
 
-def test_greedy_generation(folder):
+@pytest.mark.parametrize("name", ["mixed", "hyper", "hyper_odd"])
+def test_greedy_generation(folder, name):
     """The plugin's own generation (prompt pass, then graph-replayed steps past the windows) against greedy
     decoding of the oracle; graph replay against kernel-by-kernel launches, replayed again after a reset."""
-    path, cfg, w = folder("mixed")
+    path, cfg, w = folder(name)
     ids = tokens(cfg, 20, 2)
     want, margin = oracle_greedy(cfg, w, ids, 40)
     assert margin > 1e-4  # (no step hangs on a rounding)
@@ -433,18 +470,24 @@ def test_greedy_generation(folder):
             s.close()
 
 
-def test_sampling_is_reproducible(folder):
-    path, cfg, _ = folder("wide")
+@pytest.mark.parametrize("name", ["wide", "hyper_wide"])
+def test_sampling_is_reproducible(folder, name):
+    path, cfg, _ = folder(name)
     m = load_model(path, max_seq_len=128)
     ids, how = tokens(cfg, 12, 3), BasicGenerationConfig(max_length=30, temperature=12.0, top_k=20, top_p=0.9)
     a, b, c = (m.generate(ids, how, seed=s) for s in (1, 1, 2))
     assert a == b != c and len(a) == 30 and max(a) < cfg["vocab"]
 
 
+LONG = {"Bofirax": config(48, 60, [delta(2, 1, 16, 24, 4), latent(2, 16, 16, 24, 32, 19, ff=48), delta(2, 2, 12, 16, 3)]),
+        "Zekilix": hyper_config(48, 60, [memory(2, 16, 24), shared_kv(4, 2, 16, 19, ff=48), memory(3, 12, 16, cap=5.0)], 3)}
+
+
 @pytest.mark.parametrize("dtype", ["f32", "bf16"])
-def test_long_decoding(dtype, tmp_path):
-    """Hundreds of decoded tokens: the ring of latents comes round many times, the state keeps going."""
-    cfg = config(48, 60, [delta(2, 1, 16, 24, 4), latent(2, 16, 16, 24, 32, 19, ff=48), delta(2, 2, 12, 16, 3)])
+@pytest.mark.parametrize("design", sorted(LONG))
+def test_long_decoding(design, dtype, tmp_path):
+    """Hundreds of decoded tokens: the rings come round many times, the state keeps going."""
+    cfg = LONG[design]
     w = weights(cfg, 9)
     ids = tokens(cfg, 700, 4)
     want = L.forward(cfg, w, ids)
@@ -457,8 +500,9 @@ def test_long_decoding(dtype, tmp_path):
 
 
 @pytest.mark.parametrize("dtype", ["bfloat16", "float32"])
-def test_trace_program_on_a_model(folder, tmp_path, dtype):
-    path, cfg, w = folder("mixed")
+@pytest.mark.parametrize("name", ["mixed", "hyper"])
+def test_trace_program_on_a_model(folder, tmp_path, name, dtype):
+    path, cfg, w = folder(name)
     a, b = tokens(cfg, 40, 5), tokens(cfg, 31, 6)
     steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:30].tolist(), "want": [3, 29]}], "end": []}]
     steps += [{"step": 1 + i, "entries": [{"id": "a", "tokens": [int(a[30 + i])], "want": [0]}], "end": ["a"] if i == 9 else []}
