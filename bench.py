@@ -2,7 +2,7 @@
 """Headline benchmark: decode throughput of the transformer forward path on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload NAME] [--batch B]
-    python bench.py --layered [SIZE,..] [--steps K] [--warmup W] [--batch B]
+    python bench.py --layered [SIZE,..] [--design NAME] [--steps K] [--warmup W] [--batch B]
 
 Default workload (the 7B-shape configuration the headline target is stated on):
 7B-shape decoder, Q4_0 weights, f16 KV cache, batch 1, context filled to 4096.  A "step" is one
@@ -23,9 +23,11 @@ Prints ONE JSON line: whole-job tokens/s plus
                  Q4_0 decoder at batch 4): throughput, ms per step, the roofline of each one's
                  dominant kernel and what its outputs were checked against.
 
-With --layered it measures layered decoders instead (three gated-delta-rule layers to one windowed
-latent-attention layer, a gated feed-forward in each) beside the bf16 transformer of the same width,
-depth, heads and feed-forward: one JSON line with prompt and decode throughput of both.
+With --layered it measures layered decoders instead (three recurrent layers to one of windowed attention, a
+gated feed-forward in each) beside the bf16 transformer of the same width, depth, heads and feed-forward: one JSON
+line with prompt and decode throughput of each.  --design Bofirax (the default): gated delta rule and latent
+attention.  --design Zekilix: matrix memories and attention whose values are its keys, between four residual
+streams; the Bofirax of the same size is measured as well.
 """
 import argparse
 import json
@@ -353,8 +355,8 @@ LAYERED_SIZES = {"1024": (1024, 8, 4, 384, 256, 512, 2816, 12),
                  "4096": (4096, 32, 16, 1536, 512, 1024, 11008, 8)}
 
 
-def layered_pair(size, ctx, batch):
-    """(layered configuration, transformer configuration) of one size."""
+def layered_models(design, size, ctx):
+    """(name, family, configuration) of the models of one size that are measured together."""
     from coeus_amd import LayeredConfig, Transformer250MConfig
 
     W, H, KH, qr, kr, win, ff, L = LAYERED_SIZES[size]
@@ -362,21 +364,30 @@ def layered_pair(size, ctx, batch):
     d = {"type": "delta", "mixer": dict(heads=H, kv_heads=KH, dim=128, vdim=128, conv=4), "mlp": mlp}
     a = {"type": "latent_attention", "mlp": mlp,
          "mixer": dict(heads=H, dim=128, vdim=128, q_rank=qr, kv_rank=kr, scale=128 ** -0.5, mask={"size": win})}
-    cfg = {"architecture": "Bofirax", "vocab": 32000, "width": W, "norm": {"eps": 1e-5},
-           "layers": [a if i % 4 == 3 else d for i in range(L)]}
+    cfgs = {"Bofirax": {"architecture": "Bofirax", "vocab": 32000, "width": W, "norm": {"eps": 1e-5},
+                        "layers": [a if i % 4 == 3 else d for i in range(L)]}}
+    if design == "Zekilix":
+        mlp = {"kind": "dense", "ff": ff, "limit": 7.0}
+        d = {"type": "mlstm", "mixer": dict(heads=H, dim=128, vdim=128, gate_cap=15.0), "mlp": mlp}
+        a = {"type": "attention", "mlp": mlp,
+             "mixer": dict(heads=H, kv_heads=H // 4, dim=128, vdim=128, scale=128 ** -0.5, mask={"size": win})}
+        zek = {"architecture": "Zekilix", "vocab": 32000, "width": W, "norm": {"eps": 1e-5}, "streams": 4, "residual_mult": 0.5,
+               "embedding": {"scale": W ** 0.5}, "logit_softcap": 30.0, "layers": [a if i % 4 == 3 else d for i in range(L)]}
+        cfgs = {"Zekilix": zek, **cfgs}
     peer = Transformer250MConfig(hidden_dim=W, num_layers=L, num_heads=H, head_dim=128, intermediate_dim=ff, vocab_size=32000,
                                  max_seq_len=ctx, use_bias=False, activation="silu_gated", norm="rmsnorm", norm_scope="token",
                                  weight_dtype="bf16", kv_dtype="bf16", max_batch=16)
-    return LayeredConfig(cfg, max_seq_len=ctx, max_batch=16), peer
+    return ([("layered" if n == "Bofirax" else n.lower(), "layered_model", LayeredConfig(c, max_seq_len=ctx, max_batch=16))
+             for n, c in cfgs.items()] + [("transformer", "transformer_model", peer)])
 
 
-def layered_workload(size, B, K, W, ctx, use_graph, check):
-    """Both models of one size, measured alike: prompt pass, W warm-up steps, K timed greedy steps, the
+def layered_workload(design, size, B, K, W, ctx, use_graph, check):
+    """The models of one size, measured alike: prompt pass, W warm-up steps, K timed greedy steps, the
     decode matmuls and the mixers of a step replayed on their own."""
     from coeus_amd import PLUGINS
 
     out = {"size": size, "batch": B, "context": ctx}
-    for name, family, cfg in zip(("layered", "transformer"), ("layered_model", "transformer_model"), layered_pair(size, ctx, B)):
+    for name, family, cfg in layered_models(design, size, ctx):
         model = PLUGINS[family].create_builder().build(cfg, seed=0xC0E05)
         rng = np.random.default_rng(0xC0E06)
         sess, prompt, ids, dt, prefill_s, tok0, tok = run_decode(model, cfg, B, K, W, ctx, use_graph, rng, True)
@@ -392,7 +403,7 @@ def layered_workload(size, B, K, W, ctx, use_graph, check):
             # (a prompt pass rounds activations to bf16 where a decode step keeps f32; every sublayer of these
             # layered models adds at unit scale, so the roundings of a dozen layers weigh more than in a
             # transformer with small weights.  In f32 the two paths agree to 1e-5.)
-            leg["check"] = check_outputs(model, sess, prompt, ids, tok0, tok, W, K, ctx, bar=6e-2 if name == "layered" else 2e-2)
+            leg["check"] = check_outputs(model, sess, prompt, ids, tok0, tok, W, K, ctx, bar=2e-2 if name == "transformer" else 6e-2)
         leg["outputs_checked"] = bool(check)
         sess.close()
         model.close()
@@ -504,6 +515,7 @@ def main():
                     help="skip the other four benchmark configurations (default run of the 7B workload only)")
     ap.add_argument("--layered", nargs="?", const=",".join(sorted(LAYERED_SIZES)), metavar="SIZE,..",
                     help="layered decoders beside the transformer of the same size: " + ", ".join(sorted(LAYERED_SIZES)))
+    ap.add_argument("--design", default="Bofirax", choices=("Bofirax", "Zekilix"), help="the layered design that --layered measures")
     a = ap.parse_args()
     if a.layered and not set(a.layered.split(",")) <= set(LAYERED_SIZES):
         ap.error(f"--layered takes sizes out of {', '.join(sorted(LAYERED_SIZES))}")
@@ -517,13 +529,14 @@ def main():
         if a.steps + a.warmup + 1 >= ctx:
             print("steps + warmup must stay below the context length", file=sys.stderr)
             sys.exit(2)
-        sizes = [layered_workload(s, a.batch, a.steps, a.warmup, ctx, not a.no_graph, not a.no_check) for s in a.layered.split(",")]
-        last = sizes[-1]["layered"]["decode"]
+        sizes = [layered_workload(a.design, s, a.batch, a.steps, a.warmup, ctx, not a.no_graph, not a.no_check) for s in a.layered.split(",")]
+        name = "layered" if a.design == "Bofirax" else a.design.lower()
+        last = sizes[-1][name]["decode"]
         print(json.dumps({
             "metric": "layered decoder: decode tok/s @1 MI355X", "value": last["tok_s"], "unit": "tok/s", "n_gpus": 1,
             "steps": a.steps, "warmup": a.warmup, "ms_per_step": last["ms_per_step"], "higher_is_better": True,
             "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
-            "config": {"model": f"layered {sizes[-1]['size']}", "global_batch": a.batch, "seq_len": ctx, "parallelism": "none"},
+            "config": {"model": f"{name} {sizes[-1]['size']}", "global_batch": a.batch, "seq_len": ctx, "parallelism": "none"},
             "sizes": sizes}))
         return
 

@@ -895,10 +895,15 @@ int coeus_op_hyper_gemv(const coeus_weight *w, const coeus_hyper_step *step, con
     COEUS_TRY(limited_epilogue(epilogue, limit, y_dev, e));
     NormFuse nf;
     nf.h = x_dev; nf.h_out = x_new_dev; nf.kind = COEUS_NORM_LAYERNORM; nf.eps = h.eps;
-    nf.scale = h.norm; nf.in = h.in; nf.streams = h.streams; nf.mult = h.mult;
-    nf.y = h.y; nf.mix = h.mix; nf.out = h.out;
+    nf.scale = h.norm; nf.streams = h.streams; nf.y = h.y;
     hipStream_t st = (hipStream_t)stream;
-    return finish_op(launch_gemv(w->w, nullptr, batch, e, st, &nf), st, {}, "hyper-connections");
+    DeviceBuf fold;
+    int rc = fold.ensure(kHyperFoldFloats * 4);
+    nf.fold = (const float *)fold.p;
+    if (rc == COEUS_OK)
+        rc = launch_hyper_fold(h.y ? h.mix : nullptr, h.y ? h.out : nullptr, h.in, h.mult, h.streams, (float *)fold.p, st);
+    if (rc == COEUS_OK) rc = launch_gemv(w->w, nullptr, batch, e, st, &nf);
+    return finish_op(rc, st, {&fold}, "hyper-connections");
     COEUS_GUARD_END
 }
 

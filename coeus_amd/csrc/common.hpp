@@ -200,10 +200,9 @@ struct NormFuse {
     const float *y = nullptr, *ls = nullptr;
     float *h_out = nullptr;
     // Dense weights only, hyper-connections: h holds `streams` rows per sequence, y (nullable) the output of
-    // the sublayer before, whose mix [streams][streams], out [streams] and mult give the new streams (stored
-    // to h_out, not h); the matmul multiplies the layer norm of their sum weighted by in [streams].
-    const float *mix = nullptr, *out = nullptr, *in = nullptr;
-    float mult = 0.f;
+    // the sublayer before; the matmul multiplies the layer norm of the new streams' weighted sum, and the new
+    // streams are stored to h_out (not h).  fold: the record of the two sublayers (launch_hyper_fold).
+    const float *fold = nullptr;
     uint32_t streams = 0;
 };
 // True when launch_gemv can take `nf` for this weight and batch (quantised weights whose whole
@@ -216,6 +215,10 @@ bool gemv_can_fuse_norm_dense(const Weight &w, uint64_t batch);
 bool gemv_can_fuse_post_norm(const Weight &w, uint64_t batch);
 // ... and for hyper-connections (NormFuse::streams).
 bool gemv_can_fuse_hyper(const Weight &w, uint64_t batch, uint64_t streams);
+// What folding needs of mix, out (null in front of the first sublayer) and mult of the sublayer before and in of the
+// one behind, as kHyperFoldFloats floats on the device, 16-byte aligned; as many streams as can be folded.
+constexpr uint64_t kHyperFoldFloats = 32, kMaxFoldedStreams = 4;
+int launch_hyper_fold(const float *mix, const float *out, const float *in, float mult, uint32_t streams, float *fold, hipStream_t st);
 // The same normalisation as a launch of its own (batches too large for the folded form):
 // nf.h rows -> xq, row statistics merged from nf.stats.  Padding rows of xq are not written.
 int launch_norm_from_stats(const NormFuse &nf, uint64_t batch, uint64_t k, uint64_t k_pad, __half *xq,

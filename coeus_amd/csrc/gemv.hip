@@ -998,18 +998,10 @@ static int launch_gemv_quant(const Weight &w, const __half *xq, uint64_t batch, 
 // NORM = 3: the norm of the sublayer before stands behind it.  x is the residual stream h, y the
 // sublayer's bare output: the workgroup stages h + y / rms(y) * scale (* ls), and the first one stores
 // these rows as the new residual stream.  LDS: y rows (then the sums), [2][k] scales, h rows behind them.
-// NORM = 4: hyper-connections.  x holds `streams` rows per batch entry, y the output of the sublayer before
-// (null: none yet).  The workgroup stages the layer norm of sum_t in[t] x'_t, x'_t = sum_s mix[s][t] x_s +
-// mult out[t] y, and the first one stores the x'_t.  What a sum over t needs of the old streams is one
-// coefficient per stream, so only that workgroup forms the new ones.
 struct PostNorm {
     const float *y, *ls;
     float *h_out;
-    const float *mix, *out, *in;
-    float mult;
-    uint32_t streams;
 };
-constexpr int kFusedStreams = 4;
 template <bool BF16, int BP, int NORM>
 __global__ __launch_bounds__(1024) void gemv_dense_kernel(const void *__restrict__ wdata,
                                                           const float *__restrict__ x, uint64_t k,
@@ -1054,49 +1046,9 @@ __global__ __launch_bounds__(1024) void gemv_dense_kernel(const void *__restrict
         float ps[BP];
 #pragma unroll
         for (int b = 0; b < BP; b++) ps[b] = 0.f;
-        constexpr int NS = NORM == 4 ? kFusedStreams : 1;
-        float cs[NS], cy = 0.f;  // NORM == 4: what x_s and y contribute to the weighted sum of the new streams
-        const uint32_t S = NORM == 4 ? post.streams : 1;
-        if (NORM == 4) {
-#pragma unroll
-            for (int s = 0; s < NS; s++) {
-                cs[s] = 0.f;
-                if (s >= (int)S) continue;
-                if (!post.y) { cs[s] = post.in[s]; continue; }
-                for (uint32_t u = 0; u < S; u++) cs[s] = fmaf(post.mix[s * S + u], post.in[u], cs[s]);
-                cy = fmaf(post.mult * post.out[s], post.in[s], cy);
-            }
-        }
         for (uint64_t i = threadIdx.x; i < k; i += blockDim.x) {
             gs[i] = nscale[i];
             if (NORM == 1) bs[i] = nbias ? nbias[i] : 0.f;
-            if (NORM == 4) {
-#pragma unroll
-                for (int b = 0; b < BP; b++)
-                    if (b < (int)batch) {
-                        float xv[NS];
-#pragma unroll
-                        for (int s = 0; s < NS; s++) xv[s] = s < (int)S ? x[((uint64_t)b * S + s) * k + i] : 0.f;
-                        const float yv = post.y ? post.y[(uint64_t)b * k + i] : 0.f;
-                        float v = cy * yv;
-#pragma unroll
-                        for (int s = 0; s < NS; s++) v = fmaf(cs[s], xv[s], v);
-                        xn[(uint64_t)b * k + i] = v;
-                        ps[b] += v;
-                        if (blockIdx.x == 0 && post.y) {
-#pragma unroll
-                            for (int u = 0; u < NS; u++)
-                                if (u < (int)S) {
-                                    float nv = post.mult * post.out[u] * yv;
-#pragma unroll
-                                    for (int s = 0; s < NS; s++)
-                                        if (s < (int)S) nv = fmaf(post.mix[s * S + u], xv[s], nv);
-                                    post.h_out[((uint64_t)b * S + u) * k + i] = nv;
-                                }
-                        }
-                    }
-                continue;
-            }
             if (NORM == 3) bs[i] = post.ls ? post.ls[i] : 1.0f;
 #pragma unroll
             for (int b = 0; b < BP; b++)
@@ -1120,7 +1072,7 @@ __global__ __launch_bounds__(1024) void gemv_dense_kernel(const void *__restrict
                 for (uint32_t w = 0; w < nwaves; w++) tot += red[w * BP + lane];
             return tot;
         };
-        if (NORM == 1 || NORM == 4) {
+        if (NORM == 1) {
             const float tot = finish(ps);
             if (wave == 0 && lane < BP) stat[lane] = tot / (float)k;
             __syncthreads();
@@ -1247,18 +1199,290 @@ bool gemv_can_fuse_post_norm(const Weight &w, uint64_t batch) {
     return gemv_dense_post_lds(w.k, pad_batch(batch)) <= kDenseNormLdsLimit;
 }
 
+// ---------------------------------------------------------------- dense kernel behind hyper-connections
+// x holds `streams` rows per batch entry, y the output of the sublayer before.  A workgroup stages the layer norm
+// of sum_t in[t] x'_t, x'_t = sum_s mix[s][t] x_s + mult out[t] y, and multiplies its rows of the weight with it; the
+// first workgroup stores the x'_t.  What a sum over t needs of the old streams is one coefficient per stream
+// (hyper_fold_kernel), so only that workgroup forms the new ones.
+//
+// Five rows of f32 in front of every share of the weight are what this costs, and a compute unit's trips to memory
+// bound it: one workgroup of 16 waves per compute unit reads them once and then every rows-th row of the weight,
+// with SL steps in flight across the rows' ends.  The activation rows pass through registers (pairs of elements,
+// NIT per thread): a wave finds the mean and the squares about it of its own elements, and one barrier later every
+// wave merges the sixteen of them.  What the first loads need lies in the 64 bytes of arguments that arrive with
+// the wave.
+constexpr int kFusedStreams = (int)kMaxFoldedStreams;
+// what x_s [4] and y contribute to the weighted sum of the new streams, mult out[t] [4], mix [4][4]; zeros behind
+// the streams there are
+struct HyperFold {
+    float cs[kFusedStreams], om[kFusedStreams], mix[kFusedStreams][kFusedStreams], cy;
+};
+static_assert(sizeof(HyperFold) <= kHyperFoldFloats * 4, "size of a record");
+
+__global__ __launch_bounds__(64) void hyper_fold_kernel(const float *mix, const float *out, const float *in, float mult, uint32_t S,
+                                                        HyperFold *f) {
+    const uint32_t t = threadIdx.x;
+    if (t < 16) f->mix[t / 4][t % 4] = mix && t / 4 < S && t % 4 < S ? mix[t / 4 * S + t % 4] : 0.f;
+    if (t < 4) {
+        f->om[t] = out && t < S ? mult * out[t] : 0.f;
+        float c = 0.f;
+        if (t < S) {
+            if (!mix) c = in[t];
+            else for (uint32_t u = 0; u < S; u++) c = fmaf(mix[t * S + u], in[u], c);
+        }
+        f->cs[t] = c;
+    }
+    if (t == 0) {
+        float c = 0.f;
+        if (out)
+            for (uint32_t u = 0; u < S; u++) c = fmaf(mult * out[u], in[u], c);
+        f->cy = c;
+    }
+}
+
+int launch_hyper_fold(const float *mix, const float *out, const float *in, float mult, uint32_t streams, float *fold, hipStream_t st) {
+    if (!in || !fold || !mix != !out || streams < 1 || streams > kFusedStreams)
+        return fail(COEUS_INVALID_INPUT, "folded hyper-connections: bad arguments or too many streams");
+    hipLaunchKernelGGL(hyper_fold_kernel, dim3(1), dim3(64), 0, st, mix, out, in, mult, streams, (HyperFold *)fold);
+    COEUS_HIP(hipGetLastError());
+    return COEUS_OK;
+}
+
+template <bool BF16, int BP, int NIT>
+__global__ __launch_bounds__(1024) void gemv_hyper_kernel(const void *__restrict__ wdata, const float *__restrict__ x,
+                                                          const float *__restrict__ y, const float *__restrict__ norm,
+                                                          const HyperFold *__restrict__ fold, uint32_t k, uint32_t batch_streams,
+                                                          float *x_out, float eps, EpiArgs e) {
+    constexpr int NS = kFusedStreams, SL = 4;
+    extern __shared__ float xn[];  // [BP][k]
+    __shared__ float2 red[16][BP];
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), S = batch_streams >> 16,
+                   batch = batch_streams & 0xffffu;
+    const bool vec = (k & 7) == 0, gated = epi_gated(e.act);
+    // Unit u of this wave (a row, or the two rows of a gated pair) is unit blockIdx.x + gridDim.x (wave + 16 u) of
+    // the weight.
+    const uint32_t per = gated ? 2 : 1, units = (uint32_t)(e.n / per), first = blockIdx.x + gridDim.x * wave, stride = 16 * gridDim.x;
+    const uint32_t rows = first < units ? ((units - 1 - first) / stride + 1) * per : 0, steps = (k + 511) / 512, items = rows * steps;
+    auto row_of = [&](uint32_t i) { return gated ? 2ull * (first + stride * (i >> 1)) + (i & 1) : (uint64_t)first + (uint64_t)stride * i; };
+    // item t: step t % steps of row t / steps; a lane behind the row's end re-reads the last weights
+    uint32_t ld_row = 0, ld_step = 0;
+    auto wload = [&](uint4 &a, uint4 &b) {
+        if (ld_row >= rows) return;
+        constexpr uint32_t ES = BF16 ? 2 : 4;
+        const char *base = (const char *)wdata + row_of(ld_row) * k * ES;  // wave-uniform
+        const uint32_t off = min(lane * 8 + 512 * ld_step, k - 8) * ES;
+        if (++ld_step == steps) { ld_step = 0; ld_row++; }
+        a = load_stream((const uint4 *)(base + off));
+        if (!BF16) b = load_stream((const uint4 *)(base + off + 16));
+    };
+    // Where element i of the normalised rows lies: the two quads of every eight in halves of their own, so that the
+    // lanes of a read of quads are neighbours.
+    auto place = [&](uint32_t i) { return vec ? (i & 4 ? k / 2 : 0) + (i >> 3) * 4 + (i & 3) : i; };
+    // The streams are requested before the weights: loads return in order, and the norm needs only the streams.
+    // (No branches here: a lane behind the end re-reads the last elements, a stream that is not there the last one.)
+    float2 xv[NIT][BP][NS], yv[NIT][BP], g[NIT];
+#pragma unroll
+    for (int it = 0; it < NIT; it++) {
+        const uint32_t i = min(2 * (tid + 1024 * it), k - 2);
+        g[it] = *(const float2 *)(norm + i);
+#pragma unroll
+        for (int b = 0; b < BP; b++) {
+            const uint32_t row = min((uint32_t)b, batch - 1);
+#pragma unroll
+            for (int s = 0; s < NS; s++) xv[it][b][s] = *(const float2 *)(x + ((uint64_t)row * S + min((uint32_t)s, S - 1)) * k + i);
+            yv[it][b] = *(const float2 *)(y + (uint64_t)row * k + i);
+        }
+    }
+    __builtin_amdgcn_sched_barrier(0);
+    uint4 wa[SL], wb[SL];
+#pragma unroll
+    for (int q = 0; q < SL; q++) {
+        wa[q] = wb[q] = make_uint4(0, 0, 0, 0);
+        if (vec) wload(wa[q], wb[q]);
+    }
+    __builtin_amdgcn_sched_barrier(0);
+    float2 v[NIT][BP];
+    float cnt = 0.f;  // elements of this wave
+#pragma unroll
+    for (int it = 0; it < NIT; it++) {
+        const uint32_t i = 2 * (tid + 1024 * it), w0 = 2 * (64 * wave + 1024 * it);
+        cnt += w0 < k ? (float)min(128u, k - w0) : 0.f;
+#pragma unroll
+        for (int b = 0; b < BP; b++) {
+            float2 o = make_float2(fold->cy * yv[it][b].x, fold->cy * yv[it][b].y);
+#pragma unroll
+            for (int s = 0; s < NS; s++) { o.x = fmaf(fold->cs[s], xv[it][b][s].x, o.x); o.y = fmaf(fold->cs[s], xv[it][b][s].y, o.y); }
+            v[it][b] = i < k ? o : make_float2(0.f, 0.f);
+        }
+    }
+    if (blockIdx.x == 0 && x_out) {
+#pragma unroll
+        for (int it = 0; it < NIT; it++) {
+            const uint32_t i = 2 * (tid + 1024 * it);
+#pragma unroll
+            for (int b = 0; b < BP; b++) {
+                if (b >= (int)batch || i >= k) continue;
+#pragma unroll
+                for (int u = 0; u < NS; u++) {
+                    if (u >= (int)S) continue;
+                    float2 nv = make_float2(fold->om[u] * yv[it][b].x, fold->om[u] * yv[it][b].y);
+#pragma unroll
+                    for (int s = 0; s < NS; s++) {
+                        nv.x = fmaf(fold->mix[s][u], xv[it][b][s].x, nv.x);
+                        nv.y = fmaf(fold->mix[s][u], xv[it][b][s].y, nv.y);
+                    }
+                    *(float2 *)(x_out + ((uint64_t)b * S + u) * k + i) = nv;
+                }
+            }
+        }
+    }
+    auto row_sum = [](float t) { return xor32_sum(xor16_sum(group_sum<16>(t))); };
+    const float inv_cnt = cnt > 0.f ? 1.0f / cnt : 0.f;
+#pragma unroll
+    for (int b = 0; b < BP; b++) {
+        if (b >= (int)batch) continue;
+        float s1 = 0.f, s2 = 0.f;
+#pragma unroll
+        for (int it = 0; it < NIT; it++) s1 += v[it][b].x + v[it][b].y;
+        const float own = row_sum(s1), mw = own * inv_cnt;
+#pragma unroll
+        for (int it = 0; it < NIT; it++)
+            if (2 * (tid + 1024 * it) < k) {
+                const float dx = v[it][b].x - mw, dy = v[it][b].y - mw;
+                s2 = fmaf(dx, dx, s2); s2 = fmaf(dy, dy, s2);
+            }
+        s2 = row_sum(s2);
+        if (lane == 0) red[wave][b] = make_float2(own, s2);
+    }
+    __syncthreads();
+    {
+        // lane w of 16 takes wave w's record
+        const uint32_t w = lane & 15;
+        float cw = 0.f;
+#pragma unroll
+        for (int it = 0; it < NIT; it++) {
+            const uint32_t w0 = 2 * (64 * w + 1024 * it);
+            cw += w0 < k ? (float)min(128u, k - w0) : 0.f;
+        }
+#pragma unroll
+        for (int b = 0; b < BP; b++) {
+            if (b >= (int)batch) continue;
+            const float2 rec = red[w][b];
+            const float mean = group_sum<16>(rec.x) / (float)k, dm = cw > 0.f ? rec.x / cw - mean : 0.f;
+            const float rs = 1.0f / sqrtf(group_sum<16>(fmaf(cw * dm, dm, rec.y)) / (float)k + eps);
+#pragma unroll
+            for (int it = 0; it < NIT; it++) {
+                const uint32_t i = 2 * (tid + 1024 * it);
+                if (i < k) *(float2 *)(xn + (size_t)b * k + place(i)) = make_float2((v[it][b].x - mean) * rs * g[it].x, (v[it][b].y - mean) * rs * g[it].y);
+            }
+        }
+    }
+    __syncthreads();
+    float acc[BP], gate[BP];
+#pragma unroll
+    for (int b = 0; b < BP; b++) acc[b] = gate[b] = 0.f;
+    // a row is complete: its epilogue (the first row of a pair only keeps its sums)
+    auto finish = [&](uint32_t i) {
+#pragma unroll
+        for (int b = 0; b < BP; b++) {
+            const float sum = row_sum(acc[b]);
+            acc[b] = 0.f;
+            if (gated && (i & 1) == 0) { gate[b] = sum; continue; }
+            if (lane != 0 || b >= (int)batch) continue;
+            if (gated) epi_store_gated(e, b, row_of(i) / 2, gate[b], sum);
+            else epi_store<true>(e, b, row_of(i), sum);
+        }
+    };
+    if (vec) {
+        uint32_t row = 0, step = 0;
+        for (uint32_t t = 0; t < items; t += SL)
+#pragma unroll
+            for (int q = 0; q < SL; q++) {
+                if (t + q >= items) break;  // wave-uniform
+                const uint32_t k0 = lane * 8 + 512 * step;
+                if (k0 < k) {
+                    float wv[8];
+                    if (BF16) {
+                        const uint32_t r[4] = {wa[q].x, wa[q].y, wa[q].z, wa[q].w};
+#pragma unroll
+                        for (int j = 0; j < 4; j++) {
+                            wv[2 * j] = __uint_as_float(r[j] << 16);
+                            wv[2 * j + 1] = __uint_as_float(r[j] & 0xffff0000u);
+                        }
+                    } else {
+                        const uint32_t r[8] = {wa[q].x, wa[q].y, wa[q].z, wa[q].w, wb[q].x, wb[q].y, wb[q].z, wb[q].w};
+#pragma unroll
+                        for (int j = 0; j < 8; j++) wv[j] = __uint_as_float(r[j]);
+                    }
+#pragma unroll
+                    for (int b = 0; b < BP; b++) {
+                        if (b >= (int)batch) continue;
+                        const float *xr = xn + (size_t)b * k + k0 / 2;
+                        const float4 xa = *(const float4 *)xr, xb = *(const float4 *)(xr + k / 2);
+                        float s = acc[b];
+                        s = fmaf(wv[0], xa.x, s); s = fmaf(wv[1], xa.y, s); s = fmaf(wv[2], xa.z, s); s = fmaf(wv[3], xa.w, s);
+                        s = fmaf(wv[4], xb.x, s); s = fmaf(wv[5], xb.y, s); s = fmaf(wv[6], xb.z, s); s = fmaf(wv[7], xb.w, s);
+                        acc[b] = s;
+                    }
+                }
+                wload(wa[q], wb[q]);
+                if (++step == steps) { finish(row); step = 0; row++; }
+            }
+    } else {
+        for (uint32_t i = 0; i < rows; i++) {
+            for (uint32_t kk = lane; kk < k; kk += 64) {
+                const uint64_t at = row_of(i) * k + kk;
+                const float wv = BF16 ? bf16_bits_to_f32(((const uint16_t *)wdata)[at]) : ((const float *)wdata)[at];
+#pragma unroll
+                for (int b = 0; b < BP; b++)
+                    if (b < (int)batch) acc[b] = fmaf(wv, xn[(size_t)b * k + kk], acc[b]);
+            }
+            finish(i);
+        }
+    }
+}
+
+// pairs of elements per thread; beyond four over the batch every workgroup would read more rows than it is worth
+static uint32_t hyper_pairs(uint64_t k) { return (uint32_t)ceil_div(k, 2048); }
 bool gemv_can_fuse_hyper(const Weight &w, uint64_t batch, uint64_t streams) {
-    return streams >= 1 && streams <= kFusedStreams && gemv_can_fuse_norm_dense(w, batch);
+    if (w.dtype >= COEUS_W_Q8_0 || batch < 1 || batch > 16 || streams < 1 || streams > kFusedStreams || (w.k & 1)) return false;
+    const uint32_t bp = pad_batch(batch), nit = hyper_pairs(w.k);
+    return nit <= 3 && bp * nit <= 4;
+}
+
+template <bool BF16>
+static int launch_gemv_hyper(const Weight &w, uint64_t batch, const EpiArgs &e, hipStream_t st, const NormFuse &nf) {
+    if (!gemv_can_fuse_hyper(w, batch, nf.streams) || !nf.h || !nf.scale || !nf.fold || nf.kind != COEUS_NORM_LAYERNORM || nf.ld ||
+        nf.bias || (nf.y && (!nf.h_out || nf.h_out == nf.h)))
+        return fail(COEUS_INVALID_INPUT, "folded hyper-connections: bad arguments or too many streams");
+    const uint32_t bp = pad_batch(batch), b = (uint32_t)batch, k = (uint32_t)w.k, nit = hyper_pairs(w.k);
+    const size_t lds = (size_t)bp * k * 4;
+    const uint32_t bs = b | nf.streams << 16;
+    const HyperFold *fold = (const HyperFold *)nf.fold;
+    const float *y = nf.y ? nf.y : nf.h;  // (without an output of a sublayer before its weight is zero)
+    float *x_out = nf.y ? nf.h_out : nullptr;
+    if (w.n > 0x7fffffffull) return fail(COEUS_INVALID_INPUT, "folded hyper-connections: too many rows");
+    const uint64_t units = epi_gated(e.act) ? w.n / 2 : w.n;
+    const dim3 grid((unsigned)std::min<uint64_t>(256, units)), block(1024);  // (a workgroup per compute unit)
+#define COEUS_GH(BPV, NV) \
+    hipLaunchKernelGGL((gemv_hyper_kernel<BF16, BPV, NV>), grid, block, lds, st, w.data, nf.h, y, nf.scale, fold, k, bs, x_out, nf.eps, e)
+    if (bp == 4) COEUS_GH(4, 1);
+    else if (bp == 2 && nit == 1) COEUS_GH(2, 1);
+    else if (bp == 2) COEUS_GH(2, 2);
+    else if (nit == 1) COEUS_GH(1, 1);
+    else if (nit == 2) COEUS_GH(1, 2);
+    else COEUS_GH(1, 3);
+#undef COEUS_GH
+    COEUS_HIP(hipGetLastError());
+    return COEUS_OK;
 }
 
 template <bool BF16>
 static int launch_gemv_dense(const Weight &w, const float *x, uint64_t batch, const EpiArgs &e,
                              hipStream_t st, const NormFuse *nf) {
     const uint32_t bp = pad_batch(batch), b = (uint32_t)batch;
-    const bool hyper = nf && nf->streams, post_norm = nf && nf->y && !hyper;
-    if (hyper && (!gemv_can_fuse_hyper(w, batch, nf->streams) || !nf->in || nf->kind != COEUS_NORM_LAYERNORM || nf->ld ||
-                  (nf->y && (!nf->mix || !nf->out || !nf->h_out || nf->h_out == nf->h))))
-        return fail(COEUS_INVALID_INPUT, "folded hyper-connections: bad arguments or too many streams");
+    if (nf && nf->streams) return launch_gemv_hyper<BF16>(w, batch, e, st, *nf);
+    const bool post_norm = nf && nf->y;
     if (nf && !(post_norm ? gemv_can_fuse_post_norm(w, batch) : gemv_can_fuse_norm_dense(w, batch)))
         return fail(COEUS_INVALID_INPUT, "norm fusion needs the normalised activations to fit in LDS");
     if (post_norm && (!nf->h || !nf->scale || !nf->h_out || nf->h_out == nf->h || nf->kind != COEUS_NORM_RMSNORM))
@@ -1270,17 +1494,16 @@ static int launch_gemv_dense(const Weight &w, const float *x, uint64_t batch, co
     const uint32_t waves = nf ? 16 : 4;
     const dim3 grid((unsigned)ceil_div(w.n, waves)), block(waves * 64);
     const size_t lds = !nf ? 0 : post_norm ? gemv_dense_post_lds(w.k, bp) : gemv_dense_norm_lds(w.k, bp);
-    const int norm = !nf ? 0 : hyper ? 4 : post_norm ? 3 : nf->kind == COEUS_NORM_RMSNORM ? 2 : 1;
+    const int norm = !nf ? 0 : post_norm ? 3 : nf->kind == COEUS_NORM_RMSNORM ? 2 : 1;
     const uint64_t ldx = nf && nf->ld ? nf->ld : w.k;
-    PostNorm post{};
-    if (post_norm || hyper) post = PostNorm{nf->y, nf->ls, nf->h_out, nf->mix, nf->out, nf->in, nf->mult, nf->streams};
+    const PostNorm post = post_norm ? PostNorm{nf->y, nf->ls, nf->h_out} : PostNorm{nullptr, nullptr, nullptr};
     const float *xin = nf ? nf->h : x;
     const float *ns = nf ? nf->scale : nullptr, *nb = nf ? nf->bias : nullptr;
     const float eps = nf ? nf->eps : 0.f;
 #define COEUS_GEMVD2(BPV, NV) \
     hipLaunchKernelGGL((gemv_dense_kernel<BF16, BPV, NV>), grid, block, lds, st, w.data, xin, w.k, b, e, ns, nb, eps, ldx, post)
 #define COEUS_GEMVD(BPV) \
-    do { if (norm == 0) COEUS_GEMVD2(BPV, 0); else if (norm == 1) COEUS_GEMVD2(BPV, 1); else if (norm == 2) COEUS_GEMVD2(BPV, 2); else if (norm == 3) COEUS_GEMVD2(BPV, 3); else COEUS_GEMVD2(BPV, 4); } while (0)
+    do { if (norm == 0) COEUS_GEMVD2(BPV, 0); else if (norm == 1) COEUS_GEMVD2(BPV, 1); else if (norm == 2) COEUS_GEMVD2(BPV, 2); else COEUS_GEMVD2(BPV, 3); } while (0)
     switch (bp) {
         case 1: COEUS_GEMVD(1); break;
         case 2: COEUS_GEMVD(2); break;

@@ -34,6 +34,7 @@ LayeredStack::~LayeredStack() {
     for (LayeredLayer &l : layers)
         for (Weight *w : {&l.in, &l.o, &l.up, &l.down, &l.uq, &l.ukv}) weight_free(*w);
     if (small) (void)hipFree(small);
+    if (folds) (void)hipFree(folds);
 }
 
 // ---------------------------------------------------------------- state
@@ -163,6 +164,27 @@ struct Source {
         return COEUS_OK;
     }
 };
+
+// The records that decode steps fold hyper-connections with, in the order of the sublayers.
+int make_folds(LayeredStack &stack, hipStream_t st) {
+    const LayeredConfig &cfg = stack.cfg;
+    if (!cfg.streams || cfg.streams > kMaxFoldedStreams) return COEUS_OK;
+    COEUS_HIP(hipMalloc((void **)&stack.folds, 2 * cfg.layers.size() * kHyperFoldFloats * 4));
+    const Around *from = nullptr;
+    float *at = stack.folds;
+    auto next = [&](const Around &to) -> int {
+        COEUS_TRY(launch_hyper_fold(from ? from->mix : nullptr, from ? from->out : nullptr, to.in, cfg.residual_mult, (uint32_t)cfg.streams,
+                                    at, st));
+        from = &to;
+        at += kHyperFoldFloats;
+        return COEUS_OK;
+    };
+    for (size_t l = 0; l < cfg.layers.size(); l++) {
+        COEUS_TRY(next(stack.weights(l).around_mixer));
+        if (cfg.layers[l].ff) COEUS_TRY(next(stack.weights(l).around_ff));
+    }
+    return COEUS_OK;
+}
 
 int build(const LayeredConfig &cfg, const SafeTensors *file, uint64_t seed, const coeus_load_options &opt, Model **out) {
     if (opt.weight_dtype != COEUS_W_F32 && opt.weight_dtype != COEUS_W_BF16)
@@ -320,6 +342,7 @@ int build(const LayeredConfig &cfg, const SafeTensors *file, uint64_t seed, cons
     COEUS_HIP(hipMemcpy(stack.small, small.data(), small.size() * 4, hipMemcpyHostToDevice));
     for (auto &f : fix) *f.first = stack.small + f.second;
     m->weight_bytes += small.size() * 4;
+    COEUS_TRY(make_folds(stack, st));
 
     // ---- output projection, which may be the embedding table
     COEUS_TRY(weight_alloc(m->out, wd, cfg.width, cfg.vocab));
@@ -677,6 +700,7 @@ int layered_decode(Session &s, hipStream_t st, int only, uint64_t *launches, uin
           *att = (float *)s.datt.p, *ff = (float *)s.dff.p;
     const float eps = cfg.eps;
     const Around *pending = nullptr;
+    const float *fold = stack.folds;  // the next sublayer's record
     uint64_t n_launch = 0, n_bytes = 0;
     auto count = [&](const Weight &w, bool gated) {
         n_launch++;
@@ -706,8 +730,10 @@ int layered_decode(Session &s, hipStream_t st, int only, uint64_t *launches, uin
         return COEUS_OK;
     };
     // a matmul of what a sublayer reads (the same limit on the output rows as for norms in front of it: every
-    // workgroup of 16 rows repeats the norm)
+    // workgroup repeats the norm)
     auto stream_gemv = [&](const Weight &w, const Around &to, const Epilogue &e) -> int {
+        const float *const this_fold = fold;
+        if (fold) fold += kHyperFoldFloats;
         const bool fuse = s.fuse && w.n <= 16384 &&
                           (cfg.streams ? gemv_can_fuse_hyper(w, B, cfg.streams) : pending && gemv_can_fuse_post_norm(w, B));
         if (fuse) {
@@ -716,8 +742,7 @@ int layered_decode(Session &s, hipStream_t st, int only, uint64_t *launches, uin
             if (pending) nf.y = y;
             if (cfg.streams) {
                 nf.kind = COEUS_NORM_LAYERNORM;
-                nf.scale = to.norm; nf.in = to.in; nf.streams = (uint32_t)cfg.streams; nf.mult = cfg.residual_mult;
-                if (pending) { nf.mix = pending->mix; nf.out = pending->out; }
+                nf.scale = to.norm; nf.fold = this_fold; nf.streams = (uint32_t)cfg.streams;
             } else {
                 nf.kind = COEUS_NORM_RMSNORM;
                 nf.scale = pending->norm; nf.ls = pending->ls;

@@ -53,6 +53,7 @@ struct LayeredStack {
     LayeredConfig cfg;
     std::vector<LayeredLayer> layers;
     float *small = nullptr;  // every f32 vector of every layer
+    float *folds = nullptr;  // kHyperFoldFloats per sublayer, in their order (hyper-connections that can be folded)
     ~LayeredStack();
     const LayeredLayer &weights(size_t l) const { return layers[cfg.layers[l].source]; }
 };

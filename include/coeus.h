@@ -458,8 +458,8 @@ typedef struct coeus_hyper_step {
 /* In place on x_dev [rows][streams][hidden]; u_dev [rows][hidden] (may be y_dev). */
 int coeus_op_hyper(const coeus_hyper_step *step, float *x_dev, uint64_t rows, uint64_t hidden, float *u_dev,
                    void *stream);
-/* The same folded into the decode matmul that reads u, as decode steps run it (f32 and bf16 weights, at most 4
- * streams): y_dev [batch][n_out] = epilogue(u . W), the new streams (if y_dev of the step is set) to
+/* The same folded into the decode matmul that reads u, as decode steps run it (f32 and bf16 weights, an even k_in, at
+ * most 4 streams, few and short enough rows): y_dev [batch][n_out] = epilogue(u . W), the new streams (if y_dev of the step is set) to
  * x_new_dev, which must not be x_dev. */
 int coeus_op_hyper_gemv(const coeus_weight *w, const coeus_hyper_step *step, const float *x_dev, uint64_t batch,
                         float *x_new_dev, uint32_t epilogue, float limit, float *y_dev, void *stream);

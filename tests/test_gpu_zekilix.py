@@ -67,7 +67,8 @@ def test_hyper_output_over_its_input():
 
 @pytest.mark.parametrize("wd", [_lib.W_F32, _lib.W_BF16])
 @pytest.mark.parametrize("with_y", [True, False])
-@pytest.mark.parametrize("batch,k,n,streams", [(1, 96, 40, 3), (3, 58, 131, 2), (16, 128, 64, 4), (2, 1024, 300, 1), (1, 4096, 52, 4), (5, 250, 17, 3)])
+@pytest.mark.parametrize("batch,k,n,streams", [(1, 96, 40, 3), (3, 58, 131, 2), (4, 128, 64, 4), (2, 1024, 300, 1), (1, 4096, 52, 4), (3, 250, 17, 3),
+                                               (1, 2050, 34, 2), (2, 4000, 20, 4), (1, 6000, 18, 3), (1, 520, 8230, 4), (2, 64, 9001, 2)])
 def test_hyper_gemv(wd, with_y, batch, k, n, streams):
     rng = np.random.default_rng(k + n)
     w = rng.normal(size=(k, n)).astype(np.float32) / np.float32(np.sqrt(k))
@@ -90,6 +91,7 @@ def test_hyper_refusals():
     W = Weight(_lib.W_F32, np.zeros((64, 8), np.float32))
     y = DeviceArray((2, 8))
     assert lib.coeus_op_hyper_gemv(W.h, C.byref(t.step), dx.ptr, 2, dx.ptr, 0, 0.0, y.ptr, None) == _lib.INVALID_INPUT  # in place
+    assert lib.coeus_op_hyper_gemv(W.h, C.byref(t.step), dx.ptr, 5, u.ptr, 0, 0.0, y.ptr, None) == _lib.INVALID_INPUT
     t.step.streams = 5
     assert lib.coeus_op_hyper_gemv(W.h, C.byref(t.step), dx.ptr, 1, u.ptr, 0, 0.0, y.ptr, None) == _lib.INVALID_INPUT
     assert lib.coeus_op_matmul_limited(W.h, dx.ptr, 1, 0, _lib.EPI_CLAMP_GATE, 0.0, y.ptr, None) == _lib.INVALID_INPUT
