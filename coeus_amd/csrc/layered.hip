@@ -734,7 +734,7 @@ int layered_decode(Session &s, hipStream_t st, int only, uint64_t *launches, uin
     auto stream_gemv = [&](const Weight &w, const Around &to, const Epilogue &e) -> int {
         const float *const this_fold = fold;
         if (fold) fold += kHyperFoldFloats;
-        const bool fuse = s.fuse && w.n <= 16384 &&
+        const bool fuse = s.fuse && (cfg.streams || w.n <= 16384) &&
                           (cfg.streams ? gemv_can_fuse_hyper(w, B, cfg.streams) : pending && gemv_can_fuse_post_norm(w, B));
         if (fuse) {
             NormFuse nf;

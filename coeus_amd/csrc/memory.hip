@@ -237,25 +237,56 @@ __global__ __launch_bounds__(256) void memory_carry_kernel(MemoryDims dm, Memory
     }
 }
 
-// One workgroup of four waves per (chunk, head, sequence); wave w owns the 16-column tiles w, w + 4, .. of all 64
-// rows, so that a chunk's state is read once and the values once.
+// One workgroup of eight waves per (chunk, head, sequence); wave w owns the 16-column tiles w, w + 8, .. of all 64
+// rows, so that a chunk's state is read once and the values once.  Queries and keys are in LDS (rows of an odd
+// number of quads); the weighted scores take the keys' place.
+static uint32_t read_ld(const MemoryDims &dm) { return 16 * (uint32_t)ceil_div(dm.d, 16) + 4; }
+constexpr uint32_t kScoreLd = kChunk + 4;
+static size_t read_lds_bytes(const MemoryDims &dm) { return kChunk * (size_t)(read_ld(dm) + std::max(read_ld(dm), kScoreLd)) * 4; }
+
 template <int NCT>
-__global__ __launch_bounds__(256) void memory_read_kernel(const float *__restrict__ proj, MemoryDims dm, MemoryParams pr, MemoryState st,
+__global__ __launch_bounds__(512) void memory_read_kernel(const float *__restrict__ proj, MemoryDims dm, MemoryParams pr, MemoryState st,
                                                           uint64_t n, uint64_t t0, uint64_t seg, MemoryChunks cb,
                                                           float *__restrict__ out, uint16_t *__restrict__ out_lp, uint64_t lp_ld,
                                                           bool lp_bf16) {
-    constexpr uint32_t PLD = kChunk + 4;
-    __shared__ __attribute__((aligned(16))) float pl[kChunk * PLD];
+    constexpr uint32_t PLD = kScoreLd, W = 8;
+    extern __shared__ __attribute__((aligned(16))) float lds[];
     __shared__ double rs[kChunk], as[kChunk];  // F - m of a row, a of a column
-    __shared__ __attribute__((aligned(16))) float carry[kChunk], floor_[kChunk], psum[4][kChunk], qn[kChunk], dinv[kChunk], rsum[4][kChunk];
+    __shared__ __attribute__((aligned(16))) float carry[kChunk], floor_[kChunk], psum[4][kChunk], qn[kChunk], dinv[kChunk], rsum[W][kChunk];
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
-    const uint32_t chunk = blockIdx.x, h = blockIdx.y, H = dm.heads, d = dm.d, e = dm.e;
+    const uint32_t chunk = blockIdx.x, h = blockIdx.y, H = dm.heads, d = dm.d, e = dm.e, LD = 16 * cb.dtiles + 4;
     const uint64_t b = blockIdx.z, left = seg - (uint64_t)chunk * kChunk, row0 = b * n + t0 + (uint64_t)chunk * kChunk;
     const uint32_t live = left < kChunk ? (uint32_t)left : kChunk;
     const uint64_t unit = b * H + h, ci = unit * cb.chunks + chunk;
     const float *p = proj + row0 * dm.in_ld, *qp = p + h * d, *kp = p + dm.k_off() + h * d, *vp = p + dm.v_off() + h * e;
+    float *const ql = lds, *const kl = ql + kChunk * LD, *const pl = kl;
     const float qs = 1.0f / sqrtf((float)d);
-    if (wave == 0) {
+    // the first tiles of the state and the values are requested before anything else
+    const float *sp = cb.s + ci * cb.dtiles * cb.etiles * 256 + lane * 4;
+    auto sload = [&](uint32_t m, float4_t (&x)[NCT]) {
+#pragma unroll
+        for (int t = 0; t < NCT; t++) x[t] = *(const float4_t *)(sp + (min(m, cb.dtiles - 1) * cb.etiles + min(wave + W * t, cb.etiles - 1)) * 256);
+    };
+    float4_t s[4][NCT], v[4][NCT];
+#pragma unroll
+    for (int q = 0; q < 4; q++) sload(q, s[q]);
+#pragma unroll
+    for (int m = 0; m < 4; m++)
+#pragma unroll
+        for (int t = 0; t < NCT; t++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) v[m][t][i] = vp[(uint64_t)min(16u * m + 4 * g + i, live - 1) * dm.in_ld + min(16 * (wave + W * t) + c, e - 1)];
+    // queries and keys, half a wave per row: rows behind the end repeat the last one, dims behind the end are zero
+    for (uint32_t x = 4 * (tid & 31); x < 16 * cb.dtiles; x += 128)
+#pragma unroll
+        for (uint32_t r = tid >> 5; r < kChunk; r += 16) {
+            const uint64_t at = (uint64_t)min(r, live - 1) * dm.in_ld + min(x, d - 4);
+            float4_t qv = *(const float4_t *)(qp + at), kv = *(const float4_t *)(kp + at);
+            if (x >= d) qv = kv = float4_t{0.f, 0.f, 0.f, 0.f};
+            *(float4_t *)(ql + r * LD + x) = qv;
+            *(float4_t *)(kl + r * LD + x) = kv;
+        }
+    if (wave == W - 1) {
         const ChunkGates cg = chunk_gates(p, dm, pr, h, lane, live);
         const double m0 = (double)cb.m0[unit * (cb.chunks + 1) + chunk], top = fmax(m0, cg.top);
         rs[lane] = -top;  // F - m
@@ -264,53 +295,64 @@ __global__ __launch_bounds__(256) void memory_read_kernel(const float *__restric
         floor_[lane] = expf((float)-(cg.F + top));
         if (chunk == cb.chunks - 1 && lane == 0) st.m[unit] = cb.m0[unit * (cb.chunks + 1) + cb.chunks];
     }
-    // rows behind the end repeat the last one; dims behind the end are zero
-    auto row4 = [&](const float *base, uint32_t r, uint32_t dim) {
-        const float4_t v = *(const float4_t *)(base + (uint64_t)min(r, live - 1) * dm.in_ld + min(dim, d - 4));
-        return dim < d ? v : float4_t{0.f, 0.f, 0.f, 0.f};
-    };
+    __syncthreads();
+    auto operand = [&](const float *rows, uint32_t tile, uint32_t m) { return *(const float4_t *)(rows + (16 * tile + c) * LD + 16 * m + 4 * g); };
     // ---- Q S0
     float4_t acc[4][NCT];
 #pragma unroll
     for (int r = 0; r < 4; r++)
 #pragma unroll
         for (int t = 0; t < NCT; t++) acc[r][t] = float4_t{0.f, 0.f, 0.f, 0.f};
-    const float *sp = cb.s + ci * cb.dtiles * cb.etiles * 256 + lane * 4;
-    for (uint32_t m = 0; m < cb.dtiles; m++) {
-        float4_t q[4], s[NCT];
+    for (uint32_t m0 = 0; m0 < cb.dtiles; m0 += 4)
 #pragma unroll
-        for (int t = 0; t < NCT; t++) s[t] = *(const float4_t *)(sp + (m * cb.etiles + min(wave + 4 * t, cb.etiles - 1)) * 256);
+        for (int q = 0; q < 4; q++) {
+            const uint32_t m = m0 + q;
+            if (m >= cb.dtiles) break;
 #pragma unroll
-        for (int r = 0; r < 4; r++) q[r] = row4(qp, 16 * r + c, 16 * m + 4 * g);
+            for (int r = 0; r < 4; r++) {
+                const float4_t a = operand(ql, r, m);
 #pragma unroll
-        for (int t = 0; t < NCT; t++)
-#pragma unroll
-            for (int r = 0; r < 4; r++) acc[r][t] = mfma4(q[r], s[t], acc[r][t]);
-    }
-    // ---- q . n0, four threads a row
+                for (int t = 0; t < NCT; t++) acc[r][t] = mfma4(a, s[q][t], acc[r][t]);
+            }
+            if (m + 4 < cb.dtiles) sload(m + 4, s[q]);
+        }
+    // ---- q . n0, eight threads a row
     {
         const float *n0 = cb.n + ci * d;
         float dot = 0.f;
-        for (uint32_t dim = 4 * (tid & 3); dim < d; dim += 16) {
-            const float4_t q = row4(qp, tid >> 2, dim), v = *(const float4_t *)(n0 + dim);
-            dot = fmaf(q[0], v[0], dot); dot = fmaf(q[1], v[1], dot); dot = fmaf(q[2], v[2], dot); dot = fmaf(q[3], v[3], dot);
+        for (uint32_t dim = 4 * (tid & 7); dim < d; dim += 32) {
+            const float4_t q = *(const float4_t *)(ql + (tid >> 3) * LD + dim), x = *(const float4_t *)(n0 + dim);
+            dot = fmaf(q[0], x[0], dot); dot = fmaf(q[1], x[1], dot); dot = fmaf(q[2], x[2], dot); dot = fmaf(q[3], x[3], dot);
         }
-        dot += dpp_f32<DPP_QUAD_XOR1>(dot);
-        dot += dpp_f32<DPP_QUAD_XOR2>(dot);
-        if ((tid & 3) == 0) qn[tid >> 2] = dot;
+        dot = group_sum<8>(dot);
+        if ((tid & 7) == 0) qn[tid >> 3] = dot;
+    }
+    // ---- scores up to the diagonal: ten 16 x 16 tiles over the eight waves, then weighted
+    auto tile_of = [](uint32_t idx, uint32_t &r, uint32_t &t) {
+        r = idx < 1 ? 0 : idx < 3 ? 1 : idx < 6 ? 2 : 3;
+        t = idx - r * (r + 1) / 2;
+    };
+    float4_t sc[2];
+#pragma unroll
+    for (int u = 0; u < 2; u++) {
+        sc[u] = float4_t{0.f, 0.f, 0.f, 0.f};
+        if (wave + W * u >= 10) continue;
+        uint32_t r, t;
+        tile_of(wave + W * u, r, t);
+        for (uint32_t m = 0; m < cb.dtiles; m++) sc[u] = mfma4(operand(ql, r, m), operand(kl, t, m), sc[u]);
     }
     __syncthreads();
-    // ---- weighted scores up to the diagonal: ten 16 x 16 tiles over the four waves
-    for (uint32_t idx = wave; idx < 10; idx += 4) {
-        const uint32_t r = idx < 1 ? 0 : idx < 3 ? 1 : idx < 6 ? 2 : 3, t = idx - r * (r + 1) / 2;
-        float4_t s = {0.f, 0.f, 0.f, 0.f};
-        for (uint32_t m = 0; m < cb.dtiles; m++) s = mfma4(row4(qp, 16 * r + c, 16 * m + 4 * g), row4(kp, 16 * t + c, 16 * m + 4 * g), s);
+#pragma unroll
+    for (int u = 0; u < 2; u++) {
+        if (wave + W * u >= 10) continue;
+        uint32_t r, t;
+        tile_of(wave + W * u, r, t);
         const uint32_t j = 16 * t + c;
         const double aj = as[j];
 #pragma unroll
         for (int i = 0; i < 4; i++) {
             const uint32_t ri = 16 * r + 4 * g + i;
-            const float w = j <= ri ? qs * expf((float)(rs[ri] + aj)) * s[i] : 0.f;
+            const float w = j <= ri ? qs * expf((float)(rs[ri] + aj)) * sc[u][i] : 0.f;
             pl[ri * PLD + j] = w;
             const float sum = group_sum<16>(w);
             if (c == 0) psum[t][ri] = sum;
@@ -322,6 +364,14 @@ __global__ __launch_bounds__(256) void memory_read_kernel(const float *__restric
 #pragma unroll
         for (int t = 0; t < NCT; t++) acc[r][t] *= f;
     }
+    float4_t gate[4][NCT];
+#pragma unroll
+    for (int r = 0; r < 4; r++)
+#pragma unroll
+        for (int t = 0; t < NCT; t++)
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+                gate[r][t][i] = p[(uint64_t)min(16u * r + 4 * g + i, live - 1) * dm.in_ld + dm.gate_off() + h * e + min(16 * (wave + W * t) + c, e - 1)];
     __syncthreads();
     if (tid < kChunk) {
         float nq = qn[tid] * carry[tid];
@@ -330,19 +380,13 @@ __global__ __launch_bounds__(256) void memory_read_kernel(const float *__restric
     }
     // ---- P V
 #pragma unroll
-    for (int m = 0; m < 4; m++) {
-        float4_t pa[4];
+    for (int m = 0; m < 4; m++)
 #pragma unroll
-        for (int r = m; r < 4; r++) pa[r] = *(const float4_t *)(pl + (16 * r + c) * PLD + 16 * m + 4 * g);
+        for (int r = m; r < 4; r++) {
+            const float4_t a = *(const float4_t *)(pl + (16 * r + c) * PLD + 16 * m + 4 * g);
 #pragma unroll
-        for (int t = 0; t < NCT; t++) {
-            float4_t v;
-#pragma unroll
-            for (int i = 0; i < 4; i++) v[i] = vp[(uint64_t)min(16u * m + 4 * g + i, live - 1) * dm.in_ld + min(16 * (wave + 4 * t) + c, e - 1)];
-#pragma unroll
-            for (int r = m; r < 4; r++) acc[r][t] = mfma4(pa[r], v, acc[r][t]);
+            for (int t = 0; t < NCT; t++) acc[r][t] = mfma4(a, v[m][t], acc[r][t]);
         }
-    }
     __syncthreads();
     // ---- normaliser, norm, gate
 #pragma unroll
@@ -352,31 +396,40 @@ __global__ __launch_bounds__(256) void memory_read_kernel(const float *__restric
 #pragma unroll
         for (int t = 0; t < NCT; t++) {
             acc[r][t] *= f;
-            if (16 * (wave + 4 * t) + c < e) s2 += acc[r][t] * acc[r][t];
+            if (16 * (wave + W * t) + c < e) s2 += acc[r][t] * acc[r][t];
         }
 #pragma unroll
         for (int i = 0; i < 4; i++) {
-            const float s = group_sum<16>(s2[i]);
-            if (c == 0) rsum[wave][16 * r + 4 * g + i] = s;
+            const float x = group_sum<16>(s2[i]);
+            if (c == 0) rsum[wave][16 * r + 4 * g + i] = x;
         }
     }
     __syncthreads();
+    if (tid < kChunk) {  // (dinv has been used: the root mean square's inverse takes its place)
+        float x = 0.f;
 #pragma unroll
-    for (int r = 0; r < 4; r++)
+        for (uint32_t w = 0; w < W; w++) x += rsum[w][tid];
+        dinv[tid] = 1.0f / sqrtf(x / (float)e + pr.eps);
+    }
+    __syncthreads();
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const uint32_t ri = 16 * r + 4 * g + i;
-            if (ri >= live) continue;
-            const float f = 1.0f / sqrtf(((rsum[0][ri] + rsum[1][ri]) + (rsum[2][ri] + rsum[3][ri])) / (float)e + pr.eps);
+    for (int t = 0; t < NCT; t++) {
+        const uint32_t col = 16 * (wave + W * t) + c;
+        if (col >= e) continue;
+        const float w = pr.norm[h * e + col];
 #pragma unroll
-            for (int t = 0; t < NCT; t++) {
-                const uint32_t col = 16 * (wave + 4 * t) + c;
-                if (col >= e) continue;
-                const float o = acc[r][t][i] * f * pr.norm[h * e + col] * fast_sigmoid(p[(uint64_t)ri * dm.in_ld + dm.gate_off() + h * e + col]);
+        for (int r = 0; r < 4; r++) {
+            const float4_t f = *(const float4_t *)(dinv + 16 * r + 4 * g);
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const uint32_t ri = 16 * r + 4 * g + i;
+                if (ri >= live) continue;
+                const float o = acc[r][t][i] * f[i] * w * fast_sigmoid(gate[r][t][i]);
                 if (out) out[((row0 + ri) * H + h) * e + col] = o;
                 if (out_lp) out_lp[(row0 + ri) * lp_ld + h * e + col] = f32_to_lp_bits(o, lp_bf16);
             }
         }
+    }
 }
 
 // ---------------------------------------------------------------- token by token
@@ -498,14 +551,16 @@ int launch_memory_prompt(const float *proj, const MemoryDims &dm, const MemoryPa
             const dim3 cgrid((unsigned)ceil_div(cb.dtiles * cb.etiles * 64 + dm.d + 1, 256), dm.heads, (unsigned)batch);
             hipLaunchKernelGGL(memory_carry_kernel, cgrid, dim3(256), 0, st, dm, state, cb);
             const dim3 rgrid(cb.chunks, dm.heads, (unsigned)batch);
-#define COEUS_MR(NV) \
-    hipLaunchKernelGGL(memory_read_kernel<NV>, rgrid, dim3(256), 0, st, proj, dm, pr, state, n, t0, seg, cb, out, lp, lp_ld, lp_bf)
-            switch (ceil_div(cb.etiles, 4)) {
-                case 1: COEUS_MR(1); break;
-                case 2: COEUS_MR(2); break;
-                case 3: COEUS_MR(3); break;
-                default: COEUS_MR(4); break;
-            }
+#define COEUS_MR(NV)                                                                                                              \
+    do {                                                                                                                          \
+        static const bool once = hipFuncSetAttribute((const void *)memory_read_kernel<NV>, hipFuncAttributeMaxDynamicSharedMemorySize, \
+                                                     136 * 1024) == hipSuccess;                                                   \
+        (void)once;                                                                                                               \
+        hipLaunchKernelGGL(memory_read_kernel<NV>, rgrid, dim3(512), read_lds_bytes(dm), st, proj, dm, pr, state, n, t0, seg, cb, out, lp, \
+                           lp_ld, lp_bf);                                                                                         \
+    } while (0)
+            if (cb.etiles <= 8) COEUS_MR(1);
+            else COEUS_MR(2);
 #undef COEUS_MR
         }
         COEUS_HIP(hipGetLastError());
