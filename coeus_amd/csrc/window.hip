@@ -122,7 +122,7 @@ __global__ __launch_bounds__(256) void window_attn_kernel(const void *__restrict
 // multiplied by the key's inverse root mean square and lose slope * distance, outputs meet their gate.
 
 template <int DK, int DV, bool SHARED>
-__global__ __launch_bounds__(256) void window_prefill_kernel(const uint16_t *__restrict__ q, uint64_t q_ld,
+__global__ __launch_bounds__(256, DK + DV <= 256 ? 2 : 1) void window_prefill_kernel(const uint16_t *__restrict__ q, uint64_t q_ld,
                                                              const uint16_t *__restrict__ kv, uint64_t kv_ld,
                                                              WindowShape dm, uint32_t n, uint32_t hist,
                                                              float *__restrict__ out, uint16_t *__restrict__ out_lp,
@@ -130,7 +130,7 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(const uint16_t *__r
     constexpr int KT = 32, KLD = DK + 8, VLD = 36, NKS = DK / 16, NDT = DV / 32, KP = DK / 64, VP = (DV + 127) / 128;
     extern __shared__ __attribute__((aligned(16))) uint16_t lds16[];
     uint16_t *const ks = lds16, *const vt = lds16 + 2 * KT * KLD;  // [2][key][dim], [2][dim][key]
-    float *const rl = (float *)(vt + 2 * DV * VLD);                // SHARED: [2][key] inverse root mean squares
+    float *const rl = (float *)(vt + 2 * DV * VLD);                // SHARED: [2][key] scale / root mean square
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, qi = lane & 31, hf = lane >> 5;
     uint32_t qt, h;
     prefill_tile_of_block(qt, h);
@@ -198,7 +198,7 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(const uint16_t *__r
     };
     auto lstore = [&](uint32_t buf) {
         if (SHARED) {
-            if (tid < KT) rl[buf * KT + tid] = rr;
+            if (tid < KT) rl[buf * KT + tid] = scale2 * rr;
         } else {
             kstore(buf, 0, rk0);
             if (KP > 1) kstore(buf, 1, rk1);
@@ -231,14 +231,20 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(const uint16_t *__r
         for (int s = 0; s < NKS; s++)
             sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*(const bf16x8_t *)(kt_ + qi * KLD + 16 * s + 8 * hf), qf[s], sc, 0, 0, 0);
         float tmax = -INFINITY;
+        if (SHARED) {
+            // register i holds key k0 + 4 hf + 8 (i / 4) + i % 4
+            const float near = slope2 * (float)(int)(k0 + 4 * hf - qkey);
 #pragma unroll
-        for (int i = 0; i < 16; i++) {
-            if (SHARED) {
-                const uint32_t kl = 4 * hf + 8 * (i >> 2) + (i & 3);
-                sc[i] = fmaf(sc[i], scale2 * rl[(t & 1) * KT + kl], -slope2 * (float)(int)(qkey - k0 - kl));
-            } else {
-                sc[i] *= scale2;
+            for (int j = 0; j < 4; j++) {
+                const float4 f = *(const float4 *)(rl + (t & 1) * KT + 4 * hf + 8 * j);
+                sc[4 * j] = fmaf(sc[4 * j], f.x, fmaf(slope2, 8.f * j, near));
+                sc[4 * j + 1] = fmaf(sc[4 * j + 1], f.y, fmaf(slope2, 8.f * j + 1.f, near));
+                sc[4 * j + 2] = fmaf(sc[4 * j + 2], f.z, fmaf(slope2, 8.f * j + 2.f, near));
+                sc[4 * j + 3] = fmaf(sc[4 * j + 3], f.w, fmaf(slope2, 8.f * j + 3.f, near));
             }
+        } else {
+#pragma unroll
+            for (int i = 0; i < 16; i++) sc[i] *= scale2;
         }
         if (k0 + KT - 1 > wave_lo || (wave_hi >= W && k0 <= wave_hi - W)) {  // an edge crosses the tile
 #pragma unroll
