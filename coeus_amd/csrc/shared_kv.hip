@@ -108,7 +108,6 @@ __global__ __launch_bounds__(256) void shared_kv_decode_kernel(const float *__re
     constexpr float kLog2e = 1.4426950408889634f;
     __shared__ float2 sh[4];
     __shared__ float sm[4][HB], sl[4][HB], sacc[4][HB][DP];
-    __shared__ float rm[HB][kMaxShares], rl[HB][kMaxShares];
     __shared__ uint32_t is_last;
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, share = blockIdx.x, shares = gridDim.x;
     const uint32_t H = dm.heads, G = dm.kv_heads, d = dm.d, hpg = H / G, kvh = blockIdx.y / hblocks, hb0 = blockIdx.y % hblocks * HB;
@@ -147,7 +146,27 @@ __global__ __launch_bounds__(256) void shared_kv_decode_kernel(const float *__re
             for (int t = 0; t < 8; t++) v[t] = __uint_as_float(w[t]);
         }
     };
-    // the first tile is requested before the position is known (slots not written yet hold finite values)
+    // eight floats of a row of the projection or of the weights, the lane's dims of one head (zeros behind the end)
+    auto dims = [&](const float *row, float (&v)[8]) {
+        if (VEC) {
+            const float4 v0 = *(const float4 *)(row + dc), v1 = *(const float4 *)(row + dc + 4);
+            v[0] = v0.x; v[1] = v0.y; v[2] = v0.z; v[3] = v0.w; v[4] = v1.x; v[5] = v1.y; v[6] = v1.z; v[7] = v1.w;
+        } else {
+#pragma unroll
+            for (int t = 0; t < 8; t++) v[t] = row[min(d0 + t, d - 1)];
+        }
+    };
+    // The projection is requested first (loads return in order and it is at hand), then the first tile, before the
+    // position is known (slots not written yet hold finite values).
+    const float sq_q = squares_256<VEC>(p, H * d), sq_k = squares_256<VEC>(p + dm.k_off(), G * d);
+    float q[HB][8], wq[HB][8], slope[HB];
+#pragma unroll
+    for (int j = 0; j < HB; j++) {
+        const uint32_t h = h0 + min((uint32_t)j, nh - 1);
+        slope[j] = dm.slope_range == 0.f ? 0.f : kLog2e * exp2f(-dm.slope_range * (float)(h + 1) / (float)H);
+        dims(p + h * d, q[j]);
+        dims(wqk + h * d, wq[j]);
+    }
     uint32_t base = k_begin + wave * U * KPW;
     Raw x[U];
     float r[U];
@@ -155,19 +174,12 @@ __global__ __launch_bounds__(256) void shared_kv_decode_kernel(const float *__re
     for (int u = 0; u < U; u++) request(base + u * KPW + sub, x[u], r[u]);
     const uint32_t pos = *pos_dev, fresh = pos % cap, nv = min(pos < 0xffffffffu ? pos + 1 : pos, cap), k_end = min(nv, k_lim);
     // norms over the whole projections
-    const float2 sq = sum2_256(squares_256<VEC>(p, H * d), squares_256<VEC>(p + dm.k_off(), G * d), sh);
+    const float2 sq = sum2_256(sq_q, sq_k, sh);
     const float rq = kLog2e * dm.scale / sqrtf(sq.x / (float)(H * d) + eps), rk = 1.0f / sqrtf(sq.y / (float)(G * d) + eps);
-    float q[HB][8], slope[HB];
 #pragma unroll
-    for (int j = 0; j < HB; j++) {
-        const uint32_t h = h0 + min((uint32_t)j, nh - 1);
-        slope[j] = dm.slope_range == 0.f ? 0.f : kLog2e * exp2f(-dm.slope_range * (float)(h + 1) / (float)H);
+    for (int j = 0; j < HB; j++)
 #pragma unroll
-        for (int t = 0; t < 8; t++) {
-            const uint32_t at = h * d + min(d0 + t, d - 1);
-            q[j][t] = d0 + t < d ? p[at] * rq * wqk[at] : 0.f;  // (base 2 scores)
-        }
-    }
+        for (int t = 0; t < 8; t++) q[j][t] = d0 + t < d ? q[j][t] * rq * wq[j][t] : 0.f;  // (base 2 scores)
     float m[HB], l[HB], acc[HB][8];
 #pragma unroll
     for (int j = 0; j < HB; j++) {
@@ -185,9 +197,9 @@ __global__ __launch_bounds__(256) void shared_kv_decode_kernel(const float *__re
                 const uint64_t at = (b * cap + key) * RL;
                 float nk[8];
                 uint32_t w[8];
+                dims(p + dm.k_off() + kvh * d, nk);
 #pragma unroll
                 for (int t = 0; t < 8; t++) {
-                    nk[t] = p[dm.k_off() + kvh * d + min(d0 + t, d - 1)];
                     w[t] = BF16 ? (uint32_t)f32_to_bf16_bits(nk[t]) : __float_as_uint(nk[t]);
                     if (hb0 == 0 && d0 + t < d) {
                         if (BF16) ((uint16_t *)ring)[at + kvh * d + d0 + t] = (uint16_t)w[t];
@@ -300,28 +312,31 @@ __global__ __launch_bounds__(256) void shared_kv_decode_kernel(const float *__re
     __syncthreads();
     if (!is_last) return;
     const float *rec = part + (b * H + h0) * shares * (d + 2);
-    for (uint32_t it = tid; it < nh * shares; it += 256) {
-        const float *q0 = rec + (uint64_t)it * (d + 2);
-        rm[it / shares][it % shares] = __hip_atomic_load(q0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-        rl[it / shares][it % shares] = __hip_atomic_load(q0 + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-    }
-    __syncthreads();
     for (uint32_t it = tid; it < nh * d; it += 256) {
         const uint32_t j = it / d, c = it % d;
-        const float *q0 = rec + (uint64_t)j * shares * (d + 2) + 2 + c;
-        float mm = rm[j][0];
-        for (uint32_t s = 1; s < shares; s++) mm = fmaxf(mm, rm[j][s]);
-        float lt = 0.f, a = 0.f;
-        for (uint32_t s0 = 0; s0 < shares; s0 += 16) {
-            float y[16];
+        const float *q0 = rec + (uint64_t)j * shares * (d + 2);
+        float mm = -INFINITY, lt = 0.f, a = 0.f;
+        for (uint32_t s0 = 0; s0 < shares; s0 += 16) {  // sixteen records in one trip
+            float ym[16], yl[16], y[16];
 #pragma unroll
-            for (uint32_t s = 0; s < 16; s++)
-                y[s] = __hip_atomic_load(q0 + (uint64_t)min(s0 + s, shares - 1) * (d + 2), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+            for (uint32_t s = 0; s < 16; s++) {
+                const float *qs = q0 + (uint64_t)min(s0 + s, shares - 1) * (d + 2);
+                ym[s] = __hip_atomic_load(qs, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+                yl[s] = __hip_atomic_load(qs + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+                y[s] = __hip_atomic_load(qs + 2 + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+            }
+            float top = mm;
+#pragma unroll
+            for (uint32_t s = 0; s < 16; s++) top = fmaxf(top, ym[s]);
+            const float corr = __builtin_amdgcn_exp2f(mm - top);
+            lt *= corr;
+            a *= corr;
+            mm = top;
 #pragma unroll
             for (uint32_t s = 0; s < 16; s++) {
                 if (s0 + s >= shares) break;
-                const float f = __builtin_amdgcn_exp2f(rm[j][s0 + s] - mm);
-                lt = fmaf(rl[j][s0 + s], f, lt);
+                const float f = __builtin_amdgcn_exp2f(ym[s] - mm);
+                lt = fmaf(yl[s], f, lt);
                 a = fmaf(y[s], f, a);
             }
         }
